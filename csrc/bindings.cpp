@@ -97,7 +97,14 @@ int dllm_gqa_tile_tokens(int, int, int);
 int dllm_gqa_mfma_ok(int, int, int, int, int, int);
 int dllm_paged_gqa(const void*, const void*, const void*, int, const int*, int, int, const int*, const int*, const int*,
                    const int*, const int*, int, const void*, long, void*, int, int, int, int, int, int, float*, int, int, int,
-                   int, float, hipStream_t);
+                   int, float, int, float, const float*, long, hipStream_t);
+int dllm_rope_prep(const void*, long, int, int, int, int, int, const float*, int, int, float, const int*, const int*, void*, void*,
+                   void*, long, int, int, int, void*, long, void*, long, int, hipStream_t);
+int dllm_latent_prep(const void*, long, int, int, int, const float*, float, const int*, void*, int, int, void*, long, long,
+                     hipStream_t);
+int dllm_gate_heads(const void*, int, const void*, long, void*, long, int, int, long, hipStream_t);
+int dllm_scaled_resadd_rms(const void*, long, int, float, int, const float*, float*, const float*, void*, long, long, int, float,
+                           hipStream_t);
 int dllm_relu2_scale(const void*, int, const float*, int, int, void*, long, int, hipStream_t);
 int dllm_dense_gate(const int*, const float*, float*, long, int, int, hipStream_t);
 int dllm_latent_kv_write(const void*, long, int, int, int, const float*, float, const int*, const float*, int, const int*,
@@ -1676,7 +1683,8 @@ void attn_prep(torch::Tensor proj, int64_t H, int64_t G, int64_t d, int64_t dv, 
 void paged_gqa_attention(torch::Tensor q, torch::Tensor kc, torch::Tensor vc, torch::Tensor bt, torch::Tensor qstart,
                          torch::Tensor qlen, torch::Tensor ctx, torch::Tensor tile_seq, torch::Tensor tile_tok0,
                          c10::optional<torch::Tensor> gate, torch::Tensor out, bool mfma, int64_t splits,
-                         c10::optional<torch::Tensor> part, int64_t window, int64_t keep_first, double sink) {
+                         c10::optional<torch::Tensor> part, int64_t window, int64_t keep_first, double sink, int64_t chunk,
+                         double cap, c10::optional<torch::Tensor> sinks) {
   const bool f = act_f32(q, "q");
   TORCH_CHECK(keep_first >= 0 && sink >= 0.0, "keep_first >= 0, sink >= 0");
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous(), "q [T, H, d]");
@@ -1707,9 +1715,16 @@ void paged_gqa_attention(torch::Tensor q, torch::Tensor kc, torch::Tensor vc, to
     ldg = gate->stride(0);
   }
   const bool of32 = out.scalar_type() == torch::kFloat32;
-  TORCH_CHECK(out.is_cuda() && (of32 || out.scalar_type() == q.scalar_type()) && out.is_contiguous() && out.dim() == 2 &&
-                  out.size(0) == T && out.size(1) == H * dv,
+  check_rows2d(out, "out");      // may be the first columns of a wider matrix
+  TORCH_CHECK(out.is_cuda() && (of32 || out.scalar_type() == q.scalar_type()) && out.size(0) == T && out.size(1) == H * dv,
               "out [T, H dv] in the dtype of q or f32");
+  TORCH_CHECK(chunk >= 0 && cap >= 0.0 && !(chunk > 0 && window > 0), "chunk >= 0 (not beside a window), cap >= 0");
+  const float* sk = nullptr;
+  if (sinks) {
+    check_f32(*sinks, "sinks");
+    TORCH_CHECK(sinks->is_contiguous() && sinks->numel() == H && sink == 0.0, "sinks [H] f32, instead of a sink weight");
+    sk = sinks->data_ptr<float>();
+  }
   float* pptr = nullptr;
   TORCH_CHECK(splits >= 1 && splits <= 64 && (splits == 1 || mfma), "key splits: 1..64, matrix-core kernel only");
   if (splits > 1) {
@@ -1722,9 +1737,120 @@ void paged_gqa_attention(torch::Tensor q, torch::Tensor kc, torch::Tensor vc, to
                                 (int)kc.size(2), qstart.data_ptr<int>(), qlen.data_ptr<int>(), ctx.data_ptr<int>(),
                                 tile_seq.data_ptr<int>(), tile_tok0.data_ptr<int>(), (int)tile_seq.numel(), gp, ldg,
                                 out.data_ptr(), (int)H, (int)G, (int)d, (int)dv, (int)mfma, (int)splits, pptr, (int)window,
-                                (int)GV, (int)of32, (int)keep_first, (float)sink, stream());
+                                (int)GV, (int)of32, (int)keep_first, (float)sink, (int)chunk, (float)cap, sk,
+                                (long)out.stride(0), stream());
   TORCH_CHECK(rc != -2, "head widths do not fit the LDS");
   ok(rc, "paged_gqa_attention");
+}
+
+// ---- layers whose mixer and feed-forward read one norm and share projections (gqa.hip, latent.hip, seqmix.hip)
+// a [T, n] block of activations whose rows may be columns of a wider matrix
+static void act_rows(const torch::Tensor& t, const torch::Tensor& like, int64_t T, int64_t n, const char* what) {
+  check_rows2d(t, what);
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == like.scalar_type() && t.size(0) == T && t.size(1) == n, what,
+              ": wrong shape or dtype");
+}
+
+void rope_prep(torch::Tensor proj, int64_t H, int64_t G, int64_t d, int64_t dv, torch::Tensor cos_sin, int64_t rot, double qscale,
+               torch::Tensor pos, torch::Tensor slots, torch::Tensor kc, torch::Tensor vc, torch::Tensor q, int64_t ucol,
+               c10::optional<torch::Tensor> act, c10::optional<torch::Tensor> zero_rows) {
+  const bool f = act_f32(proj, "proj");
+  check_rows2d(proj, "proj");
+  check_f32(cos_sin, "cos_sin");
+  check_i32(pos, "positions");
+  check_i32(slots, "slots");
+  const int64_t T = proj.size(0);
+  TORCH_CHECK(H >= 1 && G >= 1 && H % G == 0 && proj.size(1) >= (H + G) * d + G * dv, "proj [T, (H + G) d + G dv + ...]");
+  TORCH_CHECK(cos_sin.dim() == 2 && cos_sin.is_contiguous() && rot >= 0 && rot % 2 == 0 && rot <= d &&
+                  (rot == 0 || cos_sin.size(1) >= rot),
+              "rotation table");
+  TORCH_CHECK(pos.numel() == T && slots.numel() == T, "positions / slots lengths");
+  for (auto* c : {&kc, &vc})
+    TORCH_CHECK(c->is_cuda() && c->scalar_type() == proj.scalar_type() && c->is_contiguous() && c->dim() == 4 && c->size(1) == G,
+                "paged caches K [blocks, G, block, d], V [blocks, G, dv, block] in the activations' dtype");
+  TORCH_CHECK(kc.size(3) == d && vc.size(2) == dv && kc.size(0) == vc.size(0) && kc.size(2) == vc.size(3), "cache widths");
+  TORCH_CHECK(q.is_cuda() && q.scalar_type() == proj.scalar_type() && q.is_contiguous() && q.numel() == T * H * d, "q [T, H, d]");
+  void *ap = nullptr, *zp = nullptr;
+  long lda = 0, ldz = 0;
+  int64_t ff = 0, zn = 0;
+  if (act) {
+    ff = act->size(1);
+    act_rows(*act, proj, T, ff, "act");
+    TORCH_CHECK(ff >= 1 && ucol >= 0 && ucol + ff <= proj.size(1), "up columns of proj");
+    ap = act->data_ptr();
+    lda = act->stride(0);
+  }
+  if (zero_rows) {
+    zn = zero_rows->size(1);
+    act_rows(*zero_rows, proj, T, zn, "zero_rows");
+    zp = zero_rows->data_ptr();
+    ldz = zero_rows->stride(0);
+  }
+  ok(dllm_rope_prep(proj.data_ptr(), proj.stride(0), f, (int)H, (int)G, (int)d, (int)dv, cos_sin.data_ptr<float>(),
+                    (int)cos_sin.size(1), (int)rot, (float)qscale, pos.data_ptr<int>(), slots.data_ptr<int>(), kc.data_ptr(),
+                    vc.data_ptr(), q.data_ptr(), (long)T, (int)kc.size(2), (int)ucol, (int)ff, ap, lda, zp, ldz, (int)zn, stream()),
+     "rope_prep");
+}
+
+void latent_prep(torch::Tensor proj, int64_t ccol, torch::Tensor w, double eps, torch::Tensor slots, torch::Tensor cache,
+                 int64_t ucol, c10::optional<torch::Tensor> act) {
+  const bool f = act_f32(proj, "proj");
+  check_rows2d(proj, "proj");
+  check_f32(w, "norm weight");
+  check_i32(slots, "slots");
+  const int64_t T = proj.size(0), rank = w.numel();
+  TORCH_CHECK(w.is_contiguous() && rank >= 1 && ccol >= 0 && ccol + rank <= proj.size(1) && slots.numel() == T, "latent columns");
+  TORCH_CHECK(cache.is_cuda() && cache.scalar_type() == proj.scalar_type() && cache.is_contiguous() && cache.dim() == 3 &&
+                  cache.size(1) == 16 && cache.size(2) == rank,
+              "cache [blocks, 16, rank] in the activations' dtype");
+  void* ap = nullptr;
+  long lda = 0;
+  int64_t ff = 0;
+  if (act) {
+    ff = act->size(1);
+    act_rows(*act, proj, T, ff, "act");
+    TORCH_CHECK(ff >= 1 && ucol >= 0 && ucol + ff <= proj.size(1), "up columns of proj");
+    ap = act->data_ptr();
+    lda = act->stride(0);
+  }
+  ok(dllm_latent_prep(proj.data_ptr(), proj.stride(0), f, (int)ccol, (int)rank, w.data_ptr<float>(), (float)eps,
+                      slots.data_ptr<int>(), cache.data_ptr(), (int)ucol, (int)ff, ap, lda, (long)T, stream()),
+     "latent_prep");
+}
+
+void gate_heads(torch::Tensor o, torch::Tensor gate, torch::Tensor out) {
+  const bool f = act_f32(o, "o");
+  TORCH_CHECK(o.dim() == 3 && o.is_contiguous(), "o [H, T, dv] contiguous");
+  const int64_t H = o.size(0), T = o.size(1), dv = o.size(2);
+  act_rows(gate, o, T, H * dv, "gate");
+  act_rows(out, o, T, H * dv, "out");
+  ok(dllm_gate_heads(o.data_ptr(), f, gate.data_ptr(), gate.stride(0), out.data_ptr(), out.stride(0), (int)H, (int)dv, (long)T,
+                     stream()),
+     "gate_heads");
+}
+
+void scaled_resadd_rms(torch::Tensor x, c10::optional<torch::Tensor> y, double mult, bool set, c10::optional<torch::Tensor> vec,
+                       c10::optional<torch::Tensor> w, double eps, c10::optional<torch::Tensor> out) {
+  check_f32(x, "x");
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous(), "x [T, width] f32 contiguous");
+  const int64_t T = x.size(0), W = x.size(1);
+  TORCH_CHECK(out.has_value() || (y.has_value() && !w.has_value()), "nothing to do");
+  TORCH_CHECK(y.has_value() || !(set || vec.has_value()), "terms without y");
+  const torch::Tensor& like = out ? *out : *y;
+  const bool f = act_f32(like, "activations");
+  auto fvec = [&](const torch::Tensor& t, const char* what) {
+    check_f32(t, what);
+    TORCH_CHECK(t.is_contiguous() && t.numel() == W, what, ": [width] f32");
+    return t.data_ptr<float>();
+  };
+  const void* yp = nullptr;
+  void* op = nullptr;
+  long ldy = 0, ldo = 0;
+  if (y) { act_rows(*y, like, T, W, "y"); yp = y->data_ptr(); ldy = y->stride(0); }
+  if (out) { act_rows(*out, like, T, W, "out"); op = out->data_ptr(); ldo = out->stride(0); }
+  ok(dllm_scaled_resadd_rms(yp, ldy, f, (float)mult, set, vec ? fvec(*vec, "vec") : nullptr, x.data_ptr<float>(),
+                            w ? fvec(*w, "norm weight") : nullptr, op, ldo, (long)T, (int)W, (float)eps, stream()),
+     "scaled_resadd_rms");
 }
 
 // ---- differential attention, Mamba-2 / mLSTM recurrences, PolyNorm, grouped router (gqa.hip, outer_scan.hip, seqmix.hip)
@@ -2190,7 +2316,12 @@ PYBIND11_MODULE(_hip_kernels, m) {
   m.def("paged_gqa_attention", &paged_gqa_attention, py::arg("q"), py::arg("k_cache"), py::arg("v_cache"),
         py::arg("block_tables"), py::arg("qstart"), py::arg("qlen"), py::arg("ctx"), py::arg("tile_seq"),
         py::arg("tile_tok0"), py::arg("gate"), py::arg("out"), py::arg("mfma"), py::arg("splits") = 1,
-        py::arg("part") = py::none(), py::arg("window") = 0, py::arg("keep_first") = 0, py::arg("sink") = 0.0);
+        py::arg("part") = py::none(), py::arg("window") = 0, py::arg("keep_first") = 0, py::arg("sink") = 0.0,
+        py::arg("chunk") = 0, py::arg("cap") = 0.0, py::arg("sinks") = py::none());
+  m.def("rope_prep", &rope_prep);
+  m.def("latent_prep", &latent_prep);
+  m.def("gate_heads", &gate_heads);
+  m.def("scaled_resadd_rms", &scaled_resadd_rms);
   m.def("gqa_tile_tokens",
         [](int64_t H, int64_t G, bool mfma) { return (int64_t)dllm_gqa_tile_tokens((int)H, (int)G, (int)mfma); });
   m.def("gqa_mfma_ok", [](bool f32, int64_t H, int64_t G, int64_t d, int64_t dv, int64_t bs) {

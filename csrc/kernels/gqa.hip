@@ -24,9 +24,15 @@
 //               own LDS patch as bf16 hi + lo parts, so the weighted sum sees them to 16 bits of
 //               mantissa through two MFMAs.  Key blocks above a wave's newest row are skipped.
 //
-// Both attention kernels take a window (a row at position p sees keys p - win < j <= p), kept first
-// keys (j < keep stays visible at any distance; the tiles between the kept keys and the window are
-// not read) and a sink (one more term exp(0) times `sink` in the denominator, with no value).
+//   rope_prep   attention inputs without a q / k norm: rotate-half positions on the first `rot` dims, q
+//               times one scale; the launch also squares the relu of a feed-forward's up columns that
+//               the same projection made (latent_prep: the same beside a normed latent).
+//
+// Both attention kernels take a window (a row at position p sees keys p - win < j <= p) or a chunk (it
+// sees the keys of its own chunk of positions, [p - p % chunk, p]), kept first keys (j < keep stays
+// visible at any distance; the tiles between the kept keys and the window are not read), a soft cap on
+// the scores (cap tanh(s / cap)) and a sink: one more term of the denominator, with no value, either
+// exp(0) times `sink` or exp(sinks[head]).
 //
 // Cache layout: K [blocks, G, block, d], V [blocks, G, dv, block] (bf16 or f32 like the activations;
 // V is kept transposed inside its page because the weighted sum runs over keys); every score,
@@ -41,6 +47,15 @@ template <> __device__ __forceinline__ float ldf<float>(const float* p) { return
 template <typename T> __device__ __forceinline__ void stf(T* p, float v);
 template <> __device__ __forceinline__ void stf<u16>(u16* p, float v) { *p = f2bf(v); }
 template <> __device__ __forceinline__ void stf<float>(float* p, float v) { *p = v; }
+
+// The oldest key a row at position p sees (kept first keys apart): its window's, its chunk's, or 0.
+__device__ __forceinline__ int oldest_key(int p, int win, int chunk) {
+  return chunk > 0 ? p - p % chunk : (win > 0 ? max(0, p - win + 1) : 0);
+}
+// cap tanh(s / cap) = cap - 2 cap / (exp(2 s / cap) + 1); an overflowing exponential gives cap
+__device__ __forceinline__ float cap_fast(float s, float cap, float two_over_cap) {
+  return cap - 2.f * cap * __builtin_amdgcn_rcpf(__expf(s * two_over_cap) + 1.f);
+}
 
 template <typename T>
 __global__ void __launch_bounds__(256) attn_prep_kernel(const T* __restrict__ proj, long ld, int H, int G, int d, int dv,
@@ -221,6 +236,84 @@ __global__ void __launch_bounds__(256) proj_norm_prep_kernel(const T* __restrict
   }
 }
 
+// Squared relu of a row's up columns (this workgroup's share): act[i] = relu(up[i])^2.  vec: rows of whole
+// 16-byte vectors on both sides.
+template <typename T>
+__device__ __forceinline__ void act_share(const T* __restrict__ up, int ff, T* __restrict__ act, int part, int parts, int tid,
+                                          bool vec) {
+  for (int i = part * 256 + tid; i < ff; i += parts * 256) {
+    const float v = fmaxf(ldf(up + i), 0.f);
+    stf(act + i, v * v);
+  }
+}
+template <>
+__device__ __forceinline__ void act_share<u16>(const u16* __restrict__ up, int ff, u16* __restrict__ act, int part, int parts,
+                                               int tid, bool vec) {
+  if (vec) {
+    for (int i = 8 * (part * 256 + tid); i < ff; i += 8 * parts * 256) {
+      float f[8];
+      unpack8(ld16(up + i), f);
+#pragma unroll
+      for (int x = 0; x < 8; ++x) { f[x] = fmaxf(f[x], 0.f); f[x] *= f[x]; }
+      st16(act + i, pack8(f));
+    }
+    return;
+  }
+  for (int i = part * 256 + tid; i < ff; i += parts * 256) {
+    const float v = fmaxf(bf2f(up[i]), 0.f);
+    act[i] = f2bf(v * v);
+  }
+}
+
+// Attention inputs without a q / k norm, and the activation of a feed-forward that shares the
+// projection.  proj row: q (H d) | k (G d) | v (G dv) | ...; a wave per q / k head: rotate-half
+// positions on the first `rot` dims (cos and sin as the table holds them), q times qscale; k and v to
+// their page slots.  act (null: no feed-forward): act[tok] = relu(proj[tok, ucol : ucol + ff])^2.
+// zrow: the first zn columns of this token's row are cleared (an attention output whose padding rows
+// no tile writes).
+template <typename T>
+__global__ void __launch_bounds__(256) rope_prep_kernel(const T* __restrict__ proj, long ld, int H, int G, int d, int dv,
+                                                        const float* __restrict__ cos_sin, int tab_w, int rot, float qscale,
+                                                        const int* __restrict__ pos, const int* __restrict__ slots,
+                                                        T* __restrict__ kc, T* __restrict__ vc, T* __restrict__ q, int BSZ,
+                                                        int ucol, int ff, T* __restrict__ act, long lda, int vec,
+                                                        T* __restrict__ zrow, long ldz, int zn) {
+  const long tok = blockIdx.x;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const T* r = proj + tok * ld;
+  const int slot = slots[tok];
+  const long blk = slot >= 0 ? slot / BSZ : 0;
+  const int off = slot >= 0 ? slot % BSZ : 0;
+  const int half = rot >> 1;
+  const float* cs = cos_sin + (long)pos[tok] * tab_w;
+  if (zrow)
+    for (int i = blockIdx.y * 256 + tid; i < zn; i += gridDim.y * 256) stf(zrow + tok * ldz + i, 0.f);
+  for (int hh = blockIdx.y * 4 + wave; hh < H + G; hh += gridDim.y * 4) {   // q heads, then k heads
+    const bool is_q = hh < H;
+    if (!is_q && slot < 0) continue;
+    const T* x = r + (long)hh * d;
+    T* dst = is_q ? q + (tok * H + hh) * d : kc + ((blk * G + (hh - H)) * BSZ + off) * d;
+    const float os = is_q ? qscale : 1.f;
+    for (int i = lane; i < d; i += 64) {
+      float v = ldf(x + i);
+      if (i < rot) {
+        const bool first = i < half;
+        const int f = first ? i : i - half;
+        const float c = cs[f], sn = cs[half + f];
+        const float p = ldf(x + (first ? i + half : i - half));
+        v = first ? v * c - p * sn : v * c + p * sn;
+      }
+      stf(dst + i, v * os);
+    }
+  }
+  if (slot >= 0) {   // values: this workgroup's share of the G * dv entries
+    const T* v = r + (long)(H + G) * d;
+    for (int i = blockIdx.y * 256 + tid; i < G * dv; i += gridDim.y * 256)
+      vc[((blk * G + i / dv) * dv + i % dv) * BSZ + off] = v[i];
+  }
+  if (act) act_share<T>(r + ucol, ff, act + tok * lda, blockIdx.y, gridDim.y, tid, vec);
+}
+
 // a [T, G, 2, R, dv] f32 (the two maps' outputs) -> out [T, G R, dv] = unit-RMS(a1 - lam a2) * scale:
 // one wave per (token, head)
 template <typename T>
@@ -253,10 +346,11 @@ __global__ void __launch_bounds__(256) paged_gqa_kernel(const T* __restrict__ q,
                                                         const int* __restrict__ tile_seq, const int* __restrict__ tile_tok0,
                                                         const T* __restrict__ gate, long ldg, T* __restrict__ out, int H,
                                                         int G, int d, int dv, int TQ, int KT, int win, int GV,
-                                                        float* __restrict__ out32, int keep, float sink) {
-  // win > 0: a row at position p sees keys p - win < j <= p, and keys j < keep.  GV value heads: key
-  // head g reads value head g / (G / GV).  out32: the output stays f32.  sink: one more term of score 0
-  // and that weight in the denominator.
+                                                        float* __restrict__ out32, int keep, float sink, int chunk,
+                                                        float cap, const float* __restrict__ sinks, long ldo) {
+  // win > 0: a row at position p sees keys p - win < j <= p, and keys j < keep; chunk > 0: keys of its
+  // own chunk.  GV value heads: key head g reads value head g / (G / GV).  out32: the output stays f32.
+  // sink: one more term of score 0 and that weight in the denominator; sinks: of score sinks[head].
   extern __shared__ float sm[];
   const int s = tile_seq[blockIdx.x];
   const int n = qlen[s];
@@ -280,20 +374,21 @@ __global__ void __launch_bounds__(256) paged_gqa_kernel(const T* __restrict__ q,
     Qs[e] = v;
   }
   float m[4], l[4], O[4][NJ];
-  int rpos[4];
+  int rpos[4], rlo[4];
 #pragma unroll
   for (int x = 0; x < 4; ++x) {
     const int rr = wave + 4 * x;
     m[x] = -INFINITY;
     l[x] = 0.f;
     rpos[x] = rr < nrows ? p0 + tok0 + rr / Rh : -1;   // -1: sees no key
+    rlo[x] = rr < nrows ? oldest_key(rpos[x], win, chunk) : 0;
 #pragma unroll
     for (int jj = 0; jj < NJ; ++jj) O[x][jj] = 0.f;
   }
   const int last = p0 + tok0 + nq - 1;   // the newest key any row sees
   const int* btr = bt + (long)s * bt_ld;
   const int gv = g / (G / GV);
-  const int first = win > 0 ? max(0, p0 + tok0 - win + 1) : 0;   // the oldest key any row sees
+  const int first = oldest_key(p0 + tok0, win, chunk);   // the oldest key any row sees
   for (int k0 = (keep > 0 ? 0 : first / KT * KT); k0 <= last; k0 += KT) {
     if (k0 >= keep && k0 + KT <= first) continue;   // between the kept keys and the window (uniform in the workgroup)
     const int nk = min(KT, last + 1 - k0);
@@ -331,8 +426,8 @@ __global__ void __launch_bounds__(256) paged_gqa_kernel(const T* __restrict__ q,
     const int pk = k0 + lane;
 #pragma unroll
     for (int x = 0; x < 4; ++x) {
-      const bool vis = lane < nk && pk <= rpos[x] && (win <= 0 || pk > rpos[x] - win || pk < keep);
-      const float sv = vis ? sc[x] : -INFINITY;
+      const bool vis = lane < nk && pk <= rpos[x] && (pk >= rlo[x] || pk < keep);
+      const float sv = !vis ? -INFINITY : cap > 0.f ? cap * tanhf(sc[x] / cap) : sc[x];
       const float mn = fmaxf(m[x], wave_max(sv));
       float p = 0.f, f = 1.f;
       if (mn > -INFINITY) {
@@ -365,15 +460,15 @@ __global__ void __launch_bounds__(256) paged_gqa_kernel(const T* __restrict__ q,
     if (rr >= nrows) continue;
     const long tok = q0 + tok0 + rr / Rh;
     const int h = g * R + r0 + rr % Rh;
-    const float inv = 1.f / (l[x] + (sink > 0.f ? sink * expf(-m[x]) : 0.f));
+    const float inv = 1.f / (l[x] + (sinks ? expf(sinks[h] - m[x]) : sink > 0.f ? sink * expf(-m[x]) : 0.f));
 #pragma unroll
     for (int jj = 0; jj < NJ; ++jj) {
       const int jx = lane + 64 * jj;
       if (jx >= dv) continue;
       float o = O[x][jj] * inv;
       if (gate) o *= 1.f / (1.f + expf(-ldf(gate + tok * ldg + (long)h * dv + jx)));
-      if (out32) out32[tok * ((long)H * dv) + (long)h * dv + jx] = o;
-      else stf(out + tok * ((long)H * dv) + (long)h * dv + jx, o);
+      if (out32) out32[tok * ldo + (long)h * dv + jx] = o;
+      else stf(out + tok * ldo + (long)h * dv + jx, o);
     }
   }
 }
@@ -412,7 +507,8 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
                                                              const int* __restrict__ tile_tok0, const u16* __restrict__ gate,
                                                              long ldg, u16* __restrict__ out, int H, int G, int d, int dv,
                                                              int TQ, int splits, float* __restrict__ part, int win, int GV,
-                                                             float* __restrict__ out32, int keep, float sink) {
+                                                             float* __restrict__ out32, int keep, float sink, int chunk,
+                                                             float cap, const float* __restrict__ sinks, long ldo) {
   constexpr int DS = SZ / 32, VB = SZ / 16, NKB = GM_KT / 16;
   constexpr int KSTR = SZ + 8, VSTR = GM_KT + 8, PSTR = GM_KT + 8;
   extern __shared__ __attribute__((aligned(16))) unsigned char smraw[];
@@ -444,13 +540,14 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
       qa[st] = __builtin_bit_cast(bf16x8, v);
     }
   }
-  int rpos[4];
+  int rpos[4], rlo[4];
   float m[4], l[4];
   f32x4 acc[VB];
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int row = 16 * wave + 4 * g4 + i;
     rpos[i] = row < nrows ? p0 + tok0 + row / R : -1;     // -1: sees no key
+    rlo[i] = row < nrows ? oldest_key(rpos[i], win, chunk) : 0;
     m[i] = -INFINITY;
     l[i] = 0.f;
   }
@@ -459,8 +556,11 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
   const int wave_last = 16 * wave < nrows ? p0 + tok0 + (min(16 * wave + 15, nrows - 1)) / R : -1;
   // the oldest row of the wave; idle rows (past nrows) are masked, so a wave that has any never skips the mask
   const int wave_first = 16 * wave + 15 < nrows ? p0 + tok0 + (16 * wave) / R : -1;
-  // with a window: the wave's oldest live row (tiles wholly before its window are skipped)
-  const int wave_old = 16 * wave < nrows ? p0 + tok0 + (16 * wave) / R : 0x3fffffff;
+  // the oldest keys the wave's oldest and newest live rows see (a tile wholly before the first is
+  // skipped; one not before the second needs no mask at its old end)
+  const int wave_lo = 16 * wave < nrows ? oldest_key(p0 + tok0 + (16 * wave) / R, win, chunk) : 0;
+  const int wave_lo_last = wave_last >= 0 ? oldest_key(wave_last, win, chunk) : 0;
+  const float cap2 = cap > 0.f ? 2.f / cap : 0.f;
   const int last = p0 + tok0 + nq - 1;   // the newest key any row sees
   const int* btr = bt + (long)s * bt_ld;
   constexpr int KCH = SZ / 8;            // 16-byte chunks of a staged key row
@@ -500,10 +600,10 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
   };
   // small grids (decode steps) split a row's key tiles over `splits` workgroups; each leaves its
   // running maximum, sum and unnormalised output in `part`, gqa_combine merges them
-  const int tfirst = win > 0 ? max(0, p0 + tok0 - win + 1) / GM_KT : 0;   // the oldest tile of the window any row sees
+  const int tfirst = oldest_key(p0 + tok0, win, chunk) / GM_KT;   // the oldest tile of the window / chunk any row sees
   // kept first keys: their tiles come before the window's in the walk; tile number v of the walk is
   // tile v of the sequence for v < nkeep, else tile tfirst + v - nkeep
-  const int nkeep = win > 0 ? min(tfirst, (keep + GM_KT - 1) / GM_KT) : 0;
+  const int nkeep = min(tfirst, (keep + GM_KT - 1) / GM_KT);
   const int ntiles = last / GM_KT + 1 - tfirst + nkeep;
   const int vbeg = (int)((long)ntiles * blockIdx.z / splits);
   const int vend = (int)((long)ntiles * (blockIdx.z + 1) / splits);   // exclusive
@@ -523,7 +623,7 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     if (vt + 1 < vend) fetch(tile_k0(vt + 1));   // the next tile's loads fly under this tile's products
     __syncthreads();
     if (k0 > wave_last) continue;   // this wave's rows see nothing of the tile (the barriers above are uniform)
-    if (win > 0 && k0 >= keep && k0 + GM_KT - 1 <= wave_old - win) continue;   // ... or the tile lies before every row's window
+    if (k0 >= keep && k0 + GM_KT <= wave_lo) continue;   // ... or the tile lies before every row's window / chunk
     f32x4 sacc[NKB];
 #pragma unroll
     for (int kb = 0; kb < NKB; ++kb) {
@@ -537,16 +637,22 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
         }
       }
     }
+    if (cap > 0.f) {
+#pragma unroll
+      for (int kb = 0; kb < NKB; ++kb)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) sacc[kb][i] = cap_fast(sacc[kb][i], cap, cap2);
+    }
     float alpha[4];
     const int key0 = k0 + 4 * lr;
     // a tile below the wave's oldest row needs no mask (wave-uniform)
-    const bool full = k0 + GM_KT - 1 <= wave_first && (win <= 0 || k0 > wave_last - win);
+    const bool full = k0 + GM_KT - 1 <= wave_first && k0 >= wave_lo_last;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       float sv[NKB];
 #pragma unroll
       for (int kb = 0; kb < NKB; ++kb)
-        sv[kb] = (full || (key0 + kb <= rpos[i] && (win <= 0 || key0 + kb > rpos[i] - win || key0 + kb < keep)))
+        sv[kb] = (full || (key0 + kb <= rpos[i] && (key0 + kb >= rlo[i] || key0 + kb < keep)))
                      ? sacc[kb][i] : -INFINITY;
       float mx = fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]));
       mx = row16_max(mx);
@@ -608,15 +714,15 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     }
     const long tok = q0 + tok0 + row / R;
     const int h = g * R + row % R;
-    const float inv = 1.f / (lt + (sink > 0.f ? sink * __expf(-m[i]) : 0.f));
+    const float inv = 1.f / (lt + (sinks ? __expf(sinks[h] - m[i]) : sink > 0.f ? sink * __expf(-m[i]) : 0.f));
 #pragma unroll
     for (int cb = 0; cb < VB; ++cb) {
       const int jx = 16 * cb + lr;
       if (jx >= dv) continue;
       float o = acc[cb][i] * inv;
       if (gate) o *= 1.f / (1.f + expf(-bf2f(gate[tok * ldg + (long)h * dv + jx])));
-      if (out32) out32[tok * ((long)H * dv) + (long)h * dv + jx] = o;
-      else out[tok * ((long)H * dv) + (long)h * dv + jx] = f2bf(o);
+      if (out32) out32[tok * ldo + (long)h * dv + jx] = o;
+      else out[tok * ldo + (long)h * dv + jx] = f2bf(o);
     }
   }
 }
@@ -627,7 +733,8 @@ __global__ void __launch_bounds__(256) gqa_combine_kernel(const float* __restric
                                                           const int* __restrict__ tile_seq,
                                                           const int* __restrict__ tile_tok0, const u16* __restrict__ gate,
                                                           long ldg, u16* __restrict__ out, int H, int G, int dv, int TQ,
-                                                          float* __restrict__ out32, float sink) {
+                                                          float* __restrict__ out32, float sink,
+                                                          const float* __restrict__ sinks, long ldo) {
   const int s = tile_seq[blockIdx.x];
   const int n = qlen[s], tok0 = tile_tok0[blockIdx.x];
   if (n <= 0 || tok0 >= n) return;
@@ -642,9 +749,9 @@ __global__ void __launch_bounds__(256) gqa_combine_kernel(const float* __restric
     const float lz = lane < splits ? pr[lane * zs + 1] : 0.f;
     const float M = wave_max(mz);
     const float wz = mz > -INFINITY ? expf(mz - M) : 0.f;
-    const float L = wave_sum(lz * wz) + (sink > 0.f ? sink * expf(-M) : 0.f);
     const long tok = qstart[s] + tok0 + row / R;
     const int h = g * R + row % R;
+    const float L = wave_sum(lz * wz) + (sinks ? expf(sinks[h] - M) : sink > 0.f ? sink * expf(-M) : 0.f);
     for (int j0 = 0; j0 < dv; j0 += 64) {     // every lane stays in the loop: the shuffles read all lanes
       const int jx = j0 + lane;
       const bool on = jx < dv;
@@ -657,8 +764,8 @@ __global__ void __launch_bounds__(256) gqa_combine_kernel(const float* __restric
       if (!on) continue;
       o /= L;
       if (gate) o *= 1.f / (1.f + expf(-bf2f(gate[tok * ldg + (long)h * dv + jx])));
-      if (out32) out32[tok * ((long)H * dv) + (long)h * dv + jx] = o;
-      else out[tok * ((long)H * dv) + (long)h * dv + jx] = f2bf(o);
+      if (out32) out32[tok * ldo + (long)h * dv + jx] = o;
+      else out[tok * ldo + (long)h * dv + jx] = f2bf(o);
     }
   }
 }
@@ -680,10 +787,10 @@ template <typename T, int NJ>
 int launch_gqa(dim3 grid, long lds, hipStream_t st, const T* q, const T* kc, const T* vc, const int* bt, int bt_ld, int BSZ,
                const int* qstart, const int* qlen, const int* ctx, const int* tile_seq, const int* tile_tok0, const T* gate,
                long ldg, T* out, int H, int G, int d, int dv, int TQ, int KT, int win, int GV, float* out32, int keep,
-               float sink) {
+               float sink, int chunk, float cap, const float* sinks, long ldo) {
   ENSURE_LDS((paged_gqa_kernel<T, NJ>), lds);
   hipLaunchKernelGGL((paged_gqa_kernel<T, NJ>), grid, dim3(256), lds, st, q, kc, vc, bt, bt_ld, BSZ, qstart, qlen, ctx, tile_seq,
-                     tile_tok0, gate, ldg, out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink);
+                     tile_tok0, gate, ldg, out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo);
   return (int)hipGetLastError();
 }
 
@@ -691,8 +798,8 @@ template <typename T>
 int launch_gqa_t(int nj, dim3 grid, long lds, hipStream_t st, const void* q, const void* kc, const void* vc, const int* bt,
                  int bt_ld, int BSZ, const int* qstart, const int* qlen, const int* ctx, const int* tile_seq,
                  const int* tile_tok0, const void* gate, long ldg, void* out, int H, int G, int d, int dv, int TQ, int KT,
-                 int win, int GV, float* out32, int keep, float sink) {
-#define GQA(NJ) return launch_gqa<T, NJ>(grid, lds, st, (const T*)q, (const T*)kc, (const T*)vc, bt, bt_ld, BSZ, qstart, qlen, ctx, tile_seq, tile_tok0, (const T*)gate, ldg, (T*)out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink)
+                 int win, int GV, float* out32, int keep, float sink, int chunk, float cap, const float* sinks, long ldo) {
+#define GQA(NJ) return launch_gqa<T, NJ>(grid, lds, st, (const T*)q, (const T*)kc, (const T*)vc, bt, bt_ld, BSZ, qstart, qlen, ctx, tile_seq, tile_tok0, (const T*)gate, ldg, (T*)out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo)
   if (nj <= 1) GQA(1);
   if (nj <= 2) GQA(2);
   GQA(4);
@@ -731,10 +838,12 @@ extern "C" int dllm_gqa_tile_tokens(int H, int G, int mfma) {
 extern "C" int dllm_paged_gqa(const void* q, const void* kc, const void* vc, int f32, const int* bt, int bt_ld, int BSZ,
                               const int* qstart, const int* qlen, const int* ctx, const int* tile_seq, const int* tile_tok0,
                               int n_tiles, const void* gate, long ldg, void* out, int H, int G, int d, int dv, int mfma,
-                              int splits, float* part, int win, int GV, int out_f32, int keep, float sink, hipStream_t st) {
+                              int splits, float* part, int win, int GV, int out_f32, int keep, float sink, int chunk, float cap,
+                              const float* sinks, long ldo, hipStream_t st) {
   if (n_tiles <= 0) return 0;
+  if (chunk < 0 || (chunk > 0 && win > 0) || cap < 0.f || ldo < (long)H * dv) return -1;
   if (G < 1 || H % G || dv > 256 || d < 1 || GV < 1 || G % GV || win < 0 || keep < 0 || sink < 0.f) return -1;
-  if (win <= 0) keep = 0;     // without a window every key is seen anyway
+  if (win <= 0 && chunk <= 0) keep = 0;     // without a bound every key is seen anyway
   float* out32 = out_f32 ? (float*)out : nullptr;
   if (mfma) {
     if (!dllm_gqa_mfma_ok(f32, H, G, d, dv, BSZ)) return -1;
@@ -749,14 +858,14 @@ extern "C" int dllm_paged_gqa(const void* q, const void* kc, const void* vc, int
     ENSURE_LDS(paged_gqa_mfma_kernel<SZ>, lds);                                                                          \
     hipLaunchKernelGGL(paged_gqa_mfma_kernel<SZ>, grid, dim3(256), lds, st, (const u16*)q, (const u16*)kc, (const u16*)vc, bt, \
                        bt_ld, qstart, qlen, ctx, tile_seq, tile_tok0, (const u16*)gate, ldg, (u16*)out, H, G, d, dv, TQ, \
-                       splits, pp, win, GV, out32, keep, sink);                                                          \
+                       splits, pp, win, GV, out32, keep, sink, chunk, cap, sinks, ldo);                                                          \
   } while (0)
     if (sz <= 64) GQM(64); else if (sz <= 128) GQM(128); else GQM(256);
 #undef GQM
     if (pp) {
       const int rows = (TQ * (H / G) < GM_ROWS ? TQ * (H / G) : GM_ROWS);
       hipLaunchKernelGGL(gqa_combine_kernel, dim3(n_tiles, G, (rows + 3) / 4), dim3(256), 0, st, pp, splits, qstart, qlen,
-                         tile_seq, tile_tok0, (const u16*)gate, ldg, (u16*)out, H, G, dv, TQ, out32, sink);
+                         tile_seq, tile_tok0, (const u16*)gate, ldg, (u16*)out, H, G, dv, TQ, out32, sink, sinks, ldo);
     }
     return (int)hipGetLastError();
   }
@@ -770,9 +879,9 @@ extern "C" int dllm_paged_gqa(const void* q, const void* kc, const void* vc, int
   const int TQ = dllm_gqa_tile_tokens(H, G, 0);
   if (f32)
     return launch_gqa_t<float>(nj, grid, lds, st, q, kc, vc, bt, bt_ld, BSZ, qstart, qlen, ctx, tile_seq, tile_tok0, gate, ldg,
-                               out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink);
+                               out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo);
   return launch_gqa_t<u16>(nj, grid, lds, st, q, kc, vc, bt, bt_ld, BSZ, qstart, qlen, ctx, tile_seq, tile_tok0, gate, ldg, out,
-                           H, G, d, dv, TQ, KT, win, GV, out32, keep, sink);
+                           H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo);
 }
 
 extern "C" int dllm_qk_norm_prep(const void* proj, long ld, int f32, const float* bias, int H, int G, int M, int d, int dv,
@@ -818,5 +927,24 @@ extern "C" int dllm_proj_norm_prep(const void* proj, long ld, int f32, int H, in
   else
     hipLaunchKernelGGL(proj_norm_prep_kernel<u16>, grid, dim3(256), 0, st, (const u16*)proj, ld, H, G, d, dv, qw, kw, cos_sin,
                        tab_w, rot, inter, eps, qscale, vnorm, pos, slots, (u16*)kc, (u16*)vc, (u16*)q, BSZ, (u16*)zrow, zn);
+  return (int)hipGetLastError();
+}
+
+extern "C" int dllm_rope_prep(const void* proj, long ld, int f32, int H, int G, int d, int dv, const float* cos_sin, int tab_w,
+                              int rot, float qscale, const int* pos, const int* slots, void* kc, void* vc, void* q, long T,
+                              int BSZ, int ucol, int ff, void* act, long lda, void* zrow, long ldz, int zn, hipStream_t st) {
+  if (T <= 0) return 0;
+  if (rot < 0 || rot > d || (rot & 1) || rot > tab_w || H < 1 || G < 1 || H % G || (act && ff < 1)) return -1;
+  const dim3 grid((unsigned)T, (H + G + 3) / 4);
+  // 16-byte vectors for the activation: every row start and the row length are multiples of 8 entries
+  const int vec = act && !f32 && ff % 8 == 0 && ucol % 8 == 0 && ld % 8 == 0 && lda % 8 == 0 && (uintptr_t)proj % 16 == 0 &&
+                  (uintptr_t)act % 16 == 0;
+  if (f32)
+    hipLaunchKernelGGL(rope_prep_kernel<float>, grid, dim3(256), 0, st, (const float*)proj, ld, H, G, d, dv, cos_sin, tab_w, rot,
+                       qscale, pos, slots, (float*)kc, (float*)vc, (float*)q, BSZ, ucol, ff, (float*)act, lda, vec, (float*)zrow,
+                       ldz, zn);
+  else
+    hipLaunchKernelGGL(rope_prep_kernel<u16>, grid, dim3(256), 0, st, (const u16*)proj, ld, H, G, d, dv, cos_sin, tab_w, rot,
+                       qscale, pos, slots, (u16*)kc, (u16*)vc, (u16*)q, BSZ, ucol, ff, (u16*)act, lda, vec, (u16*)zrow, ldz, zn);
   return (int)hipGetLastError();
 }

@@ -7,6 +7,9 @@
 //
 //   latent_kv_write   one wave per token: RMS-norm the latent (f32), rotate the shared key part
 //                     (interleaved pairs), write both into the token's cache slot
+//   latent_prep       latent_kv_write without a rotated part for a layer whose feed-forward shares the
+//                     projection: the same launch squares the relu of the up columns
+//   gate_heads        per-head outputs [H, T, dv] times sigmoid(gate), laid out token-major
 //   latent_attention  one workgroup per 16 rows (token-major (token, head) rows of one sequence):
 //                     the rows' queries staged once in LDS as f32 (rotation and the score scale
 //                     applied while staging); keys walk in tiles staged in LDS as f32;
@@ -52,6 +55,58 @@ __global__ void __launch_bounds__(64) latent_kv_write_kernel(const T* __restrict
     stf(dst + rank + 2 * i, u * c - v * sn);
     stf(dst + rank + 2 * i + 1, v * c + u * sn);
   }
+}
+
+// proj row: ... | latent (column ccol, rank wide) | ... | up (column ucol, ff wide) | ...: the latent's RMS
+// norm into the token's cache slot (wave 0 of the token's first workgroup), act[tok] = relu(up)^2
+// (shared by the token's workgroups; vec: rows of whole 16-byte vectors).
+template <typename T>
+__global__ void __launch_bounds__(256) latent_prep_kernel(const T* __restrict__ proj, long ld, int ccol, int rank,
+                                                          const float* __restrict__ w, float eps,
+                                                          const int* __restrict__ slots, T* __restrict__ cache, int ucol,
+                                                          int ff, T* __restrict__ act, long lda, int vec) {
+  const long tok = blockIdx.x;
+  const int tid = threadIdx.x;
+  const T* row = proj + tok * ld;
+  const int slot = slots[tok];
+  if (blockIdx.y == 0 && tid < 64 && slot >= 0) {
+    const T* r = row + ccol;
+    float s = 0.f;
+    for (int i = tid; i < rank; i += 64) { const float v = ldf(r + i); s += v * v; }
+    const float rs = 1.f / sqrtf(wave_sum(s) / (float)rank + eps);
+    T* dst = cache + (long)slot * rank;
+    for (int i = tid; i < rank; i += 64) stf(dst + i, ldf(r + i) * rs * w[i]);
+  }
+  if (!act) return;
+  const T* up = row + ucol;
+  T* a = act + tok * lda;
+  if constexpr (sizeof(T) == 2) {
+    if (vec) {
+      for (int i = 8 * (blockIdx.y * 256 + tid); i < ff; i += 8 * gridDim.y * 256) {
+        float f[8];
+        unpack8(ld16(up + i), f);
+#pragma unroll
+        for (int x = 0; x < 8; ++x) { f[x] = fmaxf(f[x], 0.f); f[x] *= f[x]; }
+        st16(a + i, pack8(f));
+      }
+      return;
+    }
+  }
+  for (int i = blockIdx.y * 256 + tid; i < ff; i += gridDim.y * 256) {
+    const float v = fmaxf(ldf(up + i), 0.f);
+    stf(a + i, v * v);
+  }
+}
+
+// out[t, h dv + i] = o[h, t, i] sigmoid(gate[t, h dv + i]): x over the columns, y over the tokens
+template <typename T>
+__global__ void __launch_bounds__(256) gate_heads_kernel(const T* __restrict__ o, const T* __restrict__ gate, long ldg,
+                                                         T* __restrict__ out, long ldo, int H, int dv, long Tn) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= H * dv) return;
+  const int h = c / dv, i = c - h * dv;
+  for (long t = blockIdx.y; t < Tn; t += gridDim.y)
+    stf(out + t * ldo + c, ldf(o + ((long)h * Tn + t) * dv + i) / (1.f + expf(-ldf(gate + t * ldg + c))));
 }
 
 constexpr int LROWS = 16;
@@ -746,4 +801,34 @@ extern "C" int dllm_latent_attention(const void* qa, const void* q, long ldq, in
                                 (float*)out, KT, tpe, kstride, vec, splits, part_o, part_ml);
   return launch_latent<u16>(ri, g, lds, st, (const u16*)qa, (const u16*)q, ldq, H, dim, rot, rank, Ttot, cos_sin, tab_w,
                             (const u16*)cache, bt, bt_w, qstart, qlen, ctx, tile_seq, tile_tok0, scale, (u16*)out, KT, tpe, kstride, vec, splits, part_o, part_ml);
+}
+
+extern "C" int dllm_latent_prep(const void* proj, long ld, int f32, int ccol, int rank, const float* w, float eps,
+                                const int* slots, void* cache, int ucol, int ff, void* act, long lda, long T, hipStream_t st) {
+  if (T <= 0) return 0;
+  if (rank < 1 || (act && ff < 1)) return -1;
+  const dim3 grid((unsigned)T, act ? (ff + 2047) / 2048 : 1);
+  const int vec = act && !f32 && ff % 8 == 0 && ucol % 8 == 0 && ld % 8 == 0 && lda % 8 == 0 && (uintptr_t)proj % 16 == 0 &&
+                  (uintptr_t)act % 16 == 0;
+  if (f32)
+    hipLaunchKernelGGL(latent_prep_kernel<float>, grid, dim3(256), 0, st, (const float*)proj, ld, ccol, rank, w, eps, slots,
+                       (float*)cache, ucol, ff, (float*)act, lda, vec);
+  else
+    hipLaunchKernelGGL(latent_prep_kernel<u16>, grid, dim3(256), 0, st, (const u16*)proj, ld, ccol, rank, w, eps, slots,
+                       (u16*)cache, ucol, ff, (u16*)act, lda, vec);
+  return (int)hipGetLastError();
+}
+
+extern "C" int dllm_gate_heads(const void* o, int f32, const void* gate, long ldg, void* out, long ldo, int H, int dv, long T,
+                               hipStream_t st) {
+  if (T <= 0) return 0;
+  if (H < 1 || dv < 1) return -1;
+  const dim3 grid((H * dv + 255) / 256, (unsigned)(T < 4096 ? T : 4096));
+  if (f32)
+    hipLaunchKernelGGL(gate_heads_kernel<float>, grid, dim3(256), 0, st, (const float*)o, (const float*)gate, ldg, (float*)out,
+                       ldo, H, dv, T);
+  else
+    hipLaunchKernelGGL(gate_heads_kernel<u16>, grid, dim3(256), 0, st, (const u16*)o, (const u16*)gate, ldg, (u16*)out, ldo, H,
+                       dv, T);
+  return (int)hipGetLastError();
 }

@@ -24,6 +24,8 @@
 //   softcap          cap * tanh(x / cap) in f32;  gated_group_norm: rmsnorm in parts of y silu(z)
 //   ls_resadd_ln     x (f32) += ls * (y + bias + sigmoid(g) y2 + hw h), then the layer norm (mean and
 //                    variance, weight and bias) of the next sublayer's input: one workgroup per token
+//   scaled_resadd_rms  x (f32) = x + mult y + vec (or mult y + vec alone), then the RMS norm of the next
+//                    layer's input or the rounded stream: one workgroup per token
 //   glu_act          gated activations of a fused gate | up projection: SiLU gate, or clamped with
 //                    g sigmoid(alpha g) (u + 1)
 //   route_topk       group-limited top-k routing with sigmoid or softmax scores, a correction on the
@@ -938,6 +940,36 @@ __global__ void __launch_bounds__(256) ls_resadd_ln_kernel(const T* __restrict__
   for (int i = threadIdx.x; i < H; i += 256) stf(out + row * (long)H + i, (yb[i] - mean) * r * w[i] + b[i]);
 }
 
+// ---------------------------------------------------------------- pre-norm layers with one residual add
+// One workgroup per token.  With y: x = (set ? 0 : x) + mult y + vec (vec: one f32 vector, optional).  Then
+// out = x / sqrt(mean(x^2) + eps) * w, or without w the rounded stream itself; out rows ldo apart.
+template <typename T>
+__global__ void __launch_bounds__(256) scaled_resadd_rms_kernel(const T* __restrict__ y, long ldy, float mult, int set,
+                                                                const float* __restrict__ vec, float* __restrict__ x,
+                                                                const float* __restrict__ w, T* __restrict__ out, long ldo,
+                                                                int H, float eps) {
+  __shared__ float red[16];
+  extern __shared__ float yb[];   // [H]; entry i is touched by thread i % 256 only
+  const long row = blockIdx.x;
+  float* xr = x + row * (long)H;
+  T* orow = out ? out + row * ldo : nullptr;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < H; i += 256) {
+    float v = set ? 0.f : xr[i];
+    if (y) {
+      v += mult * ldf(y + row * ldy + i);
+      if (vec) v += vec[i];
+      xr[i] = v;
+    }
+    if (w) yb[i] = v;
+    else if (orow) stf(orow + i, v);
+    ss += v * v;
+  }
+  if (!w) return;   // uniform
+  const float r = 1.f / sqrtf(block_sum(ss, red) / (float)H + eps);
+  for (int i = threadIdx.x; i < H; i += 256) stf(orow + i, yb[i] * r * w[i]);
+}
+
 // gu [rows, 2 ff] (gate columns, then up columns) + bias -> y [rows, ff].  mode 0: silu(g) u;
 // mode 1: g <- min(g, limit), u <- clamp(u, -limit, limit), y = g sigmoid(alpha g) (u + 1)
 template <typename T>
@@ -1301,5 +1333,22 @@ extern "C" int dllm_glu_act(const void* gu, long ld, int f32, const float* bias,
   BY_T(f32,
        hipLaunchKernelGGL(glu_act_kernel<u16>, grid, dim3(256), 0, st, (const u16*)gu, ld, bias, ff, mode, limit, alpha, (u16*)y, rows),
        hipLaunchKernelGGL(glu_act_kernel<float>, grid, dim3(256), 0, st, (const float*)gu, ld, bias, ff, mode, limit, alpha, (float*)y, rows))
+  return (int)hipGetLastError();
+}
+
+extern "C" int dllm_scaled_resadd_rms(const void* y, long ldy, int f32, float mult, int set, const float* vec, float* x,
+                                      const float* w, void* out, long ldo, long rows, int H, float eps, hipStream_t st) {
+  if (rows <= 0) return 0;
+  const long lds = w ? 4L * H : 0;
+  if (lds > 150 * 1024 || (w && !out) || (set && !y)) return -1;
+  if (f32) {
+    ENSURE_LDS(scaled_resadd_rms_kernel<float>, lds);
+    hipLaunchKernelGGL(scaled_resadd_rms_kernel<float>, dim3((unsigned)rows), dim3(256), lds, st, (const float*)y, ldy, mult, set,
+                       vec, x, w, (float*)out, ldo, H, eps);
+  } else {
+    ENSURE_LDS(scaled_resadd_rms_kernel<u16>, lds);
+    hipLaunchKernelGGL(scaled_resadd_rms_kernel<u16>, dim3((unsigned)rows), dim3(256), lds, st, (const u16*)y, ldy, mult, set, vec,
+                       x, w, (u16*)out, ldo, H, eps);
+  }
   return (int)hipGetLastError();
 }

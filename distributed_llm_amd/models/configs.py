@@ -93,9 +93,24 @@ def get_model_config(name: str, **overrides) -> ModelConfig:
 # folder's config.json.  ``family`` picks the model class (models.registry).
 
 @dataclass(frozen=True)
+class YarnSpec:
+    """Rotation frequencies stretched by ``factor`` beyond the ``original`` length: those that make at
+    least ``fast`` turns inside it stay, those below ``slow`` turns are divided, a ramp in between."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+    def as_scaling(self) -> Dict:
+        return {"rope_type": "yarn", "factor": self.factor, "original_max_position_embeddings": self.original,
+                "beta_fast": self.fast, "beta_slow": self.slow}
+
+
+@dataclass(frozen=True)
 class RopeSpec:
     dims: int
     base: float
+    yarn: Optional[YarnSpec] = None
 
 
 @dataclass(frozen=True)
@@ -113,7 +128,11 @@ class MixerSpec:
     heads, dim, vdim, gate_cap) or ``sink_attention`` (grouped-query softmax attention with an RMS norm
     over the whole q and k projections, rotary pairs (2i, 2i + 1), unit-RMS values, a learned number per
     head on the scores, a sliding ``window`` that also sees the first ``keep_first`` tokens, and one
-    more term of score 0 and weight ``sink`` in the softmax denominator; ``kv_from`` as above)."""
+    more term of score 0 and weight ``sink`` in the softmax denominator; ``kv_from`` as above) or
+    ``gated_attention`` (grouped-query softmax attention without q / k norms, rotate-half pairs, inside
+    ``chunk`` positions counted from 0 (0: all), scores soft-capped at ``softcap`` (0: not), one learned
+    sink score per head in the denominator, a sigmoid gate on the heads).  ``latent_attention`` with
+    ``q_rank`` 0 projects its queries directly and, with ``gate``, gates its heads."""
     kind: str
     inner: int = 0
     state: int = 0
@@ -139,6 +158,9 @@ class MixerSpec:
     gate_cap: float = 0.0
     keep_first: int = 0
     sink: float = 0.0
+    chunk: int = 0
+    softcap: float = 0.0
+    gate: bool = False
 
     @property
     def parts(self) -> Tuple["MixerSpec", ...]:
@@ -150,7 +172,7 @@ class MixerSpec:
 
     @property
     def paged(self) -> bool:
-        return any(p.kind in ("latent_attention", "softmax_attention") or
+        return any(p.kind in ("latent_attention", "softmax_attention", "gated_attention") or
                    (p.kind in ("diff_attention", "sink_attention") and p.kv_from is None) for p in self.parts)
 
 
@@ -186,8 +208,8 @@ class MoESpec:
 
 @dataclass(frozen=True)
 class DenseSpec:
-    """One dense feed-forward ``W_down act(W_up x)``, ``ff`` wide; ``act``: ``gelu`` (the erf form) or
-    ``polynorm`` (a N(z) + b N(z^2) + c N(z^3) + e with learned a, b, c, e and N the scaling of a
+    """One dense feed-forward ``W_down act(W_up x)``, ``ff`` wide; ``act``: ``gelu`` (the erf form),
+    ``relu2`` (the square of relu) or ``polynorm`` (a N(z) + b N(z^2) + c N(z^3) + e with learned a, b, c, e and N the scaling of a
     token's ff values to unit RMS), or a gated one, ``W_down (g sigmoid(1.702 g) (u + 1))`` with
     g = min(W_gate x, limit) and u = clamp(W_up x, -limit, limit) (``clamped_glu``).  ``bias``: every
     projection has one."""
@@ -201,6 +223,15 @@ class DenseSpec:
 class LayerSpec:
     mixer: MixerSpec
     mlp: Optional[Union[MoESpec, DenseSpec]] = None
+
+
+@dataclass(frozen=True)
+class LoopSpec:
+    """Layers ``start`` .. ``stop`` - 1 run ``times`` times in a row with the same weights, every pass with
+    caches and states of its own.  A pass t begins with x <- W_in [x; embedding output] + step[t]."""
+    start: int
+    stop: int
+    times: int
 
 
 @dataclass(frozen=True)
@@ -238,10 +269,26 @@ class HybridConfig:
     embed_scale: float = 1.0
     # the output projection is the embedding table
     tied_head: bool = False
+    # with pre_norm: mixer and feed-forward read the same normed input and are added together,
+    # x += residual_mult * (mixer(h) + ff(h)), h = norm(x)
+    parallel_ff: bool = False
+    residual_mult: float = 1.0
+    # the model's norm weights are stored around zero: x / rms(x) * (1 + w)
+    norm_offset: bool = False
+    loop: Optional[LoopSpec] = None
 
     @property
     def n_layers(self) -> int:
         return len(self.layers)
+
+    @property
+    def runs(self) -> Tuple[Tuple[int, Optional[int]], ...]:
+        """The layers in the order they run: (layer, the loop pass that begins with this run or None)."""
+        n, lp = len(self.layers), self.loop
+        if lp is None:
+            return tuple((i, None) for i in range(n))
+        body = [(i, t if i == lp.start else None) for t in range(lp.times) for i in range(lp.start, lp.stop)]
+        return tuple([(i, None) for i in range(lp.start)] + body + [(i, None) for i in range(lp.stop, n)])
 
     @property
     def is_moe(self) -> bool:
@@ -251,6 +298,8 @@ class HybridConfig:
         H, n = self.hidden, (1 if self.tied_head else 2) * self.vocab * self.hidden + self.hidden
         nb = 2 if self.norm_kind == "layer" else 1
         n += (nb - 1) * H
+        if self.loop is not None:
+            n += 2 * H * H + self.loop.times * H
         for L in self.layers:
             n += H * (self.input_conv + (nb - 1) + (1 if self.layer_scale else 0))
             if L.mlp is not None:
@@ -265,6 +314,11 @@ class HybridConfig:
                 if m.kind in ("retention", "lightning"):
                     n += 2 * m.heads * m.dim * H + 2 * m.heads * m.vdim * H + H * m.heads * m.vdim
                     n += m.heads * m.vdim if m.kind == "lightning" else 0
+                elif m.kind == "gated_attention":
+                    n += (m.heads + m.kv_heads) * m.dim * H + m.kv_heads * m.vdim * H + 2 * m.heads * m.vdim * H + m.heads
+                elif m.kind == "latent_attention" and not m.q_rank:
+                    n += m.heads * m.dim * H + m.kv_rank * (H + 1) + m.heads * (m.dim + m.vdim) * m.kv_rank
+                    n += (2 if m.gate else 1) * m.heads * m.vdim * H
                 elif m.kind == "latent_attention":
                     n += m.q_rank * (H + 1) + m.heads * (m.dim + m.rot_dim) * m.q_rank + (m.kv_rank + m.rot_dim) * H
                     n += m.kv_rank + m.heads * (m.dim + m.vdim) * m.kv_rank + H * m.heads * m.vdim
@@ -296,7 +350,7 @@ class HybridConfig:
             elif isinstance(L.mlp, DenseSpec):
                 f = L.mlp
                 mats = 3 if f.act == "clamped_glu" else 2
-                n += sides * H + mats * f.ff * H + (4 if f.act == "polynorm" else 0)
+                n += (0 if self.parallel_ff else sides * H) + mats * f.ff * H + (4 if f.act == "polynorm" else 0)
                 n += (2 * f.ff + H if f.bias else 0)
         if self.depth_average:
             n += sum(i + 2 for i in range(len(self.layers)))
@@ -491,9 +545,57 @@ def dogilorn_config(raw: dict, name: str = "dogilorn") -> HybridConfig:
                         embed_scale=float((raw.get("embedding") or {}).get("scale", 1.0)), tied_head=True)
 
 
+def mugipel_config(raw: dict, name: str = "mugipel") -> HybridConfig:
+    """A Mugipel config.json: ``layers`` (type ``attention`` with heads, kv_heads, dim, vdim, rot (dims,
+    base, scaling), scale, softcap, mask.size, or ``latent_attention`` with heads, dim, vdim, kv_rank,
+    scale; mlp ``dense`` with ``ff`` or null), ``loop`` (start, stop, times), ``residual_mult``,
+    ``norm.eps``, ``vocab``, ``width``.  One norm (weight around zero) ahead of a mixer and a feed-forward
+    side by side, the head tied to the embedding."""
+    layers = []
+    for i, L in enumerate(raw["layers"]):
+        m, kind = L["mixer"], L["type"]
+        heads, dim = int(m["heads"]), int(m["dim"])
+        vdim = int(m.get("vdim", dim))
+        if kind == "attention":
+            rot = m.get("rot")
+            rope = _rope(rot)
+            if rope is not None:
+                sc = rot.get("scaling")
+                if sc:
+                    rope = RopeSpec(rope.dims, rope.base, YarnSpec(float(sc["factor"]), float(sc["original"]),
+                                                                   float(sc["fast"]), float(sc["slow"])))
+                if rope.dims % 2 or rope.dims > dim:
+                    raise ValueError(f"layer {i}: rot.dims must be even and at most dim")
+            mix = MixerSpec("gated_attention", heads=heads, kv_heads=int(m.get("kv_heads", heads)), dim=dim, vdim=vdim, rot=rope,
+                            scale=float(m["scale"]), chunk=int((m.get("mask") or {}).get("size", 0)),
+                            softcap=float(m.get("softcap") or 0.0), gate=True)
+            if mix.heads % mix.kv_heads:
+                raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+        elif kind == "latent_attention":
+            mix = MixerSpec(kind, heads=heads, dim=dim, vdim=vdim, kv_rank=int(m["kv_rank"]), scale=float(m["scale"]), gate=True)
+        else:
+            raise ValueError(f"unknown mixer type {kind!r}")
+        f = L.get("mlp")
+        mlp = None
+        if f:
+            if f["kind"] != "dense":
+                raise ValueError(f"unknown feed-forward kind {f['kind']!r}")
+            mlp = DenseSpec(int(f["ff"]), act="relu2")
+        layers.append(LayerSpec(mix, mlp))
+    lp = raw.get("loop")
+    loop = None
+    if lp:
+        loop = LoopSpec(int(lp["start"]), int(lp["stop"]), int(lp["times"]))
+        if not 0 <= loop.start < loop.stop <= len(layers) or loop.times < 1:
+            raise ValueError("loop: 0 <= start < stop <= layers and times >= 1")
+    return HybridConfig(name, "mugipel", int(raw["width"]), int(raw["vocab"]), tuple(layers), rms_eps=float(raw["norm"]["eps"]),
+                        pre_norm=True, post_norm=False, parallel_ff=True, residual_mult=float(raw.get("residual_mult", 1.0)),
+                        norm_offset=True, loop=loop, tied_head=True)
+
+
 # config.json "architecture" -> parser of that design's keys
 ARCHITECTURES = {"Filevik": filevik_config, "Sedopel": sedopel_config, "Pebodra": pebodra_config,
-                 "Dogilorn": dogilorn_config}
+                 "Dogilorn": dogilorn_config, "Mugipel": mugipel_config}
 
 AnyConfig = Union[ModelConfig, HybridConfig]
 

@@ -1,4 +1,4 @@
-"""Layer-list decoders (Filevik, Sedopel, Pebodra): every layer has a token mixer (Mamba-1 selective
+"""Layer-list decoders (Filevik, Sedopel, Pebodra, Dogilorn, Mugipel): every layer has a token mixer (Mamba-1 selective
 scan, retention, latent attention, gated delta rule, grouped-query softmax attention beside lightning
 attention, differential sliding-window attention, Mamba-2, mLSTM) and an optional feed-forward
 (mixture of experts or dense), in the order config.json gives.
@@ -51,12 +51,21 @@ they do not take and for f32 models), everything between them on the HIP kernels
   experts    (softmax scores + a correction for the choice, identity experts) one f32 GEMM for the
              router logits and the shared expert's gate logit -> group-limited top-k -> SwiGLU experts;
              identity experts, the gated shared expert and the layer scale ride in the residual launch
+  gated_attn (mixer and feed-forward side by side) one fused projection q | k | v | gate | up -> rotation
+             (YaRN frequencies), k and v to their pages, relu(up)^2, in one launch -> attention inside
+             chunks with capped scores, a learned sink per head and the sigmoid gate -> one projection
+             [out | down] over the heads and the activations together
+  latent     (direct queries, gated heads) one fused projection q | latent | gate | up -> the latent's
+             norm, its page and relu(up)^2 in one launch -> absorbed latent attention as above -> value
+             up-projection per head, gate -> one projection [out | down]
 
 Layer forms: ``x += norm(sublayer(x))`` (Filevik) or, with ``cfg.pre_norm``, a norm on both sides,
 ``x += norm_b(sublayer(norm(x)))``, or without ``cfg.post_norm`` ``x += ls * sublayer(layernorm(x))``
-(layer norms with bias, a learned scale per channel); with ``cfg.depth_average`` a layer hands on a
+(layer norms with bias, a learned scale per channel), or with ``cfg.parallel_ff`` one norm and one add,
+``x += c * (mixer(norm(x)) + ff(norm(x)))``; with ``cfg.depth_average`` a layer hands on a
 learned weighted sum of the embedding output and all layer results so far (kept as an f32 stack for
-the step).
+the step); with ``cfg.loop`` some layers run several times in a row (``cfg.runs``), every run with a
+cache of its own, each pass starting from a projection of the stream and the embedding output.
 
 Per-sequence state lives in slots owned by the engine (its batch rows); paged latents use the
 engine's block tables.  No tensor parallelism.
@@ -73,7 +82,7 @@ import torch.nn.functional as F
 from .. import ops
 from ..ops import seqmix
 from ..parallel.comm import SINGLE, ParallelContext
-from .configs import DenseSpec, HybridConfig, LayerSpec, MixerSpec, MoESpec
+from .configs import DenseSpec, HybridConfig, LayerSpec, MixerSpec, MoESpec, RopeSpec
 
 
 def _mm(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
@@ -97,15 +106,26 @@ class HybridModel:
         if dtype not in (torch.bfloat16, torch.float32):
             raise ValueError("dtype must be bfloat16 or float32")
         self.cfg, self.device, self.dtype, self.par = cfg, torch.device(device), dtype, par
-        if cfg.pre_norm and not cfg.post_norm and (cfg.norm_kind != "layer" or cfg.depth_average):
+        if cfg.pre_norm and not cfg.post_norm and not cfg.parallel_ff and (cfg.norm_kind != "layer" or cfg.depth_average):
             raise ValueError(f"{cfg.name}: layers without a norm after the sublayer use layer norms and no depth average")
+        if cfg.parallel_ff:
+            for S in cfg.layers:
+                m, f = S.mixer, S.mlp
+                if m.kind != "gated_attention" and not (m.kind == "latent_attention" and not m.q_rank and not m.rot_dim and m.gate):
+                    raise ValueError(f"{cfg.name}: mixer {m.kind} is not built beside a feed-forward")
+                if f is not None and not (isinstance(f, DenseSpec) and f.act == "relu2" and not f.bias):
+                    raise ValueError(f"{cfg.name}: only dense squared-relu feed-forwards run beside a mixer")
+            if not cfg.pre_norm or cfg.post_norm or cfg.norm_kind != "rms" or cfg.depth_average or cfg.layer_scale or cfg.input_conv:
+                raise ValueError(f"{cfg.name}: parallel layers use one RMS norm ahead of both sublayers and one plain add")
+        elif cfg.loop is not None or cfg.norm_offset or cfg.residual_mult != 1.0:
+            raise ValueError(f"{cfg.name}: loops, zero-centred norms and residual multipliers are built for parallel layers")
         if cfg.norm_kind == "layer" and (not cfg.pre_norm or cfg.post_norm):
             raise ValueError(f"{cfg.name}: layer norms are built for the pre-norm layer form only")
         # the input convolution's last inputs are per-sequence state like a recurrence's
         self.has_recurrent_state = any(L.mixer.recurrent for L in cfg.layers) or cfg.input_conv > 1
         self.layers: List[Dict[str, torch.Tensor]] = []
         self.tap: Optional[list] = None      # debugging: residual stream after every layer
-        self._rot: Dict[Tuple[int, float], torch.Tensor] = {}
+        self._rot: Dict[RopeSpec, torch.Tensor] = {}
         self._max_pos = 0
         raw = self._load(weights) if weights else self._random(seed, init_std)
         self._place(raw)
@@ -127,13 +147,16 @@ class HybridModel:
         t["embed"] = rnd(cfg.vocab, W, s=1.0)
         if not cfg.tied_head:
             t["head"] = lin(cfg.vocab, W)
-        t["final.norm"] = torch.ones(W)
+        one = torch.zeros if cfg.norm_offset else torch.ones
+        t["final.norm"] = one(W)
+        if cfg.loop is not None:
+            t["loop.in"], t["loop.step"] = lin(W, 2 * W), rnd(cfg.loop.times, W, s=0.1)
         lnb = cfg.norm_kind == "layer"
         if lnb:
             t["final.norm.b"] = rnd(W, s=0.1)
         for i, L in enumerate(cfg.layers):
             p, m = f"l{i}.", L.mixer
-            t[p + "norm1"] = torch.ones(W)
+            t[p + "norm1"] = one(W)
             if lnb:
                 t[p + "norm1.b"] = rnd(W, s=0.1)
             if cfg.layer_scale:
@@ -211,6 +234,15 @@ class HybridModel:
                 t[p + "mix.q"], t[p + "mix.k"] = lin(m.heads * m.dim, W), lin(m.heads * m.dim, W)
                 t[p + "mix.v"], t[p + "mix.g"] = lin(m.heads * m.vdim, W), lin(m.heads * m.vdim, W)
                 t[p + "mix.o"] = lin(W, m.heads * m.vdim)
+            elif m.kind == "gated_attention":
+                t[p + "mix.q"], t[p + "mix.k"] = lin(m.heads * m.dim, W), lin(m.kv_heads * m.dim, W)
+                t[p + "mix.v"], t[p + "mix.sink"] = lin(m.kv_heads * m.vdim, W), rnd(m.heads, s=1.0)
+                t[p + "mix.g"], t[p + "mix.o"] = lin(m.heads * m.vdim, W), lin(W, m.heads * m.vdim)
+            elif not m.q_rank:
+                t[p + "mix.q"], t[p + "mix.dkv"] = lin(m.heads * m.dim, W), lin(m.kv_rank, W)
+                t[p + "mix.dkv.norm"] = torch.ones(m.kv_rank)
+                t[p + "mix.uk"], t[p + "mix.uv"] = lin(m.heads * m.dim, m.kv_rank), lin(m.heads * m.vdim, m.kv_rank)
+                t[p + "mix.g"], t[p + "mix.o"] = lin(m.heads * m.vdim, W), lin(W, m.heads * m.vdim)
             else:
                 t[p + "mix.dq"], t[p + "mix.dq.norm"] = lin(m.q_rank, W), torch.ones(m.q_rank)
                 t[p + "mix.uq"] = lin(m.heads * (m.dim + m.rot_dim), m.q_rank)
@@ -218,7 +250,7 @@ class HybridModel:
                 t[p + "mix.uk"], t[p + "mix.uv"] = lin(m.heads * m.dim, m.kv_rank), lin(m.heads * m.vdim, m.kv_rank)
                 t[p + "mix.o"] = lin(W, m.heads * m.vdim)
             f = L.mlp
-            if f is not None:
+            if f is not None and not cfg.parallel_ff:
                 t[p + "norm2"] = torch.ones(W)
                 if lnb:
                     t[p + "norm2.b"] = rnd(W, s=0.1)
@@ -270,7 +302,13 @@ class HybridModel:
         put = lambda x: x.to(dev, dt).contiguous()
         f32 = lambda x: x.to(dev, torch.float32).contiguous()
         W = cfg.hidden
-        self.embed, self.final_norm = put(t["embed"]), f32(t["final.norm"])
+        # norm weights stored around zero get their 1 here, in f32
+        nrm = (lambda x: f32(x) + 1.0) if cfg.norm_offset else f32
+        self.embed, self.final_norm = put(t["embed"]), nrm(t["final.norm"])
+        if cfg.loop is not None:
+            self.loop_in, self.loop_step = put(t["loop.in"]), f32(t["loop.step"])
+            if tuple(self.loop_in.shape) != (W, 2 * W) or tuple(self.loop_step.shape) != (cfg.loop.times, W):
+                raise ValueError("loop.in / loop.step do not fit config width and loop.times")
         self.lm_head = self.embed if cfg.tied_head else put(t["head"])      # tied: the table itself, unscaled
         lnb = cfg.norm_kind == "layer"
         self.final_norm_b = f32(t["final.norm.b"]) if lnb else None
@@ -278,7 +316,11 @@ class HybridModel:
             raise ValueError("embed / head do not fit config vocab x width")
         for i, L in enumerate(cfg.layers):
             p, m = f"l{i}.", L.mixer
-            D: Dict[str, torch.Tensor] = {"norm1": f32(t[p + "norm1"])}
+            D: Dict[str, torch.Tensor] = {"norm1": nrm(t[p + "norm1"])}
+            if cfg.parallel_ff:
+                self._place_parallel(D, L, t, p, put, f32)
+                self.layers.append(D)
+                continue
             if cfg.pre_norm and cfg.post_norm:
                 D["norm1b"] = f32(t[p + "norm1b"])
             if lnb:
@@ -428,15 +470,42 @@ class HybridModel:
                     assert D["sh_down"].shape[1] == f.shared_ff
             self.layers.append(D)
 
+    def _place_parallel(self, D, L: LayerSpec, t, p: str, put, f32) -> None:
+        """A layer whose mixer and feed-forward read the same input and are added together: one
+        projection for everything that reads it, one for everything that is added."""
+        m, f, W = L.mixer, L.mlp, self.cfg.hidden
+        head = ("q", "k", "v", "g") if m.kind == "gated_attention" else ("q", "dkv", "g")
+        rows = [t[p + "mix." + n] for n in head] + ([t[p + "mlp.up"]] if f is not None else [])
+        cols = [t[p + "mix.o"]] + ([t[p + "mlp.down"]] if f is not None else [])
+        D["proj"], D["out"] = put(torch.cat(rows, 0)), put(torch.cat(cols, 1))
+        if m.kind == "gated_attention":
+            D["sink"] = f32(t[p + "mix.sink"])
+            n = (m.heads + m.kv_heads) * m.dim + m.kv_heads * m.vdim
+            assert D["sink"].numel() == m.heads
+        else:
+            D["dkv_norm"] = f32(t[p + "mix.dkv.norm"])
+            D["uk"] = put(t[p + "mix.uk"].view(m.heads, m.dim, m.kv_rank))                       # [H, d, r]
+            D["uvT"] = put(t[p + "mix.uv"].view(m.heads, m.vdim, m.kv_rank).transpose(1, 2))    # [H, r, dv]
+            n = m.heads * m.dim + m.kv_rank
+            assert D["dkv_norm"].numel() == m.kv_rank
+        ff = f.ff if f is not None else 0
+        assert tuple(D["proj"].shape) == (n + m.heads * m.vdim + ff, W)
+        assert tuple(D["out"].shape) == (W, m.heads * m.vdim + ff)
+
     def weight_bytes(self) -> int:
         n = sum(x.numel() * x.element_size() for x in (self.embed, self.final_norm))
+        if self.cfg.loop is not None:
+            n += sum(x.numel() * x.element_size() for x in (self.loop_in, self.loop_step))
         n += 0 if self.cfg.tied_head else self.lm_head.numel() * self.lm_head.element_size()
         return n + sum(x.numel() * x.element_size() for L in self.layers for x in L.values() if torch.is_tensor(x))
 
     def decode_read_bytes(self, top_only: bool = True) -> int:
         """Weight bytes one decode token reads (routed experts: ``top`` of them)."""
         n = self.lm_head.numel() * self.lm_head.element_size()
-        for L, S in zip(self.layers, self.cfg.layers):
+        if self.cfg.loop is not None:
+            n += self.cfg.loop.times * self.loop_in.numel() * self.loop_in.element_size()
+        for i, _ in self.cfg.runs:      # a looped layer is read in every pass
+            L, S = self.layers[i], self.cfg.layers[i]
             for k, x in L.items():
                 if not torch.is_tensor(x):
                     continue
@@ -456,20 +525,20 @@ class HybridModel:
             for m in L.mixer.parts:
                 r = m.rot
                 if r is not None and r.dims > 0:
-                    self._rot[(r.dims, r.base)] = ops.rope_cos_sin(n, r.dims, r.base, self.device)
+                    self._rot[r] = ops.rope_cos_sin(n, r.dims, r.base, self.device, r.yarn.as_scaling() if r.yarn else None)
 
     def _table(self, m: MixerSpec) -> torch.Tensor:
-        return self._rot[(m.rot.dims, m.rot.base)]
+        return self._rot[m.rot]
 
     def block_bytes(self, block_size: int) -> int:
-        """Bytes of one paged block over all layers (latent attention layers only)."""
+        """Bytes of one paged block over all layer runs."""
         it = torch.empty((), dtype=self.dtype).element_size()
         n = 0
-        for L in self.cfg.layers:
-            for m in L.mixer.parts:
+        for i, _ in self.cfg.runs:
+            for m in self.cfg.layers[i].mixer.parts:
                 if m.kind == "latent_attention":
                     n += block_size * (m.kv_rank + m.rot_dim) * it
-                elif m.kind == "softmax_attention":
+                elif m.kind in ("softmax_attention", "gated_attention"):
                     n += block_size * m.kv_heads * (m.dim + m.vdim) * it
                 elif m.kind == "diff_attention" and m.kv_from is None:
                     n += block_size * m.kv_heads * (2 * m.dim + m.vdim) * it
@@ -478,7 +547,7 @@ class HybridModel:
         return n
 
     def alloc_caches(self, num_blocks: int, block_size: int, slots: int) -> List[tuple]:
-        """Per layer: (paged latent [blocks, block, rank + rot],) or the recurrent state of ``slots``
+        """Per layer run (``cfg.runs``): (paged latent [blocks, block, rank + rot],) or the recurrent state of ``slots``
         sequences: (conv inputs [slots, taps - 1, inner], scan state [slots, inner, state] f32) /
         (retention state [slots, heads, dim, vdim] f32,) / delta: (conv inputs [slots, taps - 1,
         q | k | v channels], state [slots, heads, vdim, dim] f32) / parallel: (paged keys [blocks,
@@ -488,13 +557,14 @@ class HybridModel:
         layer / mamba2: (conv inputs [slots, taps - 1, x | B | C channels], state [slots, heads, N,
         vdim] f32) / mlstm: (memory [slots, heads, dim, vdim] f32, normaliser and maximum [slots,
         heads, column blocks, dim + 1] f32) / sink_attention: (paged keys [blocks, kv_heads, block,
-        dim], paged values [blocks, kv_heads, vdim, block]), of the layer ``kv_from`` names if any.
+        dim], paged values [blocks, kv_heads, vdim, block]), of the layer ``kv_from`` names if any /
+        gated_attention: the same two.
         With an input convolution every layer's tuple ends with its own last inputs [slots, taps - 1,
         width]."""
         dev, out = self.device, []
-        for L in self.cfg.layers:
-            m = L.mixer
-            if m.kind == "sink_attention":
+        for i, _ in self.cfg.runs:
+            m = self.cfg.layers[i].mixer
+            if m.kind in ("sink_attention", "gated_attention"):
                 if m.kv_from is not None:
                     out.append(out[m.kv_from][:2])
                 else:
@@ -557,7 +627,7 @@ class HybridModel:
 
     def _any_table(self) -> torch.Tensor:
         if not self._rot:
-            self._rot[(2, 1.0)] = ops.rope_cos_sin(self._max_pos, 2, 1.0, self.device)
+            self._rot[RopeSpec(2, 1.0)] = ops.rope_cos_sin(self._max_pos, 2, 1.0, self.device)
         return next(iter(self._rot.values()))
 
     def _latent(self, L, m: MixerSpec, x, positions, meta, cache):
@@ -666,6 +736,79 @@ class HybridModel:
                                        None, mfma, splits, window=m.window, keep_first=m.keep_first, sink=m.sink,
                                        all_rows=self._all_rows(x, meta), out=out)
         return _mm(o, L["o"])
+
+    # ------------------------------------------------------------------ mixer and feed-forward side by side
+    def _gated_attention_ff(self, L, m: MixerSpec, f: Optional[DenseSpec], x, positions, meta, cache):
+        """mixer(x) + ff(x): one projection in, one out; the heads and the activations meet in one buffer."""
+        k_cache, v_cache = cache[0], cache[1]
+        T, hv = x.shape[0], m.heads * m.vdim
+        proj = _mm(x, L["proj"])                                        # q | k | v | gate | up
+        g0 = (m.heads + m.kv_heads) * m.dim + m.kv_heads * m.vdim
+        both = torch.empty((T, hv + (f.ff if f is not None else 0)), dtype=x.dtype, device=x.device)
+        o = both[:, :hv]
+        rot = m.rot.dims if m.rot is not None else 0
+        table = self._table(m) if rot else self._any_table()
+        all_rows = self._all_rows(x, meta)      # else the prep launch clears the attention output's padding rows
+        q = seqmix.rope_prep(proj, m.heads, m.kv_heads, m.dim, m.vdim, table, rot, m.scale, positions, meta.slots, k_cache,
+                             v_cache, g0 + hv, both[:, hv:] if f is not None else None, None if all_rows else o)
+        mfma = seqmix.gqa_use_mfma(q, m.heads, m.kv_heads, m.dim, m.vdim, k_cache.shape[2])
+        ts, tt = meta.latent_tiles(1, self.device, seqmix.gqa_tokens_per_tile(m.heads, m.kv_heads, mfma))
+        splits = seqmix.gqa_splits(int(ts.numel()), m.kv_heads, meta.max_ctx, chunk=m.chunk) if mfma else 1
+        seqmix.paged_gqa_attention(q, k_cache, v_cache, meta.block_tables, meta.qstart, meta.qlen, meta.ctx, ts, tt,
+                                   proj[:, g0:g0 + hv], mfma, splits, out=o, chunk=m.chunk, softcap=m.softcap, sinks=L["sink"])
+        return _mm(both, L["out"])
+
+    def _latent_ff(self, L, m: MixerSpec, f: Optional[DenseSpec], x, positions, meta, cache):
+        """mixer(x) + ff(x) with latent attention (absorbed form, direct queries, gated heads)."""
+        T, H, hv = x.shape[0], m.heads, m.heads * m.vdim
+        proj = _mm(x, L["proj"])                                        # q | latent | gate | up
+        c0 = H * m.dim
+        g0 = c0 + m.kv_rank
+        both = torch.empty((T, hv + (f.ff if f is not None else 0)), dtype=x.dtype, device=x.device)
+        seqmix.latent_prep(proj, c0, L["dkv_norm"], self.cfg.rms_eps, meta.slots, cache[0], g0 + hv,
+                           both[:, hv:] if f is not None else None)
+        q = proj[:, :c0]
+        qa = torch.bmm(q.unflatten(1, (H, m.dim)).transpose(0, 1), L["uk"])     # key up-projection absorbed: [H, T, rank]
+        rows = (seqmix.LAT_ROWS if meta.host_qlen is None else
+                seqmix.latent_rows(x, m.kv_rank, 0, T, len(meta.host_qlen)))
+        ts, tr = meta.latent_tiles(H, self.device, rows)
+        lat = seqmix.latent_attention(qa, q, m.dim, 0, positions, self._any_table(), cache[0], meta.block_tables, meta.qstart,
+                                      meta.qlen, meta.ctx, ts, tr, m.scale, rows=rows)
+        seqmix.gate_heads(torch.bmm(lat, L["uvT"]), proj[:, g0:g0 + hv], both[:, :hv])
+        return _mm(both, L["out"])
+
+    def _hidden_parallel(self, x, xl, positions, meta, kv_caches):
+        """The layer loop of ``parallel_ff`` models on the f32 stream x [T, width] (the embedding output):
+        a run's tail adds its output and forms what the next one reads, in one launch."""
+        cfg, eps = self.cfg, self.cfg.rms_eps
+        T, W = x.shape
+        runs = cfg.runs
+        pair = None
+        if cfg.loop is not None:     # [stream | embedding output], the input of a pass's projection
+            pair = torch.empty((T, 2 * W), dtype=self.dtype, device=x.device)
+            pair[:, W:].copy_(x if xl is None else xl)
+        h = torch.empty((T, W), dtype=self.dtype, device=x.device)
+        if runs[0][1] is None:
+            seqmix.scaled_resadd_rms(x, eps, w=self.layers[runs[0][0]]["norm1"], out=h)
+        else:
+            pair[:, :W].copy_(pair[:, W:])
+        for r, ((i, t), cache) in enumerate(zip(runs, kv_caches)):
+            L, S = self.layers[i], cfg.layers[i]
+            if t is not None:        # a pass begins: x = W_in [x; x0] + step[t]
+                h = torch.empty((T, W), dtype=self.dtype, device=x.device)
+                seqmix.scaled_resadd_rms(x, eps, y=_mm(pair, self.loop_in), set_=True, vec=self.loop_step[t], w=L["norm1"], out=h)
+            run = self._gated_attention_ff if S.mixer.kind == "gated_attention" else self._latent_ff
+            y = run(L, S.mixer, S.mlp, h, positions, meta, cache)
+            last = r + 1 == len(runs)
+            if not last and runs[r + 1][1] is not None:
+                seqmix.scaled_resadd_rms(x, eps, y=y, mult=cfg.residual_mult, out=pair[:, :W])
+            else:
+                h = torch.empty((T, W), dtype=self.dtype, device=x.device)
+                nxt = self.final_norm if last else self.layers[runs[r + 1][0]]["norm1"]
+                seqmix.scaled_resadd_rms(x, eps, y=y, mult=cfg.residual_mult, w=nxt, out=h)
+            if self.tap is not None:
+                self.tap.append(x.clone())
+        return h if meta.all_last else h.index_select(0, meta.last_idx)
 
     @staticmethod
     def _all_rows(x, meta) -> bool:
@@ -786,6 +929,8 @@ class HybridModel:
         if cfg.embed_scale != 1.0:
             x = x * cfg.embed_scale      # f32; the pre-norm layers read their own normed copy
             xl = None if xl is None else x.to(self.dtype)
+        if cfg.parallel_ff:
+            return self._hidden_parallel(x, xl, positions, meta, kv_caches)
         T, W, nL = x.shape[0], cfg.hidden, len(self.layers)
         X = None
         if cfg.depth_average:

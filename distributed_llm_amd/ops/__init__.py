@@ -87,13 +87,17 @@ def layer_norm(x: torch.Tensor, w: torch.Tensor, b: torch.Tensor, eps: float,
 # ----------------------------------------------------------------------------- rope + kv
 
 def rope_cos_sin(max_pos: int, d: int, theta: float, device=None, scaling: Optional[dict] = None) -> torch.Tensor:
-    """Host-precomputed [max_pos, d] f32 table: cos in [:d/2], sin in [d/2:]."""
+    """Host-precomputed [max_pos, d] f32 table: cos in [:d/2], sin in [d/2:].  ``scaling``
+    ``rope_type`` "llama3" or "yarn" (which also multiplies cos and sin by a factor)."""
     inv = 1.0 / (theta ** (torch.arange(0, d, 2, dtype=torch.float64) / d))
+    mul = 1.0
     if scaling and scaling.get("rope_type") == "llama3":
         inv = ref.llama3_scale_inv_freq(inv, scaling)
+    elif scaling and scaling.get("rope_type") == "yarn":
+        inv, mul = ref.yarn_scale_inv_freq(inv, d, theta, scaling)
     t = torch.arange(max_pos, dtype=torch.float64)
     f = torch.outer(t, inv)
-    return torch.cat([f.cos(), f.sin()], dim=1).float().to(device)
+    return (torch.cat([f.cos(), f.sin()], dim=1) * mul).float().to(device)
 
 
 def rope_and_cache(qkv: torch.Tensor, positions: torch.Tensor, cos_sin: torch.Tensor, slots: torch.Tensor,

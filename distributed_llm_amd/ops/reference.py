@@ -46,6 +46,21 @@ def llama3_scale_inv_freq(inv: torch.Tensor, sc: dict) -> torch.Tensor:
     return torch.where(is_mid, mid, out)
 
 
+def yarn_scale_inv_freq(inv: torch.Tensor, d: int, theta: float, sc: dict) -> Tuple[torch.Tensor, float]:
+    """YaRN: frequencies that make at least ``beta_fast`` turns inside the original length stay, those
+    below ``beta_slow`` turns are divided by ``factor``, a linear ramp over the pair index joins them;
+    cos and sin are multiplied by 0.1 ln(factor) + 1.  -> (frequencies, multiplier)"""
+    factor, old = float(sc["factor"]), float(sc["original_max_position_embeddings"])
+
+    def at(turns: float) -> float:
+        return d * math.log(old / (turns * 2 * math.pi)) / (2 * math.log(theta))
+
+    lo = max(math.floor(at(float(sc["beta_fast"]))), 0)
+    hi = min(math.ceil(at(float(sc["beta_slow"]))), d - 1)
+    ramp = ((torch.arange(inv.numel(), dtype=torch.float64) - lo) / max(hi - lo, 1e-3)).clamp(0, 1)
+    return inv / factor * ramp + inv * (1 - ramp), 0.1 * math.log(factor) + 1.0
+
+
 def _rope(x: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor) -> torch.Tensor:
     # x [T, h, d] f32; cos/sin [T, d/2]
     h = x.shape[-1] // 2
@@ -615,18 +630,22 @@ def attn_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, eps, qscale, 
 
 
 def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, gate=None, window=0, out_f32=False,
-                        keep_first=0, sink=0.0):
+                        keep_first=0, sink=0.0, chunk=0, softcap=0.0, sinks=None, out=None):
     """Causal softmax attention of q [T, heads, dim] (already scaled) over paged keys / values;
     query head h reads key head h // (heads / kv_heads); the output [T, heads * vdim] is
     multiplied by sigmoid(gate) when a gate [T, heads * vdim] is given.  ``window`` > 0: position i
     sees keys i - window < j <= i, and the keys j < ``keep_first`` whatever their distance.  A value
     cache with fewer heads than the key cache is shared by neighbouring key heads (key head g reads
     value head g // (key heads / value heads)).  ``sink``: weight of one more term of score 0 in
-    every softmax denominator (it has no value): p_j = exp(s_j) / (sink + sum exp(s_j))."""
+    every softmax denominator (it has no value): p_j = exp(s_j) / (sink + sum exp(s_j)).  ``sinks``
+    [heads] f32: that term's score per head instead, with weight 1.  ``chunk`` > 0: position i sees the
+    keys j <= i of its own chunk, j >= i - i % chunk.  ``softcap``: s <- softcap tanh(s / softcap).
+    ``out``: written there."""
     T, H, d = q.shape
     G, BSz, dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[2]
     vrep = G // v_cache.shape[1]
-    out = torch.zeros((T, H * dv), dtype=torch.float32 if out_f32 else q.dtype, device=q.device)
+    if out is None:
+        out = torch.zeros((T, H * dv), dtype=torch.float32 if out_f32 else q.dtype, device=q.device)
     qs, ql, cx = qstart.tolist(), qlen.tolist(), ctx.tolist()
     for s in range(len(qs)):
         n, c = ql[s], cx[s]
@@ -644,8 +663,16 @@ def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, ga
         if window > 0:
             keys = torch.arange(c, device=q.device)[None, :]
             mask = mask | ((keys <= pos[:, None] - window) & (keys >= keep_first))
+        if chunk > 0:
+            keys = torch.arange(c, device=q.device)[None, :]
+            mask = mask | ((keys < (pos - pos % chunk)[:, None]) & (keys >= keep_first))
+        if softcap > 0:
+            sc = softcap * torch.tanh(sc / softcap)
         sc = sc.masked_fill(mask[None], float("-inf"))
-        if sink > 0:
+        if sinks is not None:
+            sc = torch.cat([sc, sinks.float()[:, None, None].expand(H, n, 1)], -1)
+            pr = torch.softmax(sc, -1)[..., :-1]
+        elif sink > 0:
             mx = sc.max(-1, keepdim=True).values.clamp_min(0.0)
             e = torch.exp(sc - mx)
             pr = e / (e.sum(-1, keepdim=True) + sink * torch.exp(-mx))
@@ -993,3 +1020,62 @@ def glu_act(gu, bias=None, mode="swiglu", limit=0.0, alpha=1.0):
     g = g.clamp(max=limit)
     u = u.clamp(min=-limit, max=limit)
     return (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(gu.dtype)
+
+
+# ----------------------------------------------------------------------------- layers whose mixer and feed-forward share projections
+
+def scaled_resadd_rms(x, eps, y=None, mult=1.0, set_=False, vec=None, w=None, out=None):
+    """x (f32, in place) = (0 if set_ else x) + mult y + vec; out = rmsnorm(x) * w, or x itself rounded."""
+    if y is not None:
+        v = mult * y.float()
+        if not set_:
+            v = x + v
+        if vec is not None:
+            v = v + vec
+        x.copy_(v)
+    if out is not None:
+        out.copy_((x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w if w is not None else x).to(out.dtype))
+
+
+def relu2(u):
+    return torch.relu(u.float()).pow(2).to(u.dtype)
+
+
+def rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, positions, slots, k_cache, v_cache, ucol=0, act=None,
+              zero_rows=None):
+    """Rotate-half positions on the first ``rot_dims`` dims of q and k (cos and sin as the table holds
+    them), q times ``qscale``, k and v to their page slots; act = relu(proj[:, ucol:])^2."""
+    T, H, G, half = proj.shape[0], heads, kv_heads, rot_dims // 2
+    f = proj.float()
+    qk = f[:, :(H + G) * dim].reshape(T, H + G, dim).clone()
+    if rot_dims:
+        c, s = (a[:, None, :] for a in _rot_table(cos_sin, positions, half))
+        u, v = qk[..., :half].clone(), qk[..., half:rot_dims].clone()
+        qk[..., :half], qk[..., half:rot_dims] = u * c - v * s, v * c + u * s
+    ok = slots >= 0
+    BSz, sl = k_cache.shape[2], slots[ok].long()
+    k_cache[sl // BSz, :, sl % BSz] = qk[ok, H:].to(k_cache.dtype)
+    v = f[:, (H + G) * dim:(H + G) * dim + G * vdim].reshape(T, G, vdim)
+    v_cache[sl // BSz, :, :, sl % BSz] = v[ok].to(v_cache.dtype)
+    if act is not None:
+        act.copy_(relu2(proj[:, ucol:ucol + act.shape[1]]))
+    if zero_rows is not None:
+        zero_rows.zero_()
+    return (qk[:, :H] * qscale).to(proj.dtype)
+
+
+def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol=0, act=None):
+    """cache[slot] = rmsnorm(proj[:, ccol : ccol + rank]) * norm_w; act = relu(proj[:, ucol:])^2."""
+    r = norm_w.numel()
+    c = rms_rows(proj[:, ccol:ccol + r], norm_w, eps, torch.float32)
+    ok = slots >= 0
+    cache.view(-1, r)[slots[ok].long()] = c[ok].to(cache.dtype)
+    if act is not None:
+        act.copy_(relu2(proj[:, ucol:ucol + act.shape[1]]))
+
+
+def gate_heads(o, gate, out):
+    """out[t, h dv + i] = o[h, t, i] * sigmoid(gate[t, h dv + i])."""
+    H, T, dv = o.shape
+    out.copy_((o.float().transpose(0, 1).reshape(T, H * dv) * torch.sigmoid(gate.float())).to(out.dtype))
+    return out

@@ -8,7 +8,10 @@ dense form of SwiGLU experts and the logit soft cap; for pre-norm layer-norm mod
 tail with layer scale and the next layer norm in one launch, an input convolution without activation,
 attention inputs normed over the whole q / k projection, kept first keys and a softmax sink in the
 paged attention, gated activations with clamps, and top-k routing with softmax scores, a correction
-on the choice and identity experts.
+on the choice and identity experts; for layers whose mixer and feed-forward read one norm and share
+projections the attention / latent inputs with the feed-forward's activation in one launch, gated
+head outputs, and the scaled residual add with the next norm; chunks, a score soft cap and per-head
+learned sinks in the paged attention.
 
 Same dispatch rule as the rest of the op library: GPU tensors run the HIP kernel (or raise when the
 extension is missing), CPU tensors the torch reference.  Every kernel takes bf16 or f32 activations
@@ -295,19 +298,22 @@ GQA_SPLIT_TARGET = 512     # workgroups a small matrix-core attention grid is sp
 GQA_SPLIT_MAX = 16
 
 
-def gqa_splits(n_tiles: int, kv_heads: int, max_ctx: int, window: int = 0, keep_first: int = 0) -> int:
+def gqa_splits(n_tiles: int, kv_heads: int, max_ctx: int, window: int = 0, keep_first: int = 0, chunk: int = 0) -> int:
     """Key splits of a matrix-core attention launch: grids with few workgroups (decode steps at small
     batch, short portions) split every row's 64-key tiles over up to ``GQA_SPLIT_MAX`` workgroups."""
     tiles = (int(max_ctx) + 63) // 64 if max_ctx > 0 else GQA_SPLIT_MAX     # decode graphs: any context
     if window > 0:
         tiles = min(tiles, (int(window) + 62) // 64 + 1 + (int(keep_first) + 63) // 64)
+    if chunk > 0:
+        tiles = min(tiles, (int(chunk) + 62) // 64 + 1 + (int(keep_first) + 63) // 64)
     return max(1, min(GQA_SPLIT_MAX, tiles, GQA_SPLIT_TARGET // max(1, n_tiles * kv_heads)))
 
 
 def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, tile_seq, tile_tok0,
                         gate: Optional[torch.Tensor] = None, mfma: bool = False, splits: int = 1, window: int = 0,
                         out_f32: bool = False, keep_first: int = 0, sink: float = 0.0,
-                        all_rows: bool = False, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                        all_rows: bool = False, out: Optional[torch.Tensor] = None, chunk: int = 0, softcap: float = 0.0,
+                        sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal softmax attention over paged keys / values of any head widths (f32 scores, online
     softmax), output times sigmoid(gate).  ``tile_seq`` / ``tile_tok0``: one entry per
     ``gqa_tokens_per_tile(heads, kv_heads, mfma)`` new tokens of a sequence.  ``splits`` > 1
@@ -318,11 +324,15 @@ def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, ti
     denominator, with no value.  A value cache with fewer heads than the key cache is shared by
     neighbouring key heads.  ``out_f32``: the output stays f32 whatever the model dtype.  ``all_rows``:
     the tiles cover every row of q (no padding rows), so the output needs no zero fill.  ``out``: a
-    prepared output [T, heads * vdim] (its padding rows already cleared)."""
+    prepared output [T, heads * vdim] (its padding rows already cleared; may be columns of a wider
+    matrix).  ``chunk`` > 0: a position sees the keys of its own chunk of that many positions, counted
+    from 0 (older key tiles are not read).  ``softcap`` > 0: scores s become softcap tanh(s / softcap).
+    ``sinks`` [heads] f32: one more term of that score per head (neither scaled nor capped) in the
+    denominator, with no value."""
     ext = _native(q)
     if ext is None:
         return ref.paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, gate, window, out_f32,
-                                       keep_first, sink)
+                                       keep_first, sink, chunk, softcap, sinks, out)
     dv = v_cache.shape[2]
     if out is None:
         out = (torch.empty if all_rows else torch.zeros)((q.shape[0], q.shape[1] * dv),
@@ -333,7 +343,8 @@ def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, ti
         part = torch.empty(int(tile_seq.numel()) * k_cache.shape[1] * splits * GQA_ROWS_MFMA * (dv + 2),
                            dtype=torch.float32, device=q.device)
     ext.paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, tile_seq, tile_tok0, gate, out,
-                            bool(mfma), splits, part, int(window), int(keep_first), float(sink))
+                            bool(mfma), splits, part, int(window), int(keep_first), float(sink), int(chunk),
+                            float(softcap), sinks)
     return out
 
 
@@ -583,3 +594,56 @@ def glu_act(gu: torch.Tensor, bias: Optional[torch.Tensor] = None, mode: str = "
     y = torch.empty((gu.shape[0], gu.shape[1] // 2), dtype=gu.dtype, device=gu.device)
     ext.glu_act(gu, bias, 0 if mode == "swiglu" else 1, float(limit), float(alpha), y)
     return y
+
+
+# ----------------------------------------------------------------------------- layers whose mixer and feed-forward share projections
+
+def scaled_resadd_rms(x: torch.Tensor, eps: float, y: Optional[torch.Tensor] = None, mult: float = 1.0, set_: bool = False,
+                      vec: Optional[torch.Tensor] = None, w: Optional[torch.Tensor] = None,
+                      out: Optional[torch.Tensor] = None) -> None:
+    """The tail of a layer with one residual add, and the next layer's input, in one launch: the f32
+    stream x [T, width] (in place) becomes x + mult y + vec (``set_``: mult y + vec; ``vec`` f32
+    [width]); ``out`` (the model dtype, may be columns of a wider matrix) receives rmsnorm(x) * w, or
+    without ``w`` the rounded stream."""
+    ext = _native(x)
+    if ext is None:
+        return ref.scaled_resadd_rms(x, eps, y, mult, set_, vec, w, out)
+    ext.scaled_resadd_rms(x, y, float(mult), bool(set_), vec, w, float(eps), out)
+
+
+def rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, positions, slots, k_cache, v_cache, ucol: int = 0,
+              act: Optional[torch.Tensor] = None, zero_rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Attention inputs without a q / k norm: proj [T, q | k | v | ...]; rotate-half positions on the
+    first ``rot_dims`` dims of every q and k head (cos and sin as the table holds them), q times
+    ``qscale``; k and v to their page slots (k_cache [blocks, kv_heads, block, dim], v_cache [blocks,
+    kv_heads, vdim, block]).  ``act`` [T, ff] (may be columns of a wider matrix) receives
+    relu(proj[:, ucol : ucol + ff])^2, the activation of a feed-forward whose up projection is part of
+    proj.  ``zero_rows`` [T, n] is cleared in the same launch.  Returns q [T, heads, dim]."""
+    ext = _native(proj)
+    if ext is None:
+        return ref.rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, positions, slots, k_cache, v_cache,
+                             ucol, act, zero_rows)
+    q = torch.empty((proj.shape[0], heads, dim), dtype=proj.dtype, device=proj.device)     # every row is written
+    ext.rope_prep(proj, int(heads), int(kv_heads), int(dim), int(vdim), cos_sin, int(rot_dims), float(qscale), positions,
+                  slots, k_cache, v_cache, q, int(ucol), act, zero_rows)
+    return q
+
+
+def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol: int = 0, act: Optional[torch.Tensor] = None) -> None:
+    """``latent_kv_write`` for a latent without a rotated part inside a wider projection: cache [blocks,
+    block, rank] receives rmsnorm(proj[:, ccol : ccol + rank]) * norm_w at the tokens' slots; ``act``
+    as in ``rope_prep``."""
+    ext = _native(proj)
+    if ext is None:
+        return ref.latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol, act)
+    ext.latent_prep(proj, int(ccol), norm_w, float(eps), slots, cache, int(ucol), act)
+
+
+def gate_heads(o: torch.Tensor, gate: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """out[t, h vdim + i] = o[h, t, i] * sigmoid(gate[t, h vdim + i]) for head-major outputs o [heads, T,
+    vdim]; ``gate`` and ``out`` may be columns of wider matrices."""
+    ext = _native(o)
+    if ext is None:
+        return ref.gate_heads(o, gate, out)
+    ext.gate_heads(o, gate, out)
+    return out
