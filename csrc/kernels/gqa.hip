@@ -522,7 +522,8 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
   u16* ksh = reinterpret_cast<u16*>(smraw);          // [KT][KSTR]
   u16* vtr = ksh + GM_KT * KSTR;                      // [SZ][VSTR]: values transposed, [dim][key]
   u16* pw = vtr + SZ * VSTR;                          // [4 waves][hi | lo][16][PSTR]
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);   // in a scalar register: the branches on it are scalar
   const int lr = lane & 15, g4 = lane >> 4;
   u16* phi = pw + wave * (2 * 16 * PSTR);
   u16* plo = phi + 16 * PSTR;
@@ -637,11 +638,16 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
         }
       }
     }
+    float sc[NKB][4];
+#pragma unroll
+    for (int kb = 0; kb < NKB; ++kb)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) sc[kb][i] = sacc[kb][i];
     if (cap > 0.f) {
 #pragma unroll
       for (int kb = 0; kb < NKB; ++kb)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) sacc[kb][i] = cap_fast(sacc[kb][i], cap, cap2);
+        for (int i = 0; i < 4; ++i) sc[kb][i] = cap_fast(sc[kb][i], cap, cap2);
     }
     float alpha[4];
     const int key0 = k0 + 4 * lr;
@@ -650,10 +656,14 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       float sv[NKB];
+      // bitwise on purpose: a select per key.  Written with && and ||, hipcc makes a chain of exec-masked
+      // branches of it, and in the 64-wide form dropped the copy of the visible keys' scores
 #pragma unroll
-      for (int kb = 0; kb < NKB; ++kb)
-        sv[kb] = (full || (key0 + kb <= rpos[i] && (key0 + kb >= rlo[i] || key0 + kb < keep)))
-                     ? sacc[kb][i] : -INFINITY;
+      for (int kb = 0; kb < NKB; ++kb) {
+        const int key = key0 + kb;
+        const bool vis = full | ((key <= rpos[i]) & ((key >= rlo[i]) | (key < keep)));
+        sv[kb] = vis ? sc[kb][i] : -INFINITY;
+      }
       float mx = fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]));
       mx = row16_max(mx);
       const float mn = fmaxf(m[i], mx);
@@ -677,7 +687,9 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
       *reinterpret_cast<uint2*>(phi + (4 * g4 + i) * PSTR + 4 * lr) = make_uint2(h01, h23);
       *reinterpret_cast<uint2*>(plo + (4 * g4 + i) * PSTR + 4 * lr) = make_uint2(l01, l23);
     }
-    __builtin_amdgcn_wave_barrier();   // the patch is this wave's own: its LDS writes are in order before the reads
+    // the patch is this wave's own: its LDS accesses are in order, the fence keeps the compiler's order too
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
     // once the running maxima have settled no row of the wave rescales: skip the sweep over the sums
     const bool rescale = __any(alpha[0] != 1.f || alpha[1] != 1.f || alpha[2] != 1.f || alpha[3] != 1.f);
 #pragma unroll

@@ -608,3 +608,84 @@ def test_sink_attention_kernels(dt, case, H, G, d, dv, rot, win, keep):
                 got = seqmix.paged_gqa_attention(q2, kc2, vc2, bt, qstart, qlen, ctx, ts, tt, None, mfma, splits, window=win,
                                                  keep_first=keep, sink=sink).float()
                 torch.testing.assert_close(got, want, **tol(dt))
+
+
+# ----------------------------------------------------------------------------- mixer and feed-forward side by side, chunked attention with sinks
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("n", [24, 104, 328, 1000, 4104])
+@pytest.mark.parametrize("set_,vec,norm", [(False, False, True), (False, False, False), (True, True, True), (False, True, True)])
+def test_scaled_resadd_rms(dt, n, set_, vec, norm):
+    torch.manual_seed(31)
+    T = 11
+    x1 = torch.randn(T, n, device=DEV) * 3
+    x2 = x1.clone()
+    y = torch.randn(T, n + 3, device=DEV).to(dt)[:, :n]
+    v, w = (torch.randn(n, device=DEV) if vec else None), (torch.randn(n, device=DEV) if norm else None)
+    o1 = torch.zeros(T, 2 * n, device=DEV, dtype=dt)      # the output may be columns of a wider matrix
+    o2 = o1.clone()
+    seqmix.scaled_resadd_rms(x1, 1e-5, y=y, mult=0.3, set_=set_, vec=v, w=w, out=o1[:, :n])
+    ref.scaled_resadd_rms(x2, 1e-5, y=y, mult=0.3, set_=set_, vec=v, w=w, out=o2[:, :n])
+    torch.testing.assert_close(x1, x2, atol=1e-5, rtol=1e-5)
+    torch.testing.assert_close(o1.float(), o2.float(), **tol(dt))
+    seqmix.scaled_resadd_rms(x1, 1e-5, w=w, out=o1[:, n:])      # no update: the norm (or the rounding) alone
+    ref.scaled_resadd_rms(x2, 1e-5, w=w, out=o2[:, n:])
+    torch.testing.assert_close(x1, x2, atol=1e-5, rtol=1e-5)
+    torch.testing.assert_close(o1.float(), o2.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("case", CASES + [([40, 3], [90, 130]), ([1, 1], [300, 77]), ([150], [170])])
+@pytest.mark.parametrize("H,G,d,dv,rot,chunk,cap,ff", [(4, 2, 16, 8, 8, 5, 3.0, 20), (6, 2, 88, 56, 20, 64, 0.0, 64), (3, 3, 40, 72, 40, 1, 20.0, 0),
+                                                       (8, 1, 64, 64, 32, 100, 30.0, 2056), (7, 1, 56, 88, 0, 0, 2.0, 8), (2, 1, 136, 200, 64, 48, 50.0, 5)])
+def test_gated_attention_kernels(dt, case, H, G, d, dv, rot, chunk, cap, ff):
+    """Prep (rotation with scaled cos and sin, pages, squared-relu columns), then attention inside
+    chunks with capped scores, a sink per head and a gate, in both kernel forms and every split count,
+    written into the first columns of a wider matrix."""
+    from distributed_llm_amd.models.llama import AttnMeta
+    torch.manual_seed(32)
+    T, qstart, qlen, ctx, pos, bt, kc, vc, slots = _pages(case, G, d, dv, dt)
+    cols = (H + G) * d + G * dv
+    proj = torch.randn(T, (cols + H * dv + ff + 7) // 8 * 8 + (0 if d % 8 == 0 else 3), device=DEV).to(dt)
+    yarn = {"rope_type": "yarn", "factor": 4.0, "original_max_position_embeddings": 64, "beta_fast": 8.0, "beta_slow": 1.0}
+    table = ops.rope_cos_sin(512, max(rot, 2), 100.0, DEV, yarn)
+    kc1, vc1, kc2, vc2 = kc.clone(), vc.clone(), kc.clone(), vc.clone()
+    b1, b2 = (torch.full((T, H * dv + ff), 7.0, device=DEV).to(dt) for _ in range(2))
+    act = [b[:, H * dv:] if ff else None for b in (b1, b2)]
+    q1 = seqmix.rope_prep(proj, H, G, d, dv, table, rot, 0.3, pos, slots, kc1, vc1, cols + H * dv, act[0], b1[:, :H * dv])
+    q2 = ref.rope_prep(proj, H, G, d, dv, table, rot, 0.3, pos, slots, kc2, vc2, cols + H * dv, act[1], b2[:, :H * dv])
+    for a, b in ((q1, q2), (kc1, kc2), (vc1, vc2), (b1, b2)):
+        torch.testing.assert_close(a.float(), b.float(), **tol(dt))
+    sinks = torch.randn(H, device=DEV) * 2 + 1
+    gate = proj[:, cols:cols + H * dv]
+    want = ref.paged_gqa_attention(q2, kc2, vc2, bt, qstart, qlen, ctx, gate, chunk=chunk, softcap=cap, sinks=sinks).float()
+    meta = AttnMeta(slots=None, block_tables=bt, qstart=qstart, qlen=qlen, ctx=ctx, tile_seq=None, tile_tok0=None,
+                    last_idx=None, host_qlen=case[0])
+    for mfma in [False] + ([True] if seqmix.gqa_use_mfma(q2, H, G, d, dv, 16) else []):
+        ts, tt = meta.latent_tiles(1, DEV, seqmix.gqa_tokens_per_tile(H, G, mfma))
+        for splits in ((1, 2, 7) if mfma else (1,)):
+            b1[:, :H * dv] = 0
+            seqmix.paged_gqa_attention(q2, kc2, vc2, bt, qstart, qlen, ctx, ts, tt, gate, mfma, splits, out=b1[:, :H * dv],
+                                       chunk=chunk, softcap=cap, sinks=sinks)
+            torch.testing.assert_close(b1[:, :H * dv].float(), want, **tol(dt))
+            torch.testing.assert_close(b1[:, H * dv:].float(), b2[:, H * dv:].float(), **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("T,H,d,dv,rank,ff", [(1, 3, 8, 12, 24, 16), (37, 4, 16, 32, 64, 2056), (9, 2, 40, 10, 100, 5), (130, 16, 64, 64, 512, 0)])
+def test_latent_prep_and_gate(dt, T, H, d, dv, rank, ff):
+    torch.manual_seed(33)
+    proj = torch.randn(T, H * d + rank + H * dv + ff, device=DEV).to(dt)
+    w = torch.rand(rank, device=DEV) + 0.5
+    nb = (T + 15) // 16 + 1
+    slots = torch.randperm(nb * 16, device=DEV)[:T].to(torch.int32)
+    slots[0] = -1
+    c1 = torch.randn(nb, 16, rank, device=DEV).to(dt)
+    c2 = c1.clone()
+    b1, b2 = (torch.full((T, H * dv + ff), 7.0, device=DEV).to(dt) for _ in range(2))
+    for m, c, b in ((seqmix, c1, b1), (ref, c2, b2)):
+        m.latent_prep(proj, H * d, w, 1e-5, slots, c, H * d + rank + H * dv, b[:, H * dv:] if ff else None)
+        o = (torch.arange(H * T * dv, device=DEV).float() * 0.37).sin().to(dt).view(H, T, dv)
+        m.gate_heads(o, proj[:, H * d + rank:H * d + rank + H * dv], b[:, :H * dv])
+    torch.testing.assert_close(c1.float(), c2.float(), **tol(dt))
+    torch.testing.assert_close(b1.float(), b2.float(), **tol(dt))
