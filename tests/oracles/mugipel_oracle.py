@@ -153,10 +153,3 @@ def forward(tokens, W, cfg, taps=None):
     return norm(x, W["final.norm"], eps) @ W["embed"].T
 
 
-def greedy(tokens, W, cfg, n):
-    """n arg-max continuations of a prompt (the whole sequence is recomputed for every token)."""
-    seq, out = list(tokens), []
-    for _ in range(n):
-        out.append(int(forward(seq, W, cfg)[-1].argmax()))
-        seq.append(out[-1])
-    return out
