@@ -32,7 +32,7 @@
 // sees the keys of its own chunk of positions, [p - p % chunk, p]), kept first keys (j < keep stays
 // visible at any distance; the tiles between the kept keys and the window are not read), a soft cap on
 // the scores (cap tanh(s / cap)) and a sink: one more term of the denominator, with no value, either
-// exp(0) times `sink` or exp(sinks[head]).
+// exp(0) times `sink` or exp(sinks[head]).  Under a cap the matrix-core form keeps no running maximum.
 //
 // Cache layout: K [blocks, G, block, d], V [blocks, G, dv, block] (bf16 or f32 like the activations;
 // V is kept transposed inside its page because the weighted sum runs over keys); every score,
@@ -493,12 +493,16 @@ constexpr int GM_ROWS = 64, GM_KT = 64, GM_BS = 16;   // rows per workgroup, key
 typedef float f32x2v __attribute__((ext_vector_type(2)));
 typedef __bf16 bf16x2v __attribute__((ext_vector_type(2)));
 
-// SZ >= max(d, dv) in {64, 128, 256}: d is walked in SZ / 32 MFMA steps, dv in SZ / 16 column blocks
-// (steps and blocks past the real widths are skipped).  d % 8 == 0 (16-byte key rows).
+// SZ >= max(d, dv) in {64, 128, 256}: d is walked in SZ / 32 MFMA steps, dv in SZ / 16 column blocks;
+// steps and blocks past the real widths multiply zeros (a branch around each would drain the matrix
+// pipe).  d % 8 == 0 (16-byte key rows).
+// CAP: the scores are capped at 0 < cap <= CAP_MAX, so exp(score) and its sums stay inside f32 and the
+// softmax needs no running maximum (it stays 0) and no rescaling.
 // MFMA operand layout (16x16x32): with lr = lane & 15, g4 = lane >> 4, A holds row lr, contraction
 // indices 8 g4 .. 8 g4 + 7; B holds column lr, the same indices; the accumulator holds rows
 // 4 g4 .. 4 g4 + 3 of column lr.
-template <int SZ>
+constexpr float CAP_MAX = 64.f;
+template <int SZ, bool CAP>
 __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restrict__ q, const u16* __restrict__ kc,
                                                              const u16* __restrict__ vc, const int* __restrict__ bt,
                                                              int bt_ld, const int* __restrict__ qstart,
@@ -512,9 +516,10 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
   constexpr int DS = SZ / 32, VB = SZ / 16, NKB = GM_KT / 16;
   constexpr int KSTR = SZ + 8, VSTR = GM_KT + 8, PSTR = GM_KT + 8;
   extern __shared__ __attribute__((aligned(16))) unsigned char smraw[];
-  const int s = tile_seq[blockIdx.x];
+  const int tile = gridDim.x - 1 - blockIdx.x;   // later tokens see more keys: start with the long rows
+  const int s = tile_seq[tile];
   const int n = qlen[s];
-  const int tok0 = tile_tok0[blockIdx.x];
+  const int tok0 = tile_tok0[tile];
   if (n <= 0 || tok0 >= n) return;   // the whole workgroup (padding tiles)
   const int g = blockIdx.y, R = H / G;
   const int nq = min(TQ, n - tok0), nrows = nq * R;
@@ -549,7 +554,7 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     const int row = 16 * wave + 4 * g4 + i;
     rpos[i] = row < nrows ? p0 + tok0 + row / R : -1;     // -1: sees no key
     rlo[i] = row < nrows ? oldest_key(rpos[i], win, chunk) : 0;
-    m[i] = -INFINITY;
+    m[i] = CAP ? 0.f : -INFINITY;
     l[i] = 0.f;
   }
 #pragma unroll
@@ -561,7 +566,9 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
   // skipped; one not before the second needs no mask at its old end)
   const int wave_lo = 16 * wave < nrows ? oldest_key(p0 + tok0 + (16 * wave) / R, win, chunk) : 0;
   const int wave_lo_last = wave_last >= 0 ? oldest_key(wave_last, win, chunk) : 0;
-  const float cap2 = cap > 0.f ? 2.f / cap : 0.f;
+  // CAP: exponents in base 2
+  const float cap2 = cap > 0.f ? (CAP ? 2.88539008f : 2.f) / cap : 0.f;
+  const float capl = 1.44269504f * cap;
   const int last = p0 + tok0 + nq - 1;   // the newest key any row sees
   const int* btr = bt + (long)s * bt_ld;
   constexpr int KCH = SZ / 8;            // 16-byte chunks of a staged key row
@@ -627,15 +634,13 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     if (k0 >= keep && k0 + GM_KT <= wave_lo) continue;   // ... or the tile lies before every row's window / chunk
     f32x4 sacc[NKB];
 #pragma unroll
-    for (int kb = 0; kb < NKB; ++kb) {
-      sacc[kb] = f32x4{0.f, 0.f, 0.f, 0.f};
-      const u16* bp = ksh + (16 * kb + lr) * KSTR + 8 * g4;
+    for (int kb = 0; kb < NKB; ++kb) sacc[kb] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int st = 0; st < DS; ++st) {
-        if (st * 32 < d) {
-          const bf16x8 b = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(bp + st * 32));
-          sacc[kb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qa[st], b, sacc[kb], 0, 0, 0);
-        }
+    for (int st = 0; st < DS; ++st) {
+#pragma unroll
+      for (int kb = 0; kb < NKB; ++kb) {
+        const bf16x8 b = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(ksh + (16 * kb + lr) * KSTR + 8 * g4 + st * 32));
+        sacc[kb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qa[st], b, sacc[kb], 0, 0, 0);
       }
     }
     float sc[NKB][4];
@@ -643,39 +648,56 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     for (int kb = 0; kb < NKB; ++kb)
 #pragma unroll
       for (int i = 0; i < 4; ++i) sc[kb][i] = sacc[kb][i];
-    if (cap > 0.f) {
+    if (!CAP && cap > 0.f) {
 #pragma unroll
       for (int kb = 0; kb < NKB; ++kb)
 #pragma unroll
         for (int i = 0; i < 4; ++i) sc[kb][i] = cap_fast(sc[kb][i], cap, cap2);
     }
-    float alpha[4];
+    if constexpr (CAP) {   // log2(e) times the capped score
+#pragma unroll
+      for (int kb = 0; kb < NKB; ++kb)
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          sc[kb][i] = capl - 2.f * capl * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(sc[kb][i] * cap2) + 1.f);
+    }
     const int key0 = k0 + 4 * lr;
-    // a tile below the wave's oldest row needs no mask (wave-uniform)
-    const bool full = k0 + GM_KT - 1 <= wave_first && k0 >= wave_lo_last;
+    // a tile inside every row's range needs no mask (wave-uniform, a scalar branch).  The mask is bitwise on
+    // purpose, a select per key: written with && and || hipcc made a chain of exec-masked branches of it,
+    // and in the 64-wide form dropped the copy of the visible keys' scores
+    if (!(k0 + GM_KT - 1 <= wave_first && k0 >= wave_lo_last)) {
+#pragma unroll
+      for (int kb = 0; kb < NKB; ++kb)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int key = key0 + kb;
+          const bool vis = (key <= rpos[i]) & ((key >= rlo[i]) | (key < keep));
+          sc[kb][i] = vis ? sc[kb][i] : -INFINITY;
+        }
+    }
+    float alpha[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      float sv[NKB];
-      // bitwise on purpose: a select per key.  Written with && and ||, hipcc makes a chain of exec-masked
-      // branches of it, and in the 64-wide form dropped the copy of the visible keys' scores
-#pragma unroll
-      for (int kb = 0; kb < NKB; ++kb) {
-        const int key = key0 + kb;
-        const bool vis = full | ((key <= rpos[i]) & ((key >= rlo[i]) | (key < keep)));
-        sv[kb] = vis ? sc[kb][i] : -INFINITY;
-      }
-      float mx = fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]));
-      mx = row16_max(mx);
-      const float mn = fmaxf(m[i], mx);
-      const bool any = mn > -INFINITY;
-      alpha[i] = any ? __expf(m[i] - mn) : 1.f;   // m = -inf before the first visible key: 0, and acc, l are 0
-      m[i] = mn;
-      l[i] *= alpha[i];
       float p[NKB];
+      if constexpr (CAP) {
 #pragma unroll
-      for (int kb = 0; kb < NKB; ++kb) {
-        p[kb] = any ? __expf(sv[kb] - mn) : 0.f;   // exp(-inf) = 0 for masked keys
-        l[i] += p[kb];
+        for (int kb = 0; kb < NKB; ++kb) {
+          p[kb] = __builtin_amdgcn_exp2f(sc[kb][i]);   // 0 for masked keys
+          l[i] += p[kb];
+        }
+      } else {
+        float mx = fmaxf(fmaxf(sc[0][i], sc[1][i]), fmaxf(sc[2][i], sc[3][i]));
+        mx = row16_max(mx);
+        const float mn = fmaxf(m[i], mx);
+        const bool any = mn > -INFINITY;
+        alpha[i] = any ? __expf(m[i] - mn) : 1.f;   // m = -inf before the first visible key: 0, and acc, l are 0
+        m[i] = mn;
+        l[i] *= alpha[i];
+#pragma unroll
+        for (int kb = 0; kb < NKB; ++kb) {
+          p[kb] = any ? __expf(sc[kb][i] - mn) : 0.f;   // exp(-inf) = 0 for masked keys
+          l[i] += p[kb];
+        }
       }
       // p = hi + lo with both parts bf16 (the packed conversions round to nearest even)
       const uint32_t h01 = __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2v{p[0], p[1]}, bf16x2v));
@@ -690,22 +712,22 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     // the patch is this wave's own: its LDS accesses are in order, the fence keeps the compiler's order too
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     __builtin_amdgcn_wave_barrier();
-    // once the running maxima have settled no row of the wave rescales: skip the sweep over the sums
-    const bool rescale = __any(alpha[0] != 1.f || alpha[1] != 1.f || alpha[2] != 1.f || alpha[3] != 1.f);
+    if constexpr (!CAP) {
+      // once the running maxima have settled no row of the wave rescales: skip the sweep over the sums
+      if (__any(alpha[0] != 1.f || alpha[1] != 1.f || alpha[2] != 1.f || alpha[3] != 1.f)) {
 #pragma unroll
-    for (int cb = 0; cb < VB; ++cb) {
-      if (cb * 16 >= dv) continue;
-      if (rescale) {
+        for (int cb = 0; cb < VB; ++cb)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) acc[cb][i] *= alpha[i];
+          for (int i = 0; i < 4; ++i) acc[cb][i] *= alpha[i];
       }
-      const u16* bp = vtr + (16 * cb + lr) * VSTR + 8 * g4;
+    }
 #pragma unroll
-      for (int ks = 0; ks < GM_KT; ks += 32) {
-        if (k0 + ks > wave_last) continue;
-        const bf16x8 bv = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(bp + ks));
-        const bf16x8 ah = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(phi + lr * PSTR + ks + 8 * g4));
-        const bf16x8 al = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(plo + lr * PSTR + ks + 8 * g4));
+    for (int ks = 0; ks < GM_KT; ks += 32) {
+      const bf16x8 ah = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(phi + lr * PSTR + ks + 8 * g4));
+      const bf16x8 al = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(plo + lr * PSTR + ks + 8 * g4));
+#pragma unroll
+      for (int cb = 0; cb < VB; ++cb) {
+        const bf16x8 bv = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(vtr + (16 * cb + lr) * VSTR + 8 * g4 + ks));
         acc[cb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ah, bv, acc[cb], 0, 0, 0);
         acc[cb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(al, bv, acc[cb], 0, 0, 0);
       }
@@ -717,7 +739,7 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     const int row = 16 * wave + 4 * g4 + i;
     if (row >= nrows) continue;
     if (part) {
-      float* pr = part + ((((long)blockIdx.x * G + g) * splits + blockIdx.z) * GM_ROWS + row) * (dv + 2);
+      float* pr = part + ((((long)tile * G + g) * splits + blockIdx.z) * GM_ROWS + row) * (dv + 2);
       if (lr == 0) { pr[0] = m[i]; pr[1] = lt; }
 #pragma unroll
       for (int cb = 0; cb < VB; ++cb)
@@ -864,15 +886,19 @@ extern "C" int dllm_paged_gqa(const void* q, const void* kc, const void* vc, int
     const dim3 grid(n_tiles, G, splits);
     const int TQ = dllm_gqa_tile_tokens(H, G, 1);
     float* pp = splits > 1 ? part : nullptr;
-#define GQM(SZ)                                                                                                          \
+#define GQM(SZ, CAP)                                                                                                     \
   do {                                                                                                                   \
     const long lds = gqa_mfma_lds(SZ);                                                                                   \
-    ENSURE_LDS(paged_gqa_mfma_kernel<SZ>, lds);                                                                          \
-    hipLaunchKernelGGL(paged_gqa_mfma_kernel<SZ>, grid, dim3(256), lds, st, (const u16*)q, (const u16*)kc, (const u16*)vc, bt, \
-                       bt_ld, qstart, qlen, ctx, tile_seq, tile_tok0, (const u16*)gate, ldg, (u16*)out, H, G, d, dv, TQ, \
-                       splits, pp, win, GV, out32, keep, sink, chunk, cap, sinks, ldo);                                                          \
+    ENSURE_LDS((paged_gqa_mfma_kernel<SZ, CAP>), lds);                                                                   \
+    hipLaunchKernelGGL((paged_gqa_mfma_kernel<SZ, CAP>), grid, dim3(256), lds, st, (const u16*)q, (const u16*)kc,        \
+                       (const u16*)vc, bt, bt_ld, qstart, qlen, ctx, tile_seq, tile_tok0, (const u16*)gate, ldg,         \
+                       (u16*)out, H, G, d, dv, TQ, splits, pp, win, GV, out32, keep, sink, chunk, cap, sinks, ldo);      \
   } while (0)
-    if (sz <= 64) GQM(64); else if (sz <= 128) GQM(128); else GQM(256);
+    if (cap > 0.f && cap <= CAP_MAX) {
+      if (sz <= 64) GQM(64, true); else if (sz <= 128) GQM(128, true); else GQM(256, true);
+    } else {
+      if (sz <= 64) GQM(64, false); else if (sz <= 128) GQM(128, false); else GQM(256, false);
+    }
 #undef GQM
     if (pp) {
       const int rows = (TQ * (H / G) < GM_ROWS ? TQ * (H / G) : GM_ROWS);

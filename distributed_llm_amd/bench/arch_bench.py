@@ -1,9 +1,16 @@
-"""Layer-list (Filevik, Sedopel, Pebodra, Dogilorn) models beside the closest Llama-family model at equal size:
+"""Layer-list (Filevik, Sedopel, Pebodra, Dogilorn, Mugipel) models beside the closest Llama-family model at equal size:
 prefill and decode throughput through the engine, and the time of each mixer kernel against its roofline.
 
-``python bench.py --arch-bench [--arch-design filevik|sedopel|pebodra|dogilorn] [--arch-size s|m]`` (random
+``python bench.py --arch-bench [--arch-design filevik|sedopel|pebodra|dogilorn|mugipel] [--arch-size s|m]`` (random
 weights, synthetic tokens).  The default bench workload and its JSON line are untouched; this prints one
 JSON object of its own.
+
+The Mugipel stack alternates chunked grouped-query attention (capped scores, a learned sink per head,
+a sigmoid gate) and latent attention, each beside a dense squared-relu feed-forward that shares its
+projections, and runs its middle layers twice; its comparison model is a dense Llama of the same
+width, heads, depth (counting every run) and parameters a token reads, and kernel by kernel:
+attention against the Dogilorn and Sedopel attention and the Llama kernels at the same heads, latent
+attention against Filevik's, its prep and residual launches against the like launches of the others.
 
 The Dogilorn stack is attention only (grouped-query, an RMS norm over the whole q and k projections,
 a sliding window that also keeps the first tokens, a sink term in the softmax; every third layer reads
@@ -79,6 +86,112 @@ DOGILORN_SIZES = {
     "m": dict(width=2048, layers=12, heads=16, kv_heads=4, dim=128, vdim=128, rot=64, window=1024, keep_first=128, taps=4,
               experts=8, identity=2, top=2, ff=2048, shared=2048, dense_ff=8192, vocab=32000),
 }
+
+
+MUGIPEL_SIZES = {
+    "s": dict(width=1024, layers=6, loop=(2, 4, 2), heads=16, kv_heads=4, dim=64, vdim=64, rot=32, chunk=1024, kv_rank=256,
+              ff=4096, vocab=32000),
+    "m": dict(width=2048, layers=12, loop=(4, 8, 2), heads=16, kv_heads=4, dim=128, vdim=128, rot=64, chunk=1024, kv_rank=512,
+              ff=8192, vocab=32000),
+}
+
+
+def mugipel_raw(z: dict) -> dict:
+    att = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["vdim"], "scale": z["dim"] ** -0.5,
+           "softcap": 30.0, "mask": {"size": z["chunk"]},
+           "rot": {"dims": z["rot"], "base": 10000.0, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    lat = {"heads": z["heads"], "dim": z["dim"], "vdim": z["vdim"], "kv_rank": z["kv_rank"], "scale": z["dim"] ** -0.5}
+    mlp = {"kind": "dense", "ff": z["ff"]}
+    return {"architecture": "Mugipel", "width": z["width"], "vocab": z["vocab"], "norm": {"eps": 1e-5}, "residual_mult": 0.5,
+            "loop": dict(zip(("start", "stop", "times"), z["loop"])),
+            "layers": [{"type": "latent_attention", "mixer": lat, "mlp": mlp} if i % 2 else {"type": "attention", "mixer": att, "mlp": mlp}
+                       for i in range(z["layers"])]}
+
+
+def mugipel_twin(z: dict):
+    """A dense Llama that runs as many layers and reads as many parameters per token."""
+    from ..models.configs import ModelConfig, mugipel_config
+    c = mugipel_config(mugipel_raw(z))
+    mk = lambda inter: ModelConfig(f"llama-{z['width']}", z["width"], len(c.runs), z["heads"], z["kv_heads"], z["dim"], inter,
+                                   z["vocab"], 10000.0, 1e-6, 16384, tie_embeddings=True)
+    once = mugipel_config(dict(mugipel_raw(z), loop=None)).num_params()
+    body = (once - z["vocab"] * z["width"]) * len(c.runs) // c.n_layers       # every layer has about the same size
+    target = z["vocab"] * z["width"] + body + z["loop"][2] * 2 * z["width"] ** 2
+    inter = (target - mk(0).num_params()) // (3 * z["width"] * len(c.runs))
+    return mk(max(64, inter // 64 * 64))
+
+
+def mugipel_kernel_rooflines(z: dict, T: int = 4096, B: int = 64, ctx: int = 2047) -> Dict[str, dict]:
+    """Each Mugipel kernel alone (bf16): prefill of one T-token sequence, decode of B sequences at
+    ``ctx`` (the last position of a chunk); time, the bound resource's minimum time, and their ratio."""
+    from .. import ops
+    from ..models.llama import AttnMeta
+    from ..ops import seqmix
+    dev, bf = "cuda", torch.bfloat16
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)
+    res: Dict[str, dict] = {}
+
+    def rec(name, sec, bytes_, flops, peak_flops):
+        floor = max(bytes_ / PEAK_BW, flops / peak_flops)
+        res[name] = {"us": round(sec * 1e6, 1), "roofline_us": round(floor * 1e6, 2), "x_roofline": round(sec / floor, 1),
+                     "bound": "memory" if bytes_ / PEAK_BW >= flops / peak_flops else "compute"}
+
+    W, H, G, d, dv, C, r, ff = (z[k] for k in ("width", "heads", "kv_heads", "dim", "vdim", "chunk", "kv_rank", "ff"))
+    hv = H * dv
+    for tag, qlens, starts in (("prefill", [T], [0]), ("decode", [1] * B, [ctx] * B)):
+        n, S = sum(qlens), len(qlens)
+        qstart = i32([sum(qlens[:i]) for i in range(S)])
+        cxl = [a + b for a, b in zip(starts, qlens)]
+        qlen, cx = i32(qlens), i32(cxl)
+        pos = i32([p for a, m in zip(starts, qlens) for p in range(a, a + m)])
+        # causal (query, key) pairs, and those inside a chunk; keys that any row of a sequence reads
+        keys = sum((a + (m + 1) / 2) * m for a, m in zip(starts, qlens))
+        ckeys = sum(p % C + 1 for a, m in zip(starts, qlens) for p in range(a, a + m))
+        cread = sum(c - a // C * C for a, c in zip(starts, cxl))
+        nb = (max(cxl) + 15) // 16
+        bt = torch.arange(S * nb, dtype=torch.int32, device=dev).view(S, nb)
+        slots = i32([int(bt[i, p // 16]) * 16 + p % 16 for i, (a, m) in enumerate(zip(starts, qlens)) for p in range(a, a + m)])
+        meta = AttnMeta(slots=None, block_tables=bt, qstart=qstart, qlen=qlen, ctx=cx, tile_seq=None, tile_tok0=None,
+                        last_idx=None, host_qlen=qlens)
+        both = torch.empty(n, hv + ff, device=dev, dtype=bf)
+        # chunked attention and its prep
+        kc = (torch.randn(S * nb, G, 16, d, device=dev) * 0.3).to(bf)
+        vc = (torch.randn(S * nb, G, dv, 16, device=dev) * 0.3).to(bf)
+        qkv = (H + G) * d + G * dv
+        proj = torch.randn(n, qkv + hv + ff, device=dev).to(bf)
+        table = ops.rope_cos_sin(ctx + T + 8, z["rot"], 10000.0, dev)
+        prep = lambda: seqmix.rope_prep(proj, H, G, d, dv, table, z["rot"], d ** -0.5, pos, slots, kc, vc, qkv + hv, both[:, hv:])
+        q = prep()
+        rec(f"rope_prep_{tag}", _timed(prep), n * (qkv + ff) * 4, n * ((H + G) * d * 6 + ff * 2), PEAK_F32)
+        mfma = seqmix.gqa_use_mfma(q, H, G, d, dv, 16)
+        ts, tt = meta.latent_tiles(1, dev, seqmix.gqa_tokens_per_tile(H, G, mfma))
+        sp = seqmix.gqa_splits(int(ts.numel()), G, max(cxl), chunk=C) if mfma else 1
+        sinks = torch.zeros(H, device=dev)
+        rec(f"attention_{tag}",
+            _timed(lambda: seqmix.paged_gqa_attention(q, kc, vc, bt, qstart, qlen, cx, ts, tt, proj[:, qkv:qkv + hv], mfma, sp,
+                                                      out=both[:, :hv], chunk=C, softcap=30.0, sinks=sinks)),
+            cread * G * (d + dv) * 2 + n * H * (d + 2 * dv) * 2, ckeys * H * 2 * (d + dv), PEAK_BF16)
+        # latent attention, its prep, and the gated heads
+        cache = (torch.randn(S * nb, 16, r, device=dev) * 0.3).to(bf)
+        lproj = torch.randn(n, H * d + r + hv + ff, device=dev).to(bf)
+        nw = torch.ones(r, device=dev)
+        rec(f"latent_prep_{tag}", _timed(lambda: seqmix.latent_prep(lproj, H * d, nw, 1e-5, slots, cache, H * d + r + hv, both[:, hv:])),
+            n * (r + ff) * 4, n * (r * 4 + ff * 2), PEAK_F32)
+        qa = (torch.randn(H, n, r, device=dev) * 0.3).to(bf)
+        lrows = seqmix.latent_rows(qa, r, 0, n, S)
+        ls, lt = meta.latent_tiles(H, dev, lrows)
+        rec(f"latent_attention_{tag}",
+            _timed(lambda: seqmix.latent_attention(qa, lproj, d, 0, pos, table, cache, bt, qstart, qlen, cx, ls, lt, 0.1, rows=lrows), 3),
+            sum(cxl) * r * 2 + n * H * r * 4, keys * H * 4 * r, PEAK_BF16)
+        o = torch.randn(H, n, dv, device=dev).to(bf)
+        rec(f"gate_heads_{tag}", _timed(lambda: seqmix.gate_heads(o, lproj[:, H * d + r:H * d + r + hv], both[:, :hv])),
+            n * hv * 6, n * hv * 8, PEAK_F32)
+        # the layer's tail
+        x, y, w = torch.randn(n, W, device=dev), torch.randn(n, W, device=dev).to(bf), torch.ones(W, device=dev)
+        h = torch.empty(n, W, device=dev, dtype=bf)
+        rec(f"scaled_resadd_rms_{tag}", _timed(lambda: seqmix.scaled_resadd_rms(x, 1e-5, y=y, mult=0.5, w=w, out=h)), n * W * 12,
+            n * W * 6, PEAK_F32)
+    return res
 
 
 def dogilorn_raw(z: dict) -> dict:
@@ -539,7 +652,25 @@ def llama_kernel_rooflines(T: int = 4096, B: int = 64, ctx: int = 2048, nq: int 
 
 
 def run(size: str = "s", kernels_only: bool = False, design: str = "filevik") -> dict:
-    from ..models.configs import dogilorn_config, filevik_config, pebodra_config, sedopel_config
+    from ..models.configs import dogilorn_config, filevik_config, mugipel_config, pebodra_config, sedopel_config
+    if design == "mugipel":
+        z = MUGIPEL_SIZES[size]
+        out = {"bench": "arch", "design": design, "size": size, "dtype": "bf16", "data": "synthetic", "sizes": z}
+        out["mugipel_kernels"] = mugipel_kernel_rooflines(z)
+        # the like kernels at like sizes: attention inside a window (Dogilorn) and over everything (Sedopel),
+        # the Llama attention kernels, latent attention with a rotated part (Filevik)
+        out["dogilorn_kernels"] = dogilorn_kernel_rooflines(dict(DOGILORN_SIZES[size], heads=z["heads"], kv_heads=z["kv_heads"],
+                                                                 dim=z["dim"], vdim=z["vdim"], window=z["chunk"]))
+        out["filevik_kernels"] = kernel_rooflines(dict(SIZES[size], lat_heads=z["heads"], lat_dim=z["dim"], lat_v=z["vdim"],
+                                                       kv_rank=z["kv_rank"]))
+        out["llama_kernels"] = llama_kernel_rooflines(nq=z["heads"], nkv=z["kv_heads"], d=z["dim"])
+        if not kernels_only:
+            prompts, batches = [512, 2048], [1, 16, 64]
+            out["mugipel"] = engine_throughput(mugipel_config(mugipel_raw(z), name=f"mugipel-{size}"), prompts, batches, ctx=1024,
+                                               new=32, rows=64)
+            out["llama"] = engine_throughput(mugipel_twin(z), prompts, batches, ctx=1024, new=32, rows=64)
+        print(json.dumps(out))
+        return out
     if design == "dogilorn":
         z = DOGILORN_SIZES[size]
         out = {"bench": "arch", "design": design, "size": size, "dtype": "bf16", "data": "synthetic", "sizes": z}
