@@ -100,8 +100,11 @@ int dllm_paged_gqa(const void*, const void*, const void*, int, const int*, int, 
                    int, float, int, float, const float*, long, hipStream_t);
 int dllm_rope_prep(const void*, long, int, int, int, int, int, const float*, int, int, float, const int*, const int*, void*, void*,
                    void*, long, int, int, int, void*, long, void*, long, int, hipStream_t);
-int dllm_latent_prep(const void*, long, int, int, int, const float*, float, const int*, void*, int, int, void*, long, long,
-                     hipStream_t);
+int dllm_latent_prep(const void*, long, int, int, int, const float*, float, const int*, void*, int, int, void*, long, void*, int,
+                     float, long, hipStream_t);
+int dllm_latent_expand_ok(int, int, int);
+int dllm_latent_expand(const void*, const int*, int, int, int, int, const int*, int, int, int, int, const void*, const void*, void*,
+                       void*, hipStream_t);
 int dllm_gate_heads(const void*, int, const void*, long, void*, long, int, int, long, hipStream_t);
 int dllm_scaled_resadd_rms(const void*, long, int, float, int, const float*, float*, const float*, void*, long, long, int, float,
                            hipStream_t);
@@ -1793,7 +1796,7 @@ void rope_prep(torch::Tensor proj, int64_t H, int64_t G, int64_t d, int64_t dv, 
 }
 
 void latent_prep(torch::Tensor proj, int64_t ccol, torch::Tensor w, double eps, torch::Tensor slots, torch::Tensor cache,
-                 int64_t ucol, c10::optional<torch::Tensor> act) {
+                 int64_t ucol, c10::optional<torch::Tensor> act, c10::optional<torch::Tensor> q, double qscale) {
   const bool f = act_f32(proj, "proj");
   check_rows2d(proj, "proj");
   check_f32(w, "norm weight");
@@ -1813,9 +1816,42 @@ void latent_prep(torch::Tensor proj, int64_t ccol, torch::Tensor w, double eps, 
     ap = act->data_ptr();
     lda = act->stride(0);
   }
+  void* qp = nullptr;
+  int64_t nq = 0;
+  if (q) {
+    TORCH_CHECK(q->is_cuda() && q->scalar_type() == proj.scalar_type() && q->is_contiguous() && (T == 0 || q->numel() % T == 0),
+                "q [T, ...] contiguous in the activations' dtype");
+    nq = T ? q->numel() / T : 0;
+    TORCH_CHECK(nq <= proj.size(1), "q columns of proj");
+    qp = q->data_ptr();
+  }
   ok(dllm_latent_prep(proj.data_ptr(), proj.stride(0), f, (int)ccol, (int)rank, w.data_ptr<float>(), (float)eps,
-                      slots.data_ptr<int>(), cache.data_ptr(), (int)ucol, (int)ff, ap, lda, (long)T, stream()),
+                      slots.data_ptr<int>(), cache.data_ptr(), (int)ucol, (int)ff, ap, lda, qp, (int)nq, (float)qscale, (long)T,
+                      stream()),
      "latent_prep");
+}
+
+void latent_expand(torch::Tensor cache, torch::Tensor bt, torch::Tensor ctx, torch::Tensor wk, torch::Tensor wv, torch::Tensor kc,
+                   torch::Tensor vc) {
+  check_i32(bt, "block_tables");
+  check_i32(ctx, "ctx");
+  TORCH_CHECK(cache.is_cuda() && cache.scalar_type() == torch::kBFloat16 && cache.is_contiguous() && cache.dim() == 3 &&
+                  cache.size(1) == 16,
+              "cache [blocks, 16, rank] bf16");
+  const int64_t S = ctx.numel(), nb = bt.size(1), rank = cache.size(2);
+  TORCH_CHECK(bt.dim() == 2 && bt.stride(1) == 1 && bt.size(0) >= S && ctx.is_contiguous(), "block_tables [S, blocks], ctx [S]");
+  for (auto* t : {&kc, &vc, &wk, &wv})
+    TORCH_CHECK(t->is_cuda() && t->scalar_type() == torch::kBFloat16 && t->is_contiguous(), "bf16 contiguous tensors");
+  TORCH_CHECK(kc.dim() == 4 && vc.dim() == 4 && kc.size(0) == S * nb && vc.size(0) == S * nb && kc.size(1) == vc.size(1) &&
+                  kc.size(2) == 16 && vc.size(3) == 16,
+              "K [S blocks, H, 16, d], V [S blocks, H, dv, 16]");
+  const int64_t H = kc.size(1), d = kc.size(3), dv = vc.size(2);
+  TORCH_CHECK(wk.numel() == H * d * rank && wv.numel() == H * dv * rank && dllm_latent_expand_ok((int)rank, (int)d, (int)dv),
+              "weights [H d, rank], [H dv, rank]; rank % 32 == 0, d % 8 == 0");
+  ok(dllm_latent_expand(cache.data_ptr(), bt.data_ptr<int>(), (int)bt.stride(0), (int)S, (int)nb, (int)cache.size(0),
+                        ctx.data_ptr<int>(), (int)rank, (int)H, (int)d, (int)dv, wk.data_ptr(), wv.data_ptr(), kc.data_ptr(),
+                        vc.data_ptr(), stream()),
+     "latent_expand");
 }
 
 void gate_heads(torch::Tensor o, torch::Tensor gate, torch::Tensor out) {
@@ -2320,6 +2356,8 @@ PYBIND11_MODULE(_hip_kernels, m) {
         py::arg("chunk") = 0, py::arg("cap") = 0.0, py::arg("sinks") = py::none());
   m.def("rope_prep", &rope_prep);
   m.def("latent_prep", &latent_prep);
+  m.def("latent_expand", &latent_expand);
+  m.def("latent_expand_ok", [](int64_t rank, int64_t d, int64_t dv) { return dllm_latent_expand_ok((int)rank, (int)d, (int)dv) != 0; });
   m.def("gate_heads", &gate_heads);
   m.def("scaled_resadd_rms", &scaled_resadd_rms);
   m.def("gqa_tile_tokens",

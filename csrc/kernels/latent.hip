@@ -9,6 +9,8 @@
 //                     (interleaved pairs), write both into the token's cache slot
 //   latent_prep       latent_kv_write without a rotated part for a layer whose feed-forward shares the
 //                     projection: the same launch squares the relu of the up columns
+//   latent_expand     keys and values of every head from the cached latents of a step's sequences, into
+//                     pages of their own (prompt portions then run the grouped-query attention kernel)
 //   gate_heads        per-head outputs [H, T, dv] times sigmoid(gate), laid out token-major
 //   latent_attention  one workgroup per 16 rows (token-major (token, head) rows of one sequence):
 //                     the rows' queries staged once in LDS as f32 (rotation and the score scale
@@ -64,7 +66,9 @@ template <typename T>
 __global__ void __launch_bounds__(256) latent_prep_kernel(const T* __restrict__ proj, long ld, int ccol, int rank,
                                                           const float* __restrict__ w, float eps,
                                                           const int* __restrict__ slots, T* __restrict__ cache, int ucol,
-                                                          int ff, T* __restrict__ act, long lda, int vec) {
+                                                          int ff, T* __restrict__ act, long lda, int vec,
+                                                          T* __restrict__ q, int nq, float qscale) {
+  // q (optional): the row's first nq columns times qscale, as rows of a matrix of their own
   const long tok = blockIdx.x;
   const int tid = threadIdx.x;
   const T* row = proj + tok * ld;
@@ -77,6 +81,8 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(const T* __restrict__ 
     T* dst = cache + (long)slot * rank;
     for (int i = tid; i < rank; i += 64) stf(dst + i, ldf(r + i) * rs * w[i]);
   }
+  if (q)
+    for (int i = blockIdx.y * 256 + tid; i < nq; i += gridDim.y * 256) stf(q + tok * nq + i, ldf(row + i) * qscale);
   if (!act) return;
   const T* up = row + ucol;
   T* a = act + tok * lda;
@@ -95,6 +101,97 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(const T* __restrict__ 
   for (int i = blockIdx.y * 256 + tid; i < ff; i += gridDim.y * 256) {
     const float v = fmaxf(ldf(up + i), 0.f);
     stf(a + i, v * v);
+  }
+}
+
+// Keys and values of one head from 64 cached latents (four pages of one sequence): K = C Wk^T, V = C Wv^T
+// with C [64, rank] staged in LDS, Wk [H d, rank], Wv [H dv, rank] (rank % 32 == 0, d % 8 == 0).  A wave
+// owns groups of NB 16-column blocks, first the key columns', then the value columns', over all 64 latents.
+// Operands of v_mfma_f32_16x16x32_bf16 hold rows of either matrix alike (row lane & 15, contraction
+// 8 (lane >> 4) ..), so keys are made as W C^T (four key dims of a latent per lane) and values as C W^T (four
+// latents of a value dim per lane): both leave as 8-byte vectors.  Output pages: K [S nb, H, 16, d], V
+// [S nb, H, dv, 16], page (s, j) at s nb + j.
+template <int NB>
+__global__ void __launch_bounds__(256) latent_expand_kernel(const u16* __restrict__ cache, const int* __restrict__ bt, int bt_ld,
+                                                            int nb, int pages, const int* __restrict__ ctx, int rank, int H,
+                                                            int d, int dv, const u16* __restrict__ wk,
+                                                            const u16* __restrict__ wv, u16* __restrict__ kc,
+                                                            u16* __restrict__ vc) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char smx[];
+  u16* csh = reinterpret_cast<u16*>(smx);      // [64][rank + 8]
+  const int s = blockIdx.z, h = blockIdx.y, j0 = blockIdx.x * 4;
+  if (j0 * 16 >= ctx[s]) return;               // nothing of the sequence lies here (uniform)
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int lr = lane & 15, g4 = lane >> 4;
+  const int str = rank + 8, ch = rank >> 3;
+  for (int e = tid; e < 64 * ch; e += 256) {
+    const int t = e / ch, c = e - t * ch, j = j0 + (t >> 4);
+    uint4 v = make_uint4(0u, 0u, 0u, 0u);
+    if (j < nb) {
+      const int pg = bt[(long)s * bt_ld + j];
+      if (pg >= 0 && pg < pages) v = ld16(cache + ((long)pg * 16 + (t & 15)) * rank + 8 * c);
+    }
+    st16(csh + t * str + 8 * c, v);
+  }
+  __syncthreads();
+  const int kblk = (d + 15) >> 4, vblk = (dv + 15) >> 4;
+  const int kgr = (kblk + NB - 1) / NB, ngr = kgr + (vblk + NB - 1) / NB;
+  for (int gi = wave; gi < ngr; gi += 4) {
+    const bool key = gi < kgr;                 // wave-uniform
+    const int b0 = (key ? gi : gi - kgr) * NB, cols = key ? d : dv;
+    const u16* w = (key ? wk : wv) + (long)h * cols * rank;
+    const u16* wp[NB];
+#pragma unroll
+    for (int b = 0; b < NB; ++b) wp[b] = w + (long)min((b0 + b) * 16 + lr, cols - 1) * rank + 8 * g4;   // rows past the end: any
+    f32x4 acc[4][NB];
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+#pragma unroll
+      for (int b = 0; b < NB; ++b) acc[t][b] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const u16* cp = csh + lr * str + 8 * g4;
+    if (key) {
+#pragma unroll 2
+      for (int k = 0; k < rank; k += 32) {
+        bf16x8 wf[NB];
+#pragma unroll
+        for (int b = 0; b < NB; ++b) wf[b] = __builtin_bit_cast(bf16x8, ld16(wp[b] + k));
+#pragma unroll
+        for (int t = 0; t < 4; ++t) {
+          const bf16x8 cf = __builtin_bit_cast(bf16x8, ld16(cp + 16 * t * str + k));
+#pragma unroll
+          for (int b = 0; b < NB; ++b) acc[t][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[b], cf, acc[t][b], 0, 0, 0);
+        }
+      }
+    } else {
+#pragma unroll 2
+      for (int k = 0; k < rank; k += 32) {
+        bf16x8 wf[NB];
+#pragma unroll
+        for (int b = 0; b < NB; ++b) wf[b] = __builtin_bit_cast(bf16x8, ld16(wp[b] + k));
+#pragma unroll
+        for (int t = 0; t < 4; ++t) {
+          const bf16x8 cf = __builtin_bit_cast(bf16x8, ld16(cp + 16 * t * str + k));
+#pragma unroll
+          for (int b = 0; b < NB; ++b) acc[t][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cf, wf[b], acc[t][b], 0, 0, 0);
+        }
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+      if (j0 + t >= nb) continue;
+      const long page = ((long)s * nb + j0 + t) * H + h;
+#pragma unroll
+      for (int b = 0; b < NB; ++b) {
+        const f32x4 a = acc[t][b];
+        const uint2 v = make_uint2((uint32_t)f2bf(a[0]) | ((uint32_t)f2bf(a[1]) << 16), (uint32_t)f2bf(a[2]) | ((uint32_t)f2bf(a[3]) << 16));
+        const int c0 = (b0 + b) * 16;
+        if (key) {
+          if (c0 + 4 * g4 < d) *reinterpret_cast<uint2*>(kc + (page * 16 + lr) * d + c0 + 4 * g4) = v;
+        } else {
+          if (c0 + lr < dv) *reinterpret_cast<uint2*>(vc + (page * dv + c0 + lr) * 16 + 4 * g4) = v;
+        }
+      }
+    }
   }
 }
 
@@ -804,7 +901,8 @@ extern "C" int dllm_latent_attention(const void* qa, const void* q, long ldq, in
 }
 
 extern "C" int dllm_latent_prep(const void* proj, long ld, int f32, int ccol, int rank, const float* w, float eps,
-                                const int* slots, void* cache, int ucol, int ff, void* act, long lda, long T, hipStream_t st) {
+                                const int* slots, void* cache, int ucol, int ff, void* act, long lda, void* q, int nq,
+                                float qscale, long T, hipStream_t st) {
   if (T <= 0) return 0;
   if (rank < 1 || (act && ff < 1)) return -1;
   const dim3 grid((unsigned)T, act ? (ff + 2047) / 2048 : 1);
@@ -812,10 +910,10 @@ extern "C" int dllm_latent_prep(const void* proj, long ld, int f32, int ccol, in
                   (uintptr_t)act % 16 == 0;
   if (f32)
     hipLaunchKernelGGL(latent_prep_kernel<float>, grid, dim3(256), 0, st, (const float*)proj, ld, ccol, rank, w, eps, slots,
-                       (float*)cache, ucol, ff, (float*)act, lda, vec);
+                       (float*)cache, ucol, ff, (float*)act, lda, vec, (float*)q, nq, qscale);
   else
     hipLaunchKernelGGL(latent_prep_kernel<u16>, grid, dim3(256), 0, st, (const u16*)proj, ld, ccol, rank, w, eps, slots,
-                       (u16*)cache, ucol, ff, (u16*)act, lda, vec);
+                       (u16*)cache, ucol, ff, (u16*)act, lda, vec, (u16*)q, nq, qscale);
   return (int)hipGetLastError();
 }
 
@@ -830,5 +928,31 @@ extern "C" int dllm_gate_heads(const void* o, int f32, const void* gate, long ld
   else
     hipLaunchKernelGGL(gate_heads_kernel<u16>, grid, dim3(256), 0, st, (const u16*)o, (const u16*)gate, ldg, (u16*)out, ldo, H,
                        dv, T);
+  return (int)hipGetLastError();
+}
+
+// 1 when latent_expand takes the shape (bf16; the 64 latents of a workgroup fit the LDS)
+extern "C" int dllm_latent_expand_ok(int rank, int d, int dv) {
+  return rank >= 32 && rank % 32 == 0 && rank <= 1024 && d >= 8 && d % 8 == 0 && dv >= 1;
+}
+
+extern "C" int dllm_latent_expand(const void* cache, const int* bt, int bt_ld, int S, int nb, int pages, const int* ctx, int rank,
+                                  int H, int d, int dv, const void* wk, const void* wv, void* kc, void* vc, hipStream_t st) {
+  if (S <= 0 || nb <= 0) return 0;
+  if (!dllm_latent_expand_ok(rank, d, dv) || H < 1 || S > 65535 || H > 65535) return -1;
+  const long lds = 64L * (rank + 8) * 2;
+  const dim3 grid((nb + 3) / 4, H, S);
+#define LEX(NB)                                                                                                        \
+  do {                                                                                                                 \
+    static long have_ = 48 * 1024;                                                                                     \
+    if (lds > have_) {                                                                                                 \
+      hipFuncSetAttribute((const void*)latent_expand_kernel<NB>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
+      have_ = lds;                                                                                                     \
+    }                                                                                                                  \
+    hipLaunchKernelGGL(latent_expand_kernel<NB>, grid, dim3(256), lds, st, (const u16*)cache, bt, bt_ld, nb, pages, ctx, rank, H, \
+                       d, dv, (const u16*)wk, (const u16*)wv, (u16*)kc, (u16*)vc);                                     \
+  } while (0)
+  if (d >= 128 && dv >= 128) LEX(4); else if (d >= 64 || dv >= 64) LEX(2); else LEX(1);
+#undef LEX
   return (int)hipGetLastError();
 }

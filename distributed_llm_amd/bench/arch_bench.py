@@ -183,6 +183,18 @@ def mugipel_kernel_rooflines(z: dict, T: int = 4096, B: int = 64, ctx: int = 204
         rec(f"latent_attention_{tag}",
             _timed(lambda: seqmix.latent_attention(qa, lproj, d, 0, pos, table, cache, bt, qstart, qlen, cx, ls, lt, 0.1, rows=lrows), 3),
             sum(cxl) * r * 2 + n * H * r * 4, keys * H * 4 * r, PEAK_BF16)
+        if tag == "prefill":      # ... or on keys and values made from the latents (what a step of long portions runs)
+            uk, uv = (torch.randn(H, d, r, device=dev) * 0.05).to(bf), (torch.randn(H, dv, r, device=dev) * 0.05).to(bf)
+            qx = torch.randn(n, H, d, device=dev).to(bf)
+            xm = seqmix.gqa_use_mfma(qx, H, H, d, dv, 16)
+            xs, xt = meta.latent_tiles(1, dev, seqmix.gqa_tokens_per_tile(H, H, xm))
+            rec("latent_expand_prefill", _timed(lambda: seqmix.latent_expand(cache, bt, cx, uk, uv)),
+                sum(cxl) * (r + H * (d + dv)) * 2, sum(cxl) * H * (d + dv) * r * 2, PEAK_BF16)
+            ek, ev, et = seqmix.latent_expand(cache, bt, cx, uk, uv)
+            rec("latent_expanded_attention_prefill",
+                _timed(lambda: seqmix.paged_gqa_attention(qx, ek, ev, et, qstart, qlen, cx, xs, xt, lproj[:, H * d + r:H * d + r + hv],
+                                                          xm, 1, out=both[:, :hv])),
+                sum(cxl) * H * (d + dv) * 2 + n * H * (d + 2 * dv) * 2, keys * H * 2 * (d + dv), PEAK_BF16)
         o = torch.randn(H, n, dv, device=dev).to(bf)
         rec(f"gate_heads_{tag}", _timed(lambda: seqmix.gate_heads(o, lproj[:, H * d + r:H * d + r + hv], both[:, :hv])),
             n * hv * 6, n * hv * 8, PEAK_F32)

@@ -57,7 +57,9 @@ they do not take and for f32 models), everything between them on the HIP kernels
              [out | down] over the heads and the activations together
   latent     (direct queries, gated heads) one fused projection q | latent | gate | up -> the latent's
              norm, its page and relu(up)^2 in one launch -> absorbed latent attention as above -> value
-             up-projection per head, gate -> one projection [out | down]
+             up-projection per head, gate -> one projection [out | down].  Steps of longer prompt
+             portions make every head's keys and values from the latents they read, in scratch pages,
+             and run the grouped-query kernel on them instead
 
 Layer forms: ``x += norm(sublayer(x))`` (Filevik) or, with ``cfg.pre_norm``, a norm on both sides,
 ``x += norm_b(sublayer(norm(x)))``, or without ``cfg.post_norm`` ``x += ls * sublayer(layernorm(x))``
@@ -485,7 +487,8 @@ class HybridModel:
         else:
             D["dkv_norm"] = f32(t[p + "mix.dkv.norm"])
             D["uk"] = put(t[p + "mix.uk"].view(m.heads, m.dim, m.kv_rank))                       # [H, d, r]
-            D["uvT"] = put(t[p + "mix.uv"].view(m.heads, m.vdim, m.kv_rank).transpose(1, 2))    # [H, r, dv]
+            D["uv"] = put(t[p + "mix.uv"].view(m.heads, m.vdim, m.kv_rank))                      # [H, dv, r]
+            D["uvT"] = D["uv"].transpose(1, 2).contiguous()                                      # [H, r, dv]
             n = m.heads * m.dim + m.kv_rank
             assert D["dkv_norm"].numel() == m.kv_rank
         ff = f.ff if f is not None else 0
@@ -507,7 +510,7 @@ class HybridModel:
         for i, _ in self.cfg.runs:      # a looped layer is read in every pass
             L, S = self.layers[i], self.cfg.layers[i]
             for k, x in L.items():
-                if not torch.is_tensor(x):
+                if not torch.is_tensor(x) or k == "uv":      # (prompt steps read that layout of uvT)
                     continue
                 b = x.numel() * x.element_size()
                 if k in ("w1", "w2", "w2d") and top_only and isinstance(S.mlp, MoESpec):
@@ -759,14 +762,26 @@ class HybridModel:
         return _mm(both, L["out"])
 
     def _latent_ff(self, L, m: MixerSpec, f: Optional[DenseSpec], x, positions, meta, cache):
-        """mixer(x) + ff(x) with latent attention (absorbed form, direct queries, gated heads)."""
+        """mixer(x) + ff(x) with latent attention (direct queries, gated heads): on the cached latents
+        (absorbed form), or for steps of longer prompt portions on keys and values made from them."""
         T, H, hv = x.shape[0], m.heads, m.heads * m.vdim
         proj = _mm(x, L["proj"])                                        # q | latent | gate | up
         c0 = H * m.dim
         g0 = c0 + m.kv_rank
         both = torch.empty((T, hv + (f.ff if f is not None else 0)), dtype=x.dtype, device=x.device)
-        seqmix.latent_prep(proj, c0, L["dkv_norm"], self.cfg.rms_eps, meta.slots, cache[0], g0 + hv,
-                           both[:, hv:] if f is not None else None)
+        act = both[:, hv:] if f is not None else None
+        S = 0 if meta.host_qlen is None else len(meta.host_qlen)
+        if S and self._all_rows(x, meta) and seqmix.latent_expand_wanted(cache[0], H, m.dim, m.vdim, T, S, meta.block_tables.numel()):
+            q = torch.empty((T, H, m.dim), dtype=x.dtype, device=x.device)
+            seqmix.latent_prep(proj, c0, L["dkv_norm"], self.cfg.rms_eps, meta.slots, cache[0], g0 + hv, act, q, m.scale)
+            k, v, table = seqmix.latent_expand(cache[0], meta.block_tables, meta.ctx, L["uk"], L["uv"])
+            mfma = seqmix.gqa_use_mfma(q, H, H, m.dim, m.vdim, k.shape[2])
+            ts, tt = meta.latent_tiles(1, self.device, seqmix.gqa_tokens_per_tile(H, H, mfma))
+            splits = seqmix.gqa_splits(int(ts.numel()), H, meta.max_ctx) if mfma else 1
+            seqmix.paged_gqa_attention(q, k, v, table, meta.qstart, meta.qlen, meta.ctx, ts, tt, proj[:, g0:g0 + hv], mfma, splits,
+                                       out=both[:, :hv])
+            return _mm(both, L["out"])
+        seqmix.latent_prep(proj, c0, L["dkv_norm"], self.cfg.rms_eps, meta.slots, cache[0], g0 + hv, act)
         q = proj[:, :c0]
         qa = torch.bmm(q.unflatten(1, (H, m.dim)).transpose(0, 1), L["uk"])     # key up-projection absorbed: [H, T, rank]
         rows = (seqmix.LAT_ROWS if meta.host_qlen is None else

@@ -1064,8 +1064,23 @@ def rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, posit
     return (qk[:, :H] * qscale).to(proj.dtype)
 
 
-def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol=0, act=None):
-    """cache[slot] = rmsnorm(proj[:, ccol : ccol + rank]) * norm_w; act = relu(proj[:, ucol:])^2."""
+def latent_expand(cache, block_tables, wk, wv):
+    """Keys and values of every head from cached latents: page (s, j) of the block tables [S, nb] becomes
+    page s nb + j of K [S nb, heads, block, dim] and V [S nb, heads, vdim, block]; wk [heads, dim, rank],
+    wv [heads, vdim, rank]."""
+    (H, d, r), dv = wk.shape, wv.shape[1]
+    c = cache[block_tables.reshape(-1).long()]                       # [pages, block, rank]
+    P, B = c.shape[:2]
+    k = (c.reshape(P * B, r) @ wk.reshape(H * d, r).t()).view(P, B, H, d).transpose(1, 2).contiguous()
+    v = (c.reshape(P * B, r) @ wv.reshape(H * dv, r).t()).view(P, B, H, dv).permute(0, 2, 3, 1).contiguous()
+    return k, v
+
+
+def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol=0, act=None, q=None, qscale=1.0):
+    """cache[slot] = rmsnorm(proj[:, ccol : ccol + rank]) * norm_w; act = relu(proj[:, ucol:])^2; q =
+    the first columns times qscale."""
+    if q is not None:
+        q.view(proj.shape[0], -1).copy_((proj[:, :q[0].numel()].float() * qscale).to(q.dtype))
     r = norm_w.numel()
     c = rms_rows(proj[:, ccol:ccol + r], norm_w, eps, torch.float32)
     ok = slots >= 0

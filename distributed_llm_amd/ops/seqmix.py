@@ -629,14 +629,52 @@ def rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, posit
     return q
 
 
-def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol: int = 0, act: Optional[torch.Tensor] = None) -> None:
+LATENT_EXPAND_MIN = 32                 # average new tokens per sequence from which a step expands its latents
+LATENT_EXPAND_BYTES = 2 << 30          # ... and the most bytes of expanded keys and values
+
+
+def latent_expand_wanted(cache: torch.Tensor, heads: int, dim: int, vdim: int, tokens: int, seqs: int, blocks: int) -> bool:
+    """Whether a step of prompt portions makes the keys and values of every head from the latents it
+    reads and runs the grouped-query kernel on them (dim + vdim products per key and head) instead of
+    attention on the latents themselves (2 rank products): worth the extra projection when enough new
+    tokens read each latent."""
+    if tokens < LATENT_EXPAND_MIN * seqs or dim > 256 or vdim > 256 or dim + vdim > 2 * cache.shape[2]:
+        return False
+    if blocks * cache.shape[1] * heads * (dim + vdim) * cache.element_size() > LATENT_EXPAND_BYTES:
+        return False
+    if cache.is_cuda and cache.dtype == torch.bfloat16:      # the matrix-core attention or none
+        ext = _native(cache)
+        return bool(ext.gqa_mfma_ok(False, heads, heads, dim, vdim, cache.shape[1]))
+    return True
+
+
+def latent_expand(cache: torch.Tensor, block_tables: torch.Tensor, ctx: torch.Tensor, wk: torch.Tensor,
+                  wv: torch.Tensor) -> Tuple[torch.Tensor, torch.Tensor, torch.Tensor]:
+    """Keys and values of every head from the cached latents (cache [blocks, 16, rank]) that the sequences'
+    block tables [S, nb] name: K [S nb, heads, 16, dim], V [S nb, heads, vdim, 16] and their block tables,
+    for ``paged_gqa_attention``.  wk [heads, dim, rank], wv [heads, vdim, rank].  Pages past a sequence's
+    context hold nothing meaningful."""
+    S, nb = block_tables.shape
+    (H, d, r), dv = wk.shape, wv.shape[1]
+    table = torch.arange(S * nb, dtype=torch.int32, device=cache.device).view(S, nb)
+    ext = _native(cache)
+    if ext is None or cache.dtype != torch.bfloat16 or not ext.latent_expand_ok(r, d, dv):
+        return ref.latent_expand(cache, block_tables, wk, wv) + (table,)      # vendor GEMMs
+    k = torch.empty((S * nb, H, 16, d), dtype=cache.dtype, device=cache.device)
+    v = torch.empty((S * nb, H, dv, 16), dtype=cache.dtype, device=cache.device)
+    ext.latent_expand(cache, block_tables, ctx, wk, wv, k, v)
+    return k, v, table
+
+
+def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol: int = 0, act: Optional[torch.Tensor] = None,
+                q: Optional[torch.Tensor] = None, qscale: float = 1.0) -> None:
     """``latent_kv_write`` for a latent without a rotated part inside a wider projection: cache [blocks,
     block, rank] receives rmsnorm(proj[:, ccol : ccol + rank]) * norm_w at the tokens' slots; ``act``
-    as in ``rope_prep``."""
+    as in ``rope_prep``; ``q`` [T, ...] (contiguous) receives the first columns of proj times ``qscale``."""
     ext = _native(proj)
     if ext is None:
-        return ref.latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol, act)
-    ext.latent_prep(proj, int(ccol), norm_w, float(eps), slots, cache, int(ucol), act)
+        return ref.latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol, act, q, qscale)
+    ext.latent_prep(proj, int(ccol), norm_w, float(eps), slots, cache, int(ucol), act, q, float(qscale))
 
 
 def gate_heads(o: torch.Tensor, gate: torch.Tensor, out: torch.Tensor) -> torch.Tensor:

@@ -244,9 +244,12 @@ def test_first_tokens_and_long_decoding(full_model, device, dtype):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_mixed_batches_and_reuse(full_model, device, dtype):
+@pytest.mark.parametrize("expand_min", [1, 10 ** 9])      # latent layers: keys and values of every portion made from latents, or never
+def test_mixed_batches_and_reuse(full_model, monkeypatch, device, dtype, expand_min):
     """Unequal requests share steps (portions beside single tokens); more requests than batch rows
     and more tokens than pages pass through, so rows and pages are used again."""
+    from distributed_llm_amd.ops import seqmix
+    monkeypatch.setattr(seqmix, "LATENT_EXPAND_MIN", expand_min)
     eng = engine(full_model[0], device, dtype, rows=3, tokens=112)       # 7 pages of 16
     lens = [40, 9, 33, 1, 21, 30, 5]
     reqs = {f"q{i}": toks(n, seed=10 + i) for i, n in enumerate(lens)}
@@ -334,10 +337,13 @@ def test_chunk_edges(tmp_path, device, size, n):
 
 
 @pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("expand_min", [1, 10 ** 9])
 @pytest.mark.parametrize("n", [15, 16, 17, 63, 64, 65, 130, 330])
-def test_far_keys_of_the_latent_attention(tmp_path, device, n):
+def test_far_keys_of_the_latent_attention(tmp_path, monkeypatch, device, n, expand_min):
     """A softmax so sharp that one key, far back among repeated ones and on either side of a page (16)
     or key-tile (32, 64) border, carries a row; prompts and decoded rows."""
+    from distributed_llm_amd.ops import seqmix
+    monkeypatch.setattr(seqmix, "LATENT_EXPAND_MIN", expand_min)
     cfg = make_cfg([latent(heads=2, dim=8, vdim=5, rank=10, scale=2.0)], width=16)
     for seed in range(n, n + 500, 100):
         W = make_weights(cfg, seed=seed, qk_gain=2.0)
@@ -469,9 +475,12 @@ def test_unaligned_sizes(tmp_path, device, dtype):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_aligned_sizes_take_the_matrix_core_paths(tmp_path, dtype):
+@pytest.mark.parametrize("expand_min", [1, 32, 10 ** 9])
+def test_aligned_sizes_take_the_matrix_core_paths(tmp_path, monkeypatch, dtype, expand_min):
     """Sizes that the matrix-core kernels and the tuned GEMMs take (bf16), against the oracle; prompt
     portions, decoding and mixed steps; chunks that leave whole key tiles out."""
+    from distributed_llm_amd.ops import seqmix
+    monkeypatch.setattr(seqmix, "LATENT_EXPAND_MIN", expand_min)
     layers = [attn(heads=4, kv_heads=2, dim=32, vdim=64, rot=16, size=40, mlp=ff(128)), latent(heads=4, dim=32, vdim=64, rank=64, mlp=ff(64)),
               attn(heads=8, kv_heads=1, dim=48, vdim=40, rot=48, size=130, mlp=ff(64)), latent(heads=2, dim=64, vdim=32, rank=160),
               attn(heads=2, kv_heads=2, dim=128, vdim=96, rot=64, size=7)]
@@ -528,4 +537,5 @@ def test_random_weights(device):
     m = build_model(cfg, device=device, dtype=torch.float32)
     names = m._random(0, 0.02)
     assert sum(v.numel() for v in names.values()) == cfg.num_params()
-    assert m.weight_bytes() == 4 * cfg.num_params() and m.decode_read_bytes() > m.weight_bytes()
+    twice = sum(L["uv"].numel() for L in m.layers if "uv" in L)      # the value up-projections are kept in two layouts
+    assert m.weight_bytes() == 4 * (cfg.num_params() + twice) and m.decode_read_bytes() > m.weight_bytes()

@@ -683,9 +683,47 @@ def test_latent_prep_and_gate(dt, T, H, d, dv, rank, ff):
     c1 = torch.randn(nb, 16, rank, device=DEV).to(dt)
     c2 = c1.clone()
     b1, b2 = (torch.full((T, H * dv + ff), 7.0, device=DEV).to(dt) for _ in range(2))
-    for m, c, b in ((seqmix, c1, b1), (ref, c2, b2)):
-        m.latent_prep(proj, H * d, w, 1e-5, slots, c, H * d + rank + H * dv, b[:, H * dv:] if ff else None)
+    q1, q2 = (torch.zeros(T, H, d, device=DEV, dtype=dt) for _ in range(2))
+    for m, c, b, q in ((seqmix, c1, b1, q1), (ref, c2, b2, q2)):
+        m.latent_prep(proj, H * d, w, 1e-5, slots, c, H * d + rank + H * dv, b[:, H * dv:] if ff else None, q, 0.3)
         o = (torch.arange(H * T * dv, device=DEV).float() * 0.37).sin().to(dt).view(H, T, dv)
         m.gate_heads(o, proj[:, H * d + rank:H * d + rank + H * dv], b[:, :H * dv])
     torch.testing.assert_close(c1.float(), c2.float(), **tol(dt))
     torch.testing.assert_close(b1.float(), b2.float(), **tol(dt))
+    torch.testing.assert_close(q1.float(), q2.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("ctxs", [[1], [16, 5], [130, 64, 65], [300]])
+@pytest.mark.parametrize("H,d,dv,rank", [(2, 8, 5, 32), (3, 40, 72, 64), (4, 64, 64, 96), (2, 128, 128, 512), (1, 136, 200, 160), (2, 12, 4, 20)])
+def test_latent_expand(dt, ctxs, H, d, dv, rank):
+    """Keys and values from paged latents (pages out of order), then attention on them against attention
+    on the latents."""
+    torch.manual_seed(34)
+    S, nb = len(ctxs), max((c + 15) // 16 for c in ctxs)
+    bt = torch.randperm(S * nb + 2, device=DEV)[:S * nb].to(torch.int32).view(S, nb)
+    cache = torch.randn(S * nb + 2, 16, rank, device=DEV).to(dt)
+    wk, wv = (torch.randn(H, d, rank, device=DEV) / rank ** 0.5).to(dt), (torch.randn(H, dv, rank, device=DEV) / rank ** 0.5).to(dt)
+    k1, v1, table = seqmix.latent_expand(cache, bt, i32(ctxs), wk, wv)
+    k2, v2 = ref.latent_expand(cache.float(), bt, wk.float(), wv.float())
+    for s, c in enumerate(ctxs):
+        n = (c + 15) // 16
+        assert table[s].tolist() == list(range(s * nb, (s + 1) * nb))
+        torch.testing.assert_close(k1[s * nb:s * nb + n].float(), k2[s * nb:s * nb + n], **tol(dt))
+        torch.testing.assert_close(v1[s * nb:s * nb + n].float(), v2[s * nb:s * nb + n], **tol(dt))
+    if not seqmix.latent_expand_wanted(cache, H, d, dv, 1 << 20, S, S * nb):
+        return
+    from distributed_llm_amd.models.llama import AttnMeta
+    qlens = [min(c, 3) for c in ctxs]
+    T, qstart, qlen, ctx, rows, pos = batch(qlens, [c - n for c, n in zip(ctxs, qlens)])
+    q = torch.randn(T, H, d, device=DEV).to(dt)
+    meta = AttnMeta(slots=None, block_tables=bt, qstart=qstart, qlen=qlen, ctx=ctx, tile_seq=None, tile_tok0=None, last_idx=None,
+                    host_qlen=qlens)
+    mfma = seqmix.gqa_use_mfma(q, H, H, d, dv, 16)
+    ts, tt = meta.latent_tiles(1, DEV, seqmix.gqa_tokens_per_tile(H, H, mfma))
+    got = seqmix.paged_gqa_attention(q, k1, v1, table, qstart, qlen, ctx, ts, tt, None, mfma, 1).float().view(T, H, dv)
+    qa = torch.matmul(q.float().transpose(0, 1), wk.float())
+    lat = ref.latent_attention(qa, q.float().view(T, H * d), d, 0, pos, torch.zeros(512, 2, device=DEV), cache.float(), bt, qstart,
+                               qlen, ctx, 1.0)
+    want = torch.matmul(lat, wv.float().transpose(1, 2)).transpose(0, 1)
+    torch.testing.assert_close(got, want, **(dict(atol=6e-2, rtol=6e-2) if dt == torch.bfloat16 else dict(atol=1e-4, rtol=1e-4)))
