@@ -101,7 +101,7 @@ int dllm_paged_gqa(const void*, const void*, const void*, int, const int*, int, 
 int dllm_rope_prep(const void*, long, int, int, int, int, int, const float*, int, int, float, const int*, const int*, void*, void*,
                    void*, long, int, int, int, void*, long, void*, long, int, hipStream_t);
 int dllm_latent_prep(const void*, long, int, int, int, const float*, float, const int*, void*, int, int, void*, long, void*, int,
-                     float, long, hipStream_t);
+                     float, void*, int, long, hipStream_t);
 int dllm_latent_expand_ok(int, int, int);
 int dllm_latent_expand(const void*, const int*, int, int, int, int, const int*, int, int, int, int, const void*, const void*, void*,
                        void*, hipStream_t);
@@ -1796,7 +1796,8 @@ void rope_prep(torch::Tensor proj, int64_t H, int64_t G, int64_t d, int64_t dv, 
 }
 
 void latent_prep(torch::Tensor proj, int64_t ccol, torch::Tensor w, double eps, torch::Tensor slots, torch::Tensor cache,
-                 int64_t ucol, c10::optional<torch::Tensor> act, c10::optional<torch::Tensor> q, double qscale) {
+                 int64_t ucol, c10::optional<torch::Tensor> act, c10::optional<torch::Tensor> q, double qscale,
+                 c10::optional<torch::Tensor> zero) {
   const bool f = act_f32(proj, "proj");
   check_rows2d(proj, "proj");
   check_f32(w, "norm weight");
@@ -1825,9 +1826,18 @@ void latent_prep(torch::Tensor proj, int64_t ccol, torch::Tensor w, double eps, 
     TORCH_CHECK(nq <= proj.size(1), "q columns of proj");
     qp = q->data_ptr();
   }
+  void* zp = nullptr;
+  int64_t zh = 0;
+  if (zero) {
+    TORCH_CHECK(zero->is_cuda() && zero->scalar_type() == proj.scalar_type() && zero->is_contiguous() && zero->dim() == 3 &&
+                    zero->size(1) == T && zero->size(2) == rank,
+                "zero [H, T, rank] in the activations' dtype");
+    zh = zero->size(0);
+    zp = zero->data_ptr();
+  }
   ok(dllm_latent_prep(proj.data_ptr(), proj.stride(0), f, (int)ccol, (int)rank, w.data_ptr<float>(), (float)eps,
-                      slots.data_ptr<int>(), cache.data_ptr(), (int)ucol, (int)ff, ap, lda, qp, (int)nq, (float)qscale, (long)T,
-                      stream()),
+                      slots.data_ptr<int>(), cache.data_ptr(), (int)ucol, (int)ff, ap, lda, qp, (int)nq, (float)qscale, zp, (int)zh,
+                      (long)T, stream()),
      "latent_prep");
 }
 

@@ -269,8 +269,8 @@ __device__ __forceinline__ void act_share<u16>(const u16* __restrict__ up, int f
 // projection.  proj row: q (H d) | k (G d) | v (G dv) | ...; a wave per q / k head: rotate-half
 // positions on the first `rot` dims (cos and sin as the table holds them), q times qscale; k and v to
 // their page slots.  act (null: no feed-forward): act[tok] = relu(proj[tok, ucol : ucol + ff])^2.
-// zrow: the first zn columns of this token's row are cleared (an attention output whose padding rows
-// no tile writes).
+// zrow: the first zn columns of a padding token's row (slot < 0) are cleared (an attention output whose
+// padding rows no tile writes).
 template <typename T>
 __global__ void __launch_bounds__(256) rope_prep_kernel(const T* __restrict__ proj, long ld, int H, int G, int d, int dv,
                                                         const float* __restrict__ cos_sin, int tab_w, int rot, float qscale,
@@ -286,7 +286,7 @@ __global__ void __launch_bounds__(256) rope_prep_kernel(const T* __restrict__ pr
   const int off = slot >= 0 ? slot % BSZ : 0;
   const int half = rot >> 1;
   const float* cs = cos_sin + (long)pos[tok] * tab_w;
-  if (zrow)
+  if (zrow && slot < 0)
     for (int i = blockIdx.y * 256 + tid; i < zn; i += gridDim.y * 256) stf(zrow + tok * ldz + i, 0.f);
   for (int hh = blockIdx.y * 4 + wave; hh < H + G; hh += gridDim.y * 4) {   // q heads, then k heads
     const bool is_q = hh < H;

@@ -67,12 +67,16 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(const T* __restrict__ 
                                                           const float* __restrict__ w, float eps,
                                                           const int* __restrict__ slots, T* __restrict__ cache, int ucol,
                                                           int ff, T* __restrict__ act, long lda, int vec,
-                                                          T* __restrict__ q, int nq, float qscale) {
+                                                          T* __restrict__ q, int nq, float qscale, T* __restrict__ zl, int zh) {
   // q (optional): the row's first nq columns times qscale, as rows of a matrix of their own
   const long tok = blockIdx.x;
   const int tid = threadIdx.x;
   const T* row = proj + tok * ld;
   const int slot = slots[tok];
+  // zl (optional, [H, T, rank]): a padding token's rows, which no attention tile writes, are cleared
+  if (zl && slot < 0)
+    for (int i = blockIdx.y * 256 + tid; i < zh * rank; i += gridDim.y * 256)
+      stf(zl + ((long)(i / rank) * gridDim.x + tok) * rank + i % rank, 0.f);
   if (blockIdx.y == 0 && tid < 64 && slot >= 0) {
     const T* r = row + ccol;
     float s = 0.f;
@@ -498,8 +502,17 @@ __global__ void __launch_bounds__(256) latent_attention_mfma_kernel(
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int lr = lane & 15, g = lane >> 4;
   const int half = rot >> 1;
-  for (int e = tid; e < RPB * Dpad; e += 256) {
-    const int rr = e / Dpad, c = e - rr * Dpad, row = row0 + rr;
+  // queries: the latent part as 16-byte vectors where rows allow it, the rest (rotated part, padding) alone
+  const int cs0 = (rank & 7) == 0 ? rank : 0;
+  for (int e = tid; e < RPB * (cs0 >> 3); e += 256) {
+    const int rr = e / (cs0 >> 3), c = 8 * (e - rr * (cs0 >> 3)), row = row0 + rr;
+    uint4 v = make_uint4(0u, 0u, 0u, 0u);
+    if (row < nrows) v = ld16(qa + ((long)(row % H) * Ttot + q0 + tok0 + row / H) * rank + c);
+    st16(qsh + rr * qstr + c, v);
+  }
+  const int nrest = Dpad - cs0;
+  for (int e = tid; e < RPB * nrest; e += 256) {
+    const int rr = e / nrest, c = cs0 + e - rr * nrest, row = row0 + rr;
     float v = 0.f;
     if (row < nrows && c < Dp) {
       const int tl = tok0 + row / H, h = row % H;
@@ -517,7 +530,8 @@ __global__ void __launch_bounds__(256) latent_attention_mfma_kernel(
     qsh[rr * qstr + c] = f2bf(v);
   }
   // zero what no staging pass writes: the key rows' padded dims
-  for (int e = tid; e < KT * qstr; e += 256) ksh[e] = 0;
+  const int npad = Dpad - Dp;
+  for (int e = tid; e < KT * npad; e += 256) ksh[(e / npad) * qstr + Dp + e % npad] = 0;
   const int last_row = min(row0 + RPB, nrows) - 1;
   const int kmax = p0 + tok0 + last_row / H + 1;
   int rpos[LR][4];
@@ -736,17 +750,17 @@ __global__ void __launch_bounds__(256) latent_attention_mfma_kernel(
   }
 }
 
-// one wave per (entry, row): merge the splits' (max, sum, weighted latent) partials
+// one workgroup per (entry, row): merge the splits' (max, sum, weighted latent) partials.  Lane z of every
+// wave holds split z's weight (splits <= 64), a thread owns latent dims tid, tid + 256, ...
 template <typename T>
 __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __restrict__ part_o,
                                                              const float* __restrict__ part_ml, int splits, int gx,
                                                              int H, int rank, long Ttot, const int* __restrict__ qstart,
                                                              const int* __restrict__ qlen, const int* __restrict__ tile_seq,
-                                                             const int* __restrict__ tile_tok0, int tpe, long n_rows,
+                                                             const int* __restrict__ tile_tok0, int tpe,
                                                              T* __restrict__ out, int rpb) {
-  const long r = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (r >= n_rows) return;
-  const int lane = threadIdx.x & 63;
+  const long r = blockIdx.x;
+  const int tid = threadIdx.x, lane = tid & 63;
   const int rl = (int)(r % rpb);
   const long eb = r / rpb;
   const int bx = (int)(eb % gx), entry = (int)(eb / gx);
@@ -756,18 +770,24 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __rest
   const int row = bx * rpb + rl;
   if (row >= min(tpe, n - tok0) * H) return;
   const float* ml = part_ml + 2 * r * splits;
-  float M = -INFINITY;
-  for (int z = 0; z < splits; ++z) M = fmaxf(M, ml[2 * z]);
-  float L = 0.f;
-  for (int z = 0; z < splits; ++z) L += ml[2 * z] == -INFINITY ? 0.f : ml[2 * z + 1] * expf(ml[2 * z] - M);
-  const float inv = L > 0.f ? 1.f / L : 0.f;
+  const float mz = lane < splits ? ml[2 * lane] : -INFINITY, lz = lane < splits ? ml[2 * lane + 1] : 0.f;
+  const float M = wave_max(mz);
+  const float ez = mz > -INFINITY ? expf(mz - M) : 0.f;
+  const float L = wave_sum(lz * ez);
+  const float wz = L > 0.f ? ez / L : 0.f;
   const long tok = qstart[s] + tok0 + row / H;
   const int h = row % H;
-  for (int c = lane; c < rank; c += 64) {
+  const float* po = part_o + r * splits * rank;
+  for (int c0 = 0; c0 < rank; c0 += 256) {     // every lane stays in the loop: the shuffles read all lanes
+    const int c = c0 + tid;
+    const bool on = c < rank;
     float o = 0.f;
-    for (int z = 0; z < splits; ++z)
-      if (ml[2 * z] != -INFINITY) o += part_o[(r * splits + z) * rank + c] * expf(ml[2 * z] - M);
-    stf(out + ((long)h * Ttot + tok) * rank + c, o * inv);
+#pragma unroll 8
+    for (int z = 0; z < splits; ++z) {
+      const float w = __shfl(wz, z, 64);
+      if (on && w != 0.f) o += po[(long)z * rank + c] * w;     // a split that saw no key left nothing to read
+    }
+    if (on) stf(out + ((long)h * Ttot + tok) * rank + c, o);
   }
 }
 
@@ -809,8 +829,8 @@ int launch_latent(int ri, dim3 g, long lds, hipStream_t st, const T* qa, const T
 #undef LAT
   if (splits > 1) {
     const long n_rows = (long)g.y * g.x * LROWS;
-    hipLaunchKernelGGL(latent_combine_kernel<T>, dim3((unsigned)((n_rows + 3) / 4)), dim3(256), 0, st, part_o, part_ml, splits,
-                       (int)g.x, H, rank, Ttot, qstart, qlen, tile_seq, tile_tok0, tpe, n_rows, out, LROWS);
+    hipLaunchKernelGGL(latent_combine_kernel<T>, dim3((unsigned)n_rows), dim3(256), 0, st, part_o, part_ml, splits, (int)g.x, H,
+                       rank, Ttot, qstart, qlen, tile_seq, tile_tok0, tpe, out, LROWS);
   }
   return (int)hipGetLastError();
 }
@@ -849,8 +869,8 @@ int launch_latent_mfma(dim3 g, hipStream_t st, const u16* qa, const u16* q, long
 #undef LATM3
   if (splits > 1) {
     const long n_rows = (long)g.y * g.x * rows;
-    hipLaunchKernelGGL(latent_combine_kernel<u16>, dim3((unsigned)((n_rows + 3) / 4)), dim3(256), 0, st, part_o, part_ml,
-                       splits, (int)g.x, H, rank, Ttot, qstart, qlen, tile_seq, tile_tok0, tpe, n_rows, out, rows);
+    hipLaunchKernelGGL(latent_combine_kernel<u16>, dim3((unsigned)n_rows), dim3(256), 0, st, part_o, part_ml, splits, (int)g.x, H,
+                       rank, Ttot, qstart, qlen, tile_seq, tile_tok0, tpe, out, rows);
   }
   return (int)hipGetLastError();
 }
@@ -902,7 +922,7 @@ extern "C" int dllm_latent_attention(const void* qa, const void* q, long ldq, in
 
 extern "C" int dllm_latent_prep(const void* proj, long ld, int f32, int ccol, int rank, const float* w, float eps,
                                 const int* slots, void* cache, int ucol, int ff, void* act, long lda, void* q, int nq,
-                                float qscale, long T, hipStream_t st) {
+                                float qscale, void* zl, int zh, long T, hipStream_t st) {
   if (T <= 0) return 0;
   if (rank < 1 || (act && ff < 1)) return -1;
   const dim3 grid((unsigned)T, act ? (ff + 2047) / 2048 : 1);
@@ -910,10 +930,10 @@ extern "C" int dllm_latent_prep(const void* proj, long ld, int f32, int ccol, in
                   (uintptr_t)act % 16 == 0;
   if (f32)
     hipLaunchKernelGGL(latent_prep_kernel<float>, grid, dim3(256), 0, st, (const float*)proj, ld, ccol, rank, w, eps, slots,
-                       (float*)cache, ucol, ff, (float*)act, lda, vec, (float*)q, nq, qscale);
+                       (float*)cache, ucol, ff, (float*)act, lda, vec, (float*)q, nq, qscale, (float*)zl, zh);
   else
     hipLaunchKernelGGL(latent_prep_kernel<u16>, grid, dim3(256), 0, st, (const u16*)proj, ld, ccol, rank, w, eps, slots,
-                       (u16*)cache, ucol, ff, (u16*)act, lda, vec, (u16*)q, nq, qscale);
+                       (u16*)cache, ucol, ff, (u16*)act, lda, vec, (u16*)q, nq, qscale, (u16*)zl, zh);
   return (int)hipGetLastError();
 }
 

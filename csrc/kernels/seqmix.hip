@@ -970,6 +970,69 @@ __global__ void __launch_bounds__(256) scaled_resadd_rms_kernel(const T* __restr
   for (int i = threadIdx.x; i < H; i += 256) stf(orow + i, yb[i] * r * w[i]);
 }
 
+// The same for rows of whole 4-entry vectors, NV vectors a thread: the row stays in registers.
+template <typename T> struct vec4;
+template <> struct vec4<float> {
+  static __device__ __forceinline__ float4 ld(const float* p) { return *reinterpret_cast<const float4*>(p); }
+  static __device__ __forceinline__ void st(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
+};
+template <> struct vec4<u16> {
+  static __device__ __forceinline__ float4 ld(const u16* p) {
+    const uint2 w = *reinterpret_cast<const uint2*>(p);
+    return make_float4(__uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u), __uint_as_float(w.y << 16),
+                       __uint_as_float(w.y & 0xffff0000u));
+  }
+  static __device__ __forceinline__ void st(u16* p, float4 v) {
+    *reinterpret_cast<uint2*>(p) = make_uint2((uint32_t)f2bf(v.x) | ((uint32_t)f2bf(v.y) << 16),
+                                              (uint32_t)f2bf(v.z) | ((uint32_t)f2bf(v.w) << 16));
+  }
+};
+template <typename T, int NV>
+__global__ void __launch_bounds__(256) scaled_resadd_rms_vec_kernel(const T* __restrict__ y, long ldy, float mult, int set,
+                                                                    const float* __restrict__ vec, float* __restrict__ x,
+                                                                    const float* __restrict__ w, T* __restrict__ out, long ldo,
+                                                                    int H, float eps) {
+  __shared__ float red[16];
+  const long row = blockIdx.x;
+  float* xr = x + row * (long)H;
+  float4 v[NV];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = 4 * (j * 256 + (int)threadIdx.x);
+    v[j] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (c < H) {
+      if (!set) v[j] = *reinterpret_cast<const float4*>(xr + c);
+      if (y) {
+        const float4 t = vec4<T>::ld(y + row * ldy + c);
+        v[j].x += mult * t.x; v[j].y += mult * t.y; v[j].z += mult * t.z; v[j].w += mult * t.w;
+      }
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = 4 * (j * 256 + (int)threadIdx.x);
+    if (c < H) {
+      if (y) {
+        if (vec) { v[j].x += vec[c]; v[j].y += vec[c + 1]; v[j].z += vec[c + 2]; v[j].w += vec[c + 3]; }
+        *reinterpret_cast<float4*>(xr + c) = v[j];
+      }
+      if (!w && out) vec4<T>::st(out + row * ldo + c, v[j]);
+    }
+    ss += v[j].x * v[j].x + v[j].y * v[j].y + v[j].z * v[j].z + v[j].w * v[j].w;
+  }
+  if (!w) return;   // uniform
+  const float r = 1.f / sqrtf(block_sum(ss, red) / (float)H + eps);
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = 4 * (j * 256 + (int)threadIdx.x);
+    if (c < H) {
+      const float4 g = *reinterpret_cast<const float4*>(w + c);
+      vec4<T>::st(out + row * ldo + c, make_float4(v[j].x * r * g.x, v[j].y * r * g.y, v[j].z * r * g.z, v[j].w * r * g.w));
+    }
+  }
+}
+
 // gu [rows, 2 ff] (gate columns, then up columns) + bias -> y [rows, ff].  mode 0: silu(g) u;
 // mode 1: g <- min(g, limit), u <- clamp(u, -limit, limit), y = g sigmoid(alpha g) (u + 1)
 template <typename T>
@@ -1341,6 +1404,19 @@ extern "C" int dllm_scaled_resadd_rms(const void* y, long ldy, int f32, float mu
   if (rows <= 0) return 0;
   const long lds = w ? 4L * H : 0;
   if (lds > 150 * 1024 || (w && !out) || (set && !y)) return -1;
+  const long ab = f32 ? 16 : 8;     // bytes of a vector of activations
+  if (H % 4 == 0 && H <= 8192 && (uintptr_t)x % 16 == 0 && (!y || (ldy % 4 == 0 && (uintptr_t)y % ab == 0)) &&
+      (!out || (ldo % 4 == 0 && (uintptr_t)out % ab == 0)) && (!w || (uintptr_t)w % 16 == 0)) {
+    const int nv = (H + 1023) / 1024;
+#define RV(T, NV)                                                                                                         \
+  hipLaunchKernelGGL((scaled_resadd_rms_vec_kernel<T, NV>), dim3((unsigned)rows), dim3(256), 0, st, (const T*)y, ldy, mult, set, vec, \
+                     x, w, (T*)out, ldo, H, eps)
+#define RVT(T) do { if (nv <= 1) RV(T, 1); else if (nv <= 2) RV(T, 2); else if (nv <= 4) RV(T, 4); else RV(T, 8); } while (0)
+    if (f32) RVT(float); else RVT(u16);
+#undef RVT
+#undef RV
+    return (int)hipGetLastError();
+  }
   if (f32) {
     ENSURE_LDS(scaled_resadd_rms_kernel<float>, lds);
     hipLaunchKernelGGL(scaled_resadd_rms_kernel<float>, dim3((unsigned)rows), dim3(256), lds, st, (const float*)y, ldy, mult, set,

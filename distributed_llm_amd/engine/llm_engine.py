@@ -340,8 +340,14 @@ class LLMEngine:
     def _autotune(self) -> None:
         """Pick the fastest GEMM plan for every decode bucket and weight shape (before capture)."""
         m = self.model
-        if not self._paged_attn:
-            return                # layer-list models: heuristic plans (their projections are small next to the mixers)
+        if not self._paged_attn:      # layer-list models: the large weights they name, heuristic plans for the rest
+            big = [(n, k, False) for n, k in m.gemm_shapes()]
+            if big:
+                with ops.gemm.workspace_owner(self._ws_owner):
+                    ops.gemm_autotune(big, [b for b in self.buckets if b <= ops.gemm.MAX_M], self.device,
+                                      verbose=os.environ.get("DLLM_VERBOSE") == "1")
+                    ops.gemm.reserve(self.device)
+            return
         shapes = set()
         L = m.layers[0]
         for name in ("wqkv", "wqkv_f", "wo", "wgu", "wgu_f"):

@@ -495,6 +495,14 @@ class HybridModel:
         assert tuple(D["proj"].shape) == (n + m.heads * m.vdim + ff, W)
         assert tuple(D["out"].shape) == (W, m.heads * m.vdim + ff)
 
+    def gemm_shapes(self) -> List[Tuple[int, int]]:
+        """(out, in) of the large bf16 weights that run on the tuned GEMMs (the engine times their plans)."""
+        if self.dtype != torch.bfloat16 or not self.cfg.parallel_ff:
+            return []
+        ws = [L[k] for L in self.layers for k in ("proj", "out")] + [self.lm_head] + \
+            ([self.loop_in] if self.cfg.loop is not None else [])
+        return sorted({tuple(w.shape) for w in ws if w.shape[0] % 64 == 0 and w.shape[1] % 64 == 0 and w.numel() >= 1 << 22})
+
     def weight_bytes(self) -> int:
         n = sum(x.numel() * x.element_size() for x in (self.embed, self.final_norm))
         if self.cfg.loop is not None:
@@ -781,14 +789,15 @@ class HybridModel:
             seqmix.paged_gqa_attention(q, k, v, table, meta.qstart, meta.qlen, meta.ctx, ts, tt, proj[:, g0:g0 + hv], mfma, splits,
                                        out=both[:, :hv])
             return _mm(both, L["out"])
-        seqmix.latent_prep(proj, c0, L["dkv_norm"], self.cfg.rms_eps, meta.slots, cache[0], g0 + hv, act)
+        lat = torch.empty((H, T, m.kv_rank), dtype=x.dtype, device=x.device)     # padding rows cleared by the prep launch
+        seqmix.latent_prep(proj, c0, L["dkv_norm"], self.cfg.rms_eps, meta.slots, cache[0], g0 + hv, act, zero=lat)
         q = proj[:, :c0]
         qa = torch.bmm(q.unflatten(1, (H, m.dim)).transpose(0, 1), L["uk"])     # key up-projection absorbed: [H, T, rank]
         rows = (seqmix.LAT_ROWS if meta.host_qlen is None else
                 seqmix.latent_rows(x, m.kv_rank, 0, T, len(meta.host_qlen)))
         ts, tr = meta.latent_tiles(H, self.device, rows)
         lat = seqmix.latent_attention(qa, q, m.dim, 0, positions, self._any_table(), cache[0], meta.block_tables, meta.qstart,
-                                      meta.qlen, meta.ctx, ts, tr, m.scale, rows=rows)
+                                      meta.qlen, meta.ctx, ts, tr, m.scale, rows=rows, out=lat)
         seqmix.gate_heads(torch.bmm(lat, L["uvT"]), proj[:, g0:g0 + hv], both[:, :hv])
         return _mm(both, L["out"])
 

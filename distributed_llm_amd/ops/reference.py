@@ -1060,7 +1060,7 @@ def rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, posit
     if act is not None:
         act.copy_(relu2(proj[:, ucol:ucol + act.shape[1]]))
     if zero_rows is not None:
-        zero_rows.zero_()
+        zero_rows[slots < 0] = 0
     return (qk[:, :H] * qscale).to(proj.dtype)
 
 
@@ -1076,9 +1076,11 @@ def latent_expand(cache, block_tables, wk, wv):
     return k, v
 
 
-def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol=0, act=None, q=None, qscale=1.0):
+def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol=0, act=None, q=None, qscale=1.0, zero=None):
     """cache[slot] = rmsnorm(proj[:, ccol : ccol + rank]) * norm_w; act = relu(proj[:, ucol:])^2; q =
-    the first columns times qscale."""
+    the first columns times qscale; ``zero`` [heads, T, rank]: rows of tokens without a slot are cleared."""
+    if zero is not None:
+        zero[:, slots < 0] = 0
     if q is not None:
         q.view(proj.shape[0], -1).copy_((proj[:, :q[0].numel()].float() * qscale).to(q.dtype))
     r = norm_w.numel()

@@ -154,14 +154,15 @@ def latent_rows(x: torch.Tensor, rank: int, rot_dim: int, tokens: int, seqs: int
 
 def latent_attention(qa, q, dim, rot_dim, positions, cos_sin, cache, block_tables, qstart, qlen, ctx, tile_seq,
                      tile_tok0, scale, splits: Optional[int] = None, mfma: Optional[bool] = None,
-                     rows: int = LAT_ROWS) -> torch.Tensor:
-    """``mfma`` (GPU, bf16): the matrix-core kernel (default where the shape fits it;
+                     rows: int = LAT_ROWS, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``out``: a prepared output like qa (its padding rows already cleared).  ``mfma`` (GPU, bf16): the matrix-core kernel (default where the shape fits it;
     ``DLLM_LATENT_MFMA=0`` or ``mfma=False`` keeps the vector-ALU kernel that f32 models run)."""
     ext = _native(qa)
     if ext is None:
         return ref.latent_attention(qa, q, dim, rot_dim, positions, cos_sin, cache, block_tables, qstart, qlen, ctx,
                                     scale)
-    out = torch.zeros_like(qa)
+    if out is None:
+        out = torch.zeros_like(qa)
     H, n_entries = qa.shape[0], int(tile_seq.numel())
     sp = latent_splits(n_entries, H, rows) if splits is None else int(splits)
     po = pml = None
@@ -306,6 +307,8 @@ def gqa_splits(n_tiles: int, kv_heads: int, max_ctx: int, window: int = 0, keep_
         tiles = min(tiles, (int(window) + 62) // 64 + 1 + (int(keep_first) + 63) // 64)
     if chunk > 0:
         tiles = min(tiles, (int(chunk) + 62) // 64 + 1 + (int(keep_first) + 63) // 64)
+    if window > 0 or chunk > 0:
+        tiles = (tiles + 1) // 2      # few tiles: at least two a split, or merging costs more than walking them
     return max(1, min(GQA_SPLIT_MAX, tiles, GQA_SPLIT_TARGET // max(1, n_tiles * kv_heads)))
 
 
@@ -618,7 +621,8 @@ def rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, posit
     ``qscale``; k and v to their page slots (k_cache [blocks, kv_heads, block, dim], v_cache [blocks,
     kv_heads, vdim, block]).  ``act`` [T, ff] (may be columns of a wider matrix) receives
     relu(proj[:, ucol : ucol + ff])^2, the activation of a feed-forward whose up projection is part of
-    proj.  ``zero_rows`` [T, n] is cleared in the same launch.  Returns q [T, heads, dim]."""
+    proj.  ``zero_rows`` [T, n]: the rows of tokens without a slot (padding) are cleared in the same
+    launch.  Returns q [T, heads, dim]."""
     ext = _native(proj)
     if ext is None:
         return ref.rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, positions, slots, k_cache, v_cache,
@@ -667,14 +671,15 @@ def latent_expand(cache: torch.Tensor, block_tables: torch.Tensor, ctx: torch.Te
 
 
 def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol: int = 0, act: Optional[torch.Tensor] = None,
-                q: Optional[torch.Tensor] = None, qscale: float = 1.0) -> None:
+                q: Optional[torch.Tensor] = None, qscale: float = 1.0, zero: Optional[torch.Tensor] = None) -> None:
     """``latent_kv_write`` for a latent without a rotated part inside a wider projection: cache [blocks,
     block, rank] receives rmsnorm(proj[:, ccol : ccol + rank]) * norm_w at the tokens' slots; ``act``
-    as in ``rope_prep``; ``q`` [T, ...] (contiguous) receives the first columns of proj times ``qscale``."""
+    as in ``rope_prep``; ``q`` [T, ...] (contiguous) receives the first columns of proj times ``qscale``;
+    ``zero`` [heads, T, rank]: the rows of tokens without a slot (padding) are cleared."""
     ext = _native(proj)
     if ext is None:
-        return ref.latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol, act, q, qscale)
-    ext.latent_prep(proj, int(ccol), norm_w, float(eps), slots, cache, int(ucol), act, q, float(qscale))
+        return ref.latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol, act, q, qscale, zero)
+    ext.latent_prep(proj, int(ccol), norm_w, float(eps), slots, cache, int(ucol), act, q, float(qscale), zero)
 
 
 def gate_heads(o: torch.Tensor, gate: torch.Tensor, out: torch.Tensor) -> torch.Tensor:

@@ -656,6 +656,12 @@ def test_gated_attention_kernels(dt, case, H, G, d, dv, rot, chunk, cap, ff):
     q2 = ref.rope_prep(proj, H, G, d, dv, table, rot, 0.3, pos, slots, kc2, vc2, cols + H * dv, act[1], b2[:, :H * dv])
     for a, b in ((q1, q2), (kc1, kc2), (vc1, vc2), (b1, b2)):
         torch.testing.assert_close(a.float(), b.float(), **tol(dt))
+    pad = slots.clone()
+    pad[T // 2:] = -1      # padding tokens write no page, their output rows are cleared
+    kc3, z = kc2.clone(), torch.full((T, H * dv), 7.0, device=DEV).to(dt)
+    seqmix.rope_prep(proj, H, G, d, dv, table, rot, 0.3, pos, pad, kc3, vc2.clone(), zero_rows=z)
+    torch.testing.assert_close(kc3.float(), kc2.float(), **tol(dt))
+    assert float(z[T // 2:].float().abs().sum()) == 0.0 and bool((z[:T // 2] == 7.0).all())
     sinks = torch.randn(H, device=DEV) * 2 + 1
     gate = proj[:, cols:cols + H * dv]
     want = ref.paged_gqa_attention(q2, kc2, vc2, bt, qstart, qlen, ctx, gate, chunk=chunk, softcap=cap, sinks=sinks).float()
@@ -685,7 +691,9 @@ def test_latent_prep_and_gate(dt, T, H, d, dv, rank, ff):
     b1, b2 = (torch.full((T, H * dv + ff), 7.0, device=DEV).to(dt) for _ in range(2))
     q1, q2 = (torch.zeros(T, H, d, device=DEV, dtype=dt) for _ in range(2))
     for m, c, b, q in ((seqmix, c1, b1, q1), (ref, c2, b2, q2)):
-        m.latent_prep(proj, H * d, w, 1e-5, slots, c, H * d + rank + H * dv, b[:, H * dv:] if ff else None, q, 0.3)
+        z = torch.full((H, T, rank), 7.0, device=DEV).to(dt)
+        m.latent_prep(proj, H * d, w, 1e-5, slots, c, H * d + rank + H * dv, b[:, H * dv:] if ff else None, q, 0.3, z)
+        assert float(z[:, 0].float().abs().sum()) == 0.0 and bool((z[:, 1:] == 7.0).all())
         o = (torch.arange(H * T * dv, device=DEV).float() * 0.37).sin().to(dt).view(H, T, dv)
         m.gate_heads(o, proj[:, H * d + rank:H * d + rank + H * dv], b[:, :H * dv])
     torch.testing.assert_close(c1.float(), c2.float(), **tol(dt))
