@@ -637,7 +637,8 @@ def test_scaled_resadd_rms(dt, n, set_, vec, norm):
 @pytest.mark.parametrize("dt", DTYPES)
 @pytest.mark.parametrize("case", CASES + [([40, 3], [90, 130]), ([1, 1], [300, 77]), ([150], [170])])
 @pytest.mark.parametrize("H,G,d,dv,rot,chunk,cap,ff", [(4, 2, 16, 8, 8, 5, 3.0, 20), (6, 2, 88, 56, 20, 64, 0.0, 64), (3, 3, 40, 72, 40, 1, 20.0, 0),
-                                                       (8, 1, 64, 64, 32, 100, 30.0, 2056), (7, 1, 56, 88, 0, 0, 2.0, 8), (2, 1, 136, 200, 64, 48, 50.0, 5)])
+                                                       (8, 1, 64, 64, 32, 100, 30.0, 2056), (7, 1, 56, 88, 0, 0, 2.0, 8), (2, 1, 136, 200, 64, 48, 50.0, 5),
+                                                       (4, 2, 64, 32, 64, 33, 100.0, 16)])      # a cap beyond the bounded form
 def test_gated_attention_kernels(dt, case, H, G, d, dv, rot, chunk, cap, ff):
     """Prep (rotation with scaled cos and sin, pages, squared-relu columns), then attention inside
     chunks with capped scores, a sink per head and a gate, in both kernel forms and every split count,
