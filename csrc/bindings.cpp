@@ -64,6 +64,7 @@ int dllm_gated_group_norm(const float*, const void*, long, int, const float*, vo
 int dllm_outer_scan_cols();
 int dllm_ssd_scan(const void*, long, const void*, long, int, int, int, int, int, int, const float*, const float*, const float*,
                   float*, const int*, const int*, const int*, const int*, int, float*, hipStream_t);
+int dllm_latent_q_prep(const void*, long, int, int, int, int, int, const int*, const float*, int, float, void*, long, hipStream_t);
 int dllm_mlstm(const void*, long, int, int, int, int, const float*, float, float*, float*, int, float, const float*, const int*,
                const int*, const int*, const int*, int, long, float*, void*, hipStream_t);
 int dllm_qk_norm_prep(const void*, long, int, const float*, int, int, int, int, int, const float*, const float*, const float*,
@@ -84,7 +85,7 @@ int dllm_retention_chunked(const void*, long, int, int, int, int, const float*, 
 int dllm_heads_norm_gate(const float*, const void*, long, int, long, int, const float*, float, const int*, const int*, int,
                          void*, long, hipStream_t);
 int dllm_resadd_norm(const void*, long, const void*, long, int, const float*, const float*, const float*, float*,
-                     const float*, void*, int, int, float, const float*, int, hipStream_t);
+                     const float*, void*, int, int, float, const float*, int, const float*, hipStream_t);
 int dllm_depth_mix(float*, const float*, int, long, int, const float*, void*, int, float, hipStream_t);
 int dllm_gelu_erf(const void*, void*, int, long, hipStream_t);
 int dllm_conv_refill(const void*, long, int, void*, int, int, const int*, const int*, const int*, const int*, int,
@@ -97,24 +98,24 @@ int dllm_gqa_tile_tokens(int, int, int);
 int dllm_gqa_mfma_ok(int, int, int, int, int, int);
 int dllm_paged_gqa(const void*, const void*, const void*, int, const int*, int, int, const int*, const int*, const int*,
                    const int*, const int*, int, const void*, long, void*, int, int, int, int, int, int, float*, int, int, int,
-                   int, float, int, float, const float*, long, hipStream_t);
+                   int, float, int, float, const float*, long, const float*, int, hipStream_t);
 int dllm_rope_prep(const void*, long, int, int, int, int, int, const float*, int, int, float, const int*, const int*, void*, void*,
-                   void*, long, int, int, int, void*, long, void*, long, int, hipStream_t);
+                   void*, long, int, int, int, void*, long, void*, long, int, const float*, const float*, hipStream_t);
 int dllm_latent_prep(const void*, long, int, int, int, const float*, float, const int*, void*, int, int, void*, long, void*, int,
                      float, void*, int, long, hipStream_t);
-int dllm_latent_expand_ok(int, int, int);
+int dllm_latent_expand_ok(int, int, int, int);
 int dllm_latent_expand(const void*, const int*, int, int, int, int, const int*, int, int, int, int, const void*, const void*, void*,
-                       void*, hipStream_t);
-int dllm_gate_heads(const void*, int, const void*, long, void*, long, int, int, long, hipStream_t);
+                       void*, int, hipStream_t);
+int dllm_gate_heads(const void*, int, const void*, long, void*, long, int, int, long, int, hipStream_t);
 int dllm_scaled_resadd_rms(const void*, long, int, float, int, const float*, float*, const float*, void*, long, long, int, float,
                            hipStream_t);
 int dllm_relu2_scale(const void*, int, const float*, int, int, void*, long, int, hipStream_t);
 int dllm_dense_gate(const int*, const float*, float*, long, int, int, hipStream_t);
 int dllm_latent_kv_write(const void*, long, int, int, int, const float*, float, const int*, const float*, int, const int*,
-                         void*, int, hipStream_t);
+                         void*, int, int, const void*, long, int, const float*, void*, void*, int, hipStream_t);
 int dllm_latent_attention(const void*, const void*, long, int, int, int, int, int, long, const float*, int, const void*,
                           const int*, int, const int*, const int*, const int*, const int*, const int*, int, float, void*,
-                          int, float*, float*, int, int, hipStream_t);
+                          int, float*, float*, int, int, int, const float*, hipStream_t);
 int dllm_latent_mfma_ok(int, int, int);
 int dllm_car_alloc(long, void**);
 int dllm_car_get_handle(void*, char*);
@@ -1532,7 +1533,8 @@ void lightning_attention(torch::Tensor qkvg, int64_t H, int64_t d, int64_t dv, t
 void resadd_norm(torch::Tensor a, c10::optional<torch::Tensor> b, c10::optional<torch::Tensor> wa,
                  c10::optional<torch::Tensor> wb, torch::Tensor w_post, double eps, torch::Tensor x,
                  c10::optional<torch::Tensor> w_next, c10::optional<torch::Tensor> xn,
-                 c10::optional<torch::Tensor> stack, c10::optional<torch::Tensor> dw, int64_t dn) {
+                 c10::optional<torch::Tensor> stack, c10::optional<torch::Tensor> dw, int64_t dn,
+                 c10::optional<torch::Tensor> bias) {
   const bool f = act_f32(a, "a");
   check_rows2d(a, "a");
   check_f32(w_post, "w_post");
@@ -1551,7 +1553,12 @@ void resadd_norm(torch::Tensor a, c10::optional<torch::Tensor> b, c10::optional<
   TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && x.sizes() == a.sizes() && w_post.numel() == x.size(1),
               "x / a / w_post shapes");
   const void* bp = nullptr;
-  const float *wap = nullptr, *wbp = nullptr, *wnp = nullptr;
+  const float *wap = nullptr, *wbp = nullptr, *wnp = nullptr, *biasp = nullptr;
+  if (bias) {
+    check_f32(*bias, "bias");
+    TORCH_CHECK(bias->is_contiguous() && bias->numel() == x.size(1), "bias [H]");
+    biasp = bias->data_ptr<float>();
+  }
   long ldb = 0;
   if (b) {
     TORCH_CHECK(wa && wb, "two branches need both norm weights");
@@ -1578,7 +1585,7 @@ void resadd_norm(torch::Tensor a, c10::optional<torch::Tensor> b, c10::optional<
     }
   }
   ok(dllm_resadd_norm(a.data_ptr(), a.stride(0), bp, ldb, f, wap, wbp, w_post.data_ptr<float>(), x.data_ptr<float>(), wnp,
-                      xp, (int)x.size(0), (int)x.size(1), (float)eps, dwp, (int)dn, stream()),
+                      xp, (int)x.size(0), (int)x.size(1), (float)eps, dwp, (int)dn, biasp, stream()),
      "resadd_norm");
 }
 
@@ -1687,7 +1694,7 @@ void paged_gqa_attention(torch::Tensor q, torch::Tensor kc, torch::Tensor vc, to
                          torch::Tensor qlen, torch::Tensor ctx, torch::Tensor tile_seq, torch::Tensor tile_tok0,
                          c10::optional<torch::Tensor> gate, torch::Tensor out, bool mfma, int64_t splits,
                          c10::optional<torch::Tensor> part, int64_t window, int64_t keep_first, double sink, int64_t chunk,
-                         double cap, c10::optional<torch::Tensor> sinks) {
+                         double cap, c10::optional<torch::Tensor> sinks, c10::optional<torch::Tensor> slopes) {
   const bool f = act_f32(q, "q");
   TORCH_CHECK(keep_first >= 0 && sink >= 0.0, "keep_first >= 0, sink >= 0");
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous(), "q [T, H, d]");
@@ -1710,10 +1717,13 @@ void paged_gqa_attention(torch::Tensor q, torch::Tensor kc, torch::Tensor vc, to
               "metadata lengths");
   const void* gp = nullptr;
   long ldg = 0;
+  bool ghead = false;      // one gate logit per head
   if (gate) {
     check_rows2d(*gate, "gate");
-    TORCH_CHECK(gate->is_cuda() && gate->scalar_type() == q.scalar_type() && gate->size(0) == T && gate->size(1) == H * dv,
-                "gate [T, H dv]");
+    ghead = gate->size(1) == H;
+    TORCH_CHECK(gate->is_cuda() && gate->scalar_type() == q.scalar_type() && gate->size(0) == T &&
+                    (ghead || gate->size(1) == H * dv),
+                "gate [T, H dv] or [T, H]");
     gp = gate->data_ptr();
     ldg = gate->stride(0);
   }
@@ -1728,6 +1738,12 @@ void paged_gqa_attention(torch::Tensor q, torch::Tensor kc, torch::Tensor vc, to
     TORCH_CHECK(sinks->is_contiguous() && sinks->numel() == H && sink == 0.0, "sinks [H] f32, instead of a sink weight");
     sk = sinks->data_ptr<float>();
   }
+  const float* sl = nullptr;
+  if (slopes) {
+    check_f32(*slopes, "slopes");
+    TORCH_CHECK(slopes->is_contiguous() && slopes->numel() == H && cap == 0.0, "slopes [H] f32, not beside a cap");
+    sl = slopes->data_ptr<float>();
+  }
   float* pptr = nullptr;
   TORCH_CHECK(splits >= 1 && splits <= 64 && (splits == 1 || mfma), "key splits: 1..64, matrix-core kernel only");
   if (splits > 1) {
@@ -1741,7 +1757,7 @@ void paged_gqa_attention(torch::Tensor q, torch::Tensor kc, torch::Tensor vc, to
                                 tile_seq.data_ptr<int>(), tile_tok0.data_ptr<int>(), (int)tile_seq.numel(), gp, ldg,
                                 out.data_ptr(), (int)H, (int)G, (int)d, (int)dv, (int)mfma, (int)splits, pptr, (int)window,
                                 (int)GV, (int)of32, (int)keep_first, (float)sink, (int)chunk, (float)cap, sk,
-                                (long)out.stride(0), stream());
+                                (long)out.stride(0), sl, (int)ghead, stream());
   TORCH_CHECK(rc != -2, "head widths do not fit the LDS");
   ok(rc, "paged_gqa_attention");
 }
@@ -1756,7 +1772,8 @@ static void act_rows(const torch::Tensor& t, const torch::Tensor& like, int64_t 
 
 void rope_prep(torch::Tensor proj, int64_t H, int64_t G, int64_t d, int64_t dv, torch::Tensor cos_sin, int64_t rot, double qscale,
                torch::Tensor pos, torch::Tensor slots, torch::Tensor kc, torch::Tensor vc, torch::Tensor q, int64_t ucol,
-               c10::optional<torch::Tensor> act, c10::optional<torch::Tensor> zero_rows) {
+               c10::optional<torch::Tensor> act, c10::optional<torch::Tensor> zero_rows, c10::optional<torch::Tensor> bias,
+               c10::optional<torch::Tensor> qtab) {
   const bool f = act_f32(proj, "proj");
   check_rows2d(proj, "proj");
   check_f32(cos_sin, "cos_sin");
@@ -1789,9 +1806,21 @@ void rope_prep(torch::Tensor proj, int64_t H, int64_t G, int64_t d, int64_t dv, 
     zp = zero_rows->data_ptr();
     ldz = zero_rows->stride(0);
   }
+  const float *bp = nullptr, *tp = nullptr;
+  if (bias) {
+    check_f32(*bias, "bias");
+    TORCH_CHECK(bias->is_contiguous() && bias->numel() == (H + G) * d + G * dv, "bias over the q | k | v columns");
+    bp = bias->data_ptr<float>();
+  }
+  if (qtab) {
+    check_f32(*qtab, "qtab");
+    TORCH_CHECK(qtab->is_contiguous() && qtab->dim() == 1 && qtab->numel() >= cos_sin.size(0), "one query factor per position");
+    tp = qtab->data_ptr<float>();
+  }
   ok(dllm_rope_prep(proj.data_ptr(), proj.stride(0), f, (int)H, (int)G, (int)d, (int)dv, cos_sin.data_ptr<float>(),
                     (int)cos_sin.size(1), (int)rot, (float)qscale, pos.data_ptr<int>(), slots.data_ptr<int>(), kc.data_ptr(),
-                    vc.data_ptr(), q.data_ptr(), (long)T, (int)kc.size(2), (int)ucol, (int)ff, ap, lda, zp, ldz, (int)zn, stream()),
+                    vc.data_ptr(), q.data_ptr(), (long)T, (int)kc.size(2), (int)ucol, (int)ff, ap, lda, zp, ldz, (int)zn, bp, tp,
+                    stream()),
      "rope_prep");
 }
 
@@ -1847,20 +1876,21 @@ void latent_expand(torch::Tensor cache, torch::Tensor bt, torch::Tensor ctx, tor
   check_i32(ctx, "ctx");
   TORCH_CHECK(cache.is_cuda() && cache.scalar_type() == torch::kBFloat16 && cache.is_contiguous() && cache.dim() == 3 &&
                   cache.size(1) == 16,
-              "cache [blocks, 16, rank] bf16");
-  const int64_t S = ctx.numel(), nb = bt.size(1), rank = cache.size(2);
+              "cache [blocks, 16, rank + rot] bf16");
+  const int64_t S = ctx.numel(), nb = bt.size(1), rank = wk.size(-1), rot = cache.size(2) - rank;
   TORCH_CHECK(bt.dim() == 2 && bt.stride(1) == 1 && bt.size(0) >= S && ctx.is_contiguous(), "block_tables [S, blocks], ctx [S]");
   for (auto* t : {&kc, &vc, &wk, &wv})
     TORCH_CHECK(t->is_cuda() && t->scalar_type() == torch::kBFloat16 && t->is_contiguous(), "bf16 contiguous tensors");
   TORCH_CHECK(kc.dim() == 4 && vc.dim() == 4 && kc.size(0) == S * nb && vc.size(0) == S * nb && kc.size(1) == vc.size(1) &&
                   kc.size(2) == 16 && vc.size(3) == 16,
-              "K [S blocks, H, 16, d], V [S blocks, H, dv, 16]");
-  const int64_t H = kc.size(1), d = kc.size(3), dv = vc.size(2);
-  TORCH_CHECK(wk.numel() == H * d * rank && wv.numel() == H * dv * rank && dllm_latent_expand_ok((int)rank, (int)d, (int)dv),
-              "weights [H d, rank], [H dv, rank]; rank % 32 == 0, d % 8 == 0");
+              "K [S blocks, H, 16, d + rot], V [S blocks, H, dv, 16]");
+  const int64_t H = kc.size(1), d = kc.size(3) - rot, dv = vc.size(2);
+  TORCH_CHECK(rot >= 0 && d >= 1 && wk.numel() == H * d * rank && wv.numel() == H * dv * rank &&
+                  dllm_latent_expand_ok((int)rank, (int)d, (int)dv, (int)rot),
+              "weights [H d, rank], [H dv, rank]; rank % 32 == 0, d % 8 == 0, rot % 8 == 0");
   ok(dllm_latent_expand(cache.data_ptr(), bt.data_ptr<int>(), (int)bt.stride(0), (int)S, (int)nb, (int)cache.size(0),
                         ctx.data_ptr<int>(), (int)rank, (int)H, (int)d, (int)dv, wk.data_ptr(), wv.data_ptr(), kc.data_ptr(),
-                        vc.data_ptr(), stream()),
+                        vc.data_ptr(), (int)rot, stream()),
      "latent_expand");
 }
 
@@ -1868,10 +1898,11 @@ void gate_heads(torch::Tensor o, torch::Tensor gate, torch::Tensor out) {
   const bool f = act_f32(o, "o");
   TORCH_CHECK(o.dim() == 3 && o.is_contiguous(), "o [H, T, dv] contiguous");
   const int64_t H = o.size(0), T = o.size(1), dv = o.size(2);
-  act_rows(gate, o, T, H * dv, "gate");
+  const bool ghead = gate.dim() == 2 && gate.size(1) == H;      // one logit per head
+  act_rows(gate, o, T, ghead ? H : H * dv, "gate");
   act_rows(out, o, T, H * dv, "out");
   ok(dllm_gate_heads(o.data_ptr(), f, gate.data_ptr(), gate.stride(0), out.data_ptr(), out.stride(0), (int)H, (int)dv, (long)T,
-                     stream()),
+                     (int)ghead, stream()),
      "gate_heads");
 }
 
@@ -2148,7 +2179,7 @@ void ls_resadd_ln(torch::Tensor x, torch::Tensor w, torch::Tensor b, double eps,
 void glu_act(torch::Tensor gu, c10::optional<torch::Tensor> bias, int64_t mode, double limit, double alpha, torch::Tensor y) {
   const bool f = act_f32(gu, "gu");
   check_rows2d(gu, "gu");
-  TORCH_CHECK(gu.size(1) % 2 == 0 && (mode == 0 || mode == 1), "gu [T, 2 ff]; mode 0 or 1");
+  TORCH_CHECK(gu.size(1) % 2 == 0 && mode >= 0 && mode <= 2, "gu [T, 2 ff]; mode 0, 1 or 2");
   const int64_t ff = gu.size(1) / 2;
   TORCH_CHECK(y.is_cuda() && y.scalar_type() == gu.scalar_type() && y.is_contiguous() && y.dim() == 2 &&
                   y.size(0) == gu.size(0) && y.size(1) == ff,
@@ -2254,7 +2285,9 @@ void dense_gate(torch::Tensor ids, torch::Tensor wts, torch::Tensor g) {
 }
 
 void latent_kv_write(torch::Tensor ckv, int64_t rank, torch::Tensor w, double eps, torch::Tensor pos,
-                     torch::Tensor cos_sin, torch::Tensor slots, torch::Tensor cache) {
+                     torch::Tensor cos_sin, torch::Tensor slots, torch::Tensor cache, bool half,
+                     c10::optional<torch::Tensor> q_src, c10::optional<torch::Tensor> q_norm,
+                     c10::optional<torch::Tensor> q_out, c10::optional<torch::Tensor> zero) {
   const bool f = act_f32(ckv, "ckv");
   check_rows2d(ckv, "ckv");
   check_f32(w, "norm weight");
@@ -2269,17 +2302,57 @@ void latent_kv_write(torch::Tensor ckv, int64_t rank, torch::Tensor w, double ep
   TORCH_CHECK(cache.is_cuda() && cache.scalar_type() == ckv.scalar_type() && cache.is_contiguous() && cache.dim() == 3 &&
                   cache.size(1) == 16 && cache.size(2) == rank + rot,
               "cache [blocks, 16, rank + rot] in the dtype of ckv");
+  const void* qs = nullptr;
+  const float* qw = nullptr;
+  void *qd = nullptr, *zp = nullptr;
+  long ldqs = 0;
+  int64_t qn = 0, zh = 0;
+  if (q_src) {
+    TORCH_CHECK(q_norm && q_out, "a query latent needs its norm weight and its output");
+    qn = q_src->size(1);
+    act_rows(*q_src, ckv, T, qn, "q_src");
+    check_f32(*q_norm, "q_norm");
+    act_rows(*q_out, ckv, T, qn, "q_out");
+    TORCH_CHECK(qn >= 1 && q_norm->is_contiguous() && q_norm->numel() == qn && q_out->is_contiguous(), "query latent");
+    qs = q_src->data_ptr();
+    ldqs = q_src->stride(0);
+    qw = q_norm->data_ptr<float>();
+    qd = q_out->data_ptr();
+  }
+  if (zero) {
+    TORCH_CHECK(zero->is_cuda() && zero->scalar_type() == ckv.scalar_type() && zero->is_contiguous() && zero->dim() == 3 &&
+                    zero->size(1) == T && zero->size(2) == rank,
+                "zero [H, T, rank] in the activations' dtype");
+    zh = zero->size(0);
+    zp = zero->data_ptr();
+  }
   ok(dllm_latent_kv_write(ckv.data_ptr(), ckv.stride(0), f, (int)rank, (int)rot, w.data_ptr<float>(), (float)eps,
                           pos.data_ptr<int>(), cos_sin.data_ptr<float>(), (int)cos_sin.size(1), slots.data_ptr<int>(),
-                          cache.data_ptr(), T, stream()),
+                          cache.data_ptr(), T, (int)half, qs, ldqs, (int)qn, qw, qd, zp, (int)zh, stream()),
      "latent_kv_write");
+}
+
+void latent_q_prep(torch::Tensor q, int64_t H, int64_t dim, int64_t rot, bool half, torch::Tensor pos, torch::Tensor cos_sin,
+                   double scale, torch::Tensor out) {
+  const bool f = act_f32(q, "q");
+  check_rows2d(q, "q");
+  check_f32(cos_sin, "cos_sin");
+  check_i32(pos, "positions");
+  const int64_t T = q.size(0);
+  TORCH_CHECK(H >= 1 && dim >= 0 && rot >= 0 && rot % 2 == 0 && q.size(1) >= H * (dim + rot) && pos.numel() == T, "q [T, H (dim + rot)]");
+  TORCH_CHECK(cos_sin.dim() == 2 && cos_sin.is_contiguous() && cos_sin.size(1) >= rot, "rotation table");
+  TORCH_CHECK(out.is_cuda() && out.scalar_type() == q.scalar_type() && out.is_contiguous() && out.numel() == T * H * (dim + rot),
+              "out [T, H, dim + rot] contiguous");
+  ok(dllm_latent_q_prep(q.data_ptr(), q.stride(0), f, (int)H, (int)dim, (int)rot, (int)half, pos.data_ptr<int>(),
+                        cos_sin.data_ptr<float>(), (int)cos_sin.size(1), (float)scale, out.data_ptr(), (long)T, stream()),
+     "latent_q_prep");
 }
 
 void latent_attention(torch::Tensor qa, torch::Tensor q, int64_t dim, int64_t rot, torch::Tensor pos, torch::Tensor cos_sin,
                       torch::Tensor cache, torch::Tensor bt, torch::Tensor qstart, torch::Tensor qlen, torch::Tensor ctx,
                       torch::Tensor tile_seq, torch::Tensor tile_tok0, double scale, torch::Tensor out, int64_t splits,
                       c10::optional<torch::Tensor> part_o, c10::optional<torch::Tensor> part_ml, bool mfma,
-                      int64_t rows) {
+                      int64_t rows, bool half, c10::optional<torch::Tensor> sinks) {
   const bool f = act_f32(qa, "qa");
   TORCH_CHECK(rows == 16 || (rows == 32 && mfma && !f && dllm_latent_mfma_ok((int)qa.size(2), (int)rot, 32)),
               "rows per workgroup: 16, or 32 where the matrix-core kernel takes the shape");
@@ -2301,6 +2374,12 @@ void latent_attention(torch::Tensor qa, torch::Tensor q, int64_t dim, int64_t ro
   TORCH_CHECK(rank <= 512, "latent rank <= 512");
   TORCH_CHECK(out.is_cuda() && out.scalar_type() == qa.scalar_type() && out.is_contiguous() && out.sizes() == qa.sizes(),
               "out like qa");
+  const float* sk = nullptr;
+  if (sinks) {
+    check_f32(*sinks, "sinks");
+    TORCH_CHECK(sinks->is_contiguous() && sinks->numel() == H, "sinks [H] f32");
+    sk = sinks->data_ptr<float>();
+  }
   float *po = nullptr, *pml = nullptr;
   TORCH_CHECK(splits >= 1 && splits <= 64, "splits in [1, 64]");
   if (splits > 1) {
@@ -2316,7 +2395,7 @@ void latent_attention(torch::Tensor qa, torch::Tensor q, int64_t dim, int64_t ro
                            cos_sin.data_ptr<float>(), (int)cos_sin.size(1), cache.data_ptr(), bt.data_ptr<int>(),
                            (int)bt.size(1), qstart.data_ptr<int>(), qlen.data_ptr<int>(), ctx.data_ptr<int>(),
                            tile_seq.data_ptr<int>(), tile_tok0.data_ptr<int>(), (int)tile_seq.numel(), (float)scale,
-                           out.data_ptr(), (int)splits, po, pml, mfma ? 1 : 0, (int)rows, stream()),
+                           out.data_ptr(), (int)splits, po, pml, mfma ? 1 : 0, (int)rows, (int)half, sk, stream()),
      "latent_attention");
 }
 }  // namespace
@@ -2353,7 +2432,7 @@ PYBIND11_MODULE(_hip_kernels, m) {
   m.def("lightning_attention", &lightning_attention);
   m.def("resadd_norm", &resadd_norm, py::arg("a"), py::arg("b"), py::arg("wa"), py::arg("wb"), py::arg("w_post"),
         py::arg("eps"), py::arg("x"), py::arg("w_next"), py::arg("x_next"), py::arg("stack") = py::none(),
-        py::arg("depth_w") = py::none(), py::arg("depth_n") = 0);
+        py::arg("depth_w") = py::none(), py::arg("depth_n") = 0, py::arg("bias") = py::none());
   m.def("depth_mix", &depth_mix);
   m.def("gelu_erf", &gelu_erf);
   m.def("conv_state_refill", &conv_state_refill);
@@ -2363,11 +2442,14 @@ PYBIND11_MODULE(_hip_kernels, m) {
         py::arg("block_tables"), py::arg("qstart"), py::arg("qlen"), py::arg("ctx"), py::arg("tile_seq"),
         py::arg("tile_tok0"), py::arg("gate"), py::arg("out"), py::arg("mfma"), py::arg("splits") = 1,
         py::arg("part") = py::none(), py::arg("window") = 0, py::arg("keep_first") = 0, py::arg("sink") = 0.0,
-        py::arg("chunk") = 0, py::arg("cap") = 0.0, py::arg("sinks") = py::none());
+        py::arg("chunk") = 0, py::arg("cap") = 0.0, py::arg("sinks") = py::none(), py::arg("slopes") = py::none());
   m.def("rope_prep", &rope_prep);
   m.def("latent_prep", &latent_prep);
   m.def("latent_expand", &latent_expand);
-  m.def("latent_expand_ok", [](int64_t rank, int64_t d, int64_t dv) { return dllm_latent_expand_ok((int)rank, (int)d, (int)dv) != 0; });
+  m.def("latent_expand_ok",
+        [](int64_t rank, int64_t d, int64_t dv, int64_t rot) { return dllm_latent_expand_ok((int)rank, (int)d, (int)dv, (int)rot) != 0; },
+        py::arg("rank"), py::arg("d"), py::arg("dv"), py::arg("rot") = 0);
+  m.def("latent_q_prep", &latent_q_prep);
   m.def("gate_heads", &gate_heads);
   m.def("scaled_resadd_rms", &scaled_resadd_rms);
   m.def("gqa_tile_tokens",
@@ -2375,12 +2457,14 @@ PYBIND11_MODULE(_hip_kernels, m) {
   m.def("gqa_mfma_ok", [](bool f32, int64_t H, int64_t G, int64_t d, int64_t dv, int64_t bs) {
     return (bool)dllm_gqa_mfma_ok((int)f32, (int)H, (int)G, (int)d, (int)dv, (int)bs);
   });
-  m.def("latent_kv_write", &latent_kv_write);
+  m.def("latent_kv_write", &latent_kv_write, py::arg("ckv"), py::arg("rank"), py::arg("w"), py::arg("eps"), py::arg("positions"),
+        py::arg("cos_sin"), py::arg("slots"), py::arg("cache"), py::arg("half") = false, py::arg("q_src") = py::none(),
+        py::arg("q_norm") = py::none(), py::arg("q_out") = py::none(), py::arg("zero") = py::none());
   m.def("latent_attention", &latent_attention, py::arg("qa"), py::arg("q"), py::arg("dim"), py::arg("rot"),
         py::arg("positions"), py::arg("cos_sin"), py::arg("cache"), py::arg("block_tables"), py::arg("qstart"),
         py::arg("qlen"), py::arg("ctx"), py::arg("tile_seq"), py::arg("tile_tok0"), py::arg("scale"), py::arg("out"),
         py::arg("splits") = 1, py::arg("part_o") = py::none(), py::arg("part_ml") = py::none(), py::arg("mfma") = true,
-        py::arg("rows") = 16);
+        py::arg("rows") = 16, py::arg("half") = false, py::arg("sinks") = py::none());
   m.def("latent_mfma_ok", [](int64_t rank, int64_t rot, int64_t rows) { return dllm_latent_mfma_ok((int)rank, (int)rot, (int)rows) != 0; });
   m.def("encoder_attention", &encoder_attention);
   m.def("embed_ln", &embed_ln);

@@ -24,15 +24,19 @@
 //               own LDS patch as bf16 hi + lo parts, so the weighted sum sees them to 16 bits of
 //               mantissa through two MFMAs.  Key blocks above a wave's newest row are skipped.
 //
-//   rope_prep   attention inputs without a q / k norm: rotate-half positions on the first `rot` dims, q
-//               times one scale; the launch also squares the relu of a feed-forward's up columns that
-//               the same projection made (latent_prep: the same beside a normed latent).
+//   rope_prep   attention inputs without a q / k norm: optional biases, rotate-half positions on the first
+//               `rot` dims, q times one scale and optionally a number of its position; the launch also squares
+//               the relu of a feed-forward's up columns that the same projection made (latent_prep: the
+//               same beside a normed latent).
 //
 // Both attention kernels take a window (a row at position p sees keys p - win < j <= p) or a chunk (it
 // sees the keys of its own chunk of positions, [p - p % chunk, p]), kept first keys (j < keep stays
 // visible at any distance; the tiles between the kept keys and the window are not read), a soft cap on
 // the scores (cap tanh(s / cap)) and a sink: one more term of the denominator, with no value, either
 // exp(0) times `sink` or exp(sinks[head]).  Under a cap the matrix-core form keeps no running maximum.
+// slopes: a head's scores fall by slopes[head] per position between row and key (not beside a cap); the
+// matrix-core form starts its score accumulators there.  The gate has one logit per output entry or
+// (ghead) one per head.
 //
 // Cache layout: K [blocks, G, block, d], V [blocks, G, dv, block] (bf16 or f32 like the activations;
 // V is kept transposed inside its page because the weighted sum runs over keys); every score,
@@ -270,14 +274,16 @@ __device__ __forceinline__ void act_share<u16>(const u16* __restrict__ up, int f
 // positions on the first `rot` dims (cos and sin as the table holds them), q times qscale; k and v to
 // their page slots.  act (null: no feed-forward): act[tok] = relu(proj[tok, ucol : ucol + ff])^2.
 // zrow: the first zn columns of a padding token's row (slot < 0) are cleared (an attention output whose
-// padding rows no tile writes).
+// padding rows no tile writes).  bias (f32 over the q | k | v columns) is added before the rotation; qtab:
+// q is also multiplied by qtab[position].
 template <typename T>
 __global__ void __launch_bounds__(256) rope_prep_kernel(const T* __restrict__ proj, long ld, int H, int G, int d, int dv,
                                                         const float* __restrict__ cos_sin, int tab_w, int rot, float qscale,
                                                         const int* __restrict__ pos, const int* __restrict__ slots,
                                                         T* __restrict__ kc, T* __restrict__ vc, T* __restrict__ q, int BSZ,
                                                         int ucol, int ff, T* __restrict__ act, long lda, int vec,
-                                                        T* __restrict__ zrow, long ldz, int zn) {
+                                                        T* __restrict__ zrow, long ldz, int zn, const float* __restrict__ bias,
+                                                        const float* __restrict__ qtab) {
   const long tok = blockIdx.x;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const T* r = proj + tok * ld;
@@ -292,15 +298,16 @@ __global__ void __launch_bounds__(256) rope_prep_kernel(const T* __restrict__ pr
     const bool is_q = hh < H;
     if (!is_q && slot < 0) continue;
     const T* x = r + (long)hh * d;
+    const float* b = bias ? bias + (long)hh * d : nullptr;
     T* dst = is_q ? q + (tok * H + hh) * d : kc + ((blk * G + (hh - H)) * BSZ + off) * d;
-    const float os = is_q ? qscale : 1.f;
+    const float os = is_q ? (qtab ? qscale * qtab[pos[tok]] : qscale) : 1.f;
     for (int i = lane; i < d; i += 64) {
-      float v = ldf(x + i);
+      float v = ldf(x + i) + (b ? b[i] : 0.f);
       if (i < rot) {
         const bool first = i < half;
-        const int f = first ? i : i - half;
+        const int f = first ? i : i - half, j = first ? i + half : i - half;
         const float c = cs[f], sn = cs[half + f];
-        const float p = ldf(x + (first ? i + half : i - half));
+        const float p = ldf(x + j) + (b ? b[j] : 0.f);
         v = first ? v * c - p * sn : v * c + p * sn;
       }
       stf(dst + i, v * os);
@@ -308,8 +315,12 @@ __global__ void __launch_bounds__(256) rope_prep_kernel(const T* __restrict__ pr
   }
   if (slot >= 0) {   // values: this workgroup's share of the G * dv entries
     const T* v = r + (long)(H + G) * d;
-    for (int i = blockIdx.y * 256 + tid; i < G * dv; i += gridDim.y * 256)
-      vc[((blk * G + i / dv) * dv + i % dv) * BSZ + off] = v[i];
+    const float* b = bias ? bias + (long)(H + G) * d : nullptr;
+    for (int i = blockIdx.y * 256 + tid; i < G * dv; i += gridDim.y * 256) {
+      T* dst = vc + ((blk * G + i / dv) * dv + i % dv) * BSZ + off;
+      if (b) stf(dst, ldf(v + i) + b[i]);
+      else *dst = v[i];
+    }
   }
   if (act) act_share<T>(r + ucol, ff, act + tok * lda, blockIdx.y, gridDim.y, tid, vec);
 }
@@ -347,7 +358,8 @@ __global__ void __launch_bounds__(256) paged_gqa_kernel(const T* __restrict__ q,
                                                         const T* __restrict__ gate, long ldg, T* __restrict__ out, int H,
                                                         int G, int d, int dv, int TQ, int KT, int win, int GV,
                                                         float* __restrict__ out32, int keep, float sink, int chunk,
-                                                        float cap, const float* __restrict__ sinks, long ldo) {
+                                                        float cap, const float* __restrict__ sinks, long ldo,
+                                                        const float* __restrict__ slopes, int ghead) {
   // win > 0: a row at position p sees keys p - win < j <= p, and keys j < keep; chunk > 0: keys of its
   // own chunk.  GV value heads: key head g reads value head g / (G / GV).  out32: the output stays f32.
   // sink: one more term of score 0 and that weight in the denominator; sinks: of score sinks[head].
@@ -373,7 +385,7 @@ __global__ void __launch_bounds__(256) paged_gqa_kernel(const T* __restrict__ q,
     if (rr < nrows) v = ldf(q + ((long)(q0 + tok0 + rr / Rh) * H + g * R + r0 + rr % Rh) * d + i);
     Qs[e] = v;
   }
-  float m[4], l[4], O[4][NJ];
+  float m[4], l[4], O[4][NJ], slp[4];
   int rpos[4], rlo[4];
 #pragma unroll
   for (int x = 0; x < 4; ++x) {
@@ -382,6 +394,7 @@ __global__ void __launch_bounds__(256) paged_gqa_kernel(const T* __restrict__ q,
     l[x] = 0.f;
     rpos[x] = rr < nrows ? p0 + tok0 + rr / Rh : -1;   // -1: sees no key
     rlo[x] = rr < nrows ? oldest_key(rpos[x], win, chunk) : 0;
+    slp[x] = slopes && rr < nrows ? slopes[g * R + r0 + rr % Rh] : 0.f;
 #pragma unroll
     for (int jj = 0; jj < NJ; ++jj) O[x][jj] = 0.f;
   }
@@ -427,7 +440,7 @@ __global__ void __launch_bounds__(256) paged_gqa_kernel(const T* __restrict__ q,
 #pragma unroll
     for (int x = 0; x < 4; ++x) {
       const bool vis = lane < nk && pk <= rpos[x] && (pk >= rlo[x] || pk < keep);
-      const float sv = !vis ? -INFINITY : cap > 0.f ? cap * tanhf(sc[x] / cap) : sc[x];
+      const float sv = !vis ? -INFINITY : cap > 0.f ? cap * tanhf(sc[x] / cap) : slopes ? sc[x] - slp[x] * (float)(rpos[x] - pk) : sc[x];
       const float mn = fmaxf(m[x], wave_max(sv));
       float p = 0.f, f = 1.f;
       if (mn > -INFINITY) {
@@ -466,7 +479,7 @@ __global__ void __launch_bounds__(256) paged_gqa_kernel(const T* __restrict__ q,
       const int jx = lane + 64 * jj;
       if (jx >= dv) continue;
       float o = O[x][jj] * inv;
-      if (gate) o *= 1.f / (1.f + expf(-ldf(gate + tok * ldg + (long)h * dv + jx)));
+      if (gate) o *= 1.f / (1.f + expf(-ldf(gate + tok * ldg + (ghead ? (long)h : (long)h * dv + jx))));
       if (out32) out32[tok * ldo + (long)h * dv + jx] = o;
       else stf(out + tok * ldo + (long)h * dv + jx, o);
     }
@@ -502,7 +515,8 @@ typedef __bf16 bf16x2v __attribute__((ext_vector_type(2)));
 // indices 8 g4 .. 8 g4 + 7; B holds column lr, the same indices; the accumulator holds rows
 // 4 g4 .. 4 g4 + 3 of column lr.
 constexpr float CAP_MAX = 64.f;
-template <int SZ, bool CAP>
+// DIST: the scores fall with the distance (`slopes`); the score accumulators start at -slope * distance.
+template <int SZ, bool CAP, bool DIST>
 __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restrict__ q, const u16* __restrict__ kc,
                                                              const u16* __restrict__ vc, const int* __restrict__ bt,
                                                              int bt_ld, const int* __restrict__ qstart,
@@ -512,7 +526,8 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
                                                              long ldg, u16* __restrict__ out, int H, int G, int d, int dv,
                                                              int TQ, int splits, float* __restrict__ part, int win, int GV,
                                                              float* __restrict__ out32, int keep, float sink, int chunk,
-                                                             float cap, const float* __restrict__ sinks, long ldo) {
+                                                             float cap, const float* __restrict__ sinks, long ldo,
+                                                             const float* __restrict__ slopes, int ghead) {
   constexpr int DS = SZ / 32, VB = SZ / 16, NKB = GM_KT / 16;
   constexpr int KSTR = SZ + 8, VSTR = GM_KT + 8, PSTR = GM_KT + 8;
   extern __shared__ __attribute__((aligned(16))) unsigned char smraw[];
@@ -547,13 +562,14 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     }
   }
   int rpos[4], rlo[4];
-  float m[4], l[4];
+  float m[4], l[4], slp[4];
   f32x4 acc[VB];
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int row = 16 * wave + 4 * g4 + i;
     rpos[i] = row < nrows ? p0 + tok0 + row / R : -1;     // -1: sees no key
     rlo[i] = row < nrows ? oldest_key(rpos[i], win, chunk) : 0;
+    slp[i] = DIST && row < nrows ? slopes[g * R + row % R] : 0.f;
     m[i] = CAP ? 0.f : -INFINITY;
     l[i] = 0.f;
   }
@@ -633,8 +649,17 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     if (k0 > wave_last) continue;   // this wave's rows see nothing of the tile (the barriers above are uniform)
     if (k0 >= keep && k0 + GM_KT <= wave_lo) continue;   // ... or the tile lies before every row's window / chunk
     f32x4 sacc[NKB];
+    if constexpr (DIST) {
 #pragma unroll
-    for (int kb = 0; kb < NKB; ++kb) sacc[kb] = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int i = 0; i < 4; ++i) {
+        const float d0 = slp[i] * (float)(k0 + 4 * lr - rpos[i]);
+#pragma unroll
+        for (int kb = 0; kb < NKB; ++kb) sacc[kb][i] = fmaf(slp[i], (float)kb, d0);
+      }
+    } else {
+#pragma unroll
+      for (int kb = 0; kb < NKB; ++kb) sacc[kb] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
 #pragma unroll
     for (int st = 0; st < DS; ++st) {
 #pragma unroll
@@ -648,7 +673,7 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     for (int kb = 0; kb < NKB; ++kb)
 #pragma unroll
       for (int i = 0; i < 4; ++i) sc[kb][i] = sacc[kb][i];
-    if (!CAP && cap > 0.f) {
+    if (!CAP && !DIST && cap > 0.f) {
 #pragma unroll
       for (int kb = 0; kb < NKB; ++kb)
 #pragma unroll
@@ -748,13 +773,14 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     }
     const long tok = q0 + tok0 + row / R;
     const int h = g * R + row % R;
-    const float inv = 1.f / (lt + (sinks ? __expf(sinks[h] - m[i]) : sink > 0.f ? sink * __expf(-m[i]) : 0.f));
+    float inv = 1.f / (lt + (sinks ? __expf(sinks[h] - m[i]) : sink > 0.f ? sink * __expf(-m[i]) : 0.f));
+    if (gate && ghead) inv *= 1.f / (1.f + expf(-bf2f(gate[tok * ldg + h])));
 #pragma unroll
     for (int cb = 0; cb < VB; ++cb) {
       const int jx = 16 * cb + lr;
       if (jx >= dv) continue;
       float o = acc[cb][i] * inv;
-      if (gate) o *= 1.f / (1.f + expf(-bf2f(gate[tok * ldg + (long)h * dv + jx])));
+      if (gate && !ghead) o *= 1.f / (1.f + expf(-bf2f(gate[tok * ldg + (long)h * dv + jx])));
       if (out32) out32[tok * ldo + (long)h * dv + jx] = o;
       else out[tok * ldo + (long)h * dv + jx] = f2bf(o);
     }
@@ -768,7 +794,7 @@ __global__ void __launch_bounds__(256) gqa_combine_kernel(const float* __restric
                                                           const int* __restrict__ tile_tok0, const u16* __restrict__ gate,
                                                           long ldg, u16* __restrict__ out, int H, int G, int dv, int TQ,
                                                           float* __restrict__ out32, float sink,
-                                                          const float* __restrict__ sinks, long ldo) {
+                                                          const float* __restrict__ sinks, long ldo, int ghead) {
   const int s = tile_seq[blockIdx.x];
   const int n = qlen[s], tok0 = tile_tok0[blockIdx.x];
   if (n <= 0 || tok0 >= n) return;
@@ -797,7 +823,7 @@ __global__ void __launch_bounds__(256) gqa_combine_kernel(const float* __restric
       }
       if (!on) continue;
       o /= L;
-      if (gate) o *= 1.f / (1.f + expf(-bf2f(gate[tok * ldg + (long)h * dv + jx])));
+      if (gate) o *= 1.f / (1.f + expf(-bf2f(gate[tok * ldg + (ghead ? (long)h : (long)h * dv + jx)])));
       if (out32) out32[tok * ldo + (long)h * dv + jx] = o;
       else out[tok * ldo + (long)h * dv + jx] = f2bf(o);
     }
@@ -821,10 +847,11 @@ template <typename T, int NJ>
 int launch_gqa(dim3 grid, long lds, hipStream_t st, const T* q, const T* kc, const T* vc, const int* bt, int bt_ld, int BSZ,
                const int* qstart, const int* qlen, const int* ctx, const int* tile_seq, const int* tile_tok0, const T* gate,
                long ldg, T* out, int H, int G, int d, int dv, int TQ, int KT, int win, int GV, float* out32, int keep,
-               float sink, int chunk, float cap, const float* sinks, long ldo) {
+               float sink, int chunk, float cap, const float* sinks, long ldo, const float* slopes, int ghead) {
   ENSURE_LDS((paged_gqa_kernel<T, NJ>), lds);
   hipLaunchKernelGGL((paged_gqa_kernel<T, NJ>), grid, dim3(256), lds, st, q, kc, vc, bt, bt_ld, BSZ, qstart, qlen, ctx, tile_seq,
-                     tile_tok0, gate, ldg, out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo);
+                     tile_tok0, gate, ldg, out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo, slopes,
+                     ghead);
   return (int)hipGetLastError();
 }
 
@@ -832,8 +859,9 @@ template <typename T>
 int launch_gqa_t(int nj, dim3 grid, long lds, hipStream_t st, const void* q, const void* kc, const void* vc, const int* bt,
                  int bt_ld, int BSZ, const int* qstart, const int* qlen, const int* ctx, const int* tile_seq,
                  const int* tile_tok0, const void* gate, long ldg, void* out, int H, int G, int d, int dv, int TQ, int KT,
-                 int win, int GV, float* out32, int keep, float sink, int chunk, float cap, const float* sinks, long ldo) {
-#define GQA(NJ) return launch_gqa<T, NJ>(grid, lds, st, (const T*)q, (const T*)kc, (const T*)vc, bt, bt_ld, BSZ, qstart, qlen, ctx, tile_seq, tile_tok0, (const T*)gate, ldg, (T*)out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo)
+                 int win, int GV, float* out32, int keep, float sink, int chunk, float cap, const float* sinks, long ldo,
+                 const float* slopes, int ghead) {
+#define GQA(NJ) return launch_gqa<T, NJ>(grid, lds, st, (const T*)q, (const T*)kc, (const T*)vc, bt, bt_ld, BSZ, qstart, qlen, ctx, tile_seq, tile_tok0, (const T*)gate, ldg, (T*)out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo, slopes, ghead)
   if (nj <= 1) GQA(1);
   if (nj <= 2) GQA(2);
   GQA(4);
@@ -873,8 +901,9 @@ extern "C" int dllm_paged_gqa(const void* q, const void* kc, const void* vc, int
                               const int* qstart, const int* qlen, const int* ctx, const int* tile_seq, const int* tile_tok0,
                               int n_tiles, const void* gate, long ldg, void* out, int H, int G, int d, int dv, int mfma,
                               int splits, float* part, int win, int GV, int out_f32, int keep, float sink, int chunk, float cap,
-                              const float* sinks, long ldo, hipStream_t st) {
+                              const float* sinks, long ldo, const float* slopes, int ghead, hipStream_t st) {
   if (n_tiles <= 0) return 0;
+  if (slopes && cap > 0.f) return -1;
   if (chunk < 0 || (chunk > 0 && win > 0) || cap < 0.f || ldo < (long)H * dv) return -1;
   if (G < 1 || H % G || dv > 256 || d < 1 || GV < 1 || G % GV || win < 0 || keep < 0 || sink < 0.f) return -1;
   if (win <= 0 && chunk <= 0) keep = 0;     // without a bound every key is seen anyway
@@ -886,24 +915,27 @@ extern "C" int dllm_paged_gqa(const void* q, const void* kc, const void* vc, int
     const dim3 grid(n_tiles, G, splits);
     const int TQ = dllm_gqa_tile_tokens(H, G, 1);
     float* pp = splits > 1 ? part : nullptr;
-#define GQM(SZ, CAP)                                                                                                     \
+#define GQM(SZ, CAP, DIST)                                                                                               \
   do {                                                                                                                   \
     const long lds = gqa_mfma_lds(SZ);                                                                                   \
-    ENSURE_LDS((paged_gqa_mfma_kernel<SZ, CAP>), lds);                                                                   \
-    hipLaunchKernelGGL((paged_gqa_mfma_kernel<SZ, CAP>), grid, dim3(256), lds, st, (const u16*)q, (const u16*)kc,        \
+    ENSURE_LDS((paged_gqa_mfma_kernel<SZ, CAP, DIST>), lds);                                                             \
+    hipLaunchKernelGGL((paged_gqa_mfma_kernel<SZ, CAP, DIST>), grid, dim3(256), lds, st, (const u16*)q, (const u16*)kc,  \
                        (const u16*)vc, bt, bt_ld, qstart, qlen, ctx, tile_seq, tile_tok0, (const u16*)gate, ldg,         \
-                       (u16*)out, H, G, d, dv, TQ, splits, pp, win, GV, out32, keep, sink, chunk, cap, sinks, ldo);      \
+                       (u16*)out, H, G, d, dv, TQ, splits, pp, win, GV, out32, keep, sink, chunk, cap, sinks, ldo,       \
+                       slopes, ghead);                                                                                   \
   } while (0)
     if (cap > 0.f && cap <= CAP_MAX) {
-      if (sz <= 64) GQM(64, true); else if (sz <= 128) GQM(128, true); else GQM(256, true);
+      if (sz <= 64) GQM(64, true, false); else if (sz <= 128) GQM(128, true, false); else GQM(256, true, false);
+    } else if (slopes) {
+      if (sz <= 64) GQM(64, false, true); else if (sz <= 128) GQM(128, false, true); else GQM(256, false, true);
     } else {
-      if (sz <= 64) GQM(64, false); else if (sz <= 128) GQM(128, false); else GQM(256, false);
+      if (sz <= 64) GQM(64, false, false); else if (sz <= 128) GQM(128, false, false); else GQM(256, false, false);
     }
 #undef GQM
     if (pp) {
       const int rows = (TQ * (H / G) < GM_ROWS ? TQ * (H / G) : GM_ROWS);
       hipLaunchKernelGGL(gqa_combine_kernel, dim3(n_tiles, G, (rows + 3) / 4), dim3(256), 0, st, pp, splits, qstart, qlen,
-                         tile_seq, tile_tok0, (const u16*)gate, ldg, (u16*)out, H, G, dv, TQ, out32, sink, sinks, ldo);
+                         tile_seq, tile_tok0, (const u16*)gate, ldg, (u16*)out, H, G, dv, TQ, out32, sink, sinks, ldo, ghead);
     }
     return (int)hipGetLastError();
   }
@@ -917,9 +949,9 @@ extern "C" int dllm_paged_gqa(const void* q, const void* kc, const void* vc, int
   const int TQ = dllm_gqa_tile_tokens(H, G, 0);
   if (f32)
     return launch_gqa_t<float>(nj, grid, lds, st, q, kc, vc, bt, bt_ld, BSZ, qstart, qlen, ctx, tile_seq, tile_tok0, gate, ldg,
-                               out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo);
+                               out, H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo, slopes, ghead);
   return launch_gqa_t<u16>(nj, grid, lds, st, q, kc, vc, bt, bt_ld, BSZ, qstart, qlen, ctx, tile_seq, tile_tok0, gate, ldg, out,
-                           H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo);
+                           H, G, d, dv, TQ, KT, win, GV, out32, keep, sink, chunk, cap, sinks, ldo, slopes, ghead);
 }
 
 extern "C" int dllm_qk_norm_prep(const void* proj, long ld, int f32, const float* bias, int H, int G, int M, int d, int dv,
@@ -970,7 +1002,8 @@ extern "C" int dllm_proj_norm_prep(const void* proj, long ld, int f32, int H, in
 
 extern "C" int dllm_rope_prep(const void* proj, long ld, int f32, int H, int G, int d, int dv, const float* cos_sin, int tab_w,
                               int rot, float qscale, const int* pos, const int* slots, void* kc, void* vc, void* q, long T,
-                              int BSZ, int ucol, int ff, void* act, long lda, void* zrow, long ldz, int zn, hipStream_t st) {
+                              int BSZ, int ucol, int ff, void* act, long lda, void* zrow, long ldz, int zn,
+                              const float* bias, const float* qtab, hipStream_t st) {
   if (T <= 0) return 0;
   if (rot < 0 || rot > d || (rot & 1) || rot > tab_w || H < 1 || G < 1 || H % G || (act && ff < 1)) return -1;
   const dim3 grid((unsigned)T, (H + G + 3) / 4);
@@ -980,9 +1013,10 @@ extern "C" int dllm_rope_prep(const void* proj, long ld, int f32, int H, int G, 
   if (f32)
     hipLaunchKernelGGL(rope_prep_kernel<float>, grid, dim3(256), 0, st, (const float*)proj, ld, H, G, d, dv, cos_sin, tab_w, rot,
                        qscale, pos, slots, (float*)kc, (float*)vc, (float*)q, BSZ, ucol, ff, (float*)act, lda, vec, (float*)zrow,
-                       ldz, zn);
+                       ldz, zn, bias, qtab);
   else
     hipLaunchKernelGGL(rope_prep_kernel<u16>, grid, dim3(256), 0, st, (const u16*)proj, ld, H, G, d, dv, cos_sin, tab_w, rot,
-                       qscale, pos, slots, (u16*)kc, (u16*)vc, (u16*)q, BSZ, ucol, ff, (u16*)act, lda, vec, (u16*)zrow, ldz, zn);
+                       qscale, pos, slots, (u16*)kc, (u16*)vc, (u16*)q, BSZ, ucol, ff, (u16*)act, lda, vec, (u16*)zrow, ldz, zn,
+                       bias, qtab);
   return (int)hipGetLastError();
 }

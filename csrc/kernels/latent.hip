@@ -6,12 +6,16 @@
 // 16-token blocks.
 //
 //   latent_kv_write   one wave per token: RMS-norm the latent (f32), rotate the shared key part
-//                     (interleaved pairs), write both into the token's cache slot
+//                     (pairs (2i, 2i + 1) or (i, i + rot / 2)), write both into the token's cache slot; a
+//                     second wave norms the query latent that the same projection made
+//   latent_q_prep     queries of the expanded form: the rotated part rotated, everything scaled
 //   latent_prep       latent_kv_write without a rotated part for a layer whose feed-forward shares the
 //                     projection: the same launch squares the relu of the up columns
 //   latent_expand     keys and values of every head from the cached latents of a step's sequences, into
-//                     pages of their own (prompt portions then run the grouped-query attention kernel)
-//   gate_heads        per-head outputs [H, T, dv] times sigmoid(gate), laid out token-major
+//                     pages of their own (prompt portions then run the grouped-query attention kernel); the
+//                     shared rotated part is copied behind every head's key
+//   gate_heads        per-head outputs [H, T, dv] times sigmoid(gate), laid out token-major; one logit per
+//                     entry or one per head
 //   latent_attention  one workgroup per 16 rows (token-major (token, head) rows of one sequence):
 //                     the rows' queries staged once in LDS as f32 (rotation and the score scale
 //                     applied while staging); keys walk in tiles staged in LDS as f32;
@@ -21,6 +25,7 @@
 //                     phase 2: a lane owns latent dims lane, lane + 64, ... and accumulates p . c.
 //                     Each wave owns 4 of the 16 rows through both phases.  Small grids (decode) split
 //                     a row's keys over several workgroups; latent_combine merges their partials.
+//                     sinks: one more term exp(sinks[head]) of the softmax denominator, without a value.
 // Activations and the cache are bf16 or f32 (template); scores, softmax and sums are f32.
 #include "common.h"
 
@@ -33,14 +38,45 @@ template <typename T> __device__ __forceinline__ void stf(T* p, float v);
 template <> __device__ __forceinline__ void stf<u16>(u16* p, float v) { *p = f2bf(v); }
 template <> __device__ __forceinline__ void stf<float>(float* p, float v) { *p = v; }
 
+// Rotary pair of the rotated part's entry c (of `rot`): its partner, its angle index, and whether it is
+// the pair's first.  hf: pairs (i, i + rot / 2), else (2i, 2i + 1).
+__device__ __forceinline__ void rot_pair(int c, int half, int hf, int& partner, int& ang, bool& first) {
+  if (hf) { first = c < half; ang = first ? c : c - half; partner = first ? c + half : c - half; }
+  else { first = !(c & 1); ang = c >> 1; partner = c ^ 1; }
+}
 template <typename T>
-__global__ void __launch_bounds__(64) latent_kv_write_kernel(const T* __restrict__ ckv, long ld, int rank, int rot,
-                                                             const float* __restrict__ w, float eps,
-                                                             const int* __restrict__ pos,
-                                                             const float* __restrict__ cos_sin, int tab_w,
-                                                             const int* __restrict__ slots, T* __restrict__ cache) {
-  const int t = blockIdx.x, lane = threadIdx.x;
+__device__ __forceinline__ float rotated(const T* r, int c, int half, int hf, const float* cs) {
+  int p, a;
+  bool first;
+  rot_pair(c, half, hf, p, a, first);
+  const float v = ldf(r + c), w = ldf(r + p);
+  return first ? v * cs[a] - w * cs[half + a] : v * cs[a] + w * cs[half + a];
+}
+
+// wave 0: the token's latent and shared key part into its cache slot.  wave 1 (launched when qsrc):
+// qdst = rmsnorm(qsrc row) qw, the query latent.  zl (optional, [zh, tokens, rank]): a padding token's
+// rows, which no attention tile writes, are cleared.
+template <typename T>
+__global__ void __launch_bounds__(128) latent_kv_write_kernel(const T* __restrict__ ckv, long ld, int rank, int rot,
+                                                              const float* __restrict__ w, float eps,
+                                                              const int* __restrict__ pos,
+                                                              const float* __restrict__ cos_sin, int tab_w,
+                                                              const int* __restrict__ slots, T* __restrict__ cache, int hf,
+                                                              const T* __restrict__ qsrc, long ldqs, int qn,
+                                                              const float* __restrict__ qw, T* __restrict__ qdst,
+                                                              T* __restrict__ zl, int zh) {
+  const int t = blockIdx.x, lane = threadIdx.x & 63;
   const int slot = slots[t];
+  if (zl && slot < 0)
+    for (int i = threadIdx.x; i < zh * rank; i += blockDim.x) stf(zl + ((long)(i / rank) * gridDim.x + t) * rank + i % rank, 0.f);
+  if (threadIdx.x >= 64) {
+    const T* r = qsrc + (long)t * ldqs;
+    float s = 0.f;
+    for (int i = lane; i < qn; i += 64) { const float v = ldf(r + i); s += v * v; }
+    const float rs = 1.f / sqrtf(wave_sum(s) / (float)qn + eps);
+    for (int i = lane; i < qn; i += 64) stf(qdst + (long)t * qn + i, ldf(r + i) * rs * qw[i]);
+    return;
+  }
   if (slot < 0) return;
   const T* r = ckv + (long)t * ld;
   float s = 0.f;
@@ -51,11 +87,22 @@ __global__ void __launch_bounds__(64) latent_kv_write_kernel(const T* __restrict
   for (int i = lane; i < rank; i += 64) stf(dst + i, ldf(r + i) * rs * w[i]);
   const float* cs = cos_sin + (long)pos[t] * tab_w;
   const int half = rot >> 1;
-  for (int i = lane; i < half; i += 64) {
-    const float u = ldf(r + rank + 2 * i), v = ldf(r + rank + 2 * i + 1);
-    const float c = cs[i], sn = cs[half + i];
-    stf(dst + rank + 2 * i, u * c - v * sn);
-    stf(dst + rank + 2 * i + 1, v * c + u * sn);
+  for (int i = lane; i < rot; i += 64) stf(dst + rank + i, rotated(r + rank, i, half, hf, cs));
+}
+
+// out[t, h, :] = [q_h | rotated part] * scale for queries q [T, H (dim + rot)]; x over the columns, y over
+// the tokens
+template <typename T>
+__global__ void __launch_bounds__(256) latent_q_prep_kernel(const T* __restrict__ q, long ldq, int H, int dim, int rot, int hf,
+                                                            const int* __restrict__ pos, const float* __restrict__ cos_sin,
+                                                            int tab_w, float scale, T* __restrict__ out, long Tn) {
+  const int c = blockIdx.x * 256 + threadIdx.x, w = dim + rot;
+  if (c >= H * w) return;
+  const int h = c / w, i = c - h * w, half = rot >> 1;
+  for (long t = blockIdx.y; t < Tn; t += gridDim.y) {
+    const T* r = q + t * ldq + (long)h * w;
+    const float v = i < dim ? ldf(r + i) : rotated(r + dim, i - dim, half, hf, cos_sin + (long)pos[t] * tab_w);
+    stf(out + t * (long)(H * w) + c, v * scale);
   }
 }
 
@@ -113,27 +160,36 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(const T* __restrict__ 
 // owns groups of NB 16-column blocks, first the key columns', then the value columns', over all 64 latents.
 // Operands of v_mfma_f32_16x16x32_bf16 hold rows of either matrix alike (row lane & 15, contraction
 // 8 (lane >> 4) ..), so keys are made as W C^T (four key dims of a latent per lane) and values as C W^T (four
-// latents of a value dim per lane): both leave as 8-byte vectors.  Output pages: K [S nb, H, 16, d], V
+// latents of a value dim per lane): both leave as 8-byte vectors.  Cache rows are [latent | rot rotated
+// dims]; output pages: K [S nb, H, 16, d + rot] (the rotated dims copied behind every head's key), V
 // [S nb, H, dv, 16], page (s, j) at s nb + j.
 template <int NB>
 __global__ void __launch_bounds__(256) latent_expand_kernel(const u16* __restrict__ cache, const int* __restrict__ bt, int bt_ld,
                                                             int nb, int pages, const int* __restrict__ ctx, int rank, int H,
                                                             int d, int dv, const u16* __restrict__ wk,
                                                             const u16* __restrict__ wv, u16* __restrict__ kc,
-                                                            u16* __restrict__ vc) {
+                                                            u16* __restrict__ vc, int rot) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smx[];
   u16* csh = reinterpret_cast<u16*>(smx);      // [64][rank + 8]
   const int s = blockIdx.z, h = blockIdx.y, j0 = blockIdx.x * 4;
   if (j0 * 16 >= ctx[s]) return;               // nothing of the sequence lies here (uniform)
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int lr = lane & 15, g4 = lane >> 4;
-  const int str = rank + 8, ch = rank >> 3;
+  const int str = rank + 8, ch = rank >> 3, Dp = rank + rot, kd = d + rot;
+  for (int e = tid; e < 64 * (rot >> 3); e += 256) {      // the shared rotated part (rot % 8 == 0)
+    const int t = e / (rot >> 3), c = 8 * (e - t * (rot >> 3)), j = j0 + (t >> 4);
+    if (j >= nb) continue;
+    const int pg = bt[(long)s * bt_ld + j];
+    uint4 v = make_uint4(0u, 0u, 0u, 0u);
+    if (pg >= 0 && pg < pages) v = ld16(cache + ((long)pg * 16 + (t & 15)) * Dp + rank + c);
+    st16(kc + ((((long)s * nb + j) * H + h) * 16 + (t & 15)) * kd + d + c, v);
+  }
   for (int e = tid; e < 64 * ch; e += 256) {
     const int t = e / ch, c = e - t * ch, j = j0 + (t >> 4);
     uint4 v = make_uint4(0u, 0u, 0u, 0u);
     if (j < nb) {
       const int pg = bt[(long)s * bt_ld + j];
-      if (pg >= 0 && pg < pages) v = ld16(cache + ((long)pg * 16 + (t & 15)) * rank + 8 * c);
+      if (pg >= 0 && pg < pages) v = ld16(cache + ((long)pg * 16 + (t & 15)) * Dp + 8 * c);
     }
     st16(csh + t * str + 8 * c, v);
   }
@@ -190,7 +246,7 @@ __global__ void __launch_bounds__(256) latent_expand_kernel(const u16* __restric
         const uint2 v = make_uint2((uint32_t)f2bf(a[0]) | ((uint32_t)f2bf(a[1]) << 16), (uint32_t)f2bf(a[2]) | ((uint32_t)f2bf(a[3]) << 16));
         const int c0 = (b0 + b) * 16;
         if (key) {
-          if (c0 + 4 * g4 < d) *reinterpret_cast<uint2*>(kc + (page * 16 + lr) * d + c0 + 4 * g4) = v;
+          if (c0 + 4 * g4 < d) *reinterpret_cast<uint2*>(kc + (page * 16 + lr) * kd + c0 + 4 * g4) = v;
         } else {
           if (c0 + lr < dv) *reinterpret_cast<uint2*>(vc + (page * dv + c0 + lr) * 16 + 4 * g4) = v;
         }
@@ -199,15 +255,16 @@ __global__ void __launch_bounds__(256) latent_expand_kernel(const u16* __restric
   }
 }
 
-// out[t, h dv + i] = o[h, t, i] sigmoid(gate[t, h dv + i]): x over the columns, y over the tokens
+// out[t, h dv + i] = o[h, t, i] sigmoid(gate[t, h dv + i]), or gate[t, h] with `ghead`: x over the columns,
+// y over the tokens
 template <typename T>
 __global__ void __launch_bounds__(256) gate_heads_kernel(const T* __restrict__ o, const T* __restrict__ gate, long ldg,
-                                                         T* __restrict__ out, long ldo, int H, int dv, long Tn) {
+                                                         T* __restrict__ out, long ldo, int H, int dv, long Tn, int ghead) {
   const int c = blockIdx.x * 256 + threadIdx.x;
   if (c >= H * dv) return;
   const int h = c / dv, i = c - h * dv;
   for (long t = blockIdx.y; t < Tn; t += gridDim.y)
-    stf(out + t * ldo + c, ldf(o + ((long)h * Tn + t) * dv + i) / (1.f + expf(-ldf(gate + t * ldg + c))));
+    stf(out + t * ldo + c, ldf(o + ((long)h * Tn + t) * dv + i) / (1.f + expf(-ldf(gate + t * ldg + (ghead ? h : c)))));
 }
 
 constexpr int LROWS = 16;
@@ -236,7 +293,8 @@ __global__ void __launch_bounds__(256) latent_attention_kernel(
     const float* __restrict__ cos_sin, int tab_w, const T* __restrict__ cache, const int* __restrict__ bt, int bt_w,
     const int* __restrict__ qstart, const int* __restrict__ qlen, const int* __restrict__ ctx,
     const int* __restrict__ tile_seq, const int* __restrict__ tile_tok0, float scale, T* __restrict__ out, int KT,
-    int tpe, int kstride, int vec, int splits, float* __restrict__ part_o, float* __restrict__ part_ml) {
+    int tpe, int kstride, int vec, int splits, float* __restrict__ part_o, float* __restrict__ part_ml, int hf,
+    const float* __restrict__ sinks) {
   extern __shared__ float sm[];
   const int entry = blockIdx.y;
   const int s = tile_seq[entry];
@@ -265,11 +323,7 @@ __global__ void __launch_bounds__(256) latent_attention_kernel(
       if (c < rank) {
         v = ldf(qa + ((long)h * Ttot + tok) * rank + c);
       } else {
-        const int i = (c - rank) >> 1;
-        const T* qr = q + tok * ldq + (long)h * (dim + rot) + dim + 2 * i;
-        const float u = ldf(qr), w = ldf(qr + 1);
-        const float* cs = cos_sin + (long)(p0 + tl) * tab_w;
-        v = ((c - rank) & 1) ? w * cs[i] + u * cs[half + i] : u * cs[i] - w * cs[half + i];
+        v = rotated(q + tok * ldq + (long)h * (dim + rot) + dim, c - rank, half, hf, cos_sin + (long)(p0 + tl) * tab_w);
       }
       v *= scale;
     }
@@ -393,7 +447,7 @@ __global__ void __launch_bounds__(256) latent_attention_kernel(
     if (row >= nrows) continue;
     const long tok = q0 + tok0 + row / H;
     const int h = row % H;
-    const float inv = l[a] > 0.f ? 1.f / l[a] : 0.f;
+    const float inv = l[a] > 0.f ? 1.f / (l[a] + (sinks ? expf(sinks[h] - m[a]) : 0.f)) : 0.f;
 #pragma unroll
     for (int i = 0; i < RI; ++i) {
       const int c = lane + 64 * i;
@@ -476,7 +530,7 @@ __global__ void __launch_bounds__(256) latent_attention_mfma_kernel(
     const int* __restrict__ qstart, const int* __restrict__ qlen, const int* __restrict__ ctx,
     const int* __restrict__ tile_seq, const int* __restrict__ tile_tok0, float scale, u16* __restrict__ out,
     int tpe, int splits, float* __restrict__ part_o, float* __restrict__ part_ml, int Dpad, int qstr, int ktstr,
-    int pstr, int RB) {
+    int pstr, int RB, int hf, const float* __restrict__ sinks) {
   constexpr int RPB = 16 * LR;                      // rows per workgroup
   constexpr int NKB = KT >> 4;                      // 16-key blocks per tile
   constexpr int NT = (LR * NKB + 3) / 4;            // score tasks per wave
@@ -520,11 +574,7 @@ __global__ void __launch_bounds__(256) latent_attention_mfma_kernel(
       if (c < rank) {
         v = bf2f(qa[((long)h * Ttot + tok) * rank + c]);
       } else {
-        const int i = (c - rank) >> 1;
-        const u16* qr = q + tok * ldq + (long)h * (dim + rot) + dim + 2 * i;
-        const float u = bf2f(qr[0]), w = bf2f(qr[1]);
-        const float* cs = cos_sin + (long)(p0 + tl) * tab_w;
-        v = ((c - rank) & 1) ? w * cs[i] + u * cs[half + i] : u * cs[i] - w * cs[half + i];
+        v = rotated(q + tok * ldq + (long)h * (dim + rot) + dim, c - rank, half, hf, cos_sin + (long)(p0 + tl) * tab_w);
       }
     }
     qsh[rr * qstr + c] = f2bf(v);
@@ -738,7 +788,7 @@ __global__ void __launch_bounds__(256) latent_attention_mfma_kernel(
         if (row < nrows) {
           const long tok = q0 + tok0 + row / H;
           const int h = row % H;
-          const float inv = lt > 0.f ? 1.f / lt : 0.f;
+          const float inv = lt > 0.f ? 1.f / (lt + (sinks ? expf(sinks[h] - m[b][i]) : 0.f)) : 0.f;
 #pragma unroll
           for (int j = 0; j < CB; ++j) {
             const int c = (wave + 4 * j) * 16 + lr;
@@ -758,7 +808,8 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __rest
                                                              int H, int rank, long Ttot, const int* __restrict__ qstart,
                                                              const int* __restrict__ qlen, const int* __restrict__ tile_seq,
                                                              const int* __restrict__ tile_tok0, int tpe,
-                                                             T* __restrict__ out, int rpb) {
+                                                             T* __restrict__ out, int rpb,
+                                                             const float* __restrict__ sinks) {
   const long r = blockIdx.x;
   const int tid = threadIdx.x, lane = tid & 63;
   const int rl = (int)(r % rpb);
@@ -773,7 +824,8 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __rest
   const float mz = lane < splits ? ml[2 * lane] : -INFINITY, lz = lane < splits ? ml[2 * lane + 1] : 0.f;
   const float M = wave_max(mz);
   const float ez = mz > -INFINITY ? expf(mz - M) : 0.f;
-  const float L = wave_sum(lz * ez);
+  float L = wave_sum(lz * ez);
+  if (sinks && L > 0.f) L += expf(sinks[row % H] - M);
   const float wz = L > 0.f ? ez / L : 0.f;
   const long tok = qstart[s] + tok0 + row / H;
   const int h = row % H;
@@ -795,15 +847,31 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __rest
 
 extern "C" int dllm_latent_kv_write(const void* ckv, long ld, int f32, int rank, int rot, const float* w, float eps,
                                     const int* pos, const float* cos_sin, int tab_w, const int* slots, void* cache,
-                                    int T, hipStream_t st) {
+                                    int T, int hf, const void* qsrc, long ldqs, int qn, const float* qw, void* qdst, void* zl,
+                                    int zh, hipStream_t st) {
   if (T <= 0) return 0;
-  if (rot < 0 || (rot & 1) || rot > tab_w || rank < 1) return -1;
+  if (rot < 0 || (rot & 1) || rot > tab_w || rank < 1 || (qsrc && (qn < 1 || !qw || !qdst))) return -1;
+  const dim3 block(qsrc ? 128 : 64);
   if (f32)
-    hipLaunchKernelGGL(latent_kv_write_kernel<float>, dim3(T), dim3(64), 0, st, (const float*)ckv, ld, rank, rot, w, eps, pos,
-                       cos_sin, tab_w, slots, (float*)cache);
+    hipLaunchKernelGGL(latent_kv_write_kernel<float>, dim3(T), block, 0, st, (const float*)ckv, ld, rank, rot, w, eps, pos,
+                       cos_sin, tab_w, slots, (float*)cache, hf, (const float*)qsrc, ldqs, qn, qw, (float*)qdst, (float*)zl, zh);
   else
-    hipLaunchKernelGGL(latent_kv_write_kernel<u16>, dim3(T), dim3(64), 0, st, (const u16*)ckv, ld, rank, rot, w, eps, pos,
-                       cos_sin, tab_w, slots, (u16*)cache);
+    hipLaunchKernelGGL(latent_kv_write_kernel<u16>, dim3(T), block, 0, st, (const u16*)ckv, ld, rank, rot, w, eps, pos,
+                       cos_sin, tab_w, slots, (u16*)cache, hf, (const u16*)qsrc, ldqs, qn, qw, (u16*)qdst, (u16*)zl, zh);
+  return (int)hipGetLastError();
+}
+
+extern "C" int dllm_latent_q_prep(const void* q, long ldq, int f32, int H, int dim, int rot, int hf, const int* pos,
+                                  const float* cos_sin, int tab_w, float scale, void* out, long T, hipStream_t st) {
+  if (T <= 0) return 0;
+  if (H < 1 || dim < 0 || rot < 0 || (rot & 1) || rot > tab_w || dim + rot < 1) return -1;
+  const dim3 grid((H * (dim + rot) + 255) / 256, (unsigned)(T < 4096 ? T : 4096));
+  if (f32)
+    hipLaunchKernelGGL(latent_q_prep_kernel<float>, grid, dim3(256), 0, st, (const float*)q, ldq, H, dim, rot, hf, pos, cos_sin,
+                       tab_w, scale, (float*)out, T);
+  else
+    hipLaunchKernelGGL(latent_q_prep_kernel<u16>, grid, dim3(256), 0, st, (const u16*)q, ldq, H, dim, rot, hf, pos, cos_sin,
+                       tab_w, scale, (u16*)out, T);
   return (int)hipGetLastError();
 }
 
@@ -812,7 +880,8 @@ template <typename T>
 int launch_latent(int ri, dim3 g, long lds, hipStream_t st, const T* qa, const T* q, long ldq, int H, int dim, int rot,
                   int rank, long Ttot, const float* cos_sin, int tab_w, const T* cache, const int* bt, int bt_w,
                   const int* qstart, const int* qlen, const int* ctx, const int* tile_seq, const int* tile_tok0,
-                  float scale, T* out, int KT, int tpe, int kstride, int vec, int splits, float* part_o, float* part_ml) {
+                  float scale, T* out, int KT, int tpe, int kstride, int vec, int splits, float* part_o, float* part_ml, int hf,
+                  const float* sinks) {
 #define LAT(RI)                                                                                                        \
   do {                                                                                                                 \
     static long have_ = 48 * 1024; /* raised once per size: no attribute call inside a later stream capture */        \
@@ -823,14 +892,14 @@ int launch_latent(int ri, dim3 g, long lds, hipStream_t st, const T* qa, const T
     }                                                                                                                  \
     hipLaunchKernelGGL((latent_attention_kernel<T, RI>), g, dim3(256), lds, st, qa, q, ldq, H, dim, rot, rank, Ttot,   \
                        cos_sin, tab_w, cache, bt, bt_w, qstart, qlen, ctx, tile_seq, tile_tok0, scale, out, KT, tpe,   \
-                       kstride, vec, splits, part_o, part_ml);                                                         \
+                       kstride, vec, splits, part_o, part_ml, hf, sinks);                                              \
   } while (0)
   if (ri <= 1) LAT(1); else if (ri <= 2) LAT(2); else if (ri <= 4) LAT(4); else LAT(8);
 #undef LAT
   if (splits > 1) {
     const long n_rows = (long)g.y * g.x * LROWS;
     hipLaunchKernelGGL(latent_combine_kernel<T>, dim3((unsigned)n_rows), dim3(256), 0, st, part_o, part_ml, splits, (int)g.x, H,
-                       rank, Ttot, qstart, qlen, tile_seq, tile_tok0, tpe, out, LROWS);
+                       rank, Ttot, qstart, qlen, tile_seq, tile_tok0, tpe, out, LROWS, sinks);
   }
   return (int)hipGetLastError();
 }
@@ -840,7 +909,8 @@ namespace {
 int launch_latent_mfma(dim3 g, hipStream_t st, const u16* qa, const u16* q, long ldq, int H, int dim, int rot, int rank,
                        long Ttot, const float* cos_sin, int tab_w, const u16* cache, const int* bt, int bt_w,
                        const int* qstart, const int* qlen, const int* ctx, const int* tile_seq, const int* tile_tok0,
-                       float scale, u16* out, int KT, int tpe, int splits, float* part_o, float* part_ml, int rows) {
+                       float scale, u16* out, int KT, int tpe, int splits, float* part_o, float* part_ml, int rows, int hf,
+                       const float* sinks) {
   const MfmaLds L = mfma_lds(rank, rot, KT, rows);
   const int cbs = (L.RB + 3) / 4;
 #define LATM3(CB, KTC, LRC)                                                                                                 \
@@ -853,7 +923,7 @@ int launch_latent_mfma(dim3 g, hipStream_t st, const u16* qa, const u16* q, long
     }                                                                                                                  \
     hipLaunchKernelGGL((latent_attention_mfma_kernel<CB, KTC, LRC>), g, dim3(256), L.bytes, st, qa, q, ldq, H, dim, rot, \
                        rank, Ttot, cos_sin, tab_w, cache, bt, bt_w, qstart, qlen, ctx, tile_seq, tile_tok0, scale, out, \
-                       tpe, splits, part_o, part_ml, L.Dpad, L.qstr, L.ktstr, L.pstr, L.RB);                           \
+                       tpe, splits, part_o, part_ml, L.Dpad, L.qstr, L.ktstr, L.pstr, L.RB, hf, sinks);                \
   } while (0)
 #define LATM2(CB, KTC)                                                                                                 \
   do {                                                                                                                 \
@@ -870,7 +940,7 @@ int launch_latent_mfma(dim3 g, hipStream_t st, const u16* qa, const u16* q, long
   if (splits > 1) {
     const long n_rows = (long)g.y * g.x * rows;
     hipLaunchKernelGGL(latent_combine_kernel<u16>, dim3((unsigned)n_rows), dim3(256), 0, st, part_o, part_ml, splits, (int)g.x, H,
-                       rank, Ttot, qstart, qlen, tile_seq, tile_tok0, tpe, out, rows);
+                       rank, Ttot, qstart, qlen, tile_seq, tile_tok0, tpe, out, rows, sinks);
   }
   return (int)hipGetLastError();
 }
@@ -887,7 +957,8 @@ extern "C" int dllm_latent_attention(const void* qa, const void* q, long ldq, in
                                      long Ttot, const float* cos_sin, int tab_w, const void* cache, const int* bt,
                                      int bt_w, const int* qstart, const int* qlen, const int* ctx, const int* tile_seq,
                                      const int* tile_tok0, int n_entries, float scale, void* out, int splits,
-                                     float* part_o, float* part_ml, int mfma, int rows, hipStream_t st) {
+                                     float* part_o, float* part_ml, int mfma, int rows, int hf, const float* sinks,
+                                     hipStream_t st) {
   if (n_entries <= 0 || Ttot <= 0) return 0;
   if (rank < 1 || rank > 512 || rot < 0 || (rot & 1) || rot > tab_w || H < 1) return -1;
   if (splits < 1 || (splits > 1 && (!part_o || !part_ml))) return -3;
@@ -897,7 +968,7 @@ extern "C" int dllm_latent_attention(const void* qa, const void* q, long ldq, in
     const dim3 gm((tpe_m * H + rows - 1) / rows, n_entries, splits);
     return launch_latent_mfma(gm, st, (const u16*)qa, (const u16*)q, ldq, H, dim, rot, rank, Ttot, cos_sin, tab_w,
                               (const u16*)cache, bt, bt_w, qstart, qlen, ctx, tile_seq, tile_tok0, scale, (u16*)out, KTm,
-                              tpe_m, splits, part_o, part_ml, rows);
+                              tpe_m, splits, part_o, part_ml, rows, hf, sinks);
   }
   if (rows != LROWS) return -4;   // only the matrix-core kernel has the 32-row form
   // key rows in LDS: an odd stride for 4-byte reads; when the row length is a multiple of 4 a stride
@@ -915,9 +986,10 @@ extern "C" int dllm_latent_attention(const void* qa, const void* q, long ldq, in
   if (f32)
     return launch_latent<float>(ri, g, lds, st, (const float*)qa, (const float*)q, ldq, H, dim, rot, rank, Ttot, cos_sin,
                                 tab_w, (const float*)cache, bt, bt_w, qstart, qlen, ctx, tile_seq, tile_tok0, scale,
-                                (float*)out, KT, tpe, kstride, vec, splits, part_o, part_ml);
+                                (float*)out, KT, tpe, kstride, vec, splits, part_o, part_ml, hf, sinks);
   return launch_latent<u16>(ri, g, lds, st, (const u16*)qa, (const u16*)q, ldq, H, dim, rot, rank, Ttot, cos_sin, tab_w,
-                            (const u16*)cache, bt, bt_w, qstart, qlen, ctx, tile_seq, tile_tok0, scale, (u16*)out, KT, tpe, kstride, vec, splits, part_o, part_ml);
+                            (const u16*)cache, bt, bt_w, qstart, qlen, ctx, tile_seq, tile_tok0, scale, (u16*)out, KT, tpe, kstride, vec, splits, part_o, part_ml, hf,
+                            sinks);
 }
 
 extern "C" int dllm_latent_prep(const void* proj, long ld, int f32, int ccol, int rank, const float* w, float eps,
@@ -938,28 +1010,29 @@ extern "C" int dllm_latent_prep(const void* proj, long ld, int f32, int ccol, in
 }
 
 extern "C" int dllm_gate_heads(const void* o, int f32, const void* gate, long ldg, void* out, long ldo, int H, int dv, long T,
-                               hipStream_t st) {
+                               int ghead, hipStream_t st) {
   if (T <= 0) return 0;
   if (H < 1 || dv < 1) return -1;
   const dim3 grid((H * dv + 255) / 256, (unsigned)(T < 4096 ? T : 4096));
   if (f32)
     hipLaunchKernelGGL(gate_heads_kernel<float>, grid, dim3(256), 0, st, (const float*)o, (const float*)gate, ldg, (float*)out,
-                       ldo, H, dv, T);
+                       ldo, H, dv, T, ghead);
   else
     hipLaunchKernelGGL(gate_heads_kernel<u16>, grid, dim3(256), 0, st, (const u16*)o, (const u16*)gate, ldg, (u16*)out, ldo, H,
-                       dv, T);
+                       dv, T, ghead);
   return (int)hipGetLastError();
 }
 
 // 1 when latent_expand takes the shape (bf16; the 64 latents of a workgroup fit the LDS)
-extern "C" int dllm_latent_expand_ok(int rank, int d, int dv) {
-  return rank >= 32 && rank % 32 == 0 && rank <= 1024 && d >= 8 && d % 8 == 0 && dv >= 1;
+extern "C" int dllm_latent_expand_ok(int rank, int d, int dv, int rot) {
+  return rank >= 32 && rank % 32 == 0 && rank <= 1024 && d >= 8 && d % 8 == 0 && dv >= 1 && rot >= 0 && rot % 8 == 0;
 }
 
 extern "C" int dllm_latent_expand(const void* cache, const int* bt, int bt_ld, int S, int nb, int pages, const int* ctx, int rank,
-                                  int H, int d, int dv, const void* wk, const void* wv, void* kc, void* vc, hipStream_t st) {
+                                  int H, int d, int dv, const void* wk, const void* wv, void* kc, void* vc, int rot,
+                                  hipStream_t st) {
   if (S <= 0 || nb <= 0) return 0;
-  if (!dllm_latent_expand_ok(rank, d, dv) || H < 1 || S > 65535 || H > 65535) return -1;
+  if (!dllm_latent_expand_ok(rank, d, dv, rot) || H < 1 || S > 65535 || H > 65535) return -1;
   const long lds = 64L * (rank + 8) * 2;
   const dim3 grid((nb + 3) / 4, H, S);
 #define LEX(NB)                                                                                                        \
@@ -970,7 +1043,7 @@ extern "C" int dllm_latent_expand(const void* cache, const int* bt, int bt_ld, i
       have_ = lds;                                                                                                     \
     }                                                                                                                  \
     hipLaunchKernelGGL(latent_expand_kernel<NB>, grid, dim3(256), lds, st, (const u16*)cache, bt, bt_ld, nb, pages, ctx, rank, H, \
-                       d, dv, (const u16*)wk, (const u16*)wv, (u16*)kc, (u16*)vc);                                     \
+                       d, dv, (const u16*)wk, (const u16*)wv, (u16*)kc, (u16*)vc, rot);                                \
   } while (0)
   if (d >= 128 && dv >= 128) LEX(4); else if (d >= 64 || dv >= 64) LEX(2); else LEX(1);
 #undef LEX

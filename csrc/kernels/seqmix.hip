@@ -105,13 +105,15 @@ __global__ void __launch_bounds__(256) norm_resadd_kernel(const T* __restrict__ 
 //   y = a                                        (one branch)
 //   y = (rmsnorm(a) wa + rmsnorm(b) wb) / 2      (two mixers side by side)
 //   x += rmsnorm(y) w_post;  xn = rmsnorm(x) w_next  (xn = x rounded when w_next is null)
+// bias: added to y before its norm (the sublayer's output bias).
 template <typename T>
 __global__ void __launch_bounds__(256) resadd_norm_kernel(const T* __restrict__ a, long lda, const T* __restrict__ b,
                                                           long ldb, const float* __restrict__ wa,
                                                           const float* __restrict__ wb, const float* __restrict__ w_post,
                                                           float* __restrict__ x, const float* __restrict__ w_next,
                                                           T* __restrict__ xn, int H, float eps,
-                                                          const float* __restrict__ dw, int dn, long TH) {
+                                                          const float* __restrict__ dw, int dn, long TH,
+                                                          const float* __restrict__ bias) {
   __shared__ float red[16];
   extern __shared__ float yb[];   // [H]; entry i is touched by thread i % 256 only
   const long row = blockIdx.x;
@@ -132,6 +134,7 @@ __global__ void __launch_bounds__(256) resadd_norm_kernel(const T* __restrict__ 
   for (int i = threadIdx.x; i < H; i += 256) {
     float y = ldf(ar + i);
     if (br) y = 0.5f * (y * ra * wa[i] + ldf(br + i) * rb * wb[i]);
+    if (bias) y += bias[i];
     yb[i] = y;
     sy += y * y;
   }
@@ -158,6 +161,75 @@ __global__ void __launch_bounds__(256) resadd_norm_kernel(const T* __restrict__ 
   float rx = 1.f;
   if (w_next) rx = 1.f / sqrtf(block_sum(sx, red) / (float)H + eps);
   for (int i = threadIdx.x; i < H; i += 256) stf(xn + row * (long)H + i, w_next ? yb[i] * rx * w_next[i] : yb[i]);
+}
+
+// 4-entry vectors of activations (bf16 or f32) as float4
+template <typename T> struct vec4;
+template <> struct vec4<float> {
+  static __device__ __forceinline__ float4 ld(const float* p) { return *reinterpret_cast<const float4*>(p); }
+  static __device__ __forceinline__ void st(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
+};
+template <> struct vec4<u16> {
+  static __device__ __forceinline__ float4 ld(const u16* p) {
+    const uint2 w = *reinterpret_cast<const uint2*>(p);
+    return make_float4(__uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u), __uint_as_float(w.y << 16),
+                       __uint_as_float(w.y & 0xffff0000u));
+  }
+  static __device__ __forceinline__ void st(u16* p, float4 v) {
+    *reinterpret_cast<uint2*>(p) = make_uint2((uint32_t)f2bf(v.x) | ((uint32_t)f2bf(v.y) << 16),
+                                              (uint32_t)f2bf(v.z) | ((uint32_t)f2bf(v.w) << 16));
+  }
+};
+
+// resadd_norm of one branch without a sum over depth, for rows of whole 4-entry vectors, NV vectors a
+// thread: the row stays in registers.
+template <typename T, int NV>
+__global__ void __launch_bounds__(256) resadd_norm_vec_kernel(const T* __restrict__ a, long lda, const float* __restrict__ w_post,
+                                                              float* __restrict__ x, const float* __restrict__ w_next,
+                                                              T* __restrict__ xn, int H, float eps,
+                                                              const float* __restrict__ bias) {
+  __shared__ float red[16];
+  const long row = blockIdx.x;
+  float* xr = x + row * (long)H;
+  float4 y[NV], v[NV];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = 4 * (j * 256 + (int)threadIdx.x);
+    y[j] = v[j] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (c < H) {
+      y[j] = vec4<T>::ld(a + row * lda + c);
+      v[j] = *reinterpret_cast<const float4*>(xr + c);     // in flight under the first sum
+      if (bias) {
+        const float4 b = *reinterpret_cast<const float4*>(bias + c);
+        y[j].x += b.x; y[j].y += b.y; y[j].z += b.z; y[j].w += b.w;
+      }
+    }
+    ss += y[j].x * y[j].x + y[j].y * y[j].y + y[j].z * y[j].z + y[j].w * y[j].w;
+  }
+  const float ry = 1.f / sqrtf(block_sum(ss, red) / (float)H + eps);
+  ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = 4 * (j * 256 + (int)threadIdx.x);
+    if (c < H) {
+      const float4 g = *reinterpret_cast<const float4*>(w_post + c);
+      v[j].x += y[j].x * ry * g.x; v[j].y += y[j].y * ry * g.y; v[j].z += y[j].z * ry * g.z; v[j].w += y[j].w * ry * g.w;
+      *reinterpret_cast<float4*>(xr + c) = v[j];
+      if (xn && !w_next) vec4<T>::st(xn + row * (long)H + c, v[j]);
+    }
+    ss += v[j].x * v[j].x + v[j].y * v[j].y + v[j].z * v[j].z + v[j].w * v[j].w;
+  }
+  if (!xn || !w_next) return;   // uniform
+  const float rx = 1.f / sqrtf(block_sum(ss, red) / (float)H + eps);
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = 4 * (j * 256 + (int)threadIdx.x);
+    if (c < H) {
+      const float4 g = *reinterpret_cast<const float4*>(w_next + c);
+      vec4<T>::st(xn + row * (long)H + c, make_float4(v[j].x * rx * g.x, v[j].y * rx * g.y, v[j].z * rx * g.z, v[j].w * rx * g.w));
+    }
+  }
 }
 
 // X[n] = sum_{j<n} w[j] X[j] for one token per workgroup (X [slots][T][H] f32), xn = rmsnorm(X[n]) w_next
@@ -971,22 +1043,6 @@ __global__ void __launch_bounds__(256) scaled_resadd_rms_kernel(const T* __restr
 }
 
 // The same for rows of whole 4-entry vectors, NV vectors a thread: the row stays in registers.
-template <typename T> struct vec4;
-template <> struct vec4<float> {
-  static __device__ __forceinline__ float4 ld(const float* p) { return *reinterpret_cast<const float4*>(p); }
-  static __device__ __forceinline__ void st(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
-};
-template <> struct vec4<u16> {
-  static __device__ __forceinline__ float4 ld(const u16* p) {
-    const uint2 w = *reinterpret_cast<const uint2*>(p);
-    return make_float4(__uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u), __uint_as_float(w.y << 16),
-                       __uint_as_float(w.y & 0xffff0000u));
-  }
-  static __device__ __forceinline__ void st(u16* p, float4 v) {
-    *reinterpret_cast<uint2*>(p) = make_uint2((uint32_t)f2bf(v.x) | ((uint32_t)f2bf(v.y) << 16),
-                                              (uint32_t)f2bf(v.z) | ((uint32_t)f2bf(v.w) << 16));
-  }
-};
 template <typename T, int NV>
 __global__ void __launch_bounds__(256) scaled_resadd_rms_vec_kernel(const T* __restrict__ y, long ldy, float mult, int set,
                                                                     const float* __restrict__ vec, float* __restrict__ x,
@@ -1034,7 +1090,8 @@ __global__ void __launch_bounds__(256) scaled_resadd_rms_vec_kernel(const T* __r
 }
 
 // gu [rows, 2 ff] (gate columns, then up columns) + bias -> y [rows, ff].  mode 0: silu(g) u;
-// mode 1: g <- min(g, limit), u <- clamp(u, -limit, limit), y = g sigmoid(alpha g) (u + 1)
+// mode 1: g <- min(g, limit), u <- clamp(u, -limit, limit), y = g sigmoid(alpha g) (u + 1);
+// mode 2: gelu(g) u in the tanh form, 0.5 g (1 + tanh(z)) = g sigmoid(2 z), z = sqrt(2 / pi) (g + 0.044715 g^3)
 template <typename T>
 __global__ void __launch_bounds__(256) glu_act_kernel(const T* __restrict__ gu, long ld, const float* __restrict__ bias,
                                                       int ff, int mode, float limit, float alpha, T* __restrict__ y,
@@ -1047,10 +1104,12 @@ __global__ void __launch_bounds__(256) glu_act_kernel(const T* __restrict__ gu, 
   for (long r = blockIdx.y; r < rows; r += gridDim.y) {
     float g = ldf(gu + r * ld + c) + bg, u = ldf(gu + r * ld + ff + c) + bu;
     float a = 1.f;
-    if (mode != 0) {
+    if (mode == 1) {
       g = fminf(g, limit);
       u = fminf(fmaxf(u, -limit), limit) + 1.f;
       a = alpha;
+    } else if (mode == 2) {
+      a = 1.5957691216057308f * (1.f + 0.044715f * g * g);
     }
     // the result is rounded to bf16 in bf16 models: the hardware exponential and reciprocal are exact enough there
     const float den = 1.f + fastexp<T>::f(-a * g);
@@ -1104,18 +1163,31 @@ extern "C" int dllm_norm_resadd(const void* y, long ldy, int f32, const float* w
 // sum over j < dn of dw[j] * slot j, and norms that for xn
 extern "C" int dllm_resadd_norm(const void* a, long lda, const void* b, long ldb, int f32, const float* wa, const float* wb,
                                 const float* w_post, float* x, const float* w_next, void* xn, int rows, int H, float eps,
-                                const float* dw, int dn, hipStream_t st) {
+                                const float* dw, int dn, const float* bias, hipStream_t st) {
   if (rows <= 0) return rows == 0 ? 0 : -1;
   const long lds = 4L * H;
   if (lds > 150 * 1024) return -2;
+  const long ab = f32 ? 16 : 8;     // bytes of a vector of activations
+  if (!b && !dw && H % 4 == 0 && H <= 8192 && lda % 4 == 0 && (uintptr_t)a % ab == 0 && (uintptr_t)x % 16 == 0 &&
+      (uintptr_t)w_post % 16 == 0 && (!xn || (uintptr_t)xn % ab == 0) && (!w_next || (uintptr_t)w_next % 16 == 0) &&
+      (!bias || (uintptr_t)bias % 16 == 0)) {
+    const int nv = (H + 1023) / 1024;
+#define RN(T, NV)                                                                                                          \
+  hipLaunchKernelGGL((resadd_norm_vec_kernel<T, NV>), dim3(rows), dim3(256), 0, st, (const T*)a, lda, w_post, x, w_next, (T*)xn, H, eps, bias)
+#define RNT(T) do { if (nv <= 1) RN(T, 1); else if (nv <= 2) RN(T, 2); else if (nv <= 4) RN(T, 4); else RN(T, 8); } while (0)
+    if (f32) RNT(float); else RNT(u16);
+#undef RNT
+#undef RN
+    return (int)hipGetLastError();
+  }
   if (f32) {
     ENSURE_LDS(resadd_norm_kernel<float>, lds);
     hipLaunchKernelGGL(resadd_norm_kernel<float>, dim3(rows), dim3(256), lds, st, (const float*)a, lda, (const float*)b, ldb, wa,
-                       wb, w_post, x, w_next, (float*)xn, H, eps, dw, dn, (long)rows * H);
+                       wb, w_post, x, w_next, (float*)xn, H, eps, dw, dn, (long)rows * H, bias);
   } else {
     ENSURE_LDS(resadd_norm_kernel<u16>, lds);
     hipLaunchKernelGGL(resadd_norm_kernel<u16>, dim3(rows), dim3(256), lds, st, (const u16*)a, lda, (const u16*)b, ldb, wa, wb,
-                       w_post, x, w_next, (u16*)xn, H, eps, dw, dn, (long)rows * H);
+                       w_post, x, w_next, (u16*)xn, H, eps, dw, dn, (long)rows * H, bias);
   }
   return (int)hipGetLastError();
 }
@@ -1391,7 +1463,7 @@ extern "C" int dllm_glu_act(const void* gu, long ld, int f32, const float* bias,
                             void* y, long rows, hipStream_t st) {
   const long total = rows * ff;
   if (total <= 0) return 0;
-  if (mode < 0 || mode > 1) return -1;
+  if (mode < 0 || mode > 2) return -1;
   const dim3 grid((unsigned)((ff + 255) / 256), (unsigned)(rows < 2048 ? rows : 2048));
   BY_T(f32,
        hipLaunchKernelGGL(glu_act_kernel<u16>, grid, dim3(256), 0, st, (const u16*)gu, ld, bias, ff, mode, limit, alpha, (u16*)y, rows),

@@ -114,6 +114,13 @@ class RopeSpec:
 
 
 @dataclass(frozen=True)
+class QTempSpec:
+    """Queries at position p are multiplied by 1 + coef ln(floor((p + 1) / every) + 1)."""
+    coef: float
+    every: float
+
+
+@dataclass(frozen=True)
 class MixerSpec:
     """One token mixer.  ``kind``: ``mamba1`` (inner, state, dt_rank, conv), ``retention`` (heads,
     dim, vdim, decay per head, rot), ``latent_attention`` (heads, dim, rot_dim, vdim, kv_rank,
@@ -131,8 +138,13 @@ class MixerSpec:
     more term of score 0 and weight ``sink`` in the softmax denominator; ``kv_from`` as above) or
     ``gated_attention`` (grouped-query softmax attention without q / k norms, rotate-half pairs, inside
     ``chunk`` positions counted from 0 (0: all), scores soft-capped at ``softcap`` (0: not), one learned
-    sink score per head in the denominator, a sigmoid gate on the heads).  ``latent_attention`` with
-    ``q_rank`` 0 projects its queries directly and, with ``gate``, gates its heads."""
+    sink score per head in the denominator, a sigmoid gate on the heads) or ``biased_attention``
+    (grouped-query softmax attention with biases on q, k and v, inside a sliding ``window``; positions
+    enter through ``slopes``, what a head's scores lose per token of distance, and ``q_temp``, a factor
+    on the queries; with ``head_gate`` one sigmoid gate per head).  ``latent_attention`` with
+    ``q_rank`` 0 projects its queries directly and, with ``gate``, gates its heads; ``head_gate``: one gate
+    per head; ``sinks``: a learned sink score per head in the denominator; ``rot_half``: rotary pairs
+    (i, i + rot_dim / 2) instead of (2i, 2i + 1)."""
     kind: str
     inner: int = 0
     state: int = 0
@@ -161,6 +173,11 @@ class MixerSpec:
     chunk: int = 0
     softcap: float = 0.0
     gate: bool = False
+    head_gate: bool = False
+    sinks: bool = False
+    rot_half: bool = False
+    slopes: Tuple[float, ...] = ()
+    q_temp: Optional[QTempSpec] = None
 
     @property
     def parts(self) -> Tuple["MixerSpec", ...]:
@@ -172,7 +189,7 @@ class MixerSpec:
 
     @property
     def paged(self) -> bool:
-        return any(p.kind in ("latent_attention", "softmax_attention", "gated_attention") or
+        return any(p.kind in ("latent_attention", "softmax_attention", "gated_attention", "biased_attention") or
                    (p.kind in ("diff_attention", "sink_attention") and p.kv_from is None) for p in self.parts)
 
 
@@ -211,12 +228,17 @@ class DenseSpec:
     """One dense feed-forward ``W_down act(W_up x)``, ``ff`` wide; ``act``: ``gelu`` (the erf form),
     ``relu2`` (the square of relu) or ``polynorm`` (a N(z) + b N(z^2) + c N(z^3) + e with learned a, b, c, e and N the scaling of a
     token's ff values to unit RMS), or a gated one, ``W_down (g sigmoid(1.702 g) (u + 1))`` with
-    g = min(W_gate x, limit) and u = clamp(W_up x, -limit, limit) (``clamped_glu``).  ``bias``: every
+    g = min(W_gate x, limit) and u = clamp(W_up x, -limit, limit) (``clamped_glu``) or
+    ``W_down (gelu(W_gate x) * W_up x)`` with the tanh form of gelu (``gelu_glu``).  ``bias``: every
     projection has one."""
     ff: int
     act: str = "gelu"
     limit: float = 0.0
     bias: bool = False
+
+    @property
+    def gated(self) -> bool:
+        return self.act in ("clamped_glu", "gelu_glu")
 
 
 @dataclass(frozen=True)
@@ -316,12 +338,16 @@ class HybridConfig:
                     n += m.heads * m.vdim if m.kind == "lightning" else 0
                 elif m.kind == "gated_attention":
                     n += (m.heads + m.kv_heads) * m.dim * H + m.kv_heads * m.vdim * H + 2 * m.heads * m.vdim * H + m.heads
+                elif m.kind == "biased_attention":
+                    n += ((m.heads + m.kv_heads) * m.dim + m.kv_heads * m.vdim) * (H + 1) + H * m.heads * m.vdim
+                    n += m.heads * H if m.head_gate else 0
                 elif m.kind == "latent_attention" and not m.q_rank:
                     n += m.heads * m.dim * H + m.kv_rank * (H + 1) + m.heads * (m.dim + m.vdim) * m.kv_rank
                     n += (2 if m.gate else 1) * m.heads * m.vdim * H
                 elif m.kind == "latent_attention":
                     n += m.q_rank * (H + 1) + m.heads * (m.dim + m.rot_dim) * m.q_rank + (m.kv_rank + m.rot_dim) * H
                     n += m.kv_rank + m.heads * (m.dim + m.vdim) * m.kv_rank + H * m.heads * m.vdim
+                    n += (m.heads * H if m.head_gate else 0) + (m.heads if m.sinks else 0)
                 elif m.kind == "softmax_attention":
                     n += (m.heads + m.kv_heads) * m.dim * H + m.kv_heads * m.vdim * H + 2 * m.heads * m.vdim * H + m.heads
                 elif m.kind == "delta":
@@ -349,9 +375,9 @@ class HybridConfig:
                 n += f.identity * H + (f.experts + f.identity if f.correction else 0) + (H if f.shared_gate else 0)
             elif isinstance(L.mlp, DenseSpec):
                 f = L.mlp
-                mats = 3 if f.act == "clamped_glu" else 2
+                mats = 3 if f.gated else 2
                 n += (0 if self.parallel_ff else sides * H) + mats * f.ff * H + (4 if f.act == "polynorm" else 0)
-                n += (2 * f.ff + H if f.bias else 0)
+                n += ((mats - 1) * f.ff + H if f.bias else 0)
         if self.depth_average:
             n += sum(i + 2 for i in range(len(self.layers)))
         return n
@@ -593,9 +619,50 @@ def mugipel_config(raw: dict, name: str = "mugipel") -> HybridConfig:
                         norm_offset=True, loop=loop, tied_head=True)
 
 
+def figotar_config(raw: dict, name: str = "figotar") -> HybridConfig:
+    """A Figotar config.json: ``layers`` (type ``attention`` with heads, kv_heads, dim, vdim, scale, mask.size,
+    q_temp (coef, every), ``latent_attention`` with heads, dim, rot_dim, vdim, kv_rank, q_rank, rot (dims,
+    base), scale, or ``mlstm`` with heads, dim, vdim, gate_cap; mlp ``dense`` with ``ff`` or null),
+    ``norm.eps``, ``vocab``, ``width``.  A norm (weight around zero) on both sides of every sublayer."""
+    layers = []
+    for i, L in enumerate(raw["layers"]):
+        m, kind = L["mixer"], L["type"]
+        heads, dim = int(m["heads"]), int(m["dim"])
+        vdim = int(m.get("vdim", dim))
+        if kind == "attention":
+            qt = m.get("q_temp")
+            mix = MixerSpec("biased_attention", heads=heads, kv_heads=int(m.get("kv_heads", heads)), dim=dim, vdim=vdim,
+                            scale=float(m["scale"]), window=int((m.get("mask") or {}).get("size", 0)), head_gate=True,
+                            slopes=tuple(2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)),
+                            q_temp=QTempSpec(float(qt["coef"]), float(qt["every"])) if qt else None)
+            if mix.heads % mix.kv_heads:
+                raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+            if mix.q_temp is not None and mix.q_temp.every <= 0:
+                raise ValueError(f"layer {i}: q_temp.every must be positive")
+        elif kind == "latent_attention":
+            rot = _rope(m.get("rot"))
+            mix = MixerSpec(kind, heads=heads, dim=dim, rot_dim=int(m["rot_dim"]), vdim=vdim, kv_rank=int(m["kv_rank"]),
+                            q_rank=int(m["q_rank"]), scale=float(m["scale"]), rot=rot, head_gate=True, sinks=True, rot_half=True)
+            if mix.rot_dim % 2 or mix.rot_dim != (rot.dims if rot is not None else 0):
+                raise ValueError(f"layer {i}: rot_dim must be even and equal rot.dims")
+        elif kind == "mlstm":
+            mix = MixerSpec(kind, heads=heads, dim=dim, vdim=vdim, gate_cap=float(m["gate_cap"]))
+        else:
+            raise ValueError(f"unknown mixer type {kind!r}")
+        f = L.get("mlp")
+        mlp = None
+        if f:
+            if f["kind"] != "dense":
+                raise ValueError(f"unknown feed-forward kind {f['kind']!r}")
+            mlp = DenseSpec(int(f["ff"]), act="gelu_glu", bias=True)
+        layers.append(LayerSpec(mix, mlp))
+    return HybridConfig(name, "figotar", int(raw["width"]), int(raw["vocab"]), tuple(layers), rms_eps=float(raw["norm"]["eps"]),
+                        pre_norm=True, norm_offset=True)
+
+
 # config.json "architecture" -> parser of that design's keys
 ARCHITECTURES = {"Filevik": filevik_config, "Sedopel": sedopel_config, "Pebodra": pebodra_config,
-                 "Dogilorn": dogilorn_config, "Mugipel": mugipel_config}
+                 "Dogilorn": dogilorn_config, "Mugipel": mugipel_config, "Figotar": figotar_config}
 
 AnyConfig = Union[ModelConfig, HybridConfig]
 

@@ -1,4 +1,4 @@
-"""Layer-list decoders (Filevik, Sedopel, Pebodra, Dogilorn, Mugipel): every layer has a token mixer (Mamba-1 selective
+"""Layer-list decoders (Filevik, Sedopel, Pebodra, Dogilorn, Mugipel, Figotar): every layer has a token mixer (Mamba-1 selective
 scan, retention, latent attention, gated delta rule, grouped-query softmax attention beside lightning
 attention, differential sliding-window attention, Mamba-2, mLSTM) and an optional feed-forward
 (mixture of experts or dense), in the order config.json gives.
@@ -16,8 +16,11 @@ they do not take and for f32 models), everything between them on the HIP kernels
   latent     one fused down projection (query latent | key/value latent | shared rotated key) ->
              query up-projection -> the key up-projection is absorbed into the query (per-head
              batched GEMM), so attention runs over the cached latent alone (paged, written by a
-             kernel that norms the latent and rotates the shared key) -> value up-projection per
-             head -> out-proj
+             kernel that norms both latents and rotates the shared key; optional learned sinks) ->
+             value up-projection per head (optionally times one gate per head, whose logits come from
+             the down projection) -> out-proj.  Steps of longer prompt portions make every head's keys
+             and values from the latents they read, in scratch pages, and run the grouped-query kernel
+             on them instead
   experts    fused router (f32 softmax top-k, renormalised) -> grouped squared-ReLU expert GEMMs, or
              the dense form (all experts' columns, unused ones gated to zero) for f32 models and
              unaligned widths -> plus the shared expert
@@ -58,8 +61,12 @@ they do not take and for f32 models), everything between them on the HIP kernels
   latent     (direct queries, gated heads) one fused projection q | latent | gate | up -> the latent's
              norm, its page and relu(up)^2 in one launch -> absorbed latent attention as above -> value
              up-projection per head, gate -> one projection [out | down].  Steps of longer prompt
-             portions make every head's keys and values from the latents they read, in scratch pages,
-             and run the grouped-query kernel on them instead
+             portions run on expanded keys and values as above
+  biased_attn  one fused projection q | k | v | head gates -> biases, a factor on the queries that grows
+             with the position, k and v to their pages -> windowed attention whose scores fall with the
+             distance, times one gate per head -> out-proj
+  gelu_glu   one fused gate | up projection -> biases, gelu(g) u -> down-proj (its bias rides in the
+             residual launch)
 
 Layer forms: ``x += norm(sublayer(x))`` (Filevik) or, with ``cfg.pre_norm``, a norm on both sides,
 ``x += norm_b(sublayer(norm(x)))``, or without ``cfg.post_norm`` ``x += ls * sublayer(layernorm(x))``
@@ -84,7 +91,7 @@ import torch.nn.functional as F
 from .. import ops
 from ..ops import seqmix
 from ..parallel.comm import SINGLE, ParallelContext
-from .configs import DenseSpec, HybridConfig, LayerSpec, MixerSpec, MoESpec, RopeSpec
+from .configs import DenseSpec, HybridConfig, LayerSpec, MixerSpec, MoESpec, QTempSpec, RopeSpec
 
 
 def _mm(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
@@ -119,8 +126,11 @@ class HybridModel:
                     raise ValueError(f"{cfg.name}: only dense squared-relu feed-forwards run beside a mixer")
             if not cfg.pre_norm or cfg.post_norm or cfg.norm_kind != "rms" or cfg.depth_average or cfg.layer_scale or cfg.input_conv:
                 raise ValueError(f"{cfg.name}: parallel layers use one RMS norm ahead of both sublayers and one plain add")
-        elif cfg.loop is not None or cfg.norm_offset or cfg.residual_mult != 1.0:
-            raise ValueError(f"{cfg.name}: loops, zero-centred norms and residual multipliers are built for parallel layers")
+        else:
+            if cfg.loop is not None or cfg.residual_mult != 1.0:
+                raise ValueError(f"{cfg.name}: loops and residual multipliers are built for parallel layers")
+            if cfg.norm_offset and (cfg.norm_kind != "rms" or not cfg.pre_norm or not cfg.post_norm):
+                raise ValueError(f"{cfg.name}: zero-centred norms are built for RMS norms on both sides of a sublayer")
         if cfg.norm_kind == "layer" and (not cfg.pre_norm or cfg.post_norm):
             raise ValueError(f"{cfg.name}: layer norms are built for the pre-norm layer form only")
         # the input convolution's last inputs are per-sequence state like a recurrence's
@@ -128,6 +138,7 @@ class HybridModel:
         self.layers: List[Dict[str, torch.Tensor]] = []
         self.tap: Optional[list] = None      # debugging: residual stream after every layer
         self._rot: Dict[RopeSpec, torch.Tensor] = {}
+        self._qtab: Dict[QTempSpec, torch.Tensor] = {}
         self._max_pos = 0
         raw = self._load(weights) if weights else self._random(seed, init_std)
         self._place(raw)
@@ -166,7 +177,7 @@ class HybridModel:
             if cfg.input_conv:
                 t[p + "canon1"] = rnd(W, cfg.input_conv, s=0.3)
             if cfg.pre_norm and cfg.post_norm:
-                t[p + "norm1b"] = torch.ones(W)
+                t[p + "norm1b"] = one(W)
             if cfg.depth_average:
                 t[p + "dwa"] = torch.cat([rnd(i + 1, s=0.05), torch.ones(1)])
             if m.kind == "delta":
@@ -240,6 +251,12 @@ class HybridModel:
                 t[p + "mix.q"], t[p + "mix.k"] = lin(m.heads * m.dim, W), lin(m.kv_heads * m.dim, W)
                 t[p + "mix.v"], t[p + "mix.sink"] = lin(m.kv_heads * m.vdim, W), rnd(m.heads, s=1.0)
                 t[p + "mix.g"], t[p + "mix.o"] = lin(m.heads * m.vdim, W), lin(W, m.heads * m.vdim)
+            elif m.kind == "biased_attention":
+                for n_, c in (("q", m.heads * m.dim), ("k", m.kv_heads * m.dim), ("v", m.kv_heads * m.vdim)):
+                    t[p + "mix." + n_], t[p + f"mix.{n_}.b"] = lin(c, W), rnd(c, s=0.1)
+                t[p + "mix.o"] = lin(W, m.heads * m.vdim)
+                if m.head_gate:
+                    t[p + "mix.g"] = lin(m.heads, W)
             elif not m.q_rank:
                 t[p + "mix.q"], t[p + "mix.dkv"] = lin(m.heads * m.dim, W), lin(m.kv_rank, W)
                 t[p + "mix.dkv.norm"] = torch.ones(m.kv_rank)
@@ -251,23 +268,27 @@ class HybridModel:
                 t[p + "mix.dkv"], t[p + "mix.dkv.norm"] = lin(m.kv_rank + m.rot_dim, W), torch.ones(m.kv_rank)
                 t[p + "mix.uk"], t[p + "mix.uv"] = lin(m.heads * m.dim, m.kv_rank), lin(m.heads * m.vdim, m.kv_rank)
                 t[p + "mix.o"] = lin(W, m.heads * m.vdim)
+                if m.head_gate:
+                    t[p + "mix.g"] = lin(m.heads, W)
+                if m.sinks:
+                    t[p + "mix.sink"] = rnd(m.heads, s=1.0)
             f = L.mlp
             if f is not None and not cfg.parallel_ff:
-                t[p + "norm2"] = torch.ones(W)
+                t[p + "norm2"] = one(W)
                 if lnb:
                     t[p + "norm2.b"] = rnd(W, s=0.1)
                 if cfg.layer_scale:
                     t[p + "ls2"] = torch.full((W,), 0.5)
             if isinstance(f, DenseSpec):
                 if cfg.pre_norm and cfg.post_norm:
-                    t[p + "norm2b"] = torch.ones(W)
+                    t[p + "norm2b"] = one(W)
                 t[p + "mlp.up"], t[p + "mlp.down"] = lin(f.ff, W), lin(W, f.ff)
                 if f.act == "polynorm":
                     t[p + "mlp.act"] = torch.tensor([1.0, 0.5, 0.25, 0.0])
-                if f.act == "clamped_glu":
+                if f.gated:
                     t[p + "mlp.gate"] = lin(f.ff, W)
                 if f.bias:
-                    for n_, c in (("gate", f.ff), ("up", f.ff), ("down", W)):
+                    for n_, c in ((("gate", f.ff),) if f.gated else ()) + (("up", f.ff), ("down", W)):
                         t[p + f"mlp.{n_}.b"] = rnd(c, s=0.1)
             elif f is not None:
                 t[p + "mlp.router"] = lin(f.experts + f.identity, W)
@@ -302,6 +323,7 @@ class HybridModel:
         f32 copies of what the recurrences read)."""
         cfg, dev, dt = self.cfg, self.device, self.dtype
         put = lambda x: x.to(dev, dt).contiguous()
+        fuse = lambda names: self._fuse([t[n] for n in names], put)
         f32 = lambda x: x.to(dev, torch.float32).contiguous()
         W = cfg.hidden
         # norm weights stored around zero get their 1 here, in f32
@@ -324,7 +346,7 @@ class HybridModel:
                 self.layers.append(D)
                 continue
             if cfg.pre_norm and cfg.post_norm:
-                D["norm1b"] = f32(t[p + "norm1b"])
+                D["norm1b"] = nrm(t[p + "norm1b"])
             if lnb:
                 D["norm1.b"] = f32(t[p + "norm1.b"])
             if cfg.layer_scale:
@@ -391,10 +413,18 @@ class HybridModel:
                 assert D["in"].shape[0] == 2 * inner + bc + m.heads and tuple(D["conv"].shape) == (inner + bc, m.conv)
                 assert D["neg_a"].numel() == m.heads and D["gnorm"].numel() == inner
             elif m.kind == "mlstm":
-                D["proj"] = put(torch.cat([t[p + "mix." + n] for n in ("q", "k", "v", "g", "i", "f")], 0))
+                D["proj"], n = fuse([p + "mix." + x for x in ("q", "k", "v", "g", "i", "f")])
                 D["gate_b"] = f32(torch.cat([t[p + "mix.i.b"], t[p + "mix.f.b"]], 0))
                 D["hnorm"], D["o"] = f32(t[p + "mix.norm"]), put(t[p + "mix.o"])
-                assert D["proj"].shape[0] == 2 * m.heads * (m.dim + m.vdim + 1) and D["hnorm"].numel() == m.heads * m.vdim
+                assert n == 2 * m.heads * (m.dim + m.vdim + 1) and D["hnorm"].numel() == m.heads * m.vdim
+            elif m.kind == "biased_attention":
+                D["proj"], n = fuse([p + "mix." + x for x in (("q", "k", "v", "g") if m.head_gate else ("q", "k", "v"))])
+                D["bias"] = f32(torch.cat([t[p + f"mix.{x}.b"] for x in "qkv"], 0))
+                D["slopes"] = torch.tensor(m.slopes, dtype=torch.float32, device=dev)
+                D["o"] = put(t[p + "mix.o"])
+                assert D["bias"].numel() == (m.heads + m.kv_heads) * m.dim + m.kv_heads * m.vdim
+                assert n == D["bias"].numel() + (m.heads if m.head_gate else 0) and D["slopes"].numel() == m.heads
+                assert tuple(D["o"].shape) == (W, m.heads * m.vdim)
             elif m.kind == "mamba1":
                 D["in"], D["x"], D["dt"], D["o"] = (put(t[p + "mix." + n]) for n in ("in", "x", "dt", "o"))
                 D["conv"], D["conv_b"] = f32(t[p + "mix.conv"]), f32(t[p + "mix.conv.b"])
@@ -407,11 +437,17 @@ class HybridModel:
                 D["decay"] = torch.tensor(m.decay, dtype=torch.float32, device=dev)
                 assert D["decay"].numel() == m.heads
             else:
-                D["dqkv"] = put(torch.cat([t[p + "mix.dq"], t[p + "mix.dkv"]], 0))
+                D["dqkv"], n = fuse([p + "mix." + x for x in (("dq", "dkv", "g") if m.head_gate else ("dq", "dkv"))])
                 D["dq_norm"], D["dkv_norm"] = f32(t[p + "mix.dq.norm"]), f32(t[p + "mix.dkv.norm"])
                 D["uq"], D["o"] = put(t[p + "mix.uq"]), put(t[p + "mix.o"])
                 D["uk"] = put(t[p + "mix.uk"].view(m.heads, m.dim, m.kv_rank))                       # [H, d, r]
-                D["uvT"] = put(t[p + "mix.uv"].view(m.heads, m.vdim, m.kv_rank).transpose(1, 2))    # [H, r, dv]
+                D["uv"] = put(t[p + "mix.uv"].view(m.heads, m.vdim, m.kv_rank))                      # [H, dv, r]
+                D["uvT"] = D["uv"].transpose(1, 2).contiguous()                                      # [H, r, dv]
+                if m.sinks:
+                    D["sink"] = f32(t[p + "mix.sink"])
+                    assert D["sink"].numel() == m.heads
+                assert n == m.q_rank + m.kv_rank + m.rot_dim + (m.heads if m.head_gate else 0)
+                assert D["dq_norm"].numel() == m.q_rank and D["dkv_norm"].numel() == m.kv_rank
             f = L.mlp
             if f is not None:
                 if lnb:
@@ -419,25 +455,25 @@ class HybridModel:
                 if cfg.layer_scale:
                     D["ls2"] = f32(t[p + "ls2"])
             if isinstance(f, DenseSpec):
-                D["norm2"], D["down"] = f32(t[p + "norm2"]), put(t[p + "mlp.down"])
-                if f.act == "clamped_glu":     # one projection: gate rows, then up rows
+                D["norm2"], D["down"] = nrm(t[p + "norm2"]), put(t[p + "mlp.down"])
+                if f.gated:     # one projection: gate rows, then up rows
                     D["up"] = put(torch.cat([t[p + "mlp.gate"], t[p + "mlp.up"]], 0))
                     assert tuple(D["up"].shape) == (2 * f.ff, W)
                 else:
                     D["up"] = put(t[p + "mlp.up"])
                     assert tuple(D["up"].shape) == (f.ff, W)
                 if f.bias:
-                    names = ("gate", "up") if f.act == "clamped_glu" else ("up",)
+                    names = ("gate", "up") if f.gated else ("up",)
                     D["up_b"] = f32(torch.cat([t[p + f"mlp.{n}.b"] for n in names], 0))
                     D["down_b"] = f32(t[p + "mlp.down.b"])
                     assert D["up_b"].numel() == D["up"].shape[0] and D["down_b"].numel() == W
                 if cfg.pre_norm and cfg.post_norm:
-                    D["norm2b"] = f32(t[p + "norm2b"])
+                    D["norm2b"] = nrm(t[p + "norm2b"])
                 if f.act == "polynorm":
                     D["act"] = f32(t[p + "mlp.act"])
                     assert D["act"].numel() == 4
             elif f is not None:
-                D["norm2"] = f32(t[p + "norm2"])
+                D["norm2"] = nrm(t[p + "norm2"])
                 D["router"] = put(t[p + "mlp.router"])
                 if f.score == "sigmoid" or not f.renorm:
                     D["router"] = f32(t[p + "mlp.router"])     # the router runs in f32
@@ -472,6 +508,15 @@ class HybridModel:
                     assert D["sh_down"].shape[1] == f.shared_ff
             self.layers.append(D)
 
+    def _fuse(self, parts: List[torch.Tensor], put) -> Tuple[torch.Tensor, int]:
+        """One projection for several that read the same input, and its rows; bf16 models on the GPU get
+        zero rows behind them up to a multiple of 64, the output tile of the tuned GEMMs."""
+        w = torch.cat(parts, 0)
+        n = w.shape[0]
+        if self.dtype == torch.bfloat16 and self.device.type == "cuda" and n % 64 and w.shape[1] % 64 == 0:
+            w = torch.cat([w, w.new_zeros(-n % 64, w.shape[1])], 0)
+        return put(w), n
+
     def _place_parallel(self, D, L: LayerSpec, t, p: str, put, f32) -> None:
         """A layer whose mixer and feed-forward read the same input and are added together: one
         projection for everything that reads it, one for everything that is added."""
@@ -497,9 +542,10 @@ class HybridModel:
 
     def gemm_shapes(self) -> List[Tuple[int, int]]:
         """(out, in) of the large bf16 weights that run on the tuned GEMMs (the engine times their plans)."""
-        if self.dtype != torch.bfloat16 or not self.cfg.parallel_ff:
+        if self.dtype != torch.bfloat16:
             return []
-        ws = [L[k] for L in self.layers for k in ("proj", "out")] + [self.lm_head] + \
+        names = ("proj", "out", "dqkv", "uq", "o", "up", "down", "in", "x", "dt", "qkvg", "lo", "ro", "sh_up", "sh_down")
+        ws = [L[k] for L in self.layers for k in names if k in L] + [self.lm_head] + \
             ([self.loop_in] if self.cfg.loop is not None else [])
         return sorted({tuple(w.shape) for w in ws if w.shape[0] % 64 == 0 and w.shape[1] % 64 == 0 and w.numel() >= 1 << 22})
 
@@ -528,13 +574,18 @@ class HybridModel:
 
     # ------------------------------------------------------------------ positions, caches
     def ensure_positions(self, n: int) -> None:
-        """cos | sin tables (f64 on the host, stored f32) for positions < n of every rotation used."""
+        """cos | sin tables (f64 on the host, stored f32) for positions < n of every rotation used, and the
+        query factors of every temperature."""
         if n <= self._max_pos:
             return
         self._max_pos = n
         for L in self.cfg.layers:
             for m in L.mixer.parts:
                 r = m.rot
+                if m.q_temp is not None:
+                    p = torch.arange(1, n + 1, dtype=torch.float64)
+                    f = 1.0 + m.q_temp.coef * torch.log(torch.floor(p / m.q_temp.every) + 1.0)
+                    self._qtab[m.q_temp] = f.to(self.device, torch.float32)
                 if r is not None and r.dims > 0:
                     self._rot[r] = ops.rope_cos_sin(n, r.dims, r.base, self.device, r.yarn.as_scaling() if r.yarn else None)
 
@@ -549,7 +600,7 @@ class HybridModel:
             for m in self.cfg.layers[i].mixer.parts:
                 if m.kind == "latent_attention":
                     n += block_size * (m.kv_rank + m.rot_dim) * it
-                elif m.kind in ("softmax_attention", "gated_attention"):
+                elif m.kind in ("softmax_attention", "gated_attention", "biased_attention"):
                     n += block_size * m.kv_heads * (m.dim + m.vdim) * it
                 elif m.kind == "diff_attention" and m.kv_from is None:
                     n += block_size * m.kv_heads * (2 * m.dim + m.vdim) * it
@@ -569,13 +620,13 @@ class HybridModel:
         vdim] f32) / mlstm: (memory [slots, heads, dim, vdim] f32, normaliser and maximum [slots,
         heads, column blocks, dim + 1] f32) / sink_attention: (paged keys [blocks, kv_heads, block,
         dim], paged values [blocks, kv_heads, vdim, block]), of the layer ``kv_from`` names if any /
-        gated_attention: the same two.
+        gated_attention, biased_attention: the same two.
         With an input convolution every layer's tuple ends with its own last inputs [slots, taps - 1,
         width]."""
         dev, out = self.device, []
         for i, _ in self.cfg.runs:
             m = self.cfg.layers[i].mixer
-            if m.kind in ("sink_attention", "gated_attention"):
+            if m.kind in ("sink_attention", "gated_attention", "biased_attention"):
                 if m.kv_from is not None:
                     out.append(out[m.kv_from][:2])
                 else:
@@ -642,22 +693,45 @@ class HybridModel:
         return next(iter(self._rot.values()))
 
     def _latent(self, L, m: MixerSpec, x, positions, meta, cache):
-        T, H, eps = x.shape[0], m.heads, self.cfg.rms_eps
-        down = _mm(x, L["dqkv"])
-        cq = seqmix.rms_rows(down[:, :m.q_rank], L["dq_norm"], eps)
+        """Latent attention behind a query latent: on the cached latents (absorbed form), or for steps of
+        longer prompt portions on keys and values made from them."""
+        T, H, eps, rd = x.shape[0], m.heads, self.cfg.rms_eps, m.rot_dim
+        down = _mm(x, L["dqkv"])                    # query latent | latent | rotated key part (| head gates)
+        g0 = m.q_rank + m.kv_rank + rd
+        gate = down[:, g0:g0 + H] if m.head_gate else None
+        table = self._table(m) if rd else self._any_table()
+        all_rows = self._all_rows(x, meta)
+        S = 0 if meta.host_qlen is None else len(meta.host_qlen)
+        expand = bool(S) and all_rows and seqmix.latent_expand_wanted(cache[0], H, m.dim, m.vdim, T, S,
+                                                                       meta.block_tables.numel(), rd)
+        # absorbed form: padding rows of the attention output are cleared by the write launch
+        lat = None if expand else torch.empty((H, T, m.kv_rank), dtype=x.dtype, device=x.device)
+        cq = seqmix.latent_kv_write(down[:, m.q_rank:g0], m.kv_rank, L["dkv_norm"], eps, positions, table, meta.slots,
+                                    cache[0], m.rot_half, down[:, :m.q_rank], L["dq_norm"], None if all_rows else lat)
         q = _mm(cq, L["uq"])                                            # [T, H (dim + rot)]
-        table = self._table(m)
-        seqmix.latent_kv_write(down[:, m.q_rank:], m.kv_rank, L["dkv_norm"], eps, positions, table, meta.slots,
-                               cache[0])
-        qn = q.view(T, H, m.dim + m.rot_dim)[:, :, :m.dim].transpose(0, 1)
+        if expand:
+            q = seqmix.latent_q_prep(q, H, m.dim, rd, positions, table, m.scale, m.rot_half)
+            k, v, pages = seqmix.latent_expand(cache[0], meta.block_tables, meta.ctx, L["uk"], L["uv"])
+            mfma = seqmix.gqa_use_mfma(q, H, H, m.dim + rd, m.vdim, k.shape[2])
+            ts, tt = meta.latent_tiles(1, self.device, seqmix.gqa_tokens_per_tile(H, H, mfma))
+            splits = seqmix.gqa_splits(int(ts.numel()), H, meta.max_ctx) if mfma else 1
+            o = seqmix.paged_gqa_attention(q, k, v, pages, meta.qstart, meta.qlen, meta.ctx, ts, tt, gate, mfma, splits,
+                                           all_rows=True, sinks=L.get("sink"))
+            return _mm(o, L["o"])
+        qn = q.view(T, H, m.dim + rd)[:, :, :m.dim].transpose(0, 1)
         qa = torch.bmm(qn, L["uk"])                                     # key up-projection absorbed: [H, T, rank]
         rows = (seqmix.LAT_ROWS if meta.host_qlen is None else
                 seqmix.latent_rows(x, m.kv_rank, m.rot_dim, T, len(meta.host_qlen)))
         ts, tr = meta.latent_tiles(H, self.device, rows)
-        lat = seqmix.latent_attention(qa, q, m.dim, m.rot_dim, positions, table, cache[0], meta.block_tables,
-                                      meta.qstart, meta.qlen, meta.ctx, ts, tr, m.scale, rows=rows)
+        lat = seqmix.latent_attention(qa, q, m.dim, rd, positions, table, cache[0], meta.block_tables, meta.qstart,
+                                      meta.qlen, meta.ctx, ts, tr, m.scale, rows=rows, out=lat, half=m.rot_half,
+                                      sinks=L.get("sink"))
         o = torch.bmm(lat, L["uvT"])                                    # [H, T, vdim]
-        return _mm(o.transpose(0, 1).reshape(T, H * m.vdim), L["o"])
+        if gate is not None:
+            o = seqmix.gate_heads(o, gate, torch.empty((T, H * m.vdim), dtype=x.dtype, device=x.device))
+        else:
+            o = o.transpose(0, 1).reshape(T, H * m.vdim)
+        return _mm(o, L["o"])
 
     @staticmethod
     def _left_cols(a: MixerSpec) -> int:
@@ -746,6 +820,23 @@ class HybridModel:
         o = seqmix.paged_gqa_attention(q, k_cache, v_cache, meta.block_tables, meta.qstart, meta.qlen, meta.ctx, ts, tt,
                                        None, mfma, splits, window=m.window, keep_first=m.keep_first, sink=m.sink,
                                        all_rows=self._all_rows(x, meta), out=out)
+        return _mm(o, L["o"])
+
+    def _biased_attention(self, L, m: MixerSpec, x, positions, meta, cache):
+        k_cache, v_cache = cache[0], cache[1]
+        proj = _mm(x, L["proj"])                                        # q | k | v (| head gates)
+        n = (m.heads + m.kv_heads) * m.dim + m.kv_heads * m.vdim
+        gate = proj[:, n:n + m.heads] if m.head_gate else None
+        all_rows = self._all_rows(x, meta)      # else the prep launch clears the attention output's padding rows
+        out = None if all_rows else torch.empty((x.shape[0], m.heads * m.vdim), dtype=x.dtype, device=x.device)
+        q = seqmix.rope_prep(proj, m.heads, m.kv_heads, m.dim, m.vdim, self._any_table(), 0, m.scale, positions, meta.slots,
+                             k_cache, v_cache, zero_rows=out, bias=L["bias"],
+                             qtab=self._qtab[m.q_temp] if m.q_temp is not None else None)
+        mfma = seqmix.gqa_use_mfma(q, m.heads, m.kv_heads, m.dim, m.vdim, k_cache.shape[2])
+        ts, tt = meta.latent_tiles(1, self.device, seqmix.gqa_tokens_per_tile(m.heads, m.kv_heads, mfma))
+        splits = seqmix.gqa_splits(int(ts.numel()), m.kv_heads, meta.max_ctx, m.window) if mfma else 1
+        o = seqmix.paged_gqa_attention(q, k_cache, v_cache, meta.block_tables, meta.qstart, meta.qlen, meta.ctx, ts, tt,
+                                       gate, mfma, splits, window=m.window, all_rows=all_rows, out=out, slopes=L["slopes"])
         return _mm(o, L["o"])
 
     # ------------------------------------------------------------------ mixer and feed-forward side by side
@@ -865,6 +956,8 @@ class HybridModel:
         z = _mm(x, L["up"])
         if f.act == "clamped_glu":      # the down projection's bias rides in the residual launch
             a = seqmix.glu_act(z, L.get("up_b"), "clamped", f.limit, 1.702)
+        elif f.act == "gelu_glu":       # likewise
+            a = seqmix.glu_act(z, L.get("up_b"), "gelu_tanh")
         else:
             a = seqmix.polynorm(z, L["act"], self.cfg.rms_eps) if f.act == "polynorm" else seqmix.gelu_erf(z)
         return _mm(a, L["down"])
@@ -992,6 +1085,8 @@ class HybridModel:
                 y = self._mlstm(L, m, h, meta, cache)
             elif m.kind == "sink_attention":
                 y = self._sink_attention(L, m, h, positions, meta, cache)
+            elif m.kind == "biased_attention":
+                y = self._biased_attention(L, m, h, positions, meta, cache)
             else:
                 y = self._latent(L, m, h, positions, meta, cache)
             if ln:
@@ -1009,20 +1104,20 @@ class HybridModel:
                 # the sublayer's tail and the next sublayer's input norm in one launch
                 nxt = self.layers[i + 1]["norm1"] if i + 1 < nL else self.final_norm
                 pair = dict(b=y[1], wa=L["lout"], wb=L["rout"]) if isinstance(y, tuple) else {}
-                a = y[0] if isinstance(y, tuple) else y
+                a, bias = y[0] if isinstance(y, tuple) else y, None
                 if S.mlp is not None:
                     h = torch.empty((T, W), dtype=self.dtype, device=x.device)
                     seqmix.resadd_norm(a, L["norm1b"], eps, x, L["norm2"], h, **pair)
                     y = self._dense(L, S.mlp, h) if isinstance(S.mlp, DenseSpec) else self._experts(L, S.mlp, h)
-                    a, pair, post = y, {}, L["norm2b"]
+                    a, pair, post, bias = y, {}, L["norm2b"], L.get("down_b")
                 else:
                     post = L["norm1b"]
                 if X is not None:     # ... and the layer's weighted sum over depth
                     h = torch.empty((T, W), dtype=self.dtype, device=x.device)
-                    x = seqmix.resadd_norm(a, post, eps, x, nxt, h, depth=(X, L["dwa"], i + 2), **pair)
+                    x = seqmix.resadd_norm(a, post, eps, x, nxt, h, depth=(X, L["dwa"], i + 2), bias=bias, **pair)
                 else:
                     h = torch.empty((T, W), dtype=self.dtype, device=x.device)
-                    seqmix.resadd_norm(a, post, eps, x, nxt, h, **pair)
+                    seqmix.resadd_norm(a, post, eps, x, nxt, h, bias=bias, **pair)
             else:
                 ng = cfg.norm_groups
                 seqmix.norm_resadd(y, L["norm1"], eps, x, xl, groups=ng, bias=L.get("ob"))

@@ -505,20 +505,42 @@ def _rope_interleaved(x, c, s):
     return out
 
 
-def latent_kv_write(ckv, rank, norm_w, eps, positions, cos_sin, slots, cache):
-    """cache[slot] = [rmsnorm(ckv[:, :rank]) * norm_w | interleaved-rotated ckv[:, rank:]]."""
+def _rope_half(x, c, s):
+    h = x.shape[-1] // 2
+    u, w_ = x[..., :h], x[..., h:]
+    return torch.cat([u * c - w_ * s, w_ * c + u * s], -1)
+
+
+def latent_kv_write(ckv, rank, norm_w, eps, positions, cos_sin, slots, cache, half=False, q_src=None, q_norm=None, zero=None):
+    """cache[slot] = [rmsnorm(ckv[:, :rank]) * norm_w | rotated ckv[:, rank:]] (pairs (2i, 2i + 1), with
+    ``half`` (i, i + rot / 2)); returns rmsnorm(q_src) * q_norm; ``zero`` [heads, T, rank]: rows of tokens
+    without a slot are cleared."""
     dr = ckv.shape[1] - rank
     c = rms_rows(ckv[:, :rank], norm_w, eps, torch.float32)
     cs, sn = _rot_table(cos_sin, positions, dr // 2)
-    kr = _rope_interleaved(ckv[:, rank:].float(), cs, sn)
+    kr = (_rope_half if half else _rope_interleaved)(ckv[:, rank:].float(), cs, sn)
     ok = slots >= 0
     cache.view(-1, cache.shape[-1])[slots[ok].long()] = torch.cat([c, kr], 1)[ok].to(cache.dtype)
+    if zero is not None:
+        zero[:, slots < 0] = 0
+    return None if q_src is None else rms_rows(q_src, q_norm, eps)
 
 
-def latent_attention(qa, q, dim, rot_dim, positions, cos_sin, cache, block_tables, qstart, qlen, ctx, scale):
+def latent_q_prep(q, heads, dim, rot_dim, positions, cos_sin, scale, half=False):
+    """The last ``rot_dim`` dims of every head rotated, everything times ``scale``."""
+    T = q.shape[0]
+    f = q.float()[:, :heads * (dim + rot_dim)].reshape(T, heads, dim + rot_dim)
+    cs, sn = _rot_table(cos_sin, positions, rot_dim // 2)
+    qr = (_rope_half if half else _rope_interleaved)(f[..., dim:], cs[:, None, :], sn[:, None, :])
+    return (torch.cat([f[..., :dim], qr], -1) * scale).to(q.dtype)
+
+
+def latent_attention(qa, q, dim, rot_dim, positions, cos_sin, cache, block_tables, qstart, qlen, ctx, scale, half=False,
+                     sinks=None):
     """Causal softmax attention over a shared latent: row (t, h) scores key j as
     (qa[h, t] . c_j + rot(q[t, h, dim:]) . kr_j) * scale and returns sum_j p_j c_j.
-    qa [heads, T, rank], q [T, heads * (dim + rot_dim)], cache [blocks, 16, rank + rot_dim]."""
+    qa [heads, T, rank], q [T, heads * (dim + rot_dim)], cache [blocks, 16, rank + rot_dim].  ``sinks``
+    [heads]: one more score per head in the softmax, without a value."""
     Hh, T, r = qa.shape
     out = torch.zeros((Hh, T, r), dtype=qa.dtype, device=qa.device)
     flat = cache.view(-1, cache.shape[-1])
@@ -533,13 +555,15 @@ def latent_attention(qa, q, dim, rot_dim, positions, cos_sin, cache, block_table
         kv = flat[idx].float()
         cs, sn = _rot_table(cos_sin, positions[q0:q0 + n], rot_dim // 2)
         qr = q[q0:q0 + n].float().reshape(n, Hh, dim + rot_dim)[..., dim:]
-        qr = _rope_interleaved(qr, cs[:, None, :], sn[:, None, :])
+        qr = (_rope_half if half else _rope_interleaved)(qr, cs[:, None, :], sn[:, None, :])
         sc = (torch.einsum("htr,jr->htj", qa[:, q0:q0 + n].float(), kv[:, :r]) +
               torch.einsum("thr,jr->htj", qr, kv[:, r:])) * scale
         pos = positions[q0:q0 + n].long()
         mask = torch.arange(L, device=cache.device)[None, :] <= pos[:, None]
         sc = sc.masked_fill(~mask[None], float("-inf"))
-        p = torch.softmax(sc, -1)
+        if sinks is not None:
+            sc = torch.cat([sc, sinks.float()[:, None, None].expand(Hh, n, 1)], -1)
+        p = torch.softmax(sc, -1)[..., :L]
         out[:, q0:q0 + n] = torch.einsum("htj,jr->htr", p, kv[:, :r]).to(qa.dtype)
     return out
 
@@ -575,11 +599,13 @@ def dense_gate(ids, wts, E):
 
 # ----------------------------------------------------------------------------- pre/post-norm layers, depth average
 
-def resadd_norm(a, w_post, eps, x, w_next=None, x_next=None, b=None, wa=None, wb=None):
-    """x (f32 stream, in place) += rmsnorm(y) * w_post with y = a, or, with a second branch,
+def resadd_norm(a, w_post, eps, x, w_next=None, x_next=None, b=None, wa=None, wb=None, bias=None):
+    """x (f32 stream, in place) += rmsnorm(y + bias) * w_post with y = a, or, with a second branch,
     y = (rmsnorm(a) wa + rmsnorm(b) wb) / 2; ``x_next`` receives rmsnorm(x) * w_next (the plain
     rounding of x when ``w_next`` is None)."""
     y = a.float() if b is None else 0.5 * (rms_rows(a, wa, eps, torch.float32) + rms_rows(b, wb, eps, torch.float32))
+    if bias is not None:
+        y = y + bias.float()
     x += rms_rows(y, w_post, eps, torch.float32)
     if x_next is not None:
         x_next.copy_(x if w_next is None else rms_rows(x, w_next, eps, torch.float32))
@@ -630,17 +656,17 @@ def attn_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, eps, qscale, 
 
 
 def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, gate=None, window=0, out_f32=False,
-                        keep_first=0, sink=0.0, chunk=0, softcap=0.0, sinks=None, out=None):
+                        keep_first=0, sink=0.0, chunk=0, softcap=0.0, sinks=None, out=None, slopes=None):
     """Causal softmax attention of q [T, heads, dim] (already scaled) over paged keys / values;
     query head h reads key head h // (heads / kv_heads); the output [T, heads * vdim] is
-    multiplied by sigmoid(gate) when a gate [T, heads * vdim] is given.  ``window`` > 0: position i
+    multiplied by sigmoid(gate) when a gate [T, heads * vdim] or [T, heads] is given.  ``window`` > 0: position i
     sees keys i - window < j <= i, and the keys j < ``keep_first`` whatever their distance.  A value
     cache with fewer heads than the key cache is shared by neighbouring key heads (key head g reads
     value head g // (key heads / value heads)).  ``sink``: weight of one more term of score 0 in
     every softmax denominator (it has no value): p_j = exp(s_j) / (sink + sum exp(s_j)).  ``sinks``
     [heads] f32: that term's score per head instead, with weight 1.  ``chunk`` > 0: position i sees the
     keys j <= i of its own chunk, j >= i - i % chunk.  ``softcap``: s <- softcap tanh(s / softcap).
-    ``out``: written there."""
+    ``slopes`` [heads]: s <- s - slopes[head] (i - j).  ``out``: written there."""
     T, H, d = q.shape
     G, BSz, dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[2]
     vrep = G // v_cache.shape[1]
@@ -668,6 +694,8 @@ def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, ga
             mask = mask | ((keys < (pos - pos % chunk)[:, None]) & (keys >= keep_first))
         if softcap > 0:
             sc = softcap * torch.tanh(sc / softcap)
+        if slopes is not None:
+            sc = sc - slopes.float()[:, None, None] * (pos[:, None] - torch.arange(c, device=q.device)[None, :])[None]
         sc = sc.masked_fill(mask[None], float("-inf"))
         if sinks is not None:
             sc = torch.cat([sc, sinks.float()[:, None, None].expand(H, n, 1)], -1)
@@ -680,7 +708,8 @@ def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, ga
             pr = torch.softmax(sc, -1)
         o = torch.einsum("htu,uhv->thv", pr, V).reshape(n, H * dv)
         if gate is not None:
-            o = o * torch.sigmoid(gate[qs[s]:qs[s] + n].float())
+            gt = torch.sigmoid(gate[qs[s]:qs[s] + n].float())
+            o = o * (gt.repeat_interleave(dv, 1) if gt.shape[1] == H else gt)
         out[qs[s]:qs[s] + n] = o.to(out.dtype)
     return out
 
@@ -1009,7 +1038,7 @@ def proj_norm_prep(proj, heads, kv_heads, dim, vdim, qnorm_w, knorm_w, cos_sin, 
 def glu_act(gu, bias=None, mode="swiglu", limit=0.0, alpha=1.0):
     """gu [T, 2 ff] (gate columns, then up columns), ``bias`` f32 over the same columns -> [T, ff].
     "swiglu": silu(g) u.  "clamped": g <- min(g, limit), u <- clamp(u, -limit, limit), then
-    g sigmoid(alpha g) (u + 1)."""
+    g sigmoid(alpha g) (u + 1).  "gelu_tanh": gelu(g) u in its tanh form."""
     f = gu.float()
     if bias is not None:
         f = f + bias.float()
@@ -1017,6 +1046,8 @@ def glu_act(gu, bias=None, mode="swiglu", limit=0.0, alpha=1.0):
     g, u = f[:, :ff], f[:, ff:]
     if mode == "swiglu":
         return (torch.nn.functional.silu(g) * u).to(gu.dtype)
+    if mode == "gelu_tanh":
+        return (torch.nn.functional.gelu(g, approximate="tanh") * u).to(gu.dtype)
     g = g.clamp(max=limit)
     u = u.clamp(min=-limit, max=limit)
     return (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(gu.dtype)
@@ -1042,11 +1073,14 @@ def relu2(u):
 
 
 def rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, positions, slots, k_cache, v_cache, ucol=0, act=None,
-              zero_rows=None):
+              zero_rows=None, bias=None, qtab=None):
     """Rotate-half positions on the first ``rot_dims`` dims of q and k (cos and sin as the table holds
-    them), q times ``qscale``, k and v to their page slots; act = relu(proj[:, ucol:])^2."""
+    them), q times ``qscale`` (and ``qtab[position]``), k and v to their page slots; ``bias`` over the
+    q | k | v columns; act = relu(proj[:, ucol:])^2."""
     T, H, G, half = proj.shape[0], heads, kv_heads, rot_dims // 2
     f = proj.float()
+    if bias is not None:
+        f = f[:, :bias.numel()] + bias.float()
     qk = f[:, :(H + G) * dim].reshape(T, H + G, dim).clone()
     if rot_dims:
         c, s = (a[:, None, :] for a in _rot_table(cos_sin, positions, half))
@@ -1061,18 +1095,22 @@ def rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, posit
         act.copy_(relu2(proj[:, ucol:ucol + act.shape[1]]))
     if zero_rows is not None:
         zero_rows[slots < 0] = 0
-    return (qk[:, :H] * qscale).to(proj.dtype)
+    q = qk[:, :H] * qscale
+    return (q if qtab is None else q * qtab[positions.long()][:, None, None]).to(proj.dtype)
 
 
 def latent_expand(cache, block_tables, wk, wv):
     """Keys and values of every head from cached latents: page (s, j) of the block tables [S, nb] becomes
-    page s nb + j of K [S nb, heads, block, dim] and V [S nb, heads, vdim, block]; wk [heads, dim, rank],
-    wv [heads, vdim, rank]."""
+    page s nb + j of K [S nb, heads, block, dim (+ rot)] and V [S nb, heads, vdim, block]; wk [heads, dim,
+    rank], wv [heads, vdim, rank]; the rotated dims behind a latent follow every head's key."""
     (H, d, r), dv = wk.shape, wv.shape[1]
-    c = cache[block_tables.reshape(-1).long()]                       # [pages, block, rank]
+    c = cache[block_tables.reshape(-1).long()]                       # [pages, block, rank (+ rot)]
     P, B = c.shape[:2]
+    kr, c = c[..., r:], c[..., :r].contiguous()
     k = (c.reshape(P * B, r) @ wk.reshape(H * d, r).t()).view(P, B, H, d).transpose(1, 2).contiguous()
     v = (c.reshape(P * B, r) @ wv.reshape(H * dv, r).t()).view(P, B, H, dv).permute(0, 2, 3, 1).contiguous()
+    if kr.shape[-1]:
+        k = torch.cat([k, kr[:, None].expand(P, H, B, kr.shape[-1])], -1).contiguous()
     return k, v
 
 
@@ -1092,7 +1130,9 @@ def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol=0, act=None, q=None,
 
 
 def gate_heads(o, gate, out):
-    """out[t, h dv + i] = o[h, t, i] * sigmoid(gate[t, h dv + i])."""
+    """out[t, h dv + i] = o[h, t, i] * sigmoid(gate[t, h dv + i]), or gate[t, h]."""
     H, T, dv = o.shape
-    out.copy_((o.float().transpose(0, 1).reshape(T, H * dv) * torch.sigmoid(gate.float())).to(out.dtype))
+    g = torch.sigmoid(gate.float())
+    g = g.repeat_interleave(dv, 1) if g.shape[1] == H else g
+    out.copy_((o.float().transpose(0, 1).reshape(T, H * dv) * g).to(out.dtype))
     return out

@@ -11,7 +11,9 @@ paged attention, gated activations with clamps, and top-k routing with softmax s
 on the choice and identity experts; for layers whose mixer and feed-forward read one norm and share
 projections the attention / latent inputs with the feed-forward's activation in one launch, gated
 head outputs, and the scaled residual add with the next norm; chunks, a score soft cap and per-head
-learned sinks in the paged attention.
+learned sinks in the paged attention; scores that fall with the distance, queries that grow with the
+position, projection biases and one gate per head in the paged attention; rotate-half positions, sinks and
+a query latent normed in the same launch for latent attention, whose expanded form takes a rotated part.
 
 Same dispatch rule as the rest of the op library: GPU tensors run the HIP kernel (or raise when the
 extension is missing), CPU tensors the torch reference.  Every kernel takes bf16 or f32 activations
@@ -122,11 +124,32 @@ def retention(qkvg, heads, dim, vdim, cos_sin, rot_dims, decay, state, eps, posi
     return out
 
 
-def latent_kv_write(ckv, rank, norm_w, eps, positions, cos_sin, slots, cache) -> None:
+def latent_kv_write(ckv, rank, norm_w, eps, positions, cos_sin, slots, cache, half: bool = False,
+                    q_src: Optional[torch.Tensor] = None, q_norm: Optional[torch.Tensor] = None,
+                    zero: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """A token's latent (RMS norm, weight ``norm_w``) and its rotated key part (pairs (2i, 2i + 1), with
+    ``half`` (i, i + rot / 2)) into its cache slot.  ``q_src`` [T, n]: the query latent made by the same
+    projection; returns rmsnorm(q_src) * q_norm from the same launch.  ``zero`` [heads, T, rank]: the
+    rows of tokens without a slot (padding) are cleared."""
     ext = _native(ckv)
     if ext is None:
-        return ref.latent_kv_write(ckv, rank, norm_w, eps, positions, cos_sin, slots, cache)
-    ext.latent_kv_write(ckv, int(rank), norm_w, float(eps), positions, cos_sin, slots, cache)
+        return ref.latent_kv_write(ckv, rank, norm_w, eps, positions, cos_sin, slots, cache, half, q_src, q_norm, zero)
+    q_out = None if q_src is None else torch.empty(q_src.shape, dtype=q_src.dtype, device=q_src.device)
+    ext.latent_kv_write(ckv, int(rank), norm_w, float(eps), positions, cos_sin, slots, cache, bool(half), q_src, q_norm, q_out,
+                        zero)
+    return q_out
+
+
+def latent_q_prep(q, heads, dim, rot_dim, positions, cos_sin, scale, half: bool = False) -> torch.Tensor:
+    """Queries of the expanded form (``latent_expand``): q [T, heads (dim + rot_dim)], the last
+    ``rot_dim`` dims of every head rotated (layout as in ``latent_kv_write``), everything times
+    ``scale`` -> [T, heads, dim + rot_dim]."""
+    ext = _native(q)
+    if ext is None:
+        return ref.latent_q_prep(q, heads, dim, rot_dim, positions, cos_sin, scale, half)
+    out = torch.empty((q.shape[0], heads, dim + rot_dim), dtype=q.dtype, device=q.device)
+    ext.latent_q_prep(q, int(heads), int(dim), int(rot_dim), bool(half), positions, cos_sin, float(scale), out)
+    return out
 
 
 LAT_SPLIT_TARGET = 512     # workgroups a small latent-attention grid is split up to (over keys)
@@ -154,13 +177,17 @@ def latent_rows(x: torch.Tensor, rank: int, rot_dim: int, tokens: int, seqs: int
 
 def latent_attention(qa, q, dim, rot_dim, positions, cos_sin, cache, block_tables, qstart, qlen, ctx, tile_seq,
                      tile_tok0, scale, splits: Optional[int] = None, mfma: Optional[bool] = None,
-                     rows: int = LAT_ROWS, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``out``: a prepared output like qa (its padding rows already cleared).  ``mfma`` (GPU, bf16): the matrix-core kernel (default where the shape fits it;
-    ``DLLM_LATENT_MFMA=0`` or ``mfma=False`` keeps the vector-ALU kernel that f32 models run)."""
+                     rows: int = LAT_ROWS, out: Optional[torch.Tensor] = None, half: bool = False,
+                     sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``out``: a prepared output like qa (its padding rows already cleared).  ``mfma`` (GPU, bf16): the
+    matrix-core kernel (default where the shape fits it; ``DLLM_LATENT_MFMA=0`` or ``mfma=False``
+    keeps the vector-ALU kernel that f32 models run).  ``half``: layout of the rotary pairs as in
+    ``latent_kv_write``.  ``sinks`` [heads] f32: one more term of that score per head (not scaled) in the
+    denominator, with no value."""
     ext = _native(qa)
     if ext is None:
         return ref.latent_attention(qa, q, dim, rot_dim, positions, cos_sin, cache, block_tables, qstart, qlen, ctx,
-                                    scale)
+                                    scale, half, sinks)
     if out is None:
         out = torch.zeros_like(qa)
     H, n_entries = qa.shape[0], int(tile_seq.numel())
@@ -174,7 +201,7 @@ def latent_attention(qa, q, dim, rot_dim, positions, cos_sin, cache, block_table
     if mfma is None:
         mfma = os.environ.get("DLLM_LATENT_MFMA", "1") == "1"
     ext.latent_attention(qa, q, int(dim), int(rot_dim), positions, cos_sin, cache, block_tables, qstart, qlen, ctx,
-                         tile_seq, tile_tok0, float(scale), out, sp, po, pml, bool(mfma), int(rows))
+                         tile_seq, tile_tok0, float(scale), out, sp, po, pml, bool(mfma), int(rows), bool(half), sinks)
     return out
 
 
@@ -218,23 +245,24 @@ def dense_gate(ids, wts, E) -> torch.Tensor:
 def resadd_norm(a: torch.Tensor, w_post: torch.Tensor, eps: float, x: torch.Tensor,
                 w_next: Optional[torch.Tensor] = None, x_next: Optional[torch.Tensor] = None,
                 b: Optional[torch.Tensor] = None, wa: Optional[torch.Tensor] = None,
-                wb: Optional[torch.Tensor] = None, depth: Optional[Tuple[torch.Tensor, torch.Tensor, int]] = None
-                ) -> torch.Tensor:
+                wb: Optional[torch.Tensor] = None, depth: Optional[Tuple[torch.Tensor, torch.Tensor, int]] = None,
+                bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """The tail of a sublayer in one launch: ``x += rmsnorm(y) * w_post`` on the f32 stream, where y
     is the sublayer's output ``a`` or, for two mixers side by side, ``(rmsnorm(a) wa + rmsnorm(b) wb) / 2``;
     ``x_next`` (the model dtype) receives ``rmsnorm(x) * w_next``, the next sublayer's input.
     ``depth`` = (X, w, n) ends a layer of a depth-averaged model in the same launch: x is slot n - 1 of
     the f32 stack X, slot n receives ``sum_{j<n} w[j] X[j]`` (as ``depth_mix``) and ``x_next`` is
-    normed from that; returns the slot handed on."""
+    normed from that; returns the slot handed on.  ``bias`` f32 [width] (the sublayer's output bias) is
+    added to y before its norm."""
     ext = _native(a)
     if ext is None:
-        ref.resadd_norm(a, w_post, eps, x, None if depth else w_next, None if depth else x_next, b, wa, wb)
+        ref.resadd_norm(a, w_post, eps, x, None if depth else w_next, None if depth else x_next, b, wa, wb, bias)
         return ref.depth_mix(depth[0], depth[1], depth[2], w_next, eps, x_next) if depth else x
     if depth is None:
-        ext.resadd_norm(a, b, wa, wb, w_post, float(eps), x, w_next, x_next)
+        ext.resadd_norm(a, b, wa, wb, w_post, float(eps), x, w_next, x_next, bias=bias)
         return x
     X, w, n = depth
-    ext.resadd_norm(a, b, wa, wb, w_post, float(eps), x, w_next, x_next, X, w, int(n))
+    ext.resadd_norm(a, b, wa, wb, w_post, float(eps), x, w_next, x_next, X, w, int(n), bias)
     return X[n]
 
 
@@ -316,9 +344,9 @@ def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, ti
                         gate: Optional[torch.Tensor] = None, mfma: bool = False, splits: int = 1, window: int = 0,
                         out_f32: bool = False, keep_first: int = 0, sink: float = 0.0,
                         all_rows: bool = False, out: Optional[torch.Tensor] = None, chunk: int = 0, softcap: float = 0.0,
-                        sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                        sinks: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal softmax attention over paged keys / values of any head widths (f32 scores, online
-    softmax), output times sigmoid(gate).  ``tile_seq`` / ``tile_tok0``: one entry per
+    softmax), output times sigmoid(gate), one logit per entry or per head (gate [T, heads]).  ``tile_seq`` / ``tile_tok0``: one entry per
     ``gqa_tokens_per_tile(heads, kv_heads, mfma)`` new tokens of a sequence.  ``splits`` > 1
     (matrix-core kernel): a row's keys are split over that many workgroups and merged.
     ``window`` > 0: a position sees itself and the ``window - 1`` keys before it (older key tiles are
@@ -331,11 +359,12 @@ def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, ti
     matrix).  ``chunk`` > 0: a position sees the keys of its own chunk of that many positions, counted
     from 0 (older key tiles are not read).  ``softcap`` > 0: scores s become softcap tanh(s / softcap).
     ``sinks`` [heads] f32: one more term of that score per head (neither scaled nor capped) in the
-    denominator, with no value."""
+    denominator, with no value.  ``slopes`` [heads] f32 (not beside a cap): a row at position i loses
+    slopes[head] (i - j) on key j's score."""
     ext = _native(q)
     if ext is None:
         return ref.paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, gate, window, out_f32,
-                                       keep_first, sink, chunk, softcap, sinks, out)
+                                       keep_first, sink, chunk, softcap, sinks, out, slopes)
     dv = v_cache.shape[2]
     if out is None:
         out = (torch.empty if all_rows else torch.zeros)((q.shape[0], q.shape[1] * dv),
@@ -347,7 +376,7 @@ def paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, ti
                            dtype=torch.float32, device=q.device)
     ext.paged_gqa_attention(q, k_cache, v_cache, block_tables, qstart, qlen, ctx, tile_seq, tile_tok0, gate, out,
                             bool(mfma), splits, part, int(window), int(keep_first), float(sink), int(chunk),
-                            float(softcap), sinks)
+                            float(softcap), sinks, slopes)
     return out
 
 
@@ -586,16 +615,19 @@ def proj_norm_prep(proj, heads, kv_heads, dim, vdim, qnorm_w, knorm_w, cos_sin, 
     return q
 
 
+GLU_MODES = {"swiglu": 0, "clamped": 1, "gelu_tanh": 2}
+
+
 def glu_act(gu: torch.Tensor, bias: Optional[torch.Tensor] = None, mode: str = "swiglu", limit: float = 0.0,
             alpha: float = 1.0) -> torch.Tensor:
     """Gated activation of gu [T, 2 ff] (gate columns, then up columns; ``bias`` f32 over the same
-    columns) -> [T, ff]: "swiglu" silu(g) u, or "clamped": g <- min(g, limit), u <- clamp(u, -limit,
-    limit), g sigmoid(alpha g) (u + 1)."""
+    columns) -> [T, ff]: "swiglu" silu(g) u, "clamped": g <- min(g, limit), u <- clamp(u, -limit,
+    limit), g sigmoid(alpha g) (u + 1), or "gelu_tanh": gelu(g) u in its tanh form."""
     ext = _native(gu)
     if ext is None:
         return ref.glu_act(gu, bias, mode, limit, alpha)
     y = torch.empty((gu.shape[0], gu.shape[1] // 2), dtype=gu.dtype, device=gu.device)
-    ext.glu_act(gu, bias, 0 if mode == "swiglu" else 1, float(limit), float(alpha), y)
+    ext.glu_act(gu, bias, GLU_MODES[mode], float(limit), float(alpha), y)
     return y
 
 
@@ -615,21 +647,23 @@ def scaled_resadd_rms(x: torch.Tensor, eps: float, y: Optional[torch.Tensor] = N
 
 
 def rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, positions, slots, k_cache, v_cache, ucol: int = 0,
-              act: Optional[torch.Tensor] = None, zero_rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+              act: Optional[torch.Tensor] = None, zero_rows: Optional[torch.Tensor] = None,
+              bias: Optional[torch.Tensor] = None, qtab: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention inputs without a q / k norm: proj [T, q | k | v | ...]; rotate-half positions on the
     first ``rot_dims`` dims of every q and k head (cos and sin as the table holds them), q times
     ``qscale``; k and v to their page slots (k_cache [blocks, kv_heads, block, dim], v_cache [blocks,
     kv_heads, vdim, block]).  ``act`` [T, ff] (may be columns of a wider matrix) receives
     relu(proj[:, ucol : ucol + ff])^2, the activation of a feed-forward whose up projection is part of
     proj.  ``zero_rows`` [T, n]: the rows of tokens without a slot (padding) are cleared in the same
-    launch.  Returns q [T, heads, dim]."""
+    launch.  ``bias`` (f32 over the q | k | v columns) is added ahead of everything; ``qtab`` (f32, one
+    number per position): q is also multiplied by its position's.  Returns q [T, heads, dim]."""
     ext = _native(proj)
     if ext is None:
         return ref.rope_prep(proj, heads, kv_heads, dim, vdim, cos_sin, rot_dims, qscale, positions, slots, k_cache, v_cache,
-                             ucol, act, zero_rows)
+                             ucol, act, zero_rows, bias, qtab)
     q = torch.empty((proj.shape[0], heads, dim), dtype=proj.dtype, device=proj.device)     # every row is written
     ext.rope_prep(proj, int(heads), int(kv_heads), int(dim), int(vdim), cos_sin, int(rot_dims), float(qscale), positions,
-                  slots, k_cache, v_cache, q, int(ucol), act, zero_rows)
+                  slots, k_cache, v_cache, q, int(ucol), act, zero_rows, bias, qtab)
     return q
 
 
@@ -637,34 +671,37 @@ LATENT_EXPAND_MIN = 32                 # average new tokens per sequence from wh
 LATENT_EXPAND_BYTES = 2 << 30          # ... and the most bytes of expanded keys and values
 
 
-def latent_expand_wanted(cache: torch.Tensor, heads: int, dim: int, vdim: int, tokens: int, seqs: int, blocks: int) -> bool:
+def latent_expand_wanted(cache: torch.Tensor, heads: int, dim: int, vdim: int, tokens: int, seqs: int, blocks: int,
+                         rot_dim: int = 0) -> bool:
     """Whether a step of prompt portions makes the keys and values of every head from the latents it
-    reads and runs the grouped-query kernel on them (dim + vdim products per key and head) instead of
-    attention on the latents themselves (2 rank products): worth the extra projection when enough new
-    tokens read each latent."""
-    if tokens < LATENT_EXPAND_MIN * seqs or dim > 256 or vdim > 256 or dim + vdim > 2 * cache.shape[2]:
+    reads and runs the grouped-query kernel on them (dim + rot_dim + vdim products per key and head)
+    instead of attention on the latents themselves (2 rank + rot_dim products): worth the extra
+    projection when enough new tokens read each latent."""
+    kd = dim + rot_dim
+    if tokens < LATENT_EXPAND_MIN * seqs or kd > 256 or vdim > 256 or dim + vdim > 2 * (cache.shape[2] - rot_dim):
         return False
-    if blocks * cache.shape[1] * heads * (dim + vdim) * cache.element_size() > LATENT_EXPAND_BYTES:
+    if blocks * cache.shape[1] * heads * (kd + vdim) * cache.element_size() > LATENT_EXPAND_BYTES:
         return False
     if cache.is_cuda and cache.dtype == torch.bfloat16:      # the matrix-core attention or none
         ext = _native(cache)
-        return bool(ext.gqa_mfma_ok(False, heads, heads, dim, vdim, cache.shape[1]))
+        return bool(ext.gqa_mfma_ok(False, heads, heads, kd, vdim, cache.shape[1]))
     return True
 
 
 def latent_expand(cache: torch.Tensor, block_tables: torch.Tensor, ctx: torch.Tensor, wk: torch.Tensor,
                   wv: torch.Tensor) -> Tuple[torch.Tensor, torch.Tensor, torch.Tensor]:
-    """Keys and values of every head from the cached latents (cache [blocks, 16, rank]) that the sequences'
-    block tables [S, nb] name: K [S nb, heads, 16, dim], V [S nb, heads, vdim, 16] and their block tables,
-    for ``paged_gqa_attention``.  wk [heads, dim, rank], wv [heads, vdim, rank].  Pages past a sequence's
-    context hold nothing meaningful."""
+    """Keys and values of every head from the cached latents (cache [blocks, 16, rank + rot]) that the sequences'
+    block tables [S, nb] name: K [S nb, heads, 16, dim + rot] (a latent's rotated part behind every head's
+    key), V [S nb, heads, vdim, 16] and their block tables, for ``paged_gqa_attention``.  wk [heads, dim,
+    rank], wv [heads, vdim, rank].  Pages past a sequence's context hold nothing meaningful."""
     S, nb = block_tables.shape
     (H, d, r), dv = wk.shape, wv.shape[1]
     table = torch.arange(S * nb, dtype=torch.int32, device=cache.device).view(S, nb)
     ext = _native(cache)
-    if ext is None or cache.dtype != torch.bfloat16 or not ext.latent_expand_ok(r, d, dv):
+    rot = cache.shape[2] - r
+    if ext is None or cache.dtype != torch.bfloat16 or not ext.latent_expand_ok(r, d, dv, rot):
         return ref.latent_expand(cache, block_tables, wk, wv) + (table,)      # vendor GEMMs
-    k = torch.empty((S * nb, H, 16, d), dtype=cache.dtype, device=cache.device)
+    k = torch.empty((S * nb, H, 16, d + rot), dtype=cache.dtype, device=cache.device)
     v = torch.empty((S * nb, H, dv, 16), dtype=cache.dtype, device=cache.device)
     ext.latent_expand(cache, block_tables, ctx, wk, wv, k, v)
     return k, v, table
@@ -684,7 +721,7 @@ def latent_prep(proj, ccol, norm_w, eps, slots, cache, ucol: int = 0, act: Optio
 
 def gate_heads(o: torch.Tensor, gate: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
     """out[t, h vdim + i] = o[h, t, i] * sigmoid(gate[t, h vdim + i]) for head-major outputs o [heads, T,
-    vdim]; ``gate`` and ``out`` may be columns of wider matrices."""
+    vdim], or gate[t, h] for a gate [T, heads]; ``gate`` and ``out`` may be columns of wider matrices."""
     ext = _native(o)
     if ext is None:
         return ref.gate_heads(o, gate, out)
