@@ -115,7 +115,8 @@ def test_retention(dt, case, H, d, dv, rot, chunked):
 @pytest.mark.parametrize("splits", [1, 3, 16])
 @pytest.mark.parametrize("mfma", [False, True, 32])
 @pytest.mark.parametrize("H,dim,rot,rank", [(8, 32, 16, 96), (3, 16, 8, 40), (20, 32, 16, 128), (1, 8, 64, 512), (2, 8, 6, 70)])
-def test_latent_attention(dt, case, H, dim, rot, rank, splits, mfma):
+@pytest.mark.parametrize("half", [False, True])      # rotary pairs (i, i + rot / 2), and a sink per head
+def test_latent_attention(dt, case, H, dim, rot, rank, splits, mfma, half):
     if mfma and dt != torch.bfloat16:
         pytest.skip("the matrix-core kernel serves bf16 models")
     wg_rows = 32 if mfma == 32 else 16
@@ -139,8 +140,8 @@ def test_latent_attention(dt, case, H, dim, rot, rank, splits, mfma):
             continue
         ckv = torch.randn(len(ps), rank + rot + 5, device=DEV).to(dt)[:, 5:]
         wn = torch.rand(rank, device=DEV) + 0.5
-        seqmix.latent_kv_write(ckv, rank, wn, 1e-6, i32(ps), table, i32(sl), cache1)
-        ref.latent_kv_write(ckv, rank, wn, 1e-6, i32(ps), table, i32(sl), cache2)
+        seqmix.latent_kv_write(ckv, rank, wn, 1e-6, i32(ps), table, i32(sl), cache1, half)
+        ref.latent_kv_write(ckv, rank, wn, 1e-6, i32(ps), table, i32(sl), cache2, half)
     torch.testing.assert_close(cache1.float(), cache2.float(), **tol(dt))
     qa = (torch.randn(H, T, rank, device=DEV) * 0.3).to(dt)
     q = torch.randn(T, H * (dim + rot), device=DEV).to(dt)
@@ -148,9 +149,38 @@ def test_latent_attention(dt, case, H, dim, rot, rank, splits, mfma):
     meta = AttnMeta(slots=None, block_tables=perm, qstart=qstart, qlen=qlen, ctx=ctx, tile_seq=None, tile_tok0=None,
                     last_idx=None, host_qlen=qlens)
     ts, tt = meta.latent_tiles(H, DEV, wg_rows)
-    o1 = seqmix.latent_attention(qa, q, dim, rot, pos, table, cache2, perm, qstart, qlen, ctx, ts, tt, 0.2, splits=splits, mfma=bool(mfma), rows=wg_rows)
-    o2 = ref.latent_attention(qa, q, dim, rot, pos, table, cache2, perm, qstart, qlen, ctx, 0.2)
+    o1 = seqmix.latent_attention(qa, q, dim, rot, pos, table, cache2, perm, qstart, qlen, ctx, ts, tt, 0.2, splits=splits, mfma=bool(mfma),
+                                 rows=wg_rows, half=half, sinks=torch.linspace(-1.0, 4.0, H, device=DEV) if half else None)
+    o2 = ref.latent_attention(qa, q, dim, rot, pos, table, cache2, perm, qstart, qlen, ctx, 0.2, half,
+                              torch.linspace(-1.0, 4.0, H, device=DEV) if half else None)
     torch.testing.assert_close(o1.float(), o2.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("half", [False, True])
+@pytest.mark.parametrize("T,H,dim,rot,rank,qr", [(1, 3, 8, 2, 24, 10), (37, 4, 16, 12, 64, 200), (9, 2, 40, 0, 100, 64), (130, 5, 24, 64, 512, 72)])
+def test_latent_inputs(dt, half, T, H, dim, rot, rank, qr):
+    """Both latents' norms, the rotated key part and the padding rows in one launch; the rotated, scaled
+    queries of the expanded form; one gate per head on head-major outputs."""
+    torch.manual_seed(37)
+    down = torch.randn(T, qr + rank + rot + H, device=DEV).to(dt)
+    wq, wn = torch.rand(qr, device=DEV) + 0.5, torch.rand(rank, device=DEV) + 0.5
+    table = ops.rope_cos_sin(256, max(rot, 2), 300.0, DEV)
+    pos = torch.randint(0, 256, (T,), device=DEV, dtype=torch.int32)
+    nb = (T + 15) // 16 + 1
+    slots = torch.randperm(nb * 16, device=DEV)[:T].to(torch.int32)
+    slots[0] = -1
+    q = torch.randn(T, H * (dim + rot) + 3, device=DEV).to(dt)
+    o = torch.randn(H, T, dim, device=DEV).to(dt)
+    got = []
+    for m in (seqmix, ref):
+        cache, z = torch.zeros(nb, 16, rank + rot, device=DEV, dtype=dt), torch.full((H, T, rank), 7.0, device=DEV).to(dt)
+        cq = m.latent_kv_write(down[:, qr:qr + rank + rot], rank, wn, 1e-5, pos, table, slots, cache, half, down[:, :qr], wq, z)
+        assert float(z[:, 0].float().abs().sum()) == 0.0 and bool((z[:, 1:] == 7.0).all())
+        g = m.gate_heads(o, down[:, qr + rank + rot:], torch.empty(T, H * dim, device=DEV, dtype=dt))
+        got.append((cache, cq, m.latent_q_prep(q, H, dim, rot, pos, table, 0.4, half), g))
+    for a, b in zip(*got):
+        torch.testing.assert_close(a.float(), b.float(), **tol(dt))
 
 
 @pytest.mark.parametrize("dt", DTYPES)
@@ -183,11 +213,13 @@ def test_moe_relu2_grouped(T):
 # ----------------------------------------------------------------------------- pre/post-norm tails, depth average, GELU
 
 @pytest.mark.parametrize("dt", DTYPES)
-@pytest.mark.parametrize("n", [24, 200, 1032])
+@pytest.mark.parametrize("n", [24, 200, 1032, 5000])
 @pytest.mark.parametrize("pair", [False, True])
-def test_resadd_norm(dt, n, pair):
+@pytest.mark.parametrize("aligned", [False, True])      # rows of whole vectors stay in registers
+def test_resadd_norm(dt, n, pair, aligned):
     torch.manual_seed(2)
-    a = torch.randn(9, n + 5, device=DEV).to(dt)[:, 2:2 + n]
+    a = torch.randn(9, n + (8 if aligned else 5), device=DEV).to(dt)[:, :n] if aligned else torch.randn(9, n + 5, device=DEV).to(dt)[:, 2:2 + n]
+    bias = torch.randn(n, device=DEV) if n != 200 else None
     b = torch.randn(9, n, device=DEV).to(dt) if pair else None
     wa, wb, wp, wn = (torch.randn(n, device=DEV) for _ in range(4))
     for w_next in (wn, None):
@@ -195,10 +227,13 @@ def test_resadd_norm(dt, n, pair):
         x2 = x1.clone()
         h1, h2 = torch.empty(9, n, device=DEV, dtype=dt), torch.empty(9, n, device=DEV, dtype=dt)
         kw = dict(b=b, wa=wa, wb=wb) if pair else {}
-        seqmix.resadd_norm(a, wp, 1e-5, x1, w_next, h1, **kw)
-        ref.resadd_norm(a, wp, 1e-5, x2, w_next, h2, **kw)
+        seqmix.resadd_norm(a, wp, 1e-5, x1, w_next, h1, bias=bias, **kw)
+        ref.resadd_norm(a, wp, 1e-5, x2, w_next, h2, bias=bias, **kw)
         torch.testing.assert_close(x1, x2, atol=2e-5, rtol=2e-5)
         torch.testing.assert_close(h1.float(), h2.float(), **tol(dt))
+    seqmix.resadd_norm(a, wp, 1e-5, x1, bias=bias, **kw)      # the update alone
+    ref.resadd_norm(a, wp, 1e-5, x2, bias=bias, **kw)
+    torch.testing.assert_close(x1, x2, atol=2e-5, rtol=2e-5)
 
 
 @pytest.mark.parametrize("dt", DTYPES)
@@ -547,7 +582,8 @@ def test_glu_act(dt):
     for ff in (70, 72, 1024):      # 72, 1024: rows of whole 16-byte vectors
         gu = (torch.randn(33, 2 * ff + 8, device=DEV) * 3).to(dt)[:, :2 * ff]
         bias = torch.randn(2 * ff, device=DEV)
-        for kw in (dict(), dict(bias=bias), dict(bias=bias, mode="clamped", limit=1.5, alpha=1.702), dict(mode="clamped", limit=0.3, alpha=1.0)):
+        for kw in (dict(), dict(bias=bias), dict(bias=bias, mode="clamped", limit=1.5, alpha=1.702), dict(mode="clamped", limit=0.3, alpha=1.0),
+                   dict(mode="gelu_tanh"), dict(bias=bias * 4, mode="gelu_tanh")):
             torch.testing.assert_close(seqmix.glu_act(gu, **kw).float(), ref.glu_act(gu, **kw).float(), **tol(dt))
 
 
@@ -704,14 +740,16 @@ def test_latent_prep_and_gate(dt, T, H, d, dv, rank, ff):
 
 @pytest.mark.parametrize("dt", DTYPES)
 @pytest.mark.parametrize("ctxs", [[1], [16, 5], [130, 64, 65], [300]])
-@pytest.mark.parametrize("H,d,dv,rank", [(2, 8, 5, 32), (3, 40, 72, 64), (4, 64, 64, 96), (2, 128, 128, 512), (1, 136, 200, 160), (2, 12, 4, 20)])
-def test_latent_expand(dt, ctxs, H, d, dv, rank):
-    """Keys and values from paged latents (pages out of order), then attention on them against attention
-    on the latents."""
+@pytest.mark.parametrize("H,d,dv,rank,rot", [(2, 8, 5, 32, 0), (3, 40, 72, 64, 0), (4, 64, 64, 96, 0), (2, 128, 128, 512, 0),
+                                             (1, 136, 200, 160, 0), (2, 12, 4, 20, 0), (3, 40, 72, 64, 8), (2, 64, 64, 96, 32),
+                                             (2, 128, 128, 512, 64), (2, 16, 24, 32, 6), (1, 12, 4, 20, 2)])
+def test_latent_expand(dt, ctxs, H, d, dv, rank, rot):
+    """Keys and values from paged latents (pages out of order; a rotated part shared by all heads), then
+    attention with a sink per head on them against attention on the latents."""
     torch.manual_seed(34)
     S, nb = len(ctxs), max((c + 15) // 16 for c in ctxs)
     bt = torch.randperm(S * nb + 2, device=DEV)[:S * nb].to(torch.int32).view(S, nb)
-    cache = torch.randn(S * nb + 2, 16, rank, device=DEV).to(dt)
+    cache = torch.randn(S * nb + 2, 16, rank + rot, device=DEV).to(dt)
     wk, wv = (torch.randn(H, d, rank, device=DEV) / rank ** 0.5).to(dt), (torch.randn(H, dv, rank, device=DEV) / rank ** 0.5).to(dt)
     k1, v1, table = seqmix.latent_expand(cache, bt, i32(ctxs), wk, wv)
     k2, v2 = ref.latent_expand(cache.float(), bt, wk.float(), wv.float())
@@ -720,19 +758,57 @@ def test_latent_expand(dt, ctxs, H, d, dv, rank):
         assert table[s].tolist() == list(range(s * nb, (s + 1) * nb))
         torch.testing.assert_close(k1[s * nb:s * nb + n].float(), k2[s * nb:s * nb + n], **tol(dt))
         torch.testing.assert_close(v1[s * nb:s * nb + n].float(), v2[s * nb:s * nb + n], **tol(dt))
-    if not seqmix.latent_expand_wanted(cache, H, d, dv, 1 << 20, S, S * nb):
+    if not seqmix.latent_expand_wanted(cache, H, d, dv, 1 << 20, S, S * nb, rot):
         return
     from distributed_llm_amd.models.llama import AttnMeta
     qlens = [min(c, 3) for c in ctxs]
     T, qstart, qlen, ctx, rows, pos = batch(qlens, [c - n for c, n in zip(ctxs, qlens)])
-    q = torch.randn(T, H, d, device=DEV).to(dt)
+    tab, sinks = ops.rope_cos_sin(512, max(rot, 2), 100.0, DEV), torch.linspace(0.0, 5.0, H, device=DEV) if rot else None
+    raw = torch.randn(T, H * (d + rot), device=DEV).to(dt)
+    q = seqmix.latent_q_prep(raw, H, d, rot, pos, tab, 1.0, True)
     meta = AttnMeta(slots=None, block_tables=bt, qstart=qstart, qlen=qlen, ctx=ctx, tile_seq=None, tile_tok0=None, last_idx=None,
                     host_qlen=qlens)
-    mfma = seqmix.gqa_use_mfma(q, H, H, d, dv, 16)
+    mfma = seqmix.gqa_use_mfma(q, H, H, d + rot, dv, 16)
     ts, tt = meta.latent_tiles(1, DEV, seqmix.gqa_tokens_per_tile(H, H, mfma))
-    got = seqmix.paged_gqa_attention(q, k1, v1, table, qstart, qlen, ctx, ts, tt, None, mfma, 1).float().view(T, H, dv)
-    qa = torch.matmul(q.float().transpose(0, 1), wk.float())
-    lat = ref.latent_attention(qa, q.float().view(T, H * d), d, 0, pos, torch.zeros(512, 2, device=DEV), cache.float(), bt, qstart,
-                               qlen, ctx, 1.0)
+    got = seqmix.paged_gqa_attention(q, k1, v1, table, qstart, qlen, ctx, ts, tt, None, mfma, 1, sinks=sinks).float().view(T, H, dv)
+    qa = torch.matmul(raw.float().view(T, H, d + rot)[..., :d].transpose(0, 1), wk.float())
+    lat = ref.latent_attention(qa, raw.float(), d, rot, pos, tab, cache.float(), bt, qstart, qlen, ctx, 1.0, True, sinks)
     want = torch.matmul(lat, wv.float().transpose(1, 2)).transpose(0, 1)
     torch.testing.assert_close(got, want, **(dict(atol=6e-2, rtol=6e-2) if dt == torch.bfloat16 else dict(atol=1e-4, rtol=1e-4)))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("case", CASES + [([40, 3], [90, 130]), ([1, 1], [300, 77]), ([150], [170])])
+@pytest.mark.parametrize("H,G,d,dv,win", [(4, 2, 16, 8, 5), (6, 2, 88, 56, 64), (3, 3, 40, 72, 1), (8, 1, 64, 64, 100), (7, 1, 56, 88, 0),
+                                          (2, 1, 136, 200, 48), (4, 4, 96, 80, 65), (5, 5, 12, 1, 17)])
+def test_biased_attention_kernels(dt, case, H, G, d, dv, win):
+    """Prep (biases, queries times a number of their position, pages, padding rows), then windowed attention
+    whose scores fall with the distance, one gate per head, in both kernel forms and every split count."""
+    from distributed_llm_amd.models.llama import AttnMeta
+    torch.manual_seed(38)
+    T, qstart, qlen, ctx, pos, bt, kc, vc, slots = _pages(case, G, d, dv, dt)
+    cols = (H + G) * d + G * dv
+    proj = torch.randn(T, (cols + H + 7) // 8 * 8 + (0 if d % 8 == 0 else 3), device=DEV).to(dt)
+    bias, qtab = torch.randn(cols, device=DEV), 1.0 + torch.rand(512, device=DEV)
+    table = ops.rope_cos_sin(512, 2, 100.0, DEV)
+    kc1, vc1, kc2, vc2 = kc.clone(), vc.clone(), kc.clone(), vc.clone()
+    pad = slots.clone()
+    pad[T // 2:] = -1
+    z1, z2 = (torch.full((T, H * dv), 7.0, device=DEV).to(dt) for _ in range(2))
+    for sl, z in ((pad, (z1, z2)), (slots, (None, None))):
+        q1 = seqmix.rope_prep(proj, H, G, d, dv, table, 0, 0.3, pos, sl, kc1, vc1, zero_rows=z[0], bias=bias, qtab=qtab)
+        q2 = ref.rope_prep(proj, H, G, d, dv, table, 0, 0.3, pos, sl, kc2, vc2, zero_rows=z[1], bias=bias, qtab=qtab)
+        for a, b in ((q1, q2), (kc1, kc2), (vc1, vc2), (z1, z2)):
+            torch.testing.assert_close(a.float(), b.float(), **tol(dt))
+    slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / H) for h in range(H)], device=DEV)
+    gate = proj[:, cols:cols + H]
+    want = ref.paged_gqa_attention(q2, kc2, vc2, bt, qstart, qlen, ctx, gate, win, slopes=slopes).float()
+    meta = AttnMeta(slots=None, block_tables=bt, qstart=qstart, qlen=qlen, ctx=ctx, tile_seq=None, tile_tok0=None,
+                    last_idx=None, host_qlen=case[0])
+    for mfma in [False] + ([True] if seqmix.gqa_use_mfma(q2, H, G, d, dv, 16) else []):
+        ts, tt = meta.latent_tiles(1, DEV, seqmix.gqa_tokens_per_tile(H, G, mfma))
+        for splits in ((1, 2, 7) if mfma else (1,)):
+            got = seqmix.paged_gqa_attention(q2, kc2, vc2, bt, qstart, qlen, ctx, ts, tt, gate, mfma, splits, window=win, slopes=slopes)
+            torch.testing.assert_close(got.float(), want, **tol(dt))
+    with pytest.raises(RuntimeError):      # a cap on the scores has no form beside slopes
+        seqmix.paged_gqa_attention(q2, kc2, vc2, bt, qstart, qlen, ctx, ts, tt, None, mfma, 1, softcap=3.0, slopes=slopes)
