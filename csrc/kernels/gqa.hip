@@ -506,9 +506,9 @@ constexpr int GM_ROWS = 64, GM_KT = 64, GM_BS = 16;   // rows per workgroup, key
 typedef float f32x2v __attribute__((ext_vector_type(2)));
 typedef __bf16 bf16x2v __attribute__((ext_vector_type(2)));
 
-// SZ >= max(d, dv) in {64, 128, 256}: d is walked in SZ / 32 MFMA steps, dv in SZ / 16 column blocks;
-// steps and blocks past the real widths multiply zeros (a branch around each would drain the matrix
-// pipe).  d % 8 == 0 (16-byte key rows).
+// KD >= d, VD >= dv: d is walked in KD / 32 MFMA steps, dv in VD / 16 column blocks; steps and blocks past
+// the real widths multiply zeros (a branch around each would drain the matrix pipe).  d % 8 == 0
+// (16-byte key rows).
 // CAP: the scores are capped at 0 < cap <= CAP_MAX, so exp(score) and its sums stay inside f32 and the
 // softmax needs no running maximum (it stays 0) and no rescaling.
 // MFMA operand layout (16x16x32): with lr = lane & 15, g4 = lane >> 4, A holds row lr, contraction
@@ -516,7 +516,7 @@ typedef __bf16 bf16x2v __attribute__((ext_vector_type(2)));
 // 4 g4 .. 4 g4 + 3 of column lr.
 constexpr float CAP_MAX = 64.f;
 // DIST: the scores fall with the distance (`slopes`); the score accumulators start at -slope * distance.
-template <int SZ, bool CAP, bool DIST>
+template <int KD, int VD, bool CAP, bool DIST>
 __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restrict__ q, const u16* __restrict__ kc,
                                                              const u16* __restrict__ vc, const int* __restrict__ bt,
                                                              int bt_ld, const int* __restrict__ qstart,
@@ -528,8 +528,8 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
                                                              float* __restrict__ out32, int keep, float sink, int chunk,
                                                              float cap, const float* __restrict__ sinks, long ldo,
                                                              const float* __restrict__ slopes, int ghead) {
-  constexpr int DS = SZ / 32, VB = SZ / 16, NKB = GM_KT / 16;
-  constexpr int KSTR = SZ + 8, VSTR = GM_KT + 8, PSTR = GM_KT + 8;
+  constexpr int DS = KD / 32, VB = VD / 16, NKB = GM_KT / 16;
+  constexpr int KSTR = KD + 8, VSTR = GM_KT + 8, PSTR = GM_KT + 8;
   extern __shared__ __attribute__((aligned(16))) unsigned char smraw[];
   const int tile = gridDim.x - 1 - blockIdx.x;   // later tokens see more keys: start with the long rows
   const int s = tile_seq[tile];
@@ -540,8 +540,8 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
   const int nq = min(TQ, n - tok0), nrows = nq * R;
   const int q0 = qstart[s], p0 = ctx[s] - n;
   u16* ksh = reinterpret_cast<u16*>(smraw);          // [KT][KSTR]
-  u16* vtr = ksh + GM_KT * KSTR;                      // [SZ][VSTR]: values transposed, [dim][key]
-  u16* pw = vtr + SZ * VSTR;                          // [4 waves][hi | lo][16][PSTR]
+  u16* vtr = ksh + GM_KT * KSTR;                      // [VD][VSTR]: values transposed, [dim][key]
+  u16* pw = vtr + VD * VSTR;                          // [4 waves][hi | lo][16][PSTR]
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);   // in a scalar register: the branches on it are scalar
   const int lr = lane & 15, g4 = lane >> 4;
@@ -587,25 +587,29 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
   const float capl = 1.44269504f * cap;
   const int last = p0 + tok0 + nq - 1;   // the newest key any row sees
   const int* btr = bt + (long)s * bt_ld;
-  constexpr int KCH = SZ / 8;            // 16-byte chunks of a staged key row
-  constexpr int NF = SZ / 32;            // chunks of K, and of V, a thread moves per tile
+  constexpr int KCH = KD / 8;            // 16-byte chunks of a staged key row
+  constexpr int NFK = KD / 32, NFV = VD / 32;      // chunks of K, and of V, a thread moves per tile
   // Score block kb, column lr stands for key 4 lr + kb of the tile (K rows are staged in that order),
   // so a lane's four blocks are four neighbouring keys and its weights leave as 8-byte vectors.
-  uint4 pk_[NF], pv_[NF];
+  uint4 pk_[NFK], pv_[NFV];
   // A thread moves the same (key, chunk) and (dim, page, half) of every tile (tiles start at multiples
   // of 64 keys), so only the page ids change from tile to tile: offsets inside a page are kept.
-  long koff[NF], voff[NF];
-  int kkey[NF], vpg[NF];
-  bool kon[NF], von[NF];
+  long koff[NFK], voff[NFV];
+  int kkey[NFK], vpg[NFV];
+  bool kon[NFK], von[NFV];
   const long kpage = (long)G * GM_BS * d, vpage = (long)GV * dv * GM_BS;
   const int gv = g / (G / GV);
 #pragma unroll
-  for (int f = 0; f < NF; ++f) {
+  for (int f = 0; f < NFK; ++f) {
     const int e = tid + 256 * f;
     const int kk = e / KCH, c = (e % KCH) * 8;
     kkey[f] = kk;
     kon[f] = c < d;
     koff[f] = ((long)g * GM_BS + (kk & 15)) * d + c;
+  }
+#pragma unroll
+  for (int f = 0; f < NFV; ++f) {
+    const int e = tid + 256 * f;
     const int j = e / (GM_KT / 8), cc = e % (GM_KT / 8);
     vpg[f] = cc >> 1;
     von[f] = j < dv;
@@ -615,9 +619,12 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     const int nk = min(GM_KT, last + 1 - k0);
     const int* pg = btr + (k0 >> 4);
 #pragma unroll
-    for (int f = 0; f < NF; ++f) {
+    for (int f = 0; f < NFK; ++f) {
       pk_[f] = make_uint4(0u, 0u, 0u, 0u);
       if (kon[f] && kkey[f] < nk) pk_[f] = *reinterpret_cast<const uint4*>(kc + pg[kkey[f] >> 4] * kpage + koff[f]);
+    }
+#pragma unroll
+    for (int f = 0; f < NFV; ++f) {
       pv_[f] = make_uint4(0u, 0u, 0u, 0u);
       if (von[f] && 16 * vpg[f] < nk) pv_[f] = *reinterpret_cast<const uint4*>(vc + pg[vpg[f]] * vpage + voff[f]);
     }
@@ -637,10 +644,14 @@ __global__ void __launch_bounds__(256) paged_gqa_mfma_kernel(const u16* __restri
     const int k0 = tile_k0(vt);
     __syncthreads();   // the previous tile is consumed
 #pragma unroll
-    for (int f = 0; f < NF; ++f) {
+    for (int f = 0; f < NFK; ++f) {
       const int e = tid + 256 * f;
       const int kk = e / KCH, c = (e % KCH) * 8;
       *reinterpret_cast<uint4*>(ksh + (16 * (kk & 3) + (kk >> 2)) * KSTR + c) = pk_[f];
+    }
+#pragma unroll
+    for (int f = 0; f < NFV; ++f) {
+      const int e = tid + 256 * f;
       const int j = e / (GM_KT / 8), cc = e % (GM_KT / 8);
       *reinterpret_cast<uint4*>(vtr + j * VSTR + 8 * cc) = pv_[f];
     }
@@ -830,7 +841,7 @@ __global__ void __launch_bounds__(256) gqa_combine_kernel(const float* __restric
   }
 }
 
-long gqa_mfma_lds(int SZ) { return 2L * (GM_KT * (SZ + 8) + (long)SZ * (GM_KT + 8) + 4L * 2 * 16 * (GM_KT + 8)); }
+long gqa_mfma_lds(int KD, int VD) { return 2L * (GM_KT * (KD + 8) + (long)VD * (GM_KT + 8) + 4L * 2 * 16 * (GM_KT + 8)); }
 
 long gqa_lds(int d, int dv, int KT) { return 4L * (GA_ROWS * d + (long)KT * (d | 1) + (long)KT * dv + GA_ROWS * 64); }
 
@@ -910,27 +921,33 @@ extern "C" int dllm_paged_gqa(const void* q, const void* kc, const void* vc, int
   float* out32 = out_f32 ? (float*)out : nullptr;
   if (mfma) {
     if (!dllm_gqa_mfma_ok(f32, H, G, d, dv, BSZ)) return -1;
-    const int sz = d > dv ? d : dv;
     if (splits < 1 || (splits > 1 && !part)) return -1;
     const dim3 grid(n_tiles, G, splits);
     const int TQ = dllm_gqa_tile_tokens(H, G, 1);
     float* pp = splits > 1 ? part : nullptr;
-#define GQM(SZ, CAP, DIST)                                                                                               \
+#define GQM(KD, VD, CAP, DIST)                                                                                           \
   do {                                                                                                                   \
-    const long lds = gqa_mfma_lds(SZ);                                                                                   \
-    ENSURE_LDS((paged_gqa_mfma_kernel<SZ, CAP, DIST>), lds);                                                             \
-    hipLaunchKernelGGL((paged_gqa_mfma_kernel<SZ, CAP, DIST>), grid, dim3(256), lds, st, (const u16*)q, (const u16*)kc,  \
+    const long lds = gqa_mfma_lds(KD, VD);                                                                               \
+    ENSURE_LDS((paged_gqa_mfma_kernel<KD, VD, CAP, DIST>), lds);                                                         \
+    hipLaunchKernelGGL((paged_gqa_mfma_kernel<KD, VD, CAP, DIST>), grid, dim3(256), lds, st, (const u16*)q, (const u16*)kc, \
                        (const u16*)vc, bt, bt_ld, qstart, qlen, ctx, tile_seq, tile_tok0, (const u16*)gate, ldg,         \
                        (u16*)out, H, G, d, dv, TQ, splits, pp, win, GV, out32, keep, sink, chunk, cap, sinks, ldo,       \
                        slopes, ghead);                                                                                   \
   } while (0)
-    if (cap > 0.f && cap <= CAP_MAX) {
-      if (sz <= 64) GQM(64, true, false); else if (sz <= 128) GQM(128, true, false); else GQM(256, true, false);
-    } else if (slopes) {
-      if (sz <= 64) GQM(64, false, true); else if (sz <= 128) GQM(128, false, true); else GQM(256, false, true);
-    } else {
-      if (sz <= 64) GQM(64, false, false); else if (sz <= 128) GQM(128, false, false); else GQM(256, false, false);
-    }
+    // keys wider than the values (latent attention on expanded keys: unrotated and rotated parts) have forms
+    // of their own, so that the extra dims do not widen the value side
+#define GQZ(CAP, DIST)                                                                                                   \
+  do {                                                                                                                   \
+    if (d <= 64 && dv <= 64) GQM(64, 64, CAP, DIST);                                                                     \
+    else if (d <= 96 && dv <= 64) GQM(96, 64, CAP, DIST);                                                                \
+    else if (d <= 128 && dv <= 128) GQM(128, 128, CAP, DIST);                                                            \
+    else if (d <= 192 && dv <= 128) GQM(192, 128, CAP, DIST);                                                            \
+    else GQM(256, 256, CAP, DIST);                                                                                       \
+  } while (0)
+    if (cap > 0.f && cap <= CAP_MAX) GQZ(true, false);
+    else if (slopes) GQZ(false, true);
+    else GQZ(false, false);
+#undef GQZ
 #undef GQM
     if (pp) {
       const int rows = (TQ * (H / G) < GM_ROWS ? TQ * (H / G) : GM_ROWS);

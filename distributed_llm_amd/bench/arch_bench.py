@@ -1,9 +1,17 @@
-"""Layer-list (Filevik, Sedopel, Pebodra, Dogilorn, Mugipel) models beside the closest Llama-family model at equal size:
+"""Layer-list (Filevik, Sedopel, Pebodra, Dogilorn, Mugipel, Figotar) models beside the closest Llama-family model at equal size:
 prefill and decode throughput through the engine, and the time of each mixer kernel against its roofline.
 
-``python bench.py --arch-bench [--arch-design filevik|sedopel|pebodra|dogilorn|mugipel] [--arch-size s|m]`` (random
-weights, synthetic tokens).  The default bench workload and its JSON line are untouched; this prints one
+``python bench.py --arch-bench [--arch-design filevik|sedopel|pebodra|dogilorn|mugipel|figotar] [--arch-size s|m]``
+(random weights, synthetic tokens).  The default bench workload and its JSON line are untouched; this prints one
 JSON object of its own.
+
+The Figotar stack repeats windowed grouped-query attention (scores that fall with the distance, growing
+queries, a gate per head), latent attention behind a query latent (rotated part, sinks, a gate per head)
+and an mLSTM, each with a gated gelu feed-forward and norms on both sides of every sublayer; its
+comparison model is a dense Llama of the same width, heads, depth and parameter count, and kernel by
+kernel: attention against Dogilorn's windowed attention and the Llama kernels at the same heads, latent
+attention against Filevik's and, on expanded keys, Mugipel's, the mLSTM against Pebodra's and the other
+recurrences, its small launches against the like launches of the others.
 
 The Mugipel stack alternates chunked grouped-query attention (capped scores, a learned sink per head,
 a sigmoid gate) and latent attention, each beside a dense squared-relu feed-forward that shares its
@@ -94,6 +102,139 @@ MUGIPEL_SIZES = {
     "m": dict(width=2048, layers=12, loop=(4, 8, 2), heads=16, kv_heads=4, dim=128, vdim=128, rot=64, chunk=1024, kv_rank=512,
               ff=8192, vocab=32000),
 }
+
+
+FIGOTAR_SIZES = {
+    "s": dict(width=1024, layers=6, heads=16, kv_heads=4, dim=64, vdim=64, window=1024, lat_heads=16, lat_dim=64, lat_rot=32,
+              lat_v=64, kv_rank=256, q_rank=768, x_heads=8, x_dim=64, x_vdim=128, ff=2816, vocab=32000),
+    "m": dict(width=2048, layers=12, heads=16, kv_heads=4, dim=128, vdim=128, window=1024, lat_heads=16, lat_dim=128, lat_rot=64,
+              lat_v=128, kv_rank=512, q_rank=1536, x_heads=16, x_dim=128, x_vdim=128, ff=5632, vocab=32000),
+}
+
+
+def figotar_raw(z: dict) -> dict:
+    mlp = {"kind": "dense", "ff": z["ff"]}
+    kinds = [
+        {"type": "attention", "mixer": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["vdim"],
+                                        "scale": z["dim"] ** -0.5, "mask": {"size": z["window"]},
+                                        "q_temp": {"coef": 0.1, "every": 4096}}},
+        {"type": "latent_attention", "mixer": {"heads": z["lat_heads"], "dim": z["lat_dim"], "rot_dim": z["lat_rot"], "vdim": z["lat_v"],
+                                               "kv_rank": z["kv_rank"], "q_rank": z["q_rank"],
+                                               "scale": (z["lat_dim"] + z["lat_rot"]) ** -0.5,
+                                               "rot": {"dims": z["lat_rot"], "base": 10000.0}}},
+        {"type": "mlstm", "mixer": {"heads": z["x_heads"], "dim": z["x_dim"], "vdim": z["x_vdim"], "gate_cap": 15.0}},
+    ]
+    return {"architecture": "Figotar", "width": z["width"], "vocab": z["vocab"], "norm": {"eps": 1e-6},
+            "layers": [dict(kinds[i % 3], mlp=mlp) for i in range(z["layers"])]}
+
+
+def figotar_twin(z: dict):
+    """Dense Llama of the same width, depth, vocabulary, attention heads and parameter count."""
+    from ..models.configs import ModelConfig, figotar_config
+    mk = lambda inter: ModelConfig(f"llama-{z['width']}", z["width"], z["layers"], z["heads"], z["kv_heads"], z["dim"], inter,
+                                   z["vocab"], 10000.0, 1e-6, 16384)
+    inter = (figotar_config(figotar_raw(z)).num_params() - mk(0).num_params()) // (3 * z["width"] * z["layers"])
+    return mk(max(64, inter // 64 * 64))
+
+
+def figotar_kernel_rooflines(z: dict, T: int = 4096, B: int = 64, ctx: int = 2048) -> Dict[str, dict]:
+    """Each Figotar kernel alone (bf16): prefill of one T-token sequence, decode of B sequences at
+    ``ctx``; time, the bound resource's minimum time, and their ratio."""
+    from .. import ops
+    from ..models.llama import AttnMeta
+    from ..ops import seqmix
+    dev, bf = "cuda", torch.bfloat16
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)
+    res: Dict[str, dict] = {}
+
+    def rec(name, sec, bytes_, flops, peak_flops):
+        floor = max(bytes_ / PEAK_BW, flops / peak_flops)
+        res[name] = {"us": round(sec * 1e6, 1), "roofline_us": round(floor * 1e6, 2), "x_roofline": round(sec / floor, 1),
+                     "bound": "memory" if bytes_ / PEAK_BW >= flops / peak_flops else "compute"}
+
+    W, H, G, d, dv, Wn, ff = (z[k] for k in ("width", "heads", "kv_heads", "dim", "vdim", "window", "ff"))
+    Hl, dl, rd, dvl, r, qr = (z[k] for k in ("lat_heads", "lat_dim", "lat_rot", "lat_v", "kv_rank", "q_rank"))
+    for tag, qlens, starts in (("prefill", [T], [0]), ("decode", [1] * B, [ctx] * B)):
+        n, S = sum(qlens), len(qlens)
+        qstart = i32([sum(qlens[:i]) for i in range(S)])
+        cxl = [a + b for a, b in zip(starts, qlens)]
+        qlen, cx, rows = i32(qlens), i32(cxl), i32(list(range(S)))
+        pos = i32([p for a, m in zip(starts, qlens) for p in range(a, a + m)])
+        keys = sum((a + (m + 1) / 2) * m for a, m in zip(starts, qlens))                      # causal (query, key) pairs
+        pairs = sum(min(p + 1, Wn) for a, m in zip(starts, qlens) for p in range(a, a + m))   # ... inside the window
+        seen = sum(min(c, Wn + m - 1) for c, m in zip(cxl, qlens))                            # keys any row of a sequence sees
+        nb = (max(cxl) + 15) // 16
+        bt = torch.arange(S * nb, dtype=torch.int32, device=dev).view(S, nb)
+        slots = i32([int(bt[i, p // 16]) * 16 + p % 16 for i, (a, m) in enumerate(zip(starts, qlens)) for p in range(a, a + m)])
+        meta = AttnMeta(slots=None, block_tables=bt, qstart=qstart, qlen=qlen, ctx=cx, tile_seq=None, tile_tok0=None,
+                        last_idx=None, host_qlen=qlens)
+        # windowed attention and its prep
+        kc = (torch.randn(S * nb, G, 16, d, device=dev) * 0.3).to(bf)
+        vc = (torch.randn(S * nb, G, dv, 16, device=dev) * 0.3).to(bf)
+        cols = (H + G) * d + G * dv
+        proj = torch.randn(n, (cols + H + 63) // 64 * 64, device=dev).to(bf)
+        bias, qtab = torch.zeros(cols, device=dev), torch.ones(ctx + T + 8, device=dev)
+        table = ops.rope_cos_sin(ctx + T + 8, rd, 10000.0, dev)
+        prep = lambda: seqmix.rope_prep(proj, H, G, d, dv, table, 0, d ** -0.5, pos, slots, kc, vc, bias=bias, qtab=qtab)
+        q = prep()
+        rec(f"rope_prep_{tag}", _timed(prep), n * cols * 4, n * cols * 3, PEAK_F32)
+        mfma = seqmix.gqa_use_mfma(q, H, G, d, dv, 16)
+        ts, tt = meta.latent_tiles(1, dev, seqmix.gqa_tokens_per_tile(H, G, mfma))
+        sp = seqmix.gqa_splits(int(ts.numel()), G, max(cxl), Wn) if mfma else 1
+        slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / H) for h in range(H)], device=dev)
+        rec(f"attention_{tag}",
+            _timed(lambda: seqmix.paged_gqa_attention(q, kc, vc, bt, qstart, qlen, cx, ts, tt, proj[:, cols:cols + H], mfma, sp,
+                                                      window=Wn, slopes=slopes), 3),
+            seen * G * (d + dv) * 2 + n * H * (d + dv) * 2, pairs * H * 2 * (d + dv), PEAK_BF16)
+        # latent attention: inputs, absorbed form, expanded form
+        cache = (torch.randn(S * nb, 16, r + rd, device=dev) * 0.3).to(bf)
+        down = torch.randn(n, (qr + r + rd + Hl + 63) // 64 * 64, device=dev).to(bf)
+        gate = down[:, qr + r + rd:qr + r + rd + Hl]
+        nw, nq = torch.ones(r, device=dev), torch.ones(qr, device=dev)
+        sinks = torch.zeros(Hl, device=dev)
+        rec(f"latent_kv_write_{tag}",
+            _timed(lambda: seqmix.latent_kv_write(down[:, qr:qr + r + rd], r, nw, 1e-6, pos, table, slots, cache, True, down[:, :qr], nq)),
+            n * (qr + r + rd) * 4, n * (qr + r + rd) * 4, PEAK_F32)
+        qa = (torch.randn(Hl, n, r, device=dev) * 0.3).to(bf)
+        ql = torch.randn(n, Hl * (dl + rd), device=dev).to(bf)
+        lrows = seqmix.latent_rows(qa, r, rd, n, S)
+        ls, lt = meta.latent_tiles(Hl, dev, lrows)
+        rec(f"latent_attention_{tag}",
+            _timed(lambda: seqmix.latent_attention(qa, ql, dl, rd, pos, table, cache, bt, qstart, qlen, cx, ls, lt, 0.1, rows=lrows,
+                                                   half=True, sinks=sinks), 3),
+            sum(cxl) * (r + rd) * 2 + n * Hl * (2 * r + rd) * 2, keys * Hl * 2 * (2 * r + rd), PEAK_BF16)
+        if tag == "prefill":      # what a step of long portions runs
+            uk, uv = (torch.randn(Hl, dl, r, device=dev) * 0.05).to(bf), (torch.randn(Hl, dvl, r, device=dev) * 0.05).to(bf)
+            rec("latent_q_prep_prefill", _timed(lambda: seqmix.latent_q_prep(ql, Hl, dl, rd, pos, table, 0.1, True)),
+                n * Hl * (dl + rd) * 4, n * Hl * (dl + 4 * rd), PEAK_F32)
+            rec("latent_expand_prefill", _timed(lambda: seqmix.latent_expand(cache, bt, cx, uk, uv)),
+                sum(cxl) * (r + rd + Hl * (dl + rd + dvl)) * 2, sum(cxl) * Hl * (dl + dvl) * r * 2, PEAK_BF16)
+            qx = seqmix.latent_q_prep(ql, Hl, dl, rd, pos, table, 0.1, True)
+            ek, ev, et = seqmix.latent_expand(cache, bt, cx, uk, uv)
+            xm = seqmix.gqa_use_mfma(qx, Hl, Hl, dl + rd, dvl, 16)
+            xs, xt = meta.latent_tiles(1, dev, seqmix.gqa_tokens_per_tile(Hl, Hl, xm))
+            rec("latent_expanded_attention_prefill",
+                _timed(lambda: seqmix.paged_gqa_attention(qx, ek, ev, et, qstart, qlen, cx, xs, xt, gate, xm, 1, all_rows=True, sinks=sinks)),
+                sum(cxl) * Hl * (dl + rd + dvl) * 2 + n * Hl * (dl + rd + dvl) * 2, keys * Hl * 2 * (dl + rd + dvl), PEAK_BF16)
+        o = torch.randn(Hl, n, dvl, device=dev).to(bf)
+        oh = torch.empty(n, Hl * dvl, device=dev, dtype=bf)
+        rec(f"gate_heads_{tag}", _timed(lambda: seqmix.gate_heads(o, gate, oh)), n * Hl * dvl * 4, n * Hl * dvl * 2, PEAK_F32)
+        # mLSTM
+        Hx, dx, dvx = z["x_heads"], z["x_dim"], z["x_vdim"]
+        px = torch.randn(n, 2 * Hx * (dx + dvx + 1), device=dev).to(bf)
+        sx = torch.zeros(S, Hx, dx, dvx, device=dev)
+        nm = torch.zeros(S, Hx, seqmix.scan_col_blocks(dvx), dx + 1, device=dev)
+        gb, hw = torch.zeros(2 * Hx, device=dev), torch.ones(Hx * dvx, device=dev)
+        rec(f"mlstm_{tag}", _timed(lambda: seqmix.mlstm(px, Hx, dx, dvx, gb, 15.0, sx, nm, 1e-6, hw, qstart, qlen, cx, rows)),
+            n * (2 * Hx * dx + 3 * Hx * dvx) * 2 + (S * Hx * dx * dvx * 8 if tag == "decode" else 0),
+            n * Hx * dx * (dvx + 1) * 4, PEAK_F32)
+        # gated gelu, a sublayer's tail
+        gu, gbias = torch.randn(n, 2 * ff, device=dev).to(bf), torch.zeros(2 * ff, device=dev)
+        rec(f"glu_act_{tag}", _timed(lambda: seqmix.glu_act(gu, gbias, "gelu_tanh")), n * ff * 6, n * ff * 14, PEAK_F32)
+        x, y, w = torch.randn(n, W, device=dev), torch.randn(n, W, device=dev).to(bf), torch.ones(W, device=dev)
+        h = torch.empty(n, W, device=dev, dtype=bf)
+        rec(f"resadd_norm_{tag}", _timed(lambda: seqmix.resadd_norm(y, w, 1e-6, x, w, h, bias=w)), n * W * 12, n * W * 10, PEAK_F32)
+    return res
 
 
 def mugipel_raw(z: dict) -> dict:
@@ -664,7 +805,30 @@ def llama_kernel_rooflines(T: int = 4096, B: int = 64, ctx: int = 2048, nq: int 
 
 
 def run(size: str = "s", kernels_only: bool = False, design: str = "filevik") -> dict:
-    from ..models.configs import dogilorn_config, filevik_config, mugipel_config, pebodra_config, sedopel_config
+    from ..models.configs import (dogilorn_config, figotar_config, filevik_config, mugipel_config, pebodra_config,
+                                  sedopel_config)
+    if design == "figotar":
+        z = FIGOTAR_SIZES[size]
+        out = {"bench": "arch", "design": design, "size": size, "dtype": "bf16", "data": "synthetic", "sizes": z}
+        out["figotar_kernels"] = figotar_kernel_rooflines(z)
+        # the like kernels at like sizes: attention inside a window (Dogilorn) and the Llama kernels at the same
+        # heads, latent attention with a rotated part (Filevik) and on expanded keys (Mugipel), mLSTM (Pebodra)
+        out["dogilorn_kernels"] = dogilorn_kernel_rooflines(dict(DOGILORN_SIZES[size], heads=z["heads"], kv_heads=z["kv_heads"],
+                                                                 dim=z["dim"], vdim=z["vdim"], window=z["window"], dense_ff=z["ff"]))
+        out["filevik_kernels"] = kernel_rooflines(dict(SIZES[size], lat_heads=z["lat_heads"], lat_dim=z["lat_dim"], lat_rot=z["lat_rot"],
+                                                       lat_v=z["lat_v"], kv_rank=z["kv_rank"]))
+        out["mugipel_kernels"] = mugipel_kernel_rooflines(dict(MUGIPEL_SIZES[size], heads=z["lat_heads"], kv_heads=z["kv_heads"],
+                                                               dim=z["lat_dim"], vdim=z["lat_v"], kv_rank=z["kv_rank"], ff=z["ff"]))
+        out["pebodra_kernels"] = pebodra_kernel_rooflines(dict(PEBODRA_SIZES[size], x_heads=z["x_heads"], x_dim=z["x_dim"],
+                                                               x_vdim=z["x_vdim"]))
+        out["llama_kernels"] = llama_kernel_rooflines(nq=z["heads"], nkv=z["kv_heads"], d=z["dim"])
+        if not kernels_only:
+            prompts, batches = [512, 2048], [1, 16, 64]
+            out["figotar"] = engine_throughput(figotar_config(figotar_raw(z), name=f"figotar-{size}"), prompts, batches, ctx=1024,
+                                               new=32, rows=64)
+            out["llama"] = engine_throughput(figotar_twin(z), prompts, batches, ctx=1024, new=32, rows=64)
+        print(json.dumps(out))
+        return out
     if design == "mugipel":
         z = MUGIPEL_SIZES[size]
         out = {"bench": "arch", "design": design, "size": size, "dtype": "bf16", "data": "synthetic", "sizes": z}
