@@ -66,7 +66,8 @@ int dllm_ssd_scan(const void*, long, const void*, long, int, int, int, int, int,
                   float*, const int*, const int*, const int*, const int*, int, float*, hipStream_t);
 int dllm_latent_q_prep(const void*, long, int, int, int, int, int, const int*, const float*, int, float, void*, long, hipStream_t);
 int dllm_mlstm(const void*, long, int, int, int, int, const float*, float, float*, float*, int, float, const float*, const int*,
-               const int*, const int*, const int*, int, long, float*, void*, hipStream_t);
+               const int*, const int*, const int*, int, long, float*, void*, int, hipStream_t);
+int dllm_mlstm_chunk_ok(int, long, int, int);
 int dllm_qk_norm_prep(const void*, long, int, const float*, int, int, int, int, int, const float*, const float*, const float*,
                       int, int, float, float, const int*, const int*, void*, void*, void*, long, int, hipStream_t);
 int dllm_diff_combine(const float*, void*, int, long, int, int, int, float, float, float, hipStream_t);
@@ -2015,9 +2016,11 @@ void ssd_scan(torch::Tensor xbc, torch::Tensor proj, int64_t dt_col, int64_t H, 
 
 void mlstm(torch::Tensor proj, int64_t H, int64_t d, int64_t dv, torch::Tensor gate_b, double cap, torch::Tensor state,
            torch::Tensor nm, double eps, torch::Tensor norm_w, torch::Tensor qstart, torch::Tensor qlen, torch::Tensor ctx,
-           torch::Tensor rows, torch::Tensor raw, torch::Tensor out) {
+           torch::Tensor rows, torch::Tensor raw, torch::Tensor out, bool chunked) {
   const bool f = act_f32(proj, "proj");
   check_rows2d(proj, "proj");
+  TORCH_CHECK(!chunked || (dllm_mlstm_chunk_ok(f, proj.stride(0), (int)d, (int)dv) && (uintptr_t)proj.data_ptr() % 16 == 0),
+              "shape outside the chunk form's range");
   check_f32(gate_b, "gate biases");
   check_f32(state, "state");
   check_f32(nm, "normaliser state");
@@ -2038,7 +2041,8 @@ void mlstm(torch::Tensor proj, int64_t H, int64_t d, int64_t dv, torch::Tensor g
   auto m = seq_meta(qstart, qlen, ctx, rows, state.size(0));
   const int rc = dllm_mlstm(proj.data_ptr(), proj.stride(0), f, (int)H, (int)d, (int)dv, gate_b.data_ptr<float>(), (float)cap,
                             state.data_ptr<float>(), nm.data_ptr<float>(), (int)ncb, (float)eps, norm_w.data_ptr<float>(),
-                            m.qstart, m.qlen, m.ctx, m.rows, m.S, (long)T, raw.data_ptr<float>(), out.data_ptr(), stream());
+                            m.qstart, m.qlen, m.ctx, m.rows, m.S, (long)T, raw.data_ptr<float>(), out.data_ptr(), (int)chunked,
+                            stream());
   TORCH_CHECK(rc != -2, "key width outside the kernel's range");
   ok(rc, "mlstm");
 }
@@ -2418,7 +2422,10 @@ PYBIND11_MODULE(_hip_kernels, m) {
   m.def("gated_group_norm", &gated_group_norm);
   m.def("outer_scan_cols", []() { return dllm_outer_scan_cols(); });
   m.def("ssd_scan", &ssd_scan);
-  m.def("mlstm", &mlstm);
+  m.def("mlstm", &mlstm, py::arg("proj"), py::arg("heads"), py::arg("dim"), py::arg("vdim"), py::arg("gate_b"), py::arg("cap"),
+        py::arg("state"), py::arg("nm"), py::arg("eps"), py::arg("norm_w"), py::arg("qstart"), py::arg("qlen"), py::arg("ctx"),
+        py::arg("rows"), py::arg("raw"), py::arg("out"), py::arg("chunked") = false);
+  m.def("mlstm_chunk_ok", [](bool f32, int64_t ld, int64_t d, int64_t dv) { return dllm_mlstm_chunk_ok(f32, ld, (int)d, (int)dv) != 0; });
   m.def("qk_norm_prep", &qk_norm_prep);
   m.def("diff_combine", &diff_combine);
   m.def("causal_conv_silu", &causal_conv_silu, py::arg("x"), py::arg("w"), py::arg("b"), py::arg("state"), py::arg("qstart"),

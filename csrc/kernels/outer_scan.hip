@@ -9,7 +9,7 @@
 //              (0 at the start): m' = max(f + m, i), a = exp(f + m - m'), b = exp(i - m');  a
 //              normaliser n_t = a n + b k rides along as one more value column (v = 1), and
 //              y = S^T q / (max(|n . q|, exp(-m')) + 1e-6).  mlstm_finish: heads to unit RMS, weight,
-//              sigmoid gate.
+//              sigmoid gate.  Prompt portions of bf16 models run the chunk-parallel form (mlstm_chunk.hip).
 //
 // One workgroup per (16 value columns, head, sequence); thread = (column, strip of state rows): a
 // thread keeps rows strip, strip + strips, ... of its column in registers.  Tokens run in groups of
@@ -266,21 +266,27 @@ extern "C" int dllm_ssd_scan(const void* xbc, long ld, const void* gates, long l
                                       N, dv);
 }
 
-// proj [T, ld] = q | k | v | output gate | input-gate logits | forget-gate logits; gate_b = both gates' biases
+extern "C" int dllm_mlstm_chunk(const void*, long, int, int, int, const float*, float, float*, float*, int, const int*, const int*,
+                                const int*, const int*, int, float*, hipStream_t);
+
+// proj [T, ld] = q | k | v | output gate | input-gate logits | forget-gate logits; gate_b = both gates' biases;
+// chunked: the chunk-parallel form (bf16)
 extern "C" int dllm_mlstm(const void* proj, long ld, int f32, int H, int d, int dv, const float* gate_b, float cap,
                           float* state, float* nm, int NCB, float eps, const float* norm_w, const int* qstart,
                           const int* qlen, const int* ctx, const int* rows, int S, long T, float* raw, void* out,
-                          hipStream_t st) {
+                          int chunked, hipStream_t st) {
   if (T <= 0) return 0;
-  if (H < 1 || d < 1 || dv < 1 || !(cap > 0.f) || NCB != (dv + OS_COLS - 1) / OS_COLS) return -1;
+  if (H < 1 || d < 1 || dv < 1 || !(cap > 0.f) || NCB != (dv + OS_COLS - 1) / OS_COLS || (chunked && f32)) return -1;
   const long lds = outer_lds<true>(d);
-  if (lds > 150 * 1024) return -2;
+  if (!chunked && lds > 150 * 1024) return -2;
   const dim3 grid(NCB, H, S);
   const int kc = H * d, vc = 2 * H * d, gc = 2 * H * d + H * dv, ic = gc + H * dv, fc = ic + H;
   const float qs = 1.f / sqrtf((float)d);
   int rc = 0;
   if (S > 0) {
-    if (f32)
+    if (chunked)
+      rc = dllm_mlstm_chunk(proj, ld, H, d, dv, gate_b, cap, state, nm, NCB, qstart, qlen, ctx, rows, S, raw, st);
+    else if (f32)
       rc = launch_outer_npt<float, true>(d, grid, lds, st, proj, ld, kc, 0, 1, proj, ld, vc, proj, ld, ic, fc, gate_b, gate_b + H,
                                          (const float*)nullptr, cap, qs, state, nm, NCB, qstart, qlen, ctx, rows, raw, H, d, dv);
     else

@@ -449,20 +449,28 @@ def gated_group_norm(y, z, w, groups, eps, out_dtype) -> torch.Tensor:
     return out
 
 
-def mlstm(proj, heads, dim, vdim, gate_b, cap, state, nm, eps, norm_w, qstart, qlen, ctx, rows) -> torch.Tensor:
+MLSTM_CHUNK_MIN = 8    # average new tokens per sequence from which the chunk-parallel kernel runs (bf16)
+
+
+def mlstm(proj, heads, dim, vdim, gate_b, cap, state, nm, eps, norm_w, qstart, qlen, ctx, rows,
+          chunked: Optional[bool] = None) -> torch.Tensor:
     """Matrix-memory LSTM over proj [T, q | k | v | output gate | input-gate logits | forget-gate
     logits] (``gate_b``: the two gates' biases): capped exponential input gate, sigmoid forget gate in
     log space, running maximum from 0, normaliser max(|n . q|, exp(-m)) + 1e-6; heads to unit RMS times
     ``norm_w`` times sigmoid(gate).  state [slots, heads, dim, vdim] f32, nm [slots, heads,
-    scan_col_blocks(vdim), dim + 1] f32 (n and m)."""
+    scan_col_blocks(vdim), dim + 1] f32 (n and m).  ``chunked`` (GPU, bf16): the chunk-parallel kernel on the
+    matrix cores or the token-by-token one; default by the step's tokens per sequence and the shape."""
     ext = _native(proj)
     if ext is None:
         return ref.mlstm(proj, heads, dim, vdim, gate_b, cap, state, nm, eps, norm_w, qstart, qlen, ctx, rows)
     T = proj.shape[0]
     raw = torch.zeros((T, heads * vdim), dtype=torch.float32, device=proj.device)
     out = torch.empty((T, heads * vdim), dtype=proj.dtype, device=proj.device)      # the finish kernel writes every row
+    if chunked is None:
+        chunked = (T >= MLSTM_CHUNK_MIN * qstart.numel() and os.environ.get("DLLM_MLSTM_CHUNK", "1") == "1" and
+                   proj.data_ptr() % 16 == 0 and ext.mlstm_chunk_ok(proj.dtype == torch.float32, proj.stride(0), int(dim), int(vdim)))
     ext.mlstm(proj, int(heads), int(dim), int(vdim), gate_b, float(cap), state, nm, float(eps), norm_w, qstart, qlen,
-              ctx, rows, raw, out)
+              ctx, rows, raw, out, bool(chunked))
     return out
 
 

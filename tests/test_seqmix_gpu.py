@@ -495,6 +495,35 @@ def test_mlstm(dt, case, H, d, dv):
     torch.testing.assert_close(nm1, nm2, atol=2e-4, rtol=2e-4)
 
 
+@pytest.mark.parametrize("case", CASES + [([200, 63, 1, 64], [0, 5, 9, 130]), ([129, 128], [0, 7])])
+@pytest.mark.parametrize("H,d,dv", [(4, 40, 48), (3, 64, 8), (2, 128, 128), (1, 8, 72), (2, 96, 40)])
+@pytest.mark.parametrize("cap,gain", [(3.0, 4.0), (15.0, 8.0), (6.0, 0.5)])
+def test_mlstm_chunk_form(case, H, d, dv, cap, gain):
+    """The chunk-parallel kernel against the reference and the token-by-token kernel: portions of any length
+    that start from zero or from a slot, weak and strong gates; outputs, memory, normaliser, maximum."""
+    torch.manual_seed(39)
+    qlens, starts = case
+    T, qstart, qlen, ctx, rows, _ = batch(qlens, starts)
+    slots, n = len(qlens) + 1, 2 * H * (d + dv + 1)
+    proj = torch.randn(T, (n + 7) // 8 * 8 + 8, device=DEV).to(torch.bfloat16)
+    proj[:, 2 * H * (d + dv):] *= gain
+    gate_b = torch.cat([torch.randn(H), 2.0 + torch.randn(H)]).to(DEV)
+    w = torch.rand(H * dv, device=DEV) + 0.5
+    st = torch.randn(slots, H, d, dv, device=DEV)
+    nm = torch.randn(slots, H, 1, d + 1, device=DEV).repeat(1, 1, seqmix.scan_col_blocks(dv), 1).contiguous()
+    res = []
+    for form in (True, False, None):
+        s, m = st.clone(), nm.clone()
+        args = (proj, H, d, dv, gate_b, cap, s, m, 1e-5, w, qstart, qlen, ctx, rows)
+        res.append((ref.mlstm(*args) if form is None else seqmix.mlstm(*args, chunked=form), s, m))
+    for o, s, m in res[:2]:
+        # (a head's output is scaled to unit RMS: where normaliser and output are near zero together their rounding is not)
+        diff = (o.float() - res[2][0].float()).abs()
+        assert float((diff > 2e-2 + 2e-2 * res[2][0].float().abs()).float().mean()) < 1e-3
+        torch.testing.assert_close(s, res[2][1], atol=1e-3, rtol=1e-3)
+        torch.testing.assert_close(m, res[2][2], atol=1e-3, rtol=1e-3)
+
+
 @pytest.mark.parametrize("dt", DTYPES)
 def test_polynorm_swiglu_softcap(dt):
     torch.manual_seed(17)
