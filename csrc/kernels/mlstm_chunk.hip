@@ -15,7 +15,8 @@
 // split into bf16 hi + lo parts (two MFMAs, 16 bits of mantissa): the weights P, the weighted values, the
 // state as the queries read it.  The state itself stays in f32 accumulators from chunk to chunk.  The
 // normaliser is a 33rd value column whose values are 1.  The next chunk's rows are fetched into registers
-// under the current chunk's products.
+// under the current chunk's products.  Exponents are kept in base 2 (E, R, m, F times log2 e), gates use the
+// hardware exponential, logarithm and reciprocal.
 #include "common.h"
 
 namespace {
@@ -59,7 +60,14 @@ __device__ __forceinline__ void split4(const float (&x)[4], uint2& hi, uint2& lo
 }
 __device__ __forceinline__ bf16x8 frag(const u16* p) { return __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(p)); }
 
-__device__ __forceinline__ float logsigmoid_f(float x) { return x < 0.f ? x - log1pf(expf(x)) : -log1pf(expf(-x)); }
+constexpr float LOG2E = 1.44269504088896f;
+__device__ __forceinline__ float ex2(float x) { return __builtin_amdgcn_exp2f(x); }
+// log2(e) cap tanh(x / cap), from cap - 2 cap / (exp(2 x / cap) + 1); an overflowing exponential gives cap
+__device__ __forceinline__ float cap2(float x, float cap) {
+  return LOG2E * cap * (1.f - 2.f * __builtin_amdgcn_rcpf(ex2(2.f * LOG2E * x / cap) + 1.f));
+}
+// log2 sigmoid(y / log2 e)
+__device__ __forceinline__ float logsigmoid2(float y) { return fminf(y, 0.f) - __builtin_amdgcn_logf(1.f + ex2(-fabsf(y))); }
 
 template <int KD> constexpr long mc_lds() {
   return 2L * (2 * MC_L * (KD + 8) + KD * MC_PS + 3 * MC_V * MC_PS + 4 * 2 * 16 * MC_PS + 2 * (MC_V + 1) * (KD + 8) + 2 * MC_L) +
@@ -93,7 +101,7 @@ __global__ void __launch_bounds__(256) mlstm_chunk_kernel(const u16* __restrict_
   u16* stl = sth + (MC_V + 1) * KST;
   u16* wnh = stl + (MC_V + 1) * KST;               // [L]: exp(E_s - R_L), hi and lo
   u16* wnl = wnh + MC_L;
-  float* Es = reinterpret_cast<float*>(wnl + MC_L);   // [L] each: E, R, qs exp(m - R), exp(-m_t)
+  float* Es = reinterpret_cast<float*>(wnl + MC_L);   // [L] each: E + log2 qs, R, qs exp(m - R), exp(-m_t)
   float* Rs = Es + MC_L;
   float* Xs = Rs + MC_L;
   float* Ds = Xs + MC_L;
@@ -123,7 +131,8 @@ __global__ void __launch_bounds__(256) mlstm_chunk_kernel(const u16* __restrict_
         }
         S[j][cb][i] = v;
       }
-  float m = p0 > 0 ? np[d] : 0.f;
+  float m = p0 > 0 ? np[d] * LOG2E : 0.f;
+  const float lqs = __builtin_amdgcn_logf(qs);
   const bf16x8 zero8 = __builtin_bit_cast(bf16x8, make_uint4(0u, 0u, 0u, 0u));
   const bf16x8 ones8 = __builtin_bit_cast(bf16x8, lr == 0 ? make_uint4(0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u)
                                                           : make_uint4(0u, 0u, 0u, 0u));
@@ -158,22 +167,22 @@ __global__ void __launch_bounds__(256) mlstm_chunk_kernel(const u16* __restrict_
     // gates, a lane per token (every wave for itself)
     float ig = -INFINITY, fg = 0.f;
     if (lane < nt) {
-      ig = cap * tanhf((bf2f(gi) + bi) / cap);
-      fg = logsigmoid_f(cap * tanhf((bf2f(gf) + bf) / cap));
+      ig = cap2(bf2f(gi) + bi, cap);
+      fg = logsigmoid2(cap2(bf2f(gf) + bf, cap));
     }
     const float F = scan_add(fg), E = ig - F, R = fmaxf(m, scan_max(E));
-    const float RL = last_lane(R), decay = expf(m - RL), wlast = expf(E - RL);
+    const float RL = last_lane(R), decay = ex2(m - RL), wlast = ex2(E - RL);
     const float wv = __shfl(wlast, 16 * wave + (lane >> 2));     // the weight of the token whose values this thread moves
     __syncthreads();     // the previous chunk is consumed
     if (wave == 0) {
-      Es[lane] = E;
+      Es[lane] = E + lqs;
       Rs[lane] = R;
-      Xs[lane] = qs * expf(m - R);
-      Ds[lane] = expf(-(F + R));
+      Xs[lane] = qs * ex2(m - R);
+      Ds[lane] = ex2(-(F + R));
     } else if (wave == 1) {
-      const u16 hi = f2bf(wlast);
-      wnh[lane] = hi;
-      wnl[lane] = f2bf(wlast - bf2f(hi));
+      const uint32_t hi = pack2(wlast, 0.f);
+      wnh[lane] = (u16)hi;
+      wnl[lane] = (u16)pack2(wlast - __uint_as_float(hi << 16), 0.f);
     }
     m = last_lane(F) + RL;
 #pragma unroll
@@ -183,15 +192,18 @@ __global__ void __launch_bounds__(256) mlstm_chunk_kernel(const u16* __restrict_
       *reinterpret_cast<uint4*>(ksh + (16 * (t & 3) + (t >> 2)) * KST + c) = pk[f];
     }
     {
-      const u16* pe = reinterpret_cast<const u16*>(&pv);
+      const uint32_t pe[4] = {pv.x, pv.y, pv.z, pv.w};
 #pragma unroll
-      for (int x = 0; x < 8; ++x) {
-        const float w = wv * bf2f(pe[x]);
-        const u16 hi = f2bf(w);
-        const int o = (vc8 + x) * MC_PS + vtok;
-        vt[o] = pe[x];
-        wh[o] = hi;
-        wl[o] = f2bf(w - bf2f(hi));
+      for (int x = 0; x < 4; ++x) {
+        const float w0 = wv * __uint_as_float(pe[x] << 16), w1 = wv * __uint_as_float(pe[x] & 0xffff0000u);
+        const uint32_t hi = pack2(w0, w1), lo = pack2(w0 - __uint_as_float(hi << 16), w1 - __uint_as_float(hi & 0xffff0000u));
+        const int o = (vc8 + 2 * x) * MC_PS + vtok;
+        vt[o] = (u16)pe[x];
+        vt[o + MC_PS] = (u16)(pe[x] >> 16);
+        wh[o] = (u16)hi;
+        wh[o + MC_PS] = (u16)(hi >> 16);
+        wl[o] = (u16)lo;
+        wl[o + MC_PS] = (u16)(lo >> 16);
       }
     }
 #pragma unroll
@@ -241,7 +253,7 @@ __global__ void __launch_bounds__(256) mlstm_chunk_kernel(const u16* __restrict_
       float p[4];
 #pragma unroll
       for (int kb = 0; kb < 4; ++kb) {
-        const float w = sacc[kb][i] * qs * expf(ev[kb] - rv[i]);
+        const float w = sacc[kb][i] * ex2(ev[kb] - rv[i]);
         p[kb] = 4 * lr + kb <= row0 + i ? w : 0.f;
       }
       uint2 hi, lo;
@@ -283,7 +295,7 @@ __global__ void __launch_bounds__(256) mlstm_chunk_kernel(const u16* __restrict_
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const float nq = __shfl(oi[2][i] + xv[i] * os[2][i], lane & 48);      // the row's normaliser: column 0 of its block
-        const float inv = 1.f / (fmaxf(fabsf(nq), dn[i]) + 1e-6f);
+        const float inv = __builtin_amdgcn_rcpf(fmaxf(fabsf(nq), dn[i]) + 1e-6f);
         const int t = row0 + i;
         if (t >= nt) continue;
         float* dst = raw + (long)(q0 + t0 + t) * ((long)H * dv) + (long)h * dv + v0 + lr;
@@ -330,8 +342,8 @@ __global__ void __launch_bounds__(256) mlstm_chunk_kernel(const u16* __restrict_
         }
       }
   if (tid == 0) {
-    np[d] = m;
-    if (2 * (int)blockIdx.x + 1 < NCB) np[2 * d + 1] = m;
+    np[d] = m / LOG2E;
+    if (2 * (int)blockIdx.x + 1 < NCB) np[2 * d + 1] = m / LOG2E;
   }
 }
 
