@@ -5,9 +5,9 @@
 // up-projection follows as a per-head batched GEMM).  Only [c_j | kr_j] is cached, paged in
 // 16-token blocks.
 //
-//   latent_kv_write   one wave per token: RMS-norm the latent (f32), rotate the shared key part
-//                     (pairs (2i, 2i + 1) or (i, i + rot / 2)), write both into the token's cache slot; a
-//                     second wave norms the query latent that the same projection made
+//   latent_kv_write   one workgroup per token: RMS-norm the latent (f32), rotate the shared key part
+//                     (pairs (2i, 2i + 1) or (i, i + rot / 2)), write both into the token's cache slot, and
+//                     norm the query latent that the same projection made
 //   latent_q_prep     queries of the expanded form: the rotated part rotated, everything scaled
 //   latent_prep       latent_kv_write without a rotated part for a layer whose feed-forward shares the
 //                     projection: the same launch squares the relu of the up columns
@@ -53,11 +53,12 @@ __device__ __forceinline__ float rotated(const T* r, int c, int half, int hf, co
   return first ? v * cs[a] - w * cs[half + a] : v * cs[a] + w * cs[half + a];
 }
 
-// wave 0: the token's latent and shared key part into its cache slot.  wave 1 (launched when qsrc):
-// qdst = rmsnorm(qsrc row) qw, the query latent.  zl (optional, [zh, tokens, rank]): a padding token's
-// rows, which no attention tile writes, are cleared.
+// wave 0: the token's latent and shared key part into its cache slot.  waves 1 to 3 (launched when qsrc):
+// qdst = rmsnorm(qsrc row) qw, the query latent.  Rows of up to 8 values a lane stay in registers between
+// the sum and the store.  zl (optional, [zh, tokens, rank]): a padding token's rows, which no attention
+// tile writes, are cleared.
 template <typename T>
-__global__ void __launch_bounds__(128) latent_kv_write_kernel(const T* __restrict__ ckv, long ld, int rank, int rot,
+__global__ void __launch_bounds__(256) latent_kv_write_kernel(const T* __restrict__ ckv, long ld, int rank, int rot,
                                                               const float* __restrict__ w, float eps,
                                                               const int* __restrict__ pos,
                                                               const float* __restrict__ cos_sin, int tab_w,
@@ -65,26 +66,37 @@ __global__ void __launch_bounds__(128) latent_kv_write_kernel(const T* __restric
                                                               const T* __restrict__ qsrc, long ldqs, int qn,
                                                               const float* __restrict__ qw, T* __restrict__ qdst,
                                                               T* __restrict__ zl, int zh) {
-  const int t = blockIdx.x, lane = threadIdx.x & 63;
+  constexpr int NR = 8;      // values a lane keeps
+  __shared__ float red[3];
+  const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int slot = slots[t];
   if (zl && slot < 0)
     for (int i = threadIdx.x; i < zh * rank; i += blockDim.x) stf(zl + ((long)(i / rank) * gridDim.x + t) * rank + i % rank, 0.f);
-  if (threadIdx.x >= 64) {
-    const T* r = qsrc + (long)t * ldqs;
-    float s = 0.f;
-    for (int i = lane; i < qn; i += 64) { const float v = ldf(r + i); s += v * v; }
-    const float rs = 1.f / sqrtf(wave_sum(s) / (float)qn + eps);
-    for (int i = lane; i < qn; i += 64) stf(qdst + (long)t * qn + i, ldf(r + i) * rs * qw[i]);
-    return;
+  const bool is_q = wave > 0;
+  const T* r = is_q ? qsrc + (long)t * ldqs : ckv + (long)t * ld;
+  const int n = is_q ? qn : rank, i0 = is_q ? threadIdx.x - 64 : lane, step = is_q ? 192 : 64;
+  float v[NR], s = 0.f;
+#pragma unroll
+  for (int j = 0; j < NR; ++j) {
+    v[j] = i0 + j * step < n ? ldf(r + i0 + j * step) : 0.f;
+    s += v[j] * v[j];
   }
-  if (slot < 0) return;
-  const T* r = ckv + (long)t * ld;
-  float s = 0.f;
-  for (int i = lane; i < rank; i += 64) { const float v = ldf(r + i); s += v * v; }
+  for (int i = i0 + NR * step; i < n; i += step) { const float x = ldf(r + i); s += x * x; }
   s = wave_sum(s);
-  const float rs = 1.f / sqrtf(s / (float)rank + eps);
-  T* dst = cache + (long)slot * (rank + rot);
-  for (int i = lane; i < rank; i += 64) stf(dst + i, ldf(r + i) * rs * w[i]);
+  if (qsrc) {      // uniform: the query latent's sum over its three waves
+    if (is_q && lane == 0) red[wave - 1] = s;
+    __syncthreads();
+    if (is_q) s = red[0] + red[1] + red[2];
+  }
+  if (!is_q && slot < 0) return;
+  const float rs = 1.f / sqrtf(s / (float)n + eps);
+  const float* g = is_q ? qw : w;
+  T* dst = is_q ? qdst + (long)t * qn : cache + (long)slot * (rank + rot);
+#pragma unroll
+  for (int j = 0; j < NR; ++j)
+    if (i0 + j * step < n) stf(dst + i0 + j * step, v[j] * rs * g[i0 + j * step]);
+  for (int i = i0 + NR * step; i < n; i += step) stf(dst + i, ldf(r + i) * rs * g[i]);
+  if (is_q) return;
   const float* cs = cos_sin + (long)pos[t] * tab_w;
   const int half = rot >> 1;
   for (int i = lane; i < rot; i += 64) stf(dst + rank + i, rotated(r + rank, i, half, hf, cs));
@@ -851,7 +863,7 @@ extern "C" int dllm_latent_kv_write(const void* ckv, long ld, int f32, int rank,
                                     int zh, hipStream_t st) {
   if (T <= 0) return 0;
   if (rot < 0 || (rot & 1) || rot > tab_w || rank < 1 || (qsrc && (qn < 1 || !qw || !qdst))) return -1;
-  const dim3 block(qsrc ? 128 : 64);
+  const dim3 block(qsrc ? 256 : 64);
   if (f32)
     hipLaunchKernelGGL(latent_kv_write_kernel<float>, dim3(T), block, 0, st, (const float*)ckv, ld, rank, rot, w, eps, pos,
                        cos_sin, tab_w, slots, (float*)cache, hf, (const float*)qsrc, ldqs, qn, qw, (float*)qdst, (float*)zl, zh);

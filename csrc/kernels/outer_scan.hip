@@ -172,16 +172,24 @@ __global__ void __launch_bounds__(256) outer_scan_kernel(const T* __restrict__ k
   }
 }
 
-// each head's row of `raw` to unit RMS, times w[head, :], times sigmoid(gate): one wave per (token, head)
+// each head's row of `raw` to unit RMS, times w[head, :], times sigmoid(gate): one wave per (token, head);
+// rows of no sequence (graph padding, `raw` not written) become zeros
 template <typename T>
 __global__ void __launch_bounds__(256) head_norm_gate_kernel(const float* __restrict__ raw, const T* __restrict__ gate, long ldg,
                                                              const float* __restrict__ w, T* __restrict__ out, long units,
-                                                             int H, int dv, float eps) {
+                                                             int H, int dv, float eps, const int* __restrict__ qstart,
+                                                             const int* __restrict__ qlen, int S) {
   const long u = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   const int lane = threadIdx.x & 63;
   if (u >= units) return;
   const long tok = u / H;
   const int h = (int)(u % H);
+  bool live = false;
+  for (int s = lane; s < S; s += 64) live |= tok >= qstart[s] && tok < qstart[s] + qlen[s];
+  if (!__any(live)) {
+    for (int i = lane; i < dv; i += 64) stf(out + u * dv + i, 0.f);
+    return;
+  }
   const float* r = raw + u * dv;
   float s = 0.f;
   for (int i = lane; i < dv; i += 64) s += r[i] * r[i];
@@ -298,9 +306,9 @@ extern "C" int dllm_mlstm(const void* proj, long ld, int f32, int H, int d, int 
   const dim3 g2((unsigned)((units + 3) / 4));
   if (f32)
     hipLaunchKernelGGL(head_norm_gate_kernel<float>, g2, dim3(256), 0, st, raw, (const float*)proj + gc, ld, norm_w, (float*)out,
-                       units, H, dv, eps);
+                       units, H, dv, eps, qstart, qlen, S);
   else
     hipLaunchKernelGGL(head_norm_gate_kernel<u16>, g2, dim3(256), 0, st, raw, (const u16*)proj + gc, ld, norm_w, (u16*)out, units,
-                       H, dv, eps);
+                       H, dv, eps, qstart, qlen, S);
   return (int)hipGetLastError();
 }

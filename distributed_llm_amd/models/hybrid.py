@@ -1062,7 +1062,8 @@ class HybridModel:
         if ln:
             h = seqmix.ls_resadd_ln(x, self.layers[0]["norm1"], self.layers[0]["norm1.b"], eps, self.dtype)
         elif cfg.pre_norm:
-            h = seqmix.rms_rows(x, self.layers[0]["norm1"], eps, out_dtype=self.dtype)
+            h = torch.empty((T, W), dtype=self.dtype, device=x.device)
+            seqmix.scaled_resadd_rms(x, eps, w=self.layers[0]["norm1"], out=h)
         for i, (L, S, cache) in enumerate(zip(self.layers, cfg.layers, kv_caches)):
             m = S.mixer
             if not cfg.pre_norm:

@@ -464,7 +464,7 @@ def mlstm(proj, heads, dim, vdim, gate_b, cap, state, nm, eps, norm_w, qstart, q
     if ext is None:
         return ref.mlstm(proj, heads, dim, vdim, gate_b, cap, state, nm, eps, norm_w, qstart, qlen, ctx, rows)
     T = proj.shape[0]
-    raw = torch.zeros((T, heads * vdim), dtype=torch.float32, device=proj.device)
+    raw = torch.empty((T, heads * vdim), dtype=torch.float32, device=proj.device)   # read for live tokens only
     out = torch.empty((T, heads * vdim), dtype=proj.dtype, device=proj.device)      # the finish kernel writes every row
     if chunked is None:
         chunked = (T >= MLSTM_CHUNK_MIN * qstart.numel() and os.environ.get("DLLM_MLSTM_CHUNK", "1") == "1" and
