@@ -118,6 +118,39 @@ __global__ void __launch_bounds__(256) latent_q_prep_kernel(const T* __restrict_
   }
 }
 
+// The same for bf16 rows of whole 16-byte vectors and rotate-half pairs (dim % 8 == 0, rot % 16 == 0): a
+// thread owns 8 neighbouring unrotated dims, or 8 rotary pairs.
+__global__ void __launch_bounds__(256) latent_q_prep_vec_kernel(const u16* __restrict__ q, long ldq, int H, int dim, int rot,
+                                                                const int* __restrict__ pos, const float* __restrict__ cos_sin,
+                                                                int tab_w, float scale, u16* __restrict__ out, long Tn) {
+  const int w = dim + rot, half = rot >> 1, per = (dim + half) >> 3;      // vectors (or pairs of vectors) of a head
+  const int u = blockIdx.x * 256 + threadIdx.x;
+  if (u >= H * per) return;
+  const int h = u / per, c = 8 * (u - h * per);
+  for (long t = blockIdx.y; t < Tn; t += gridDim.y) {
+    const u16* r = q + t * ldq + (long)h * w;
+    u16* o = out + t * (long)(H * w) + (long)h * w;
+    float a[8];
+    unpack8(ld16(r + c), a);
+    if (c >= dim) {
+      float b[8];
+      unpack8(ld16(r + c + half), b);
+      const float* cs = cos_sin + (long)pos[t] * tab_w + (c - dim);
+#pragma unroll
+      for (int x = 0; x < 8; ++x) {
+        const float cc = cs[x] * scale, sn = cs[half + x] * scale, va = a[x];
+        a[x] = va * cc - b[x] * sn;
+        b[x] = b[x] * cc + va * sn;
+      }
+      st16(o + c + half, pack8(b));
+    } else {
+#pragma unroll
+      for (int x = 0; x < 8; ++x) a[x] *= scale;
+    }
+    st16(o + c, pack8(a));
+  }
+}
+
 // proj row: ... | latent (column ccol, rank wide) | ... | up (column ucol, ff wide) | ...: the latent's RMS
 // norm into the token's cache slot (wave 0 of the token's first workgroup), act[tok] = relu(up)^2
 // (shared by the token's workgroups; vec: rows of whole 16-byte vectors).
@@ -277,6 +310,28 @@ __global__ void __launch_bounds__(256) gate_heads_kernel(const T* __restrict__ o
   const int h = c / dv, i = c - h * dv;
   for (long t = blockIdx.y; t < Tn; t += gridDim.y)
     stf(out + t * ldo + c, ldf(o + ((long)h * Tn + t) * dv + i) / (1.f + expf(-ldf(gate + t * ldg + (ghead ? h : c)))));
+}
+
+// ... for bf16 rows of whole 16-byte vectors (dv % 8 == 0): a thread owns 8 neighbouring entries of a head
+__global__ void __launch_bounds__(256) gate_heads_vec_kernel(const u16* __restrict__ o, const u16* __restrict__ gate, long ldg,
+                                                             u16* __restrict__ out, long ldo, int H, int dv, long Tn, int ghead) {
+  const int c = 8 * (blockIdx.x * 256 + threadIdx.x);
+  if (c >= H * dv) return;
+  const int h = c / dv, i = c - h * dv;
+  for (long t = blockIdx.y; t < Tn; t += gridDim.y) {
+    float v[8], g[8];
+    unpack8(ld16(o + ((long)h * Tn + t) * dv + i), v);
+    if (ghead) {
+      const float s = 1.f / (1.f + __expf(-bf2f(gate[t * ldg + h])));
+#pragma unroll
+      for (int x = 0; x < 8; ++x) v[x] *= s;
+    } else {
+      unpack8(ld16(gate + t * ldg + c), g);
+#pragma unroll
+      for (int x = 0; x < 8; ++x) v[x] *= __builtin_amdgcn_rcpf(1.f + __expf(-g[x]));
+    }
+    st16(out + t * ldo + c, pack8(v));
+  }
 }
 
 constexpr int LROWS = 16;
@@ -877,6 +932,12 @@ extern "C" int dllm_latent_q_prep(const void* q, long ldq, int f32, int H, int d
                                   const float* cos_sin, int tab_w, float scale, void* out, long T, hipStream_t st) {
   if (T <= 0) return 0;
   if (H < 1 || dim < 0 || rot < 0 || (rot & 1) || rot > tab_w || dim + rot < 1) return -1;
+  if (!f32 && (hf || !rot) && dim % 8 == 0 && rot % 16 == 0 && ldq % 8 == 0 && (uintptr_t)q % 16 == 0 && (uintptr_t)out % 16 == 0) {
+    const int units = H * ((dim + rot / 2) / 8);
+    hipLaunchKernelGGL(latent_q_prep_vec_kernel, dim3((units + 255) / 256, (unsigned)(T < 4096 ? T : 4096)), dim3(256), 0, st,
+                       (const u16*)q, ldq, H, dim, rot, pos, cos_sin, tab_w, scale, (u16*)out, T);
+    return (int)hipGetLastError();
+  }
   const dim3 grid((H * (dim + rot) + 255) / 256, (unsigned)(T < 4096 ? T : 4096));
   if (f32)
     hipLaunchKernelGGL(latent_q_prep_kernel<float>, grid, dim3(256), 0, st, (const float*)q, ldq, H, dim, rot, hf, pos, cos_sin,
@@ -1025,6 +1086,12 @@ extern "C" int dllm_gate_heads(const void* o, int f32, const void* gate, long ld
                                int ghead, hipStream_t st) {
   if (T <= 0) return 0;
   if (H < 1 || dv < 1) return -1;
+  if (!f32 && dv % 8 == 0 && ldo % 8 == 0 && (uintptr_t)o % 16 == 0 && (uintptr_t)out % 16 == 0 &&
+      (ghead || (ldg % 8 == 0 && (uintptr_t)gate % 16 == 0))) {
+    hipLaunchKernelGGL(gate_heads_vec_kernel, dim3((H * dv / 8 + 255) / 256, (unsigned)(T < 4096 ? T : 4096)), dim3(256), 0, st,
+                       (const u16*)o, (const u16*)gate, ldg, (u16*)out, ldo, H, dv, T, ghead);
+    return (int)hipGetLastError();
+  }
   const dim3 grid((H * dv + 255) / 256, (unsigned)(T < 4096 ? T : 4096));
   if (f32)
     hipLaunchKernelGGL(gate_heads_kernel<float>, grid, dim3(256), 0, st, (const float*)o, (const float*)gate, ldg, (float*)out,

@@ -158,7 +158,8 @@ def test_latent_attention(dt, case, H, dim, rot, rank, splits, mfma, half):
 
 @pytest.mark.parametrize("dt", DTYPES)
 @pytest.mark.parametrize("half", [False, True])
-@pytest.mark.parametrize("T,H,dim,rot,rank,qr", [(1, 3, 8, 2, 24, 10), (37, 4, 16, 12, 64, 200), (9, 2, 40, 0, 100, 64), (130, 5, 24, 64, 512, 72)])
+@pytest.mark.parametrize("T,H,dim,rot,rank,qr", [(1, 3, 8, 2, 24, 10), (37, 4, 16, 12, 64, 200), (9, 2, 40, 0, 100, 64), (130, 5, 24, 64, 512, 72),
+                                                 (50, 8, 32, 16, 64, 2000)])      # whole vectors everywhere; a query latent beyond the registers
 def test_latent_inputs(dt, half, T, H, dim, rot, rank, qr):
     """Both latents' norms, the rotated key part and the padding rows in one launch; the rotated, scaled
     queries of the expanded form; one gate per head on head-major outputs."""
@@ -170,7 +171,7 @@ def test_latent_inputs(dt, half, T, H, dim, rot, rank, qr):
     nb = (T + 15) // 16 + 1
     slots = torch.randperm(nb * 16, device=DEV)[:T].to(torch.int32)
     slots[0] = -1
-    q = torch.randn(T, H * (dim + rot) + 3, device=DEV).to(dt)
+    q = torch.randn(T, H * (dim + rot) + (8 if T == 50 else 3), device=DEV).to(dt)
     o = torch.randn(H, T, dim, device=DEV).to(dt)
     got = []
     for m in (seqmix, ref):
