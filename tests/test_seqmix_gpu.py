@@ -810,7 +810,7 @@ def test_latent_expand(dt, ctxs, H, d, dv, rank, rot):
 @pytest.mark.parametrize("dt", DTYPES)
 @pytest.mark.parametrize("case", CASES + [([40, 3], [90, 130]), ([1, 1], [300, 77]), ([150], [170])])
 @pytest.mark.parametrize("H,G,d,dv,win", [(4, 2, 16, 8, 5), (6, 2, 88, 56, 64), (3, 3, 40, 72, 1), (8, 1, 64, 64, 100), (7, 1, 56, 88, 0),
-                                          (2, 1, 136, 200, 48), (4, 4, 96, 80, 65), (5, 5, 12, 1, 17)])
+                                          (2, 1, 136, 200, 48), (4, 4, 104, 72, 65), (5, 5, 12, 1, 17)])
 def test_biased_attention_kernels(dt, case, H, G, d, dv, win):
     """Prep (biases, queries times a number of their position, pages, padding rows), then windowed attention
     whose scores fall with the distance, one gate per head, in both kernel forms and every split count."""
